@@ -8,7 +8,11 @@ form a *group*: the group has its own pool of pages, and a request has one
 block table per group, shared by all cache ids of the group — page p holds the
 same token slots in each of them.  A group that keeps all keys gives pages back
 when the request ends; a group with a window also gives back every page the
-window has passed, after each step.
+window has passed, after each step.  A group whose spec names block sizes
+(``pools``) also holds, per request and block size, a table of pages with one
+slot per whole block of so many tokens, for the mean keys and values that
+outlive the tokens; these pages come from the same pool, and the tokens of an
+unfinished block stay until it is whole.
 
 Device layout per group: one tensor ``kv[cache index, 0 = K / 1 = V, page, ...]``;
 a key page is ``[kv head, slot in page, head element]``, a value page is kept
@@ -30,6 +34,7 @@ import torch
 
 from ..parts.base import KVCacheSpec, StateSpec
 from .block_pool import BlockPool, OutOfPages
+from .sizing import pool_pages, state_id
 from .state_slots import StateSlots
 
 
@@ -40,6 +45,7 @@ class CacheGroup:
     pool: BlockPool
     cache_ids: list = field(default_factory=list)
     tables: dict = field(default_factory=dict)   # request -> [page id or -1 per logical block]
+    pool_tables: dict = field(default_factory=dict)   # request -> per block size of the spec, [page ids]
     kv: torch.Tensor | None = None
 
     def index_of(self, cache_id: int) -> int:
@@ -59,8 +65,9 @@ class CacheManager:
     def __init__(self, requirements, page_size: int, num_pages, max_seqs: int,
                  dtype: torch.dtype | None = None, device=None):
         """``requirements``: (cache id, writes, KVCacheSpec | None, StateSpec | None)
-        per layer call.  ``num_pages``: pages of every group's pool, or a dict
-        {KVCacheSpec: pages}.  Device memory is taken only if ``device`` is given."""
+        per layer call, and the state's id where it is not the cache's.  ``num_pages``: pages for the
+        tokens of every group (a group that keeps keys of blocks gets those of its blocks on top),
+        or a dict {KVCacheSpec: all pages of the group's pool}.  Device memory is taken only if ``device`` is given."""
         if page_size <= 0 or page_size % 8:
             raise ValueError(f"page size {page_size} must be a positive multiple of 8")
         self.page_size = int(page_size)
@@ -74,7 +81,9 @@ class CacheManager:
         self.state_tensors: dict[int, torch.Tensor] = {}
         spec_of: dict[int, KVCacheSpec] = {}
         writers = set()
-        for cache_id, writes, kv_spec, state_spec in requirements:
+        for row in requirements:
+            cache_id, writes, kv_spec, state_spec = row[:4]
+            sid = state_id(row)
             if kv_spec is not None:
                 if cache_id in spec_of and spec_of[cache_id] != kv_spec:
                     raise ValueError(f"layer calls sharing cache {cache_id} ask for different caches: "
@@ -83,9 +92,9 @@ class CacheManager:
                 if writes:
                     writers.add(cache_id)
             if state_spec is not None:
-                if cache_id in self._state_specs and self._state_specs[cache_id] != state_spec:
-                    raise ValueError(f"layer calls sharing state {cache_id} ask for different states")
-                self._state_specs[cache_id] = state_spec
+                if sid in self._state_specs and self._state_specs[sid] != state_spec:
+                    raise ValueError(f"layer calls sharing state {sid} ask for different states")
+                self._state_specs[sid] = state_spec
         for cache_id in spec_of:
             if cache_id not in writers:
                 raise ValueError(f"cache {cache_id} is read but no layer call writes it")
@@ -94,7 +103,11 @@ class CacheManager:
             spec = spec_of[cache_id]
             g = by_spec.get(spec)
             if g is None:
-                n = num_pages[spec] if isinstance(num_pages, dict) else num_pages
+                if isinstance(num_pages, dict):
+                    n = num_pages[spec]
+                else:
+                    tokens = int(num_pages) * self.page_size
+                    n = int(num_pages) + sum(-(-(tokens // p) // self.page_size) + self.max_seqs for p in spec.pools)
                 g = CacheGroup(spec, self.page_size, BlockPool(int(n)))
                 by_spec[spec] = g
                 self.groups.append(g)
@@ -146,6 +159,10 @@ class CacheManager:
     def block_table(self, group: int, req) -> list[int]:
         return self.groups[group].tables[req]
 
+    def pool_table(self, group: int, req, which: int) -> list[int]:
+        """Pages of the request's blocks of size ``groups[group].spec.pools[which]``."""
+        return self.groups[group].pool_tables[req][which]
+
     # ---- life of a request ----------------------------------------------
     def add_request(self, req) -> int:
         if req in self.requests:
@@ -155,6 +172,7 @@ class CacheManager:
         self.requests[req] = RequestCacheState(slot, life=self._lives)
         for g in self.groups:
             g.tables[req] = []
+            g.pool_tables[req] = [[] for _ in g.spec.pools]
         for t in self.state_tensors.values():
             t[slot].zero_()
         return slot
@@ -162,8 +180,35 @@ class CacheManager:
     def pages_needed(self, req, n_new: int) -> list[int]:
         """Pages each group must still take so that ``n_new`` more tokens fit."""
         st = self.requests[req]
-        blocks = -(-(st.num_tokens + n_new) // self.page_size)
-        return [max(0, blocks - len(g.tables[req])) for g in self.groups]
+        total = st.num_tokens + n_new
+        blocks = -(-total // self.page_size)
+        return [max(0, blocks - len(g.tables[req])) + sum(self._pool_pages_missing(g, req, total)) for g in self.groups]
+
+    def _pool_pages_missing(self, g: CacheGroup, req, tokens: int) -> list[int]:
+        """Per block size of the group, the pages the whole blocks of ``tokens`` tokens still lack."""
+        return [max(0, -(-(tokens // p) // self.page_size) - len(t)) for p, t in zip(g.spec.pools, g.pool_tables[req])]
+
+    def fit(self, req, want: int, free: list[int]) -> int:
+        """Most new tokens up to ``want`` whose pages the groups' counts ``free`` allow; ``req`` None: for
+        a request that is not live yet."""
+        ps = self.page_size
+        tokens = 0 if req is None else self.requests[req].num_tokens
+        n = want
+        for gi, g in enumerate(self.groups):
+            have = 0 if req is None else len(g.tables[req])
+            n = min(n, (have + free[gi]) * ps - tokens)
+        if n > 0 and any(g.spec.pools for g in self.groups):
+            def fits(k: int) -> bool:
+                if req is not None:
+                    return self.can_reserve(req, k, free)
+                return all(-(-k // ps) + pool_pages(g.spec, k, ps) <= f for g, f in zip(self.groups, free))
+
+            lo, hi = 0, n + 1       # (the pages needed never fall as tokens are added)
+            while hi - lo > 1:
+                mid = (lo + hi) // 2
+                lo, hi = (mid, hi) if fits(mid) else (lo, mid)
+            n = lo
+        return max(0, n)
 
     def can_reserve(self, req, n_new: int, spare: list[int] | None = None) -> bool:
         need = self.pages_needed(req, n_new)
@@ -178,8 +223,12 @@ class CacheManager:
                 raise OutOfPages(
                     f"request {req!r} needs {n} more pages for {n_new} tokens, "
                     f"{g.pool.num_free} of {g.pool.num_pages} free (group {g.spec})")
+        total = self.requests[req].num_tokens + n_new
         for n, g in zip(need, self.groups):
-            g.tables[req].extend(g.pool.allocate(n))
+            missing = self._pool_pages_missing(g, req, total)
+            g.tables[req].extend(g.pool.allocate(n - sum(missing)))
+            for k, t in zip(missing, g.pool_tables[req]):
+                t.extend(g.pool.allocate(k))
 
     def rollback(self, req, keep_new: int = 0) -> int:
         """Gives back the pages that ``reserve`` took beyond what ``keep_new`` more tokens need
@@ -195,6 +244,11 @@ class CacheManager:
                 g.pool.free(gone)
                 n += len(gone)
             del table[keep:]
+            for p, t in zip(g.spec.pools, g.pool_tables[req]):
+                whole = -(-((st.num_tokens + keep_new) // p) // self.page_size)
+                g.pool.free(t[whole:])
+                n += len(t[whole:])
+                del t[whole:]
         return n
 
     def commit(self, req, n_new: int) -> None:
@@ -212,7 +266,9 @@ class CacheManager:
                                    f"{len(g.tables[req]) * ps}")
             w = g.spec.window
             if w > 0:
-                dead = max(0, (st.num_tokens - w + 1) // ps)
+                # (the tokens of a block that is not whole yet stay, however small the window is)
+                passed = min([st.num_tokens - w + 1] + [st.num_tokens // p * p for p in g.spec.pools])
+                dead = max(0, passed // ps)
                 kept = -(-g.spec.keep_first // ps)      # blocks that hold tokens every later token reads
                 table = g.tables[req]
                 gone = [table[b] for b in range(kept, min(dead, len(table))) if table[b] >= 0]
@@ -226,6 +282,8 @@ class CacheManager:
         st = self.requests.pop(req)
         for g in self.groups:
             g.pool.free([p for p in g.tables.pop(req) if p >= 0])
+            for t in g.pool_tables.pop(req):
+                g.pool.free(t)
         self.slots.release(st.slot)
 
     def slot_mapping(self, group: int, req, start: int, n: int) -> list[int]:
@@ -246,6 +304,7 @@ class CacheManager:
         for g in self.groups:
             g.pool.check()
             held = [p for t in g.tables.values() for p in t if p >= 0]
+            held += [p for ts in g.pool_tables.values() for t in ts for p in t]
             assert len(held) == len(set(held)), "a page is held by two requests"
             assert len(held) == g.pool.num_used, "pages in tables and used count differ"
         assert set(self.requests) == set().union(*[set(g.tables) for g in self.groups]) or not self.groups

@@ -18,7 +18,7 @@ def group_layers(requirements) -> dict[KVCacheSpec, int]:
     """Cache spec -> number of caches (layer calls that write one) of that spec, in the
     order the cache manager forms its groups."""
     spec_of = {}
-    for cache_id, _writes, kv_spec, _state in requirements:
+    for cache_id, _writes, kv_spec, *_ in requirements:
         if kv_spec is not None:
             spec_of[cache_id] = kv_spec
     out: dict[KVCacheSpec, int] = {}
@@ -27,12 +27,18 @@ def group_layers(requirements) -> dict[KVCacheSpec, int]:
     return out
 
 
+def state_id(row) -> int:
+    """The number of a layer call's state: the row's fifth element where it has one, else its cache's number."""
+    return row[4] if len(row) > 4 else row[0]
+
+
 def state_bytes(requirements, max_seqs: int) -> int:
     """Device bytes of the per-request state tensors (one row more than there are requests)."""
     seen, total = set(), 0
-    for cache_id, _writes, _kv, st in requirements:
-        if st is not None and cache_id not in seen:
-            seen.add(cache_id)
+    for row in requirements:
+        st, sid = row[3], state_id(row)
+        if st is not None and sid not in seen:
+            seen.add(sid)
             total += (max_seqs + 1) * math.prod(st.shape) * st.dtype.itemsize
     return total
 
@@ -53,6 +59,19 @@ def window_pool_pages(window: int, page_size: int, max_seqs: int, token_budget: 
             + -(-token_budget // page_size))
 
 
+def pool_pages(spec: KVCacheSpec, tokens: int, page_size: int) -> int:
+    """Pages a request of ``tokens`` tokens holds for the whole blocks of all of the cache's block sizes."""
+    return sum(-(-(tokens // p) // page_size) for p in spec.pools)
+
+
+def request_pages(spec: KVCacheSpec, tokens: int, page_size: int) -> int:
+    """Pages a request must be able to hold in this cache to reach ``tokens`` tokens one at a time."""
+    n = -(-tokens // page_size)
+    if spec.window > 0:
+        n = min(n, min_window_pages(spec.reach, page_size, spec.keep_first))
+    return n + pool_pages(spec, tokens, page_size)
+
+
 def bytes_per_page(spec: KVCacheSpec, layers: int, page_size: int, elem_size: int) -> int:
     return 2 * layers * spec.num_kv_heads * spec.head_dim * page_size * elem_size
 
@@ -68,6 +87,9 @@ def plan_pages(requirements, page_size: int, elem_size: int, max_seqs: int, toke
     groups = group_layers(requirements)
     if not groups:
         return {}
+    if any(s.pools for s in groups):
+        return _plan_pages_with_blocks(requirements, groups, page_size, elem_size, max_seqs, token_budget, tokens,
+                                       kv_bytes, free_bytes)
     full = [s for s in groups if s.window <= 0]
     want_full = None if tokens is None else -(-tokens // page_size) + max_seqs
     pages = {}
@@ -104,3 +126,40 @@ def plan_pages(requirements, page_size: int, elem_size: int, max_seqs: int, toke
     if bad:
         raise ValueError(f"the memory given to the cache holds no page of {page_size} tokens for {bad[0]}")
     return pages
+
+
+def _plan_pages_with_blocks(requirements, groups, page_size, elem_size, max_seqs, token_budget, tokens, kv_bytes,
+                            free_bytes) -> dict[KVCacheSpec, int]:
+    """The same where some groups keep a key per block of tokens for good: those pages grow with the
+    tokens held, so the most tokens that fit the bytes are found by bisection."""
+    def pages_for(n: int) -> dict:
+        full = -(-n // page_size) + max_seqs
+        out = {}
+        for s in groups:
+            own = full
+            if s.window > 0:
+                own = min(full, window_pool_pages(s.reach, page_size, max_seqs, token_budget, s.keep_first))
+            out[s] = own + sum(-(-(n // p) // page_size) + max_seqs for p in s.pools)
+        return out
+
+    budget = None if kv_bytes is None else int(kv_bytes)
+    if free_bytes is not None:
+        cap = max(0, int(free_bytes) - state_bytes(requirements, max_seqs))
+        budget = cap if budget is None else min(budget, cap)
+    if budget is None and tokens is None:
+        raise ValueError("the cache needs a size: tokens, bytes or the free memory")
+
+    def fits(n: int) -> bool:
+        return budget is None or sum(k * bytes_per_page(s, groups[s], page_size, elem_size)
+                                     for s, k in pages_for(n).items()) <= budget
+
+    hi = int(tokens) if tokens is not None else 1 << 40
+    if fits(hi):
+        return pages_for(hi)
+    lo = page_size
+    if not fits(lo):
+        raise ValueError(f"the memory given to the cache holds no page of {page_size} tokens a request")
+    while hi - lo > 1:
+        mid = (lo + hi) // 2
+        lo, hi = (mid, hi) if fits(mid) else (lo, mid)
+    return pages_for(lo)

@@ -47,11 +47,14 @@ class LayerCall:
     ``writes_cache=False`` makes the call a reader of a cache another call
     fills.  ``offset`` >= 0: that row of the model's table of stream offsets
     (``ModelConfig.stream_offset_rows``) is added to the stream before the call.
+    ``state`` >= 0: the state this call works on, where it is not the one of the
+    cache's number (a call that borrows keys and values and has a state of its own).
     """
     layer: int
     cache: int
     writes_cache: bool = True
     offset: int = -1
+    state: int = -1
 
 
 class ModelConfig:

@@ -83,7 +83,20 @@ struct AttnFuse {
     const float* sinks;
     // A cap on the scores: s <- cap * tanh(s / cap) after the scale and before the mask.  0: none.
     float softcap;
+    // Keys of whole blocks of `pool` tokens that stand before the window's (0: none), in pages of the same
+    // cache that the rows of pool_tables name, pt_stride numbers apart: block b is seen from position i if its
+    // last token (b + 1) pool - 1 <= i - window.  The kernels with POOL work through those keys first, as keys
+    // 0 .. seen - 1 of a table of their own, then through the tokens'.
+    const int32_t* pool_tables;
+    int pt_stride;
+    int pool;
 };
+
+// The last block that position pos sees (-1: none).
+__device__ __forceinline__ int attn_last_block(int pos, int window, int pool) {
+    const int before = pos - window + 1;
+    return before >= pool ? before / pool - 1 : -1;
+}
 
 // tanh by one exponential: 1 - 2 / (1 + e^(2x)), which ends at 1 and -1 as e^(2x) overflows and vanishes.
 __device__ __forceinline__ float attn_tanh(float x) {
@@ -164,7 +177,7 @@ __device__ __forceinline__ void norm_rope_fragments(bf16x8 (&f)[(DT * 16 + 31) /
 // A wave alone streams some 16 GB/s, eight of them on a CU together as much as the CU takes
 // (≈ 100 GB/s), so this pays once there are entries x kv heads enough for the blocks to saturate
 // HBM between them (64 and more); with fewer, the keys are split over blocks as before.
-template <int DT, bool SPLIT, int RING, bool FUSED = false, int BW = 1>
+template <int DT, bool SPLIT, int RING, bool FUSED = false, int BW = 1, bool POOL = false>
 __global__ __launch_bounds__(64 * BW, 1) void attn_wave_kernel(
     const bf16_t* __restrict__ q, int q_stride, bf16_t* __restrict__ out, float* __restrict__ part_o,
     float* __restrict__ part_ml, const bf16_t* __restrict__ k_cache,
@@ -175,6 +188,7 @@ __global__ __launch_bounds__(64 * BW, 1) void attn_wave_kernel(
     constexpr int D = DT * 16;
     constexpr int KS = (D + 31) / 32;
     static_assert(BW == 1 || (FUSED && !SPLIT), "blocks of several waves are for fused decode steps, and merge in LDS");
+    static_assert(!POOL || !FUSED, "keys of blocks are for finished queries and filled pages");
     constexpr int BT_LEN = BW == 1 ? ATTN_WAVE_BT : ATTN_WAVE_BT / 4;     // page numbers a wave keeps at a time
     __shared__ int32_t bt_all[BW * BT_LEN];
     __shared__ __attribute__((aligned(16))) float fz_all[BW * (FUSED ? 3 * D : 4)];   // q weight, k weight, (cos, sin) pairs
@@ -236,15 +250,23 @@ __global__ __launch_bounds__(64 * BW, 1) void attn_wave_kernel(
     const int tl = cc / G;
     const int c_tok = tok0 + tl;
     const int c_head = g * G + (cc - tl * G);
-    const int c_pos = c_ok ? P + tl : -1;   // a missing column sees no key
-    const int c_lo = window > 0 ? max(0, P + tl - window + 1) : 0;
+    int c_pos = c_ok ? P + tl : -1;   // a missing column sees no key
+    int c_lo = window > 0 ? max(0, P + tl - window + 1) : 0;
     // keys any column of this wave can see
     const int tl_first = col0 / G;
     const int tl_last = (min(col0 + 16, ncols) - 1) / G;
     const int kmin = window > 0 ? max(0, P + tl_first - window + 1) : 0;
-    const int kmax = P + tl_last;
-    const int kb0 = (kmin / 32) * 32;
-    const int nsteps = (kmax - kb0) / 32 + 1;
+    int kmax = P + tl_last;
+    int kb0 = (kmin / 32) * 32;
+    int nsteps = (kmax - kb0) / 32 + 1;
+    // (POOL: the steps of the blocks' keys come before the tokens')
+    int pool_steps = 0, pool_last = -1, c_pool = -1;
+    if constexpr (POOL) {
+        pool_last = attn_last_block(kmax, window, fz.pool);
+        pool_steps = pool_last >= 0 ? pool_last / 32 + 1 : 0;
+        c_pool = c_ok ? attn_last_block(P + tl, window, fz.pool) : -1;
+        nsteps += pool_steps;
+    }
     int s_begin = 0, s_end = nsteps;
     if (by_runs) {
         s_begin = min(nsteps, max(0, (run.y - kb0) >> 5));
@@ -301,7 +323,7 @@ __global__ __launch_bounds__(64 * BW, 1) void attn_wave_kernel(
     // for the addresses of the keys (norm weights, angles, the raw q, k and v) is put to use
     // after the first keys and values are on their way.
     int new_page = 0, first_page = 0, first_count = 0;
-    if (s_begin < s_end) {
+    if (!POOL && s_begin < s_end) {
         pi0 = page_index(kb0 + s_begin * 32, page_size, page_shift);
         first_count = page_index(min(kmax, kb0 + min(s_end, s_begin + seg_steps) * 32 - 1), page_size, page_shift) - pi0 + 1;
         if (lane < first_count) first_page = bt[pi0 + lane];
@@ -419,12 +441,17 @@ __global__ __launch_bounds__(64 * BW, 1) void attn_wave_kernel(
     const float slack = 8.0f / sl2;
     // a cap c on the scores, in raw score units: s <- (c / scale) tanh(s scale / c), so that s scale is capped
     const float cap_in = fz.softcap > 0.f ? scale / fz.softcap : 0.f, cap_out = fz.softcap > 0.f ? fz.softcap / scale : 0.f;
-    int w_min_pos = c_ok ? c_pos : 0x7fffffff, w_max_lo = c_ok ? c_lo : 0;   // over the wave's columns
+    int w_min_pos, w_max_lo;   // over the wave's columns
+    auto edges = [&]() {
+        w_min_pos = c_ok ? c_pos : 0x7fffffff;
+        w_max_lo = c_ok ? c_lo : 0;
 #pragma unroll
-    for (int o = 32; o > 0; o >>= 1) {
-        w_min_pos = min(w_min_pos, __shfl_xor(w_min_pos, o, 64));
-        w_max_lo = max(w_max_lo, __shfl_xor(w_max_lo, o, 64));
-    }
+        for (int o = 32; o > 0; o >>= 1) {
+            w_min_pos = min(w_min_pos, __shfl_xor(w_min_pos, o, 64));
+            w_max_lo = max(w_max_lo, __shfl_xor(w_max_lo, o, 64));
+        }
+    };
+    if constexpr (!POOL) edges();
 #define TFF_WAVE_COMPUTE(buf, step)                                                                 \
     {                                                                                               \
         const int kb_ = kb0 + (step) * 32;                                                          \
@@ -475,9 +502,22 @@ __global__ __launch_bounds__(64 * BW, 1) void attn_wave_kernel(
             oacc[dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[buf][dt], pv_, oacc[dt], 0, 0, 0); \
     }
 
+    const int token_kmax = kmax, token_kb0 = kb0, token_pos = c_pos, token_lo = c_lo, all_begin = s_begin, all_end = s_end;
+    for (int part = POOL ? 0 : 1; part < 2; ++part) {
+    if constexpr (POOL) {
+        s_begin = part == 0 ? all_begin : max(all_begin, pool_steps) - pool_steps;
+        s_end = part == 0 ? min(all_end, pool_steps) : all_end - pool_steps;
+        if (s_begin >= s_end) continue;
+        kmax = part == 0 ? pool_last : token_kmax;
+        kb0 = part == 0 ? 0 : token_kb0;
+        c_pos = part == 0 ? c_pool : token_pos;
+        c_lo = part == 0 ? 0 : token_lo;
+        bt = part == 0 ? fz.pool_tables + (size_t)r * fz.pt_stride : block_tables + (size_t)r * bt_stride;
+        edges();
+    }
     for (int seg0 = s_begin; seg0 < s_end; seg0 += seg_steps) {
         const int seg1 = min(s_end, seg0 + seg_steps);
-        if (seg0 > s_begin) {
+        if (POOL || seg0 > s_begin) {
             wave_sync();            // the segment before is read
             fill_pages(seg0, seg1, 0);
             wave_sync();
@@ -537,6 +577,7 @@ __global__ __launch_bounds__(64 * BW, 1) void attn_wave_kernel(
                 TFF_WAVE_COMPUTE(u, s + u)
             }
     }
+    }   // blocks' keys, tokens' keys
 #undef TFF_WAVE_PAGE
 #undef TFF_WAVE_PATCH
 #undef TFF_WAVE_LOAD
@@ -865,14 +906,15 @@ __device__ __forceinline__ float max3_raw(float a, float b, float c) {
 #define ATTN_STAGES 4
 constexpr int attn_vmcnt_imm(int v) { return (v & 15) | (7 << 4) | (15 << 8) | ((v >> 4) << 14); }
 
-template <int DT, int NQT, int NW, int KGRP>
+template <int DT, int NQT, int NW, int KGRP, bool POOL = false>
 __global__ __launch_bounds__(64 * NW * KGRP, (NW * KGRP <= 4 ? 2 : 1)) void attn_mfma_block_kernel(
     const bf16_t* __restrict__ q, int q_stride, bf16_t* __restrict__ out,
     const bf16_t* __restrict__ k_cache, const bf16_t* __restrict__ v_cache,
     const int32_t* __restrict__ block_tables, int bt_stride, const int32_t* __restrict__ cu_tokens,
     const int32_t* __restrict__ start_pos, const int32_t* __restrict__ work,
     const int32_t* __restrict__ block_items, int nq, int nkv, int page_size, int page_shift,
-    int window, float scale, const float* __restrict__ sinks, float softcap) {
+    int window, float scale, const float* __restrict__ sinks, float softcap, const int32_t* __restrict__ pool_tables,
+    int pt_stride, int pool) {
     constexpr int D = DT * 16;
     constexpr int KS = (D + 31) / 32;
     constexpr int KFR = 2 * KS, VFR = DT, FR = KFR + VFR;   // 1 KB fragments per slice
@@ -926,9 +968,9 @@ __global__ __launch_bounds__(64 * NW * KGRP, (NW * KGRP <= 4 ? 2 : 1)) void attn
     const int tl_first = bcol0 / G;
     const int tl_last = (min(bcol0 + BCOLS, ncols) - 1) / G;
     const int kmin = window > 0 ? max(0, P + tl_first - window + 1) : 0;
-    const int kmax = P + tl_last;
-    const int kb0 = (kmin / 32) * 32;
-    const int nsteps = (kmax - kb0) / 32 + 1;
+    int kmax = P + tl_last;
+    int kb0 = (kmin / 32) * 32;
+    int nsteps = (kmax - kb0) / 32 + 1;
     // The page numbers of the block's keys come from LDS, always (a lookup in the table itself
     // is a memory load, and to wait for it is to wait for every copy in flight).  Keys beyond
     // what ATTN_BT_LDS pages hold are worked through in segments, each with its own page numbers
@@ -978,7 +1020,7 @@ __global__ __launch_bounds__(64 * NW * KGRP, (NW * KGRP <= 4 ? 2 : 1)) void attn
     const uint32_t page_stride = (uint32_t)nkv * page_size * D;      // elements of a page, K or V (the host checks that it fits)
     const bf16_t* kbase = k_cache + (size_t)g * page_size * D;
     const bf16_t* vbase = v_cache + (size_t)g * D * page_size;
-    const int vkmax = (kmax >> 3) << 3;
+    int vkmax = (kmax >> 3) << 3;
     int cp_F[LPW], cp_sub[LPW], cp_key[LPW], cp_off[LPW];
     bool cp_is_k[LPW];
 #pragma unroll
@@ -1026,24 +1068,48 @@ __global__ __launch_bounds__(64 * NW * KGRP, (NW * KGRP <= 4 ? 2 : 1)) void attn
     // a cap c on the scores, in raw score units: s <- (c / scale) tanh(s scale / c), so that s scale is capped
     const float cap_in = softcap > 0.f ? scale / softcap : 0.f, cap_out = softcap > 0.f ? softcap / scale : 0.f;
     int t_min_pos[NQT], t_max_lo[NQT];
+    auto edges = [&]() {
 #pragma unroll
-    for (int t = 0; t < NQT; ++t) {
-        int mn = c_pos[t], mx = c_lo[t];
+        for (int t = 0; t < NQT; ++t) {
+            int mn = c_pos[t], mx = c_lo[t];
 #pragma unroll
-        for (int o = 32; o > 0; o >>= 1) {
-            mn = min(mn, __shfl_xor(mn, o, 64));
-            mx = max(mx, __shfl_xor(mx, o, 64));
+            for (int o = 32; o > 0; o >>= 1) {
+                mn = min(mn, __shfl_xor(mn, o, 64));
+                mx = max(mx, __shfl_xor(mx, o, 64));
+            }
+            t_min_pos[t] = mn;
+            t_max_lo[t] = mx;
         }
-        t_min_pos[t] = mn;
-        t_max_lo[t] = mx;
-    }
+    };
+    if constexpr (!POOL) edges();
 
+    // (POOL: first the keys of the blocks before the window, then the tokens'; each part has a pipeline of copies of its own)
+    bool copies_out = false;
+    for (int part = POOL ? 0 : 1; part < 2; ++part) {
+    if constexpr (POOL) {
+        const int last = attn_last_block(P + tl_last, window, pool);
+        if (part == 0 && last < 0) continue;        // (the same for the whole block)
+        kmax = part == 0 ? last : P + tl_last;
+        kb0 = part == 0 ? 0 : (kmin / 32) * 32;
+        nsteps = (kmax - kb0) / 32 + 1;
+        vkmax = (kmax >> 3) << 3;
+        bt = part == 0 ? pool_tables + (size_t)r * pt_stride : block_tables + (size_t)r * bt_stride;
+#pragma unroll
+        for (int t = 0; t < NQT; ++t) {
+            const int c = col0 + t * 16 + qc;
+            const int pos = P + (c < ncols ? c : ncols - 1) / G;
+            c_pos[t] = c < ncols ? (part == 0 ? attn_last_block(pos, window, pool) : pos) : -1;
+            c_lo[t] = part == 0 ? 0 : max(0, pos - window + 1);
+        }
+        edges();
+    }
     for (int seg0 = 0; seg0 < nsteps; seg0 += seg_steps) {
     const int seg1 = min(nsteps, seg0 + seg_steps);
-    if (seg0 > 0) {
+    if (POOL ? copies_out : seg0 > 0) {
         __builtin_amdgcn_s_waitcnt(vmcnt_imm0());   // the segment before: its copies past the end have landed,
         __syncthreads();                            // its slices and page numbers are read
     }
+    copies_out = true;
     pg0 = page_index(kb0 + seg0 * 32, page_size, page_shift);
     {
         const int npg = page_index(min(kmax, kb0 + seg1 * 32 - 1), page_size, page_shift) - pg0 + 1;
@@ -1147,6 +1213,7 @@ __global__ __launch_bounds__(64 * NW * KGRP, (NW * KGRP <= 4 ? 2 : 1)) void attn
         }
     }
     }   // segments
+    }   // blocks' keys, tokens' keys
 #undef ATTN_ISSUE
 #undef ATTN_PAGE
     __builtin_amdgcn_s_waitcnt(vmcnt_imm0());   // the copies past the end must not outlive the block
@@ -1219,7 +1286,8 @@ static int launch_attn(const bf16_t* q, int q_stride, bf16_t* out, float* part_o
                        int tiles_per_entry, int cols_per_wave,
                        int splits, int nq, int nkv, int page_size, int window, float scale,
                        int T_total, hipStream_t s, const AttnFuse* fuse = nullptr, int key_groups = 2,
-                       const AttnFuse* runs_only = nullptr, const float* sinks = nullptr, float softcap = 0.f) {
+                       const AttnFuse* runs_only = nullptr, const float* sinks = nullptr, float softcap = 0.f,
+                       const int32_t* pool_tables = nullptr, int pt_stride = 0, int pool = 0) {
     int page_shift = 0;   // the page size is a power of two (tff_attention_mfma_supported)
     while ((1 << page_shift) < page_size) ++page_shift;
     if (cols_per_wave == 256) {
@@ -1229,11 +1297,25 @@ static int launch_attn(const bf16_t* q, int q_stride, bf16_t* out, float* part_o
         if constexpr (DT <= 8) {
             attn_mfma_block_kernel<DT, 2, 8, 1><<<dim3(num_blocks, nkv), 512, 0, s>>>(
                 q, q_stride, out, k_cache, v_cache, block_tables, bt_stride, cu_tokens, start_pos, work,
-                block_items, nq, nkv, page_size, page_shift, window, scale, sinks, softcap);
+                block_items, nq, nkv, page_size, page_shift, window, scale, sinks, softcap, pool_tables, pt_stride, pool);
             return tff_check_launch("attention_mfma_block256");
         } else {
             return tff_fail("attention_mfma: blocks of 256 columns take head sizes up to 128");
         }
+    }
+    if (pool > 0 && cols_per_wave == 128) {
+        if constexpr (DT <= 7) {       // (two groups of waves at a head size of 128 have no registers left for the second table)
+            if (key_groups == 2) {
+                attn_mfma_block_kernel<DT, 1, 8, 2, true><<<dim3(num_blocks, nkv), 1024, 0, s>>>(
+                    q, q_stride, out, k_cache, v_cache, block_tables, bt_stride, cu_tokens, start_pos, work,
+                    block_items, nq, nkv, page_size, page_shift, window, scale, sinks, softcap, pool_tables, pt_stride, pool);
+                return tff_check_launch("attention_mfma_block_pool");
+            }
+        }
+        attn_mfma_block_kernel<DT, 1, 8, 1, true><<<dim3(num_blocks, nkv), 512, 0, s>>>(
+            q, q_stride, out, k_cache, v_cache, block_tables, bt_stride, cu_tokens, start_pos, work,
+            block_items, nq, nkv, page_size, page_shift, window, scale, sinks, softcap, pool_tables, pt_stride, pool);
+        return tff_check_launch("attention_mfma_block_pool");
     }
     if (cols_per_wave == 128) {   // blocks of eight waves that share their keys through LDS
         // Two groups of eight waves that take every other slice, where LDS holds their stages:
@@ -1244,15 +1326,15 @@ static int launch_attn(const bf16_t* q, int q_stride, bf16_t* out, float* part_o
             if (key_groups == 2)
                 attn_mfma_block_kernel<DT, 1, 8, 2><<<dim3(num_blocks, nkv), 1024, 0, s>>>(
                     q, q_stride, out, k_cache, v_cache, block_tables, bt_stride, cu_tokens, start_pos, work,
-                    block_items, nq, nkv, page_size, page_shift, window, scale, sinks, softcap);
+                    block_items, nq, nkv, page_size, page_shift, window, scale, sinks, softcap, pool_tables, pt_stride, pool);
             else
                 attn_mfma_block_kernel<DT, 1, 8, 1><<<dim3(num_blocks, nkv), 512, 0, s>>>(
                     q, q_stride, out, k_cache, v_cache, block_tables, bt_stride, cu_tokens, start_pos, work,
-                    block_items, nq, nkv, page_size, page_shift, window, scale, sinks, softcap);
+                    block_items, nq, nkv, page_size, page_shift, window, scale, sinks, softcap, pool_tables, pt_stride, pool);
         } else
             attn_mfma_block_kernel<DT, 1, 8, 1><<<dim3(num_blocks, nkv), 512, 0, s>>>(
                 q, q_stride, out, k_cache, v_cache, block_tables, bt_stride, cu_tokens, start_pos, work,
-                block_items, nq, nkv, page_size, page_shift, window, scale, sinks, softcap);
+                block_items, nq, nkv, page_size, page_shift, window, scale, sinks, softcap, pool_tables, pt_stride, pool);
         return tff_check_launch("attention_mfma_block");
     }
     const dim3 grid(num_work, nkv, max(splits, 1));
@@ -1261,9 +1343,17 @@ static int launch_attn(const bf16_t* q, int q_stride, bf16_t* out, float* part_o
                                            : AttnFuse{nullptr, nullptr, nullptr, nullptr, nullptr, nullptr, 0.f, 0, nullptr, nullptr};
     if (sinks) fz.sinks = sinks;
     if (softcap > 0.f) fz.softcap = softcap;
+    fz.pool_tables = pool_tables;
+    fz.pt_stride = pt_stride;
+    fz.pool = pool;
 #define TFF_ATTN_ARGS                                                                              \
     q, q_stride, out, part_o, part_ml, k_cache, v_cache, block_tables, bt_stride, cu_tokens,       \
         start_pos, work, tiles_per_entry, nq, nkv, page_size, page_shift, window, scale, T_total
+    if (pool > 0) {
+        if (splits > 1) attn_wave_kernel<DT, true, (DT <= 8 ? 4 : DT <= 12 ? 2 : 1), false, 1, true><<<grid, 64, 0, s>>>(TFF_ATTN_ARGS, fz);
+        else attn_wave_kernel<DT, false, (DT <= 8 ? 4 : DT <= 12 ? 2 : 1), false, 1, true><<<grid, 64, 0, s>>>(TFF_ATTN_ARGS, fz);
+        return tff_check_launch("attention_mfma_pool");
+    }
     if (fuse && splits == 0) {
         // a block of eight waves per entry (or run of keys dealt by the host) and kv head: the keys split
         // among its waves, merged in LDS
@@ -1312,9 +1402,12 @@ TFF_API int tff_attention_mfma(const void* q, int q_stride, void* out, float* pa
                                const int32_t* block_items, int num_blocks,
                                int tiles_per_entry, int cols_per_wave, int key_groups, int splits, int T_total,
                                int nq, int nkv, int d, int page_size, int num_pages, int window,
-                               float scale, const float* sinks, float softcap, tff_stream_t stream) {
+                               float scale, const float* sinks, float softcap, const int32_t* pool_tables, int pt_stride,
+                               int pool, tff_stream_t stream) {
     TFF_REQUIRE(q && out && k_cache && v_cache && block_tables && cu_tokens && start_pos,
                 "attention_mfma: null pointer");
+    TFF_REQUIRE(pool >= 0 && (pool == 0 || (window > 0 && pool_tables && pt_stride > 0 && cols_per_wave != 256)),
+                "attention_mfma: keys of blocks of %d tokens stand before a window and need their tables", pool);
     TFF_REQUIRE(key_groups == 1 || key_groups == 2, "attention_mfma: %d key groups (1 or 2)", key_groups);
     TFF_REQUIRE(!(softcap > 0.f) || d <= 192, "attention_mfma: a cap on the scores with head sizes up to 192, not %d", d);
     TFF_REQUIRE(nq > 0 && nkv > 0 && nq % nkv == 0,
@@ -1355,7 +1448,7 @@ TFF_API int tff_attention_mfma(const void* q, int q_stride, void* out, float* pa
                                 bt_stride, cu_tokens, start_pos, work, num_work, block_items,       \
                                 num_blocks, tiles_per_entry,                                        \
                                 cols_per_wave, splits, nq, nkv, page_size, window, scale, T_total, s, \
-                                nullptr, key_groups, nullptr, splits > 1 ? nullptr : sinks, softcap);
+                                nullptr, key_groups, nullptr, splits > 1 ? nullptr : sinks, softcap, pool_tables, pt_stride, pool);
     switch (d) {
         TFF_ATTN_CASE(1) TFF_ATTN_CASE(2) TFF_ATTN_CASE(3) TFF_ATTN_CASE(4) TFF_ATTN_CASE(5)
         TFF_ATTN_CASE(6) TFF_ATTN_CASE(7) TFF_ATTN_CASE(8) TFF_ATTN_CASE(12) TFF_ATTN_CASE(16)

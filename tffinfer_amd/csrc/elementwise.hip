@@ -23,7 +23,7 @@ int tff_check_launch(const char* what) {
     return 0;
 }
 TFF_API const char* tff_last_error() { return g_error; }
-TFF_API int tff_abi_version() { return 34; }
+TFF_API int tff_abi_version() { return 35; }
 
 // ----------------------------------------------------------------- embed ---
 // x[t, :] = E[token[t], :]   (reference: src/kernel/cpu/embedding.cpp:34-49,
@@ -612,17 +612,17 @@ TFF_API int tff_qk_norm_rope_kv(void* qkv, int T, int nq, int nkv, int d, const 
 // m = silu(g) * u, silu(x) = x / (1 + exp(-x))  (reference:
 // src/kernel/cuda/unary.cu:10-27, x1 = gate, x2 = up).
 template <typename T>
-__global__ void swiglu_kernel(const T* __restrict__ gu, T* __restrict__ out, int64_t total, int I) {
+__global__ void swiglu_kernel(const T* __restrict__ gu, const float* __restrict__ bias, T* __restrict__ out, int64_t total, int I) {
     const int64_t idx = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (idx >= total) return;
     const int64_t t = idx / I;
     const int i = (int)(idx - t * I);
-    const float g = to_f32(gu[t * 2 * I + i]);
-    const float u = to_f32(gu[t * 2 * I + I + i]);
+    const float g = to_f32(gu[t * 2 * I + i]) + (bias ? bias[i] : 0.f);
+    const float u = to_f32(gu[t * 2 * I + I + i]) + (bias ? bias[I + i] : 0.f);
     out[idx] = from_f32<T>(g / (1.0f + expf(-g)) * u);
 }
 
-TFF_API int tff_swiglu(const void* gu, void* out, int T, int I, int dtype, tff_stream_t stream) {
+TFF_API int tff_swiglu(const void* gu, const float* bias, void* out, int T, int I, int dtype, tff_stream_t stream) {
     TFF_REQUIRE(gu && out, "swiglu: null pointer");
     TFF_REQUIRE(T >= 0 && I > 0, "swiglu: bad sizes T=%d I=%d", T, I);
     if (T == 0) return 0;
@@ -631,9 +631,9 @@ TFF_API int tff_swiglu(const void* gu, void* out, int T, int I, int dtype, tff_s
     TFF_REQUIRE(blocks < 2147483647LL, "swiglu: too many elements");
     hipStream_t s = (hipStream_t)stream;
     if (dtype == TFF_F32)
-        swiglu_kernel<float><<<(unsigned)blocks, 256, 0, s>>>((const float*)gu, (float*)out, total, I);
+        swiglu_kernel<float><<<(unsigned)blocks, 256, 0, s>>>((const float*)gu, bias, (float*)out, total, I);
     else if (dtype == TFF_BF16)
-        swiglu_kernel<bf16_t><<<(unsigned)blocks, 256, 0, s>>>((const bf16_t*)gu, (bf16_t*)out, total, I);
+        swiglu_kernel<bf16_t><<<(unsigned)blocks, 256, 0, s>>>((const bf16_t*)gu, bias, (bf16_t*)out, total, I);
     else
         return tff_fail("swiglu: unknown dtype %d", dtype);
     return tff_check_launch("swiglu");

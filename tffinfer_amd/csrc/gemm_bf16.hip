@@ -49,6 +49,13 @@ __device__ __forceinline__ floatx4 silu_mul(const floatx4& g, const floatx4& u) 
     return o;
 }
 
+// Four neighbouring numbers of a bias in the order of W's rows (16 NB of them), for a lane's four columns from n
+// on; columns past the end, whose results are never stored, take the last ones.
+__device__ __forceinline__ floatx4 bias4(const float* __restrict__ bias, int n, int NB) {
+    const float4 b = *reinterpret_cast<const float4*>(bias + min(n, NB * 16 - 4));
+    return floatx4{b.x, b.y, b.z, b.w};
+}
+
 // ------------------------------------------------------- tiled, async copy ---
 // Block tile (WGM*WTM*16) x (WGN*WTN*16) x (32 KPS) on WGM x WGN waves, each wave
 // WTM x WTN MFMA tiles.  Both operands are staged in LDS in fragment order; the
@@ -68,7 +75,7 @@ constexpr int vmcnt_imm(int v) { return (v & 15) | (7 << 4) | (15 << 8) | ((v >>
 template <int WGM, int WGN, int WTM, int WTN, int STAGES, bool GLU, typename TC, int KPS = 2, bool EARLY = false>
 __global__ __launch_bounds__(64 * WGM * WGN) void gemm_bf16_async_kernel(
     const bf16_t* __restrict__ A, const bf16_t* __restrict__ Wp, TC* __restrict__ C, int M, int N,
-    int K, int lda, int KB, int n_out, float* __restrict__ part) {
+    int K, int lda, int KB, int n_out, float* __restrict__ part, const float* __restrict__ bias) {
     // WGM x WGN waves, each WTM x WTN MFMA tiles of 16 x 16
     constexpr int NW = WGM * WGN;
     constexpr int BM = WGM * WTM * 16, BN = WGN * WTN * 16;
@@ -123,6 +130,14 @@ __global__ __launch_bounds__(64 * WGM * WGN) void gemm_bf16_async_kernel(
     for (int i = 0; i < WTN; ++i)
 #pragma unroll
         for (int j = 0; j < WTM; ++j) acc[i][j] = floatx4{0.f, 0.f, 0.f, 0.f};
+    if (bias && blockIdx.z == 0) {
+#pragma unroll
+        for (int i = 0; i < WTN; ++i) {
+            const floatx4 b = bias4(bias, n0 + (wn * WTN + i) * 16 + fg * 4, NB);
+#pragma unroll
+            for (int j = 0; j < WTM; ++j) acc[i][j] = b;
+        }
+    }
 
     // this wave's copies: fragments f = wave + NW j of a stage; f < AF is of A, else of W
     const bf16_t* src[LPW];
@@ -295,7 +310,7 @@ __global__ __launch_bounds__(256) void gemm_splitk_reduce_kernel(const float* __
 // splits > 1: the blocks of a tile split K among them; part holds splits * M * N floats
 template <int WGM, int WGN, int WTM, int WTN, int STAGES, bool GLU = false, int KPS = 2, bool EARLY = false>
 static int launch_async_g(const bf16_t* A, const bf16_t* Wp, void* C, int M, int N, int K, int lda,
-                          int c_dtype, int n_out, hipStream_t s, int splits = 1, float* part = nullptr,
+                          const float* bias, int c_dtype, int n_out, hipStream_t s, int splits = 1, float* part = nullptr,
                           bool reduce = true) {
     const int KB = (K + 31) / 32;
     constexpr int BM = WGM * WTM * 16, BN = WGN * WTN * 16;
@@ -306,10 +321,10 @@ static int launch_async_g(const bf16_t* A, const bf16_t* Wp, void* C, int M, int
     const dim3 grid((unsigned)tiles, 1, splits);
     if (c_dtype == TFF_F32)
         gemm_bf16_async_kernel<WGM, WGN, WTM, WTN, STAGES, GLU, float, KPS, EARLY>
-            <<<grid, 64 * WGM * WGN, 0, s>>>(A, Wp, (float*)C, M, N, K, lda, KB, n_out, part);
+            <<<grid, 64 * WGM * WGN, 0, s>>>(A, Wp, (float*)C, M, N, K, lda, KB, n_out, part, bias);
     else
         gemm_bf16_async_kernel<WGM, WGN, WTM, WTN, STAGES, GLU, bf16_t, KPS, EARLY>
-            <<<grid, 64 * WGM * WGN, 0, s>>>(A, Wp, (bf16_t*)C, M, N, K, lda, KB, n_out, part);
+            <<<grid, 64 * WGM * WGN, 0, s>>>(A, Wp, (bf16_t*)C, M, N, K, lda, KB, n_out, part, bias);
     if (int rc = tff_check_launch("gemm_bf16_async")) return rc;
     if (splits > 1 && reduce) {
         const int No = GLU ? n_out : N;
@@ -445,7 +460,7 @@ struct W4Scale {
 template <int WTN, int NWS, bool GLU, typename TC, int WGM = 2, bool SCALE = false, int WTM = 8>
 __global__ __launch_bounds__(256) void gemm_bf16_w4_kernel(
     const bf16_t* __restrict__ A, const bf16_t* __restrict__ Wp, TC* __restrict__ C, int M, int N,
-    int K, int lda, int KB, int n_out, W4Scale sc) {
+    int K, int lda, int KB, int n_out, W4Scale sc, const float* __restrict__ bias) {
     static_assert(!SCALE || WGM == 1, "rows that lack their norm's factor: up to 16, one row tile");
     // WGM: waves along the rows, 2 (a block tile of 256 rows, two waves side by side) or 1 (128 rows, four side by side)
     // WTM: row groups of 16 a wave, 8, or with the waves side by side 4 or 2 (a block tile of 64 or 32 rows)
@@ -498,6 +513,14 @@ __global__ __launch_bounds__(256) void gemm_bf16_w4_kernel(
     for (int i = 0; i < WTN; ++i)
 #pragma unroll
         for (int jj = 0; jj < WTM; ++jj) acc[i][jj] = floatx4{0.f, 0.f, 0.f, 0.f};
+    if (bias && blockIdx.z == 0) {
+#pragma unroll
+        for (int i = 0; i < WTN; ++i) {
+            const floatx4 b = bias4(bias, n0 + (wn * WTN + i) * 16 + fg * 4, NB);
+#pragma unroll
+            for (int jj = 0; jj < WTM; ++jj) acc[i][jj] = b;
+        }
+    }
     // (a lane's results are four columns of row fr of each row group: of row fr itself in the first,
     // the only one that counts with up to 16 rows; the four lanes of a row share out its sums)
     float row_ss = 0.f;
@@ -670,7 +693,7 @@ __global__ __launch_bounds__(256) void gemm_bf16_w4_kernel(
 
 // splits > 1: the blocks of a tile split K among them in units of 64; part holds splits * M * N floats
 template <int WTN, int NWS, bool GLU = false, int WGM = 2, bool SCALE = false, int WTM = 8>
-static int launch_w4(const bf16_t* A, const bf16_t* Wp, void* C, int M, int N, int K, int lda, int c_dtype,
+static int launch_w4(const bf16_t* A, const bf16_t* Wp, void* C, int M, int N, int K, int lda, const float* bias, int c_dtype,
                      int n_out, hipStream_t s, int splits = 1, float* part = nullptr, bool reduce = true,
                      W4Scale sc = W4Scale{nullptr, 0, 0, 0.f, 0.f}) {
     TFF_REQUIRE(!SCALE || (M <= 16 && sc.ss && (splits <= 1 || !part)),
@@ -687,11 +710,11 @@ static int launch_w4(const bf16_t* A, const bf16_t* Wp, void* C, int M, int N, i
     const dim3 grid((unsigned)tiles, 1, splits);
     // the blocks of a split K leave plain float32 sums, plane by plane; a gate is applied when they are added up
     if (splits > 1)
-        gemm_bf16_w4_kernel<WTN, NWS, false, float, WGM, false, WTM><<<grid, 256, 0, s>>>(A, Wp, part, M, N, K, lda, KB, 0, sc);
+        gemm_bf16_w4_kernel<WTN, NWS, false, float, WGM, false, WTM><<<grid, 256, 0, s>>>(A, Wp, part, M, N, K, lda, KB, 0, sc, bias);
     else if (c_dtype == TFF_F32)
-        gemm_bf16_w4_kernel<WTN, NWS, GLU, float, WGM, SCALE, WTM><<<grid, 256, 0, s>>>(A, Wp, (float*)C, M, N, K, lda, KB, n_out, sc);
+        gemm_bf16_w4_kernel<WTN, NWS, GLU, float, WGM, SCALE, WTM><<<grid, 256, 0, s>>>(A, Wp, (float*)C, M, N, K, lda, KB, n_out, sc, bias);
     else
-        gemm_bf16_w4_kernel<WTN, NWS, GLU, bf16_t, WGM, SCALE, WTM><<<grid, 256, 0, s>>>(A, Wp, (bf16_t*)C, M, N, K, lda, KB, n_out, sc);
+        gemm_bf16_w4_kernel<WTN, NWS, GLU, bf16_t, WGM, SCALE, WTM><<<grid, 256, 0, s>>>(A, Wp, (bf16_t*)C, M, N, K, lda, KB, n_out, sc, bias);
     if (int rc = tff_check_launch("gemm_bf16_w4")) return rc;
     if (splits > 1 && reduce) {
         const int No = GLU ? n_out : N;
@@ -753,7 +776,7 @@ struct SkinnyFuse {
 template <int MT, int R, int UNROLL, int KSPLIT, int NSETS, bool GLU, typename TC, bool RING = false, int EPI = 0>
 __global__ __launch_bounds__(64 * KSPLIT * NSETS) void gemm_bf16_skinny_kernel(
     const bf16_t* __restrict__ A, const bf16_t* __restrict__ Wp, TC* __restrict__ C, int M, int N,
-    int K, int lda, int KB, int n_out, SkinnyFuse fz) {
+    int K, int lda, int KB, int n_out, SkinnyFuse fz, const float* __restrict__ bias) {
     static_assert(EPI == 0 || MT == 1, "the fused norm is for up to 16 rows");
     static_assert(EPI < 2 || !GLU, "the product before a norm has a plain float32 result");
     constexpr int SK_WAVES = KSPLIT * NSETS;
@@ -770,6 +793,14 @@ __global__ __launch_bounds__(64 * KSPLIT * NSETS) void gemm_bf16_skinny_kernel(
     for (int r = 0; r < R; ++r)
 #pragma unroll
         for (int t = 0; t < MT; ++t) acc[r][t] = floatx4{0.f, 0.f, 0.f, 0.f};
+    if (bias && wave == 0) {        // (the first of the waves that split K)
+#pragma unroll
+        for (int r = 0; r < R; ++r) {
+            const floatx4 b = bias4(bias, (nb0 + r) * 16 + fg * 4, NB);
+#pragma unroll
+            for (int t = 0; t < MT; ++t) acc[r][t] = b;
+        }
+    }
 
     // k-steps of 32 are dealt out to the waves in contiguous runs
     const int per = (KB + KSPLIT - 1) / KSPLIT;
@@ -1005,17 +1036,17 @@ __global__ __launch_bounds__(64 * KSPLIT * NSETS) void gemm_bf16_skinny_kernel(
 
 template <int MT, int R, int UNROLL, int KSPLIT, int NSETS = 1, bool GLU = false, bool RING = false, int EPI = 0>
 static int launch_skinny(const bf16_t* A, const bf16_t* Wp, void* C, int M, int N, int K, int lda,
-                         int c_dtype, int n_out, hipStream_t s, const SkinnyFuse* fuse = nullptr) {
+                         const float* bias, int c_dtype, int n_out, hipStream_t s, const SkinnyFuse* fuse = nullptr) {
     const int NB = (N + 15) / 16, KB = (K + 31) / 32;
     const int per_block = NSETS * R;
     const dim3 grid((NB + per_block - 1) / per_block);
     const SkinnyFuse fz = fuse ? *fuse : SkinnyFuse{nullptr, 0, 0, 0.f, 0.f, nullptr, nullptr, nullptr, nullptr, 0, nullptr, 0.f};
     if (c_dtype == TFF_F32)
         gemm_bf16_skinny_kernel<MT, R, UNROLL, KSPLIT, NSETS, GLU, float, RING, EPI>
-            <<<grid, 64 * KSPLIT * NSETS, 0, s>>>(A, Wp, (float*)C, M, N, K, lda, KB, n_out, fz);
+            <<<grid, 64 * KSPLIT * NSETS, 0, s>>>(A, Wp, (float*)C, M, N, K, lda, KB, n_out, fz, bias);
     else if constexpr (EPI < 2)
         gemm_bf16_skinny_kernel<MT, R, UNROLL, KSPLIT, NSETS, GLU, bf16_t, RING, EPI>
-            <<<grid, 64 * KSPLIT * NSETS, 0, s>>>(A, Wp, (bf16_t*)C, M, N, K, lda, KB, n_out, fz);
+            <<<grid, 64 * KSPLIT * NSETS, 0, s>>>(A, Wp, (bf16_t*)C, M, N, K, lda, KB, n_out, fz, bias);
     else
         return tff_fail("gemm: the product before a norm has a float32 result");
     return tff_check_launch("gemm_bf16_skinny");
@@ -1201,19 +1232,19 @@ TFF_API int tff_gemm_plan(int M, int N, int K, int glu, int keep_partials, int* 
 // a group's whole K through a ring (384 such waves, at N = 6,144, are too few: 3 % slower).  Plain: more waves per block where there are few blocks
 // (small N) or long rows (large K), fewer and deeper ones in between.
 template <int EPI>
-static int skinny_for(const bf16_t* A, const bf16_t* Wp, void* C, int M, int N, int K, int lda, int c_dtype,
+static int skinny_for(const bf16_t* A, const bf16_t* Wp, void* C, int M, int N, int K, int lda, const float* bias, int c_dtype,
                       int glu_out, hipStream_t s, const SkinnyFuse* fuse) {
     if (glu_out > 0) {
         if constexpr (EPI < 2) {
             if (N >= 8 * 1024)
-                return launch_skinny<1, 1, 8, 1, 2, true, true, EPI>(A, Wp, C, M, N, K, lda, c_dtype, glu_out, s, fuse);
+                return launch_skinny<1, 1, 8, 1, 2, true, true, EPI>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, fuse);
             // A wave takes a quarter of K in groups of k-steps whose loads are issued together, and
             // the steps that are left when a group is not full go one at a time: groups of eight
             // where a quarter of K is fewer than 32 steps, of 32 (with the norm's factor taken in,
             // which needs registers of its own, 24) otherwise.
             if (K < 4096)
-                return launch_skinny<1, 1, 8, 4, 2, true, false, EPI>(A, Wp, C, M, N, K, lda, c_dtype, glu_out, s, fuse);
-            return launch_skinny<1, 1, (EPI == 1 ? 24 : 32), 4, 2, true, false, EPI>(A, Wp, C, M, N, K, lda, c_dtype, glu_out, s, fuse);
+                return launch_skinny<1, 1, 8, 4, 2, true, false, EPI>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, fuse);
+            return launch_skinny<1, 1, (EPI == 1 ? 24 : 32), 4, 2, true, false, EPI>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, fuse);
         } else {
             return tff_fail("gemm: a gated product does not come before a norm");
         }
@@ -1227,7 +1258,7 @@ static int skinny_for(const bf16_t* A, const bf16_t* Wp, void* C, int M, int N, 
     // 39.8 against 42.9 / 42.8 at 1 / 8 rows (at 16 rows the tiles are ahead, see plan_for).  Not for
     // the product after a norm: the row factors' registers do not fit beside two row groups.
     if constexpr (EPI != 1) {
-        if (two_row_groups(N)) return launch_skinny<1, 2, 4, 16, 1, false, false, EPI>(A, Wp, C, M, N, K, lda, c_dtype, 0, s, fuse);
+        if (two_row_groups(N)) return launch_skinny<1, 2, 4, 16, 1, false, false, EPI>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, fuse);
     }
     // A very wide product (an output head) has thousands of blocks, each of which fetches all of A's
     // rows: with many rows and a long K that traffic shows (152k columns, K = 4,096: 196 / 217 / 281 us
@@ -1235,23 +1266,25 @@ static int skinny_for(const bf16_t* A, const bf16_t* Wp, void* C, int M, int N, 
     // 8 / 16 rows 264 / 303 us against 278 / 366; with fewer rows one group a block stays ahead.
     if constexpr (EPI == 0) {
         if (N >= 32 * 1024 && (long)M * K >= 40000)
-            return launch_skinny<1, 2, 4, 8, 1, false, false, 0>(A, Wp, C, M, N, K, lda, c_dtype, 0, s, fuse);
+            return launch_skinny<1, 2, 4, 8, 1, false, false, 0>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, fuse);
     }
     // (K up to 1,024: sixteen waves would have two k-steps each, less than a group of four)
     if (N >= 32 * 1024 || K <= 1024)
-        return launch_skinny<1, 1, 4, 8, 1, false, false, EPI>(A, Wp, C, M, N, K, lda, c_dtype, 0, s, fuse);
+        return launch_skinny<1, 1, 4, 8, 1, false, false, EPI>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, fuse);
     if (K >= 8192 || N <= 4096)
-        return launch_skinny<1, 1, 4, 16, 1, false, false, EPI>(A, Wp, C, M, N, K, lda, c_dtype, 0, s, fuse);
-    return launch_skinny<1, 1, 8, 4, 1, false, false, EPI>(A, Wp, C, M, N, K, lda, c_dtype, 0, s, fuse);
+        return launch_skinny<1, 1, 4, 16, 1, false, false, EPI>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, fuse);
+    return launch_skinny<1, 1, 8, 4, 1, false, false, EPI>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, fuse);
 }
 
 // glu_out > 0: W holds gate and up groups in turn (N = 2 * ceil16(glu_out) rows) and C is
 // [M, glu_out] = silu(gate) * up.  workspace: room for partial sums (tff_gemm_workspace_bytes);
 // with less the blocks do not split K.
+// bias (may be null): ceil16(N) float32 numbers in the order of W's rows, added to the product (before the gate's
+// activation): the accumulators start from them (of a split K, the first part's).
 // keep_partials: where the plan splits K, the partial sums stay in the workspace
 // ([splits, M, N] float32) for the caller to add up, and C is not written.
 int tff_gemm_bf16(const bf16_t* A, const bf16_t* Wp, void* C, int M, int N, int K, int lda,
-                  int c_dtype, int glu_out, float* workspace, size_t workspace_bytes,
+                  const float* bias, int c_dtype, int glu_out, float* workspace, size_t workspace_bytes,
                   int keep_partials, hipStream_t s) {
     TFF_REQUIRE(K % 8 == 0 && lda % 8 == 0,
                 "gemm: the bfloat16 product needs the inner size (K=%d, row stride %d) to be a multiple of 8",
@@ -1269,64 +1302,64 @@ int tff_gemm_bf16(const bf16_t* A, const bf16_t* Wp, void* C, int M, int N, int 
     if (glu_out > 0) {
         TFF_REQUIRE(N % 32 == 0 && glu_out <= N / 2 && glu_out > N / 2 - 16,
                     "gemm: a gated weight of %d rows does not fit %d output columns", N, glu_out);
-        if (plan.tile == 0) return skinny_for<0>(A, Wp, C, M, N, K, lda, c_dtype, glu_out, s, nullptr);
+        if (plan.tile == 0) return skinny_for<0>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, nullptr);
         if (plan.tile <= 64 && K % 64 == 0) {                // the four waves side by side on 64 or 32 rows
-            if (plan.tile == 32 && plan.bn == 128) return launch_w4<2, 5, true, 1, false, 2>(A, Wp, C, M, N, K, lda, c_dtype, glu_out, s, S, workspace);
-            if (plan.tile == 32) return launch_w4<4, 5, true, 1, false, 2>(A, Wp, C, M, N, K, lda, c_dtype, glu_out, s, S, workspace);
-            if (plan.bn == 128) return launch_w4<2, 5, true, 1, false, 4>(A, Wp, C, M, N, K, lda, c_dtype, glu_out, s, S, workspace);
-            return launch_w4<4, 5, true, 1, false, 4>(A, Wp, C, M, N, K, lda, c_dtype, glu_out, s, S, workspace);
+            if (plan.tile == 32 && plan.bn == 128) return launch_w4<2, 5, true, 1, false, 2>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, S, workspace);
+            if (plan.tile == 32) return launch_w4<4, 5, true, 1, false, 2>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, S, workspace);
+            if (plan.bn == 128) return launch_w4<2, 5, true, 1, false, 4>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, S, workspace);
+            return launch_w4<4, 5, true, 1, false, 4>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, S, workspace);
         }
         if (plan.tile == 64)
-            return launch_async_g<2, 2, 2, 4, 3, true>(A, Wp, C, M, N, K, lda, c_dtype, glu_out, s, S, workspace);
+            return launch_async_g<2, 2, 2, 4, 3, true>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, S, workspace);
         if (K % 64 == 0) {
             if (plan.tile == 128) {
-                if (plan.bn == 128) return launch_w4<2, 5, true, 1>(A, Wp, C, M, N, K, lda, c_dtype, glu_out, s, S, workspace);
-                if (plan.bn == 256) return launch_w4<4, 5, true, 1>(A, Wp, C, M, N, K, lda, c_dtype, glu_out, s, S, workspace);
-                return launch_w4<6, 4, true, 1>(A, Wp, C, M, N, K, lda, c_dtype, glu_out, s, S, workspace);
+                if (plan.bn == 128) return launch_w4<2, 5, true, 1>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, S, workspace);
+                if (plan.bn == 256) return launch_w4<4, 5, true, 1>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, S, workspace);
+                return launch_w4<6, 4, true, 1>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, S, workspace);
             }
-            if (plan.bn == 128) return launch_w4<4, 5, true>(A, Wp, C, M, N, K, lda, c_dtype, glu_out, s, S, workspace);
-            if (plan.bn == 192) return launch_w4<6, 5, true>(A, Wp, C, M, N, K, lda, c_dtype, glu_out, s, S, workspace);
-            return launch_w4<8, 4, true>(A, Wp, C, M, N, K, lda, c_dtype, glu_out, s, S, workspace);
+            if (plan.bn == 128) return launch_w4<4, 5, true>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, S, workspace);
+            if (plan.bn == 192) return launch_w4<6, 5, true>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, S, workspace);
+            return launch_w4<8, 4, true>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, S, workspace);
         }
         if (plan.tile == 128 && plan.bn == 128)
-            return launch_async_g<2, 2, 4, 4, 3, true>(A, Wp, C, M, N, K, lda, c_dtype, glu_out, s, S, workspace);
+            return launch_async_g<2, 2, 4, 4, 3, true>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, S, workspace);
         if (plan.tile == 128)
-            return launch_async_g<2, 4, 4, 4, 3, true>(A, Wp, C, M, N, K, lda, c_dtype, glu_out, s, S, workspace);
-        return launch_async_g<4, 4, 4, 4, 5, true, 1, true>(A, Wp, C, M, N, K, lda, c_dtype, glu_out, s, S, workspace);
+            return launch_async_g<2, 4, 4, 4, 3, true>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, S, workspace);
+        return launch_async_g<4, 4, 4, 4, 5, true, 1, true>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, S, workspace);
     }
-    if (plan.tile == 0) return skinny_for<0>(A, Wp, C, M, N, K, lda, c_dtype, 0, s, nullptr);
+    if (plan.tile == 0) return skinny_for<0>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, nullptr);
     if (plan.tile == 64 || plan.tile == 32) {
         // few columns and no room for partial sums: the streaming kernel, whose blocks split K
         // among their waves
         if (S == 1 && planned_splits > 1 && M <= 64) {
-            if (M <= 32) return launch_skinny<2, 2, 4, 8>(A, Wp, C, M, N, K, lda, c_dtype, 0, s);
-            return launch_skinny<4, 2, 4, 8>(A, Wp, C, M, N, K, lda, c_dtype, 0, s);
+            if (M <= 32) return launch_skinny<2, 2, 4, 8>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s);
+            return launch_skinny<4, 2, 4, 8>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s);
         }
         if (K % 64 == 0) {                                   // the four waves side by side on 64 or 32 rows
-            if (plan.tile == 32 && plan.bn == 128) return launch_w4<2, 5, false, 1, false, 2>(A, Wp, C, M, N, K, lda, c_dtype, 0, s, S, workspace, red);
-            if (plan.tile == 32) return launch_w4<4, 5, false, 1, false, 2>(A, Wp, C, M, N, K, lda, c_dtype, 0, s, S, workspace, red);
-            if (plan.bn == 128) return launch_w4<2, 5, false, 1, false, 4>(A, Wp, C, M, N, K, lda, c_dtype, 0, s, S, workspace, red);
-            return launch_w4<4, 5, false, 1, false, 4>(A, Wp, C, M, N, K, lda, c_dtype, 0, s, S, workspace, red);
+            if (plan.tile == 32 && plan.bn == 128) return launch_w4<2, 5, false, 1, false, 2>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, S, workspace, red);
+            if (plan.tile == 32) return launch_w4<4, 5, false, 1, false, 2>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, S, workspace, red);
+            if (plan.bn == 128) return launch_w4<2, 5, false, 1, false, 4>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, S, workspace, red);
+            return launch_w4<4, 5, false, 1, false, 4>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, S, workspace, red);
         }
-        return launch_async_g<2, 2, 2, 4, 3>(A, Wp, C, M, N, K, lda, c_dtype, 0, s, S, workspace, red);
+        return launch_async_g<2, 2, 2, 4, 3>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, S, workspace, red);
     }
     if (K % 64 == 0) {
         if (plan.tile == 128) {
-            if (plan.bn == 128) return launch_w4<2, 5, false, 1>(A, Wp, C, M, N, K, lda, c_dtype, 0, s, S, workspace, red);
-            if (plan.bn == 256) return launch_w4<4, 5, false, 1>(A, Wp, C, M, N, K, lda, c_dtype, 0, s, S, workspace, red);
-            return launch_w4<6, 4, false, 1>(A, Wp, C, M, N, K, lda, c_dtype, 0, s, S, workspace, red);
+            if (plan.bn == 128) return launch_w4<2, 5, false, 1>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, S, workspace, red);
+            if (plan.bn == 256) return launch_w4<4, 5, false, 1>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, S, workspace, red);
+            return launch_w4<6, 4, false, 1>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, S, workspace, red);
         }
-        if (plan.bn == 128) return launch_w4<4, 5>(A, Wp, C, M, N, K, lda, c_dtype, 0, s, S, workspace, red);
-        if (plan.bn == 192) return launch_w4<6, 5>(A, Wp, C, M, N, K, lda, c_dtype, 0, s, S, workspace, red);
-        return launch_w4<8, 4>(A, Wp, C, M, N, K, lda, c_dtype, 0, s, S, workspace, red);
+        if (plan.bn == 128) return launch_w4<4, 5>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, S, workspace, red);
+        if (plan.bn == 192) return launch_w4<6, 5>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, S, workspace, red);
+        return launch_w4<8, 4>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, S, workspace, red);
     }
     if (plan.tile == 128 && plan.bn == 128)
-        return launch_async_g<2, 2, 4, 4, 3>(A, Wp, C, M, N, K, lda, c_dtype, 0, s, S, workspace, red);
+        return launch_async_g<2, 2, 4, 4, 3>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, S, workspace, red);
     if (plan.tile == 128)
-        return launch_async_g<2, 4, 4, 4, 3>(A, Wp, C, M, N, K, lda, c_dtype, 0, s, S, workspace, red);
+        return launch_async_g<2, 4, 4, 4, 3>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, S, workspace, red);
     if (plan.bn == 192)
-        return launch_async_g<4, 4, 4, 3, 5, false, 1, true>(A, Wp, C, M, N, K, lda, c_dtype, 0, s, S, workspace, red);
-    return launch_async_g<4, 4, 4, 4, 5, false, 1, true>(A, Wp, C, M, N, K, lda, c_dtype, 0, s, S, workspace, red);
+        return launch_async_g<4, 4, 4, 3, 5, false, 1, true>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, S, workspace, red);
+    return launch_async_g<4, 4, 4, 4, 5, false, 1, true>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, S, workspace, red);
 }
 
 // ---- the norm between two products of up to 16 rows, taken into them ----
@@ -1353,7 +1386,7 @@ TFF_API int tff_gemm_residual_prenorm(const void* A, const void* Wp, int M, int 
     TFF_REQUIRE(((uintptr_t)resid % 16) == 0 && ((uintptr_t)norm_w % 16) == 0 && ((uintptr_t)x_out % 8) == 0,
                 "gemm_residual_prenorm: operands must be 16-byte aligned");
     SkinnyFuse fz{nullptr, 0, 0, 0.f, 0.f, resid, norm_w, (bf16_t*)x_out, ss_out, ss_stride, nullptr, 0.f};
-    return skinny_for<2>((const bf16_t*)A, (const bf16_t*)Wp, resid, M, N, K, lda, TFF_F32, 0, (hipStream_t)stream, &fz);
+    return skinny_for<2>((const bf16_t*)A, (const bf16_t*)Wp, resid, M, N, K, lda, nullptr, TFF_F32, 0, (hipStream_t)stream, &fz);
 }
 
 // resid[M, N] += A . W^T (bfloat16 A and packed W, float32 sums); x_out[M, N] = bfloat16 of
@@ -1367,7 +1400,7 @@ TFF_API int tff_gemm_residual_dyt(const void* A, const void* Wp, int M, int N, i
     TFF_REQUIRE(((uintptr_t)resid % 16) == 0 && ((uintptr_t)norm_w % 16) == 0 && ((uintptr_t)bias % 16) == 0 &&
                 ((uintptr_t)x_out % 8) == 0, "gemm_residual_dyt: operands must be 16-byte aligned");
     SkinnyFuse fz{nullptr, 0, 0, 0.f, 0.f, resid, norm_w, (bf16_t*)x_out, nullptr, 0, bias, alpha};
-    return skinny_for<3>((const bf16_t*)A, (const bf16_t*)Wp, resid, M, N, K, lda, TFF_F32, 0, (hipStream_t)stream, &fz);
+    return skinny_for<3>((const bf16_t*)A, (const bf16_t*)Wp, resid, M, N, K, lda, nullptr, TFF_F32, 0, (hipStream_t)stream, &fz);
 }
 
 // C = rstd[m] * (A . W^T) with rstd[m] = rsqrt(sum_g ss[m][g] / dim + eps), g < ss_count: the product
@@ -1391,32 +1424,33 @@ TFF_API int tff_gemm_row_scaled(const void* A, const void* Wp, void* C, int M, i
         const bf16_t* w = (const bf16_t*)Wp;
         hipStream_t s = (hipStream_t)stream;
         if (plan_rows32(N, K) == 128)
-            return launch_w4<2, 5, true, 1, true, 2>(a, w, C, M, N, K, lda, c_dtype, glu_out, s, 1, nullptr, true, sc);
-        return launch_w4<4, 5, true, 1, true, 2>(a, w, C, M, N, K, lda, c_dtype, glu_out, s, 1, nullptr, true, sc);
+            return launch_w4<2, 5, true, 1, true, 2>(a, w, C, M, N, K, lda, nullptr, c_dtype, glu_out, s, 1, nullptr, true, sc);
+        return launch_w4<4, 5, true, 1, true, 2>(a, w, C, M, N, K, lda, nullptr, c_dtype, glu_out, s, 1, nullptr, true, sc);
     }
     SkinnyFuse fz{ss, ss_stride, ss_count, 1.0f / (float)dim, eps, nullptr, nullptr, nullptr, nullptr, 0, nullptr, 0.f};
-    return skinny_for<1>((const bf16_t*)A, (const bf16_t*)Wp, C, M, N, K, lda, c_dtype, glu_out, (hipStream_t)stream, &fz);
+    return skinny_for<1>((const bf16_t*)A, (const bf16_t*)Wp, C, M, N, K, lda, nullptr, c_dtype, glu_out, (hipStream_t)stream, &fz);
 }
 
 int tff_gemm_f32(const float* A, const float* W, void* C, int M, int N, int K, int lda,
                  int c_dtype, hipStream_t s);
 
 TFF_API int tff_gemm(const void* A, const void* W, void* C, int M, int N, int K, int lda,
-                     int ab_dtype, int c_dtype, int w_packed, int glu_out, void* workspace,
+                     int ab_dtype, int c_dtype, int w_packed, int glu_out, const float* bias, void* workspace,
                      size_t workspace_bytes, int keep_partials, tff_stream_t stream) {
     TFF_REQUIRE(A && W && C, "gemm: null pointer");
     TFF_REQUIRE(M >= 0 && N > 0 && K > 0 && lda >= K, "gemm: bad sizes M=%d N=%d K=%d lda=%d", M, N, K, lda);
     if (M == 0) return 0;
     hipStream_t s = (hipStream_t)stream;
     if (ab_dtype == TFF_F32) {
-        TFF_REQUIRE(!w_packed && glu_out == 0 && !keep_partials,
-                    "gemm: the float32 product takes a plain row-major weight and keeps no partial sums");
+        TFF_REQUIRE(!w_packed && glu_out == 0 && !keep_partials && !bias,
+                    "gemm: the float32 product takes a plain row-major weight, no bias and keeps no partial sums");
         return tff_gemm_f32((const float*)A, (const float*)W, C, M, N, K, lda, c_dtype, s);
     }
     if (ab_dtype == TFF_BF16) {
         TFF_REQUIRE(w_packed, "gemm: the bfloat16 product takes a weight in fragment order");
         TFF_REQUIRE(((uintptr_t)workspace % 16) == 0, "gemm: the workspace must be 16-byte aligned");
-        return tff_gemm_bf16((const bf16_t*)A, (const bf16_t*)W, C, M, N, K, lda, c_dtype, glu_out,
+        TFF_REQUIRE(((uintptr_t)bias % 16) == 0, "gemm: the bias must be 16-byte aligned");
+        return tff_gemm_bf16((const bf16_t*)A, (const bf16_t*)W, C, M, N, K, lda, bias, c_dtype, glu_out,
                              (float*)workspace, workspace ? workspace_bytes : 0, keep_partials, s);
     }
     return tff_fail("gemm: unknown operand type %d", ab_dtype);

@@ -1,0 +1,183 @@
+// What stands around the paged attention kernels in a grouped attention whose queries carry a temperature that grows
+// with the position and whose window has the mean keys of whole blocks of tokens before it.
+//
+// tff_grouped_qkv_store:  from the joint projection (float32): rotation of q and k, the temperature on q, q laid out
+//                         with the cache's head size, the token's key and value into its slot.
+// tff_pool_keys:          for every token of the step that ends a block of P tokens: the means of the block's P keys and
+//                         values, as the pages hold them, into the block's slot.
+// tff_gate_heads:         a head's output times one gate per head, heads brought together.
+#include "common.h"
+#include "tffinfer_kernels.h"
+
+struct GroupedRot {
+    const float* cs;     // the position's [pair][cos, sin], or null
+    int dims;            // rotated elements of a head (even)
+    int pairing;         // 0: (i, i + dims/2), 1: (2i, 2i+1)
+};
+
+__device__ __forceinline__ float grouped_rotated(const float* __restrict__ x, int e, const GroupedRot r) {
+    const float v = x[e];
+    if (!r.cs || e >= r.dims) return v;
+    int i, other;
+    bool first;
+    if (r.pairing == 0) {
+        const int half = r.dims >> 1;
+        first = e < half;
+        i = first ? e : e - half;
+        other = first ? e + half : e - half;
+    } else {
+        first = !(e & 1);
+        i = e >> 1;
+        other = e ^ 1;
+    }
+    const float o = x[other], c = r.cs[2 * i], s = r.cs[2 * i + 1];
+    // the pair (u, w) becomes (u c - w s, w c + u s)
+    return first ? fmaf(v, c, -(o * s)) : fmaf(v, c, o * s);
+}
+
+// Blocks (token, y): y < q_blocks works through GQ_HEADS query heads; the others are one kv head each: its key row and
+// its value row into the token's slot.  Elements past a head's own size are zeros.
+#define GQ_THREADS 128
+#define GQ_HEADS 8
+
+template <typename TC>
+__global__ __launch_bounds__(GQ_THREADS) void grouped_qkv_store_kernel(
+    const float* __restrict__ proj, size_t row, const float* __restrict__ cos_sin, int rot_dims, int pairing, int max_pos,
+    float temp_coef, int temp_every, const int32_t* __restrict__ positions, const int32_t* __restrict__ slots,
+    TC* __restrict__ q_out, TC* __restrict__ k_cache, TC* __restrict__ v_cache, int page_size, int H, int G, int D, int E, int P,
+    int q_blocks) {
+    const int t = blockIdx.x, y = blockIdx.y, tid = threadIdx.x;
+    const float* x = proj + (size_t)t * row;
+    const int pos = max(positions[t], 0), tpos = min(pos, max(max_pos - 1, 0));
+    const GroupedRot rot{(cos_sin && rot_dims) ? cos_sin + (size_t)tpos * rot_dims : nullptr, rot_dims, pairing};
+    if (y < q_blocks) {
+        const float temp = temp_coef != 0.f ? 1.0f + temp_coef * logf((float)((pos + 1) / temp_every + 1)) : 1.0f;
+        TC* qo = q_out + (size_t)t * H * P;
+        const int h0 = y * GQ_HEADS, h1 = min(H, h0 + GQ_HEADS);
+        for (int h = h0; h < h1; ++h)
+            for (int e = tid; e < P; e += GQ_THREADS)
+                qo[(size_t)h * P + e] = from_f32<TC>(e < D ? grouped_rotated(x + (size_t)h * D, e, rot) * temp : 0.f);
+        return;
+    }
+    const int slot = slots[t];
+    if (slot < 0) return;      // (the whole block: a token that writes no key)
+    const int g = y - q_blocks;
+    const int page = slot / page_size, off = slot - page * page_size;
+    const float* xk = x + (size_t)H * D + (size_t)g * D;
+    const float* xv = x + (size_t)H * D + (size_t)G * D + (size_t)g * E;
+    TC* kd = k_cache + (((size_t)page * G + g) * page_size + off) * P;
+    TC* vd = v_cache + ((size_t)page * G + g) * P * page_size + off;
+    for (int e = tid; e < P; e += GQ_THREADS) {
+        kd[e] = from_f32<TC>(e < D ? grouped_rotated(xk, e, rot) : 0.f);
+        vd[(size_t)e * page_size] = from_f32<TC>(e < E ? xv[e] : 0.f);
+    }
+}
+
+TFF_API int tff_grouped_qkv_store(const float* proj, size_t row, const float* cos_sin, int rot_dims, int pairing, int max_pos,
+                                  float temp_coef, int temp_every, const int32_t* positions, const int32_t* slots, void* q_out,
+                                  void* k_cache, void* v_cache, int page_size, int num_pages, int T, int H, int G, int D, int E,
+                                  int P, int store, int dtype, tff_stream_t stream) {
+    TFF_REQUIRE(proj && positions && q_out && (!store || (slots && k_cache && v_cache)), "grouped_qkv_store: null pointer");
+    TFF_REQUIRE(T >= 0 && H > 0 && G > 0 && H % G == 0 && D > 0 && E > 0 && P >= D && P >= E && temp_every > 0,
+                "grouped_qkv_store: bad sizes H=%d G=%d D=%d E=%d P=%d", H, G, D, E, P);
+    TFF_REQUIRE(row >= (size_t)H * D + (store ? (size_t)G * (D + E) : 0), "grouped_qkv_store: rows of %zu are too short", row);
+    TFF_REQUIRE(rot_dims >= 0 && rot_dims <= D && rot_dims % 2 == 0 && (rot_dims == 0 || (cos_sin && max_pos > 0)) &&
+                (pairing == 0 || pairing == 1), "grouped_qkv_store: %d rotated elements of a head of %d need an even count and a table", rot_dims, D);
+    TFF_REQUIRE(page_size > 0 && num_pages > 0, "grouped_qkv_store: bad cache geometry");
+    if (T == 0) return 0;
+    hipStream_t s = (hipStream_t)stream;
+    const int q_blocks = (H + GQ_HEADS - 1) / GQ_HEADS, kv_blocks = store ? G : 0;
+    TFF_REQUIRE(q_blocks + kv_blocks <= 65535, "grouped_qkv_store: too many heads");
+    const dim3 grid(T, q_blocks + kv_blocks);
+#define GQ_LAUNCH(TC)                                                                                                          \
+    grouped_qkv_store_kernel<TC><<<grid, GQ_THREADS, 0, s>>>(proj, row, cos_sin, rot_dims, pairing, max_pos, temp_coef, temp_every, \
+                                                             positions, slots, (TC*)q_out, (TC*)k_cache, (TC*)v_cache, page_size, H, \
+                                                             G, D, E, P, q_blocks)
+    if (dtype == TFF_F32) GQ_LAUNCH(float);
+    else if (dtype == TFF_BF16) GQ_LAUNCH(bf16_t);
+    else return tff_fail("grouped_qkv_store: unknown dtype %d", dtype);
+#undef GQ_LAUNCH
+    return tff_check_launch("grouped_qkv_store");
+}
+
+// Blocks (token, kv head).  The sum runs over the block's tokens in their order; a thread takes elements tid, tid + 128, ...
+#define PK_THREADS 128
+
+template <typename TC>
+__global__ __launch_bounds__(PK_THREADS) void pool_keys_kernel(TC* __restrict__ k_cache, TC* __restrict__ v_cache,
+                                                               const int32_t* __restrict__ block_tables, int bt_stride,
+                                                               const int32_t* __restrict__ pool_tables, int pt_stride,
+                                                               const int32_t* __restrict__ token_req,
+                                                               const int32_t* __restrict__ positions,
+                                                               const int32_t* __restrict__ slots, int page_size, int pool, int G,
+                                                               int d) {
+    const int t = blockIdx.x, g = blockIdx.y;
+    const int pos = positions[t];
+    if (slots[t] < 0 || (pos + 1) % pool) return;      // (the whole block)
+    const int r = token_req[t], blk = pos / pool, first = pos + 1 - pool;
+    const int32_t* bt = block_tables + (size_t)r * bt_stride;
+    const int dpage = pool_tables[(size_t)r * pt_stride + blk / page_size], dslot = blk % page_size;
+    const float f = 1.0f / (float)pool;
+    for (int e = threadIdx.x; e < d; e += PK_THREADS) {
+        float ks = 0.f, vs = 0.f;
+#pragma unroll 4
+        for (int i = 0; i < pool; ++i) {
+            const int j = first + i, slot = j % page_size;
+            const size_t head = ((size_t)bt[j / page_size] * G + g) * page_size * d;
+            ks += to_f32(k_cache[head + (size_t)slot * d + e]);
+            vs += to_f32(v_cache[head + (size_t)e * page_size + slot]);
+        }
+        const size_t head = ((size_t)dpage * G + g) * page_size * d;
+        k_cache[head + (size_t)dslot * d + e] = from_f32<TC>(ks * f);
+        v_cache[head + (size_t)e * page_size + dslot] = from_f32<TC>(vs * f);
+    }
+}
+
+TFF_API int tff_pool_keys(void* k_cache, void* v_cache, const int32_t* block_tables, int bt_stride, const int32_t* pool_tables,
+                          int pt_stride, const int32_t* token_req, const int32_t* positions, const int32_t* slots, int page_size,
+                          int num_pages, int pool, int T, int G, int d, int dtype, tff_stream_t stream) {
+    TFF_REQUIRE(k_cache && v_cache && block_tables && pool_tables && token_req && positions && slots, "pool_keys: null pointer");
+    TFF_REQUIRE(T >= 0 && G > 0 && G <= 65535 && d > 0 && pool > 0 && page_size > 0 && num_pages > 0 && bt_stride > 0 && pt_stride > 0,
+                "pool_keys: bad sizes");
+    if (T == 0) return 0;
+    hipStream_t s = (hipStream_t)stream;
+    const dim3 grid(T, G);
+    if (dtype == TFF_F32)
+        pool_keys_kernel<float><<<grid, PK_THREADS, 0, s>>>((float*)k_cache, (float*)v_cache, block_tables, bt_stride, pool_tables, pt_stride,
+                                                            token_req, positions, slots, page_size, pool, G, d);
+    else if (dtype == TFF_BF16)
+        pool_keys_kernel<bf16_t><<<grid, PK_THREADS, 0, s>>>((bf16_t*)k_cache, (bf16_t*)v_cache, block_tables, bt_stride, pool_tables,
+                                                             pt_stride, token_req, positions, slots, page_size, pool, G, d);
+    else
+        return tff_fail("pool_keys: unknown dtype %d", dtype);
+    return tff_check_launch("pool_keys");
+}
+
+// out[t, h E + e] = o[t, h P + e] * sigmoid(g[t, h])      (g null: the heads brought together only)
+template <typename T>
+__global__ __launch_bounds__(256) void gate_heads_kernel(const T* __restrict__ o, size_t o_row, int P, const float* __restrict__ g,
+                                                         size_t g_row, T* __restrict__ out, int HE, int E, size_t count) {
+    const size_t id = (size_t)blockIdx.x * 256 + threadIdx.x;
+    if (id >= count) return;
+    const size_t t = id / HE;
+    const int c = (int)(id - t * HE), h = c / E, e = c - h * E;
+    const float f = g ? 1.0f / (1.0f + expf(-g[t * g_row + h])) : 1.0f;
+    out[t * HE + c] = from_f32<T>(to_f32(o[t * o_row + (size_t)h * P + e]) * f);
+}
+
+TFF_API int tff_gate_heads(const void* o, size_t o_row, int P, const float* g, size_t g_row, void* out, int T, int H, int E,
+                           int dtype, tff_stream_t stream) {
+    TFF_REQUIRE(o && out, "gate_heads: null pointer");
+    TFF_REQUIRE(T >= 0 && H > 0 && E > 0 && P >= E && o_row >= (size_t)H * P && (!g || g_row >= (size_t)H), "gate_heads: bad sizes");
+    if (T == 0) return 0;
+    hipStream_t s = (hipStream_t)stream;
+    const size_t count = (size_t)T * H * E;
+    const unsigned blocks = (unsigned)((count + 255) / 256);
+    if (dtype == TFF_F32)
+        gate_heads_kernel<float><<<blocks, 256, 0, s>>>((const float*)o, o_row, P, g, g_row, (float*)out, H * E, E, count);
+    else if (dtype == TFF_BF16)
+        gate_heads_kernel<bf16_t><<<blocks, 256, 0, s>>>((const bf16_t*)o, o_row, P, g, g_row, (bf16_t*)out, H * E, E, count);
+    else
+        return tff_fail("gate_heads: unknown dtype %d", dtype);
+    return tff_check_launch("gate_heads");
+}

@@ -10,6 +10,8 @@
 // tff_experts_down: out[t] = sum over the token's experts, in the order they were chosen, of
 //                   weight * (Wd y), float32.
 //
+// Experts numbered E and beyond have no matrices: such an expert hands its input on, f_e = h.
+//
 // The two expert kernels give every (token, expert) pair waves of its own that stream the
 // expert's rows once: what a step of few tokens is bound by.  Each output element is one
 // wave's dot product in a fixed order of k, so a token's result does not depend on what else
@@ -176,12 +178,13 @@ template <typename T>
 __global__ __launch_bounds__(64 * EX_WAVES) void experts_gate_up_kernel(
     const T* __restrict__ h, int h_row, const T* __restrict__ Wg, const T* __restrict__ Wu,
     const int32_t* __restrict__ idx, int top, int width, int ff, int ldw, float limit, float act_alpha, float up_offset,
-    const float* __restrict__ in_wts, T* __restrict__ y) {
+    const float* __restrict__ in_wts, T* __restrict__ y, int E) {
     // Wg null: experts without a gate, y = max(Wu h, 0)^2.  in_wts: the pair's weight multiplies what goes into the
     // expert, W (w h) = w (W h): both products times w before clamps and activation.
     const int pair = blockIdx.x;                  // token * top + k
     const int t = pair / top;
     const int e = idx[pair];
+    if (e >= E) return;                           // (an expert without matrices)
     const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
     const T* hr = h + (size_t)t * h_row;
     const T* wg = Wg ? Wg + (size_t)e * ff * ldw : nullptr;
@@ -212,7 +215,7 @@ __global__ __launch_bounds__(64 * EX_WAVES) void experts_gate_up_kernel(
 template <typename T>
 __global__ __launch_bounds__(64 * EX_WAVES) void experts_down_kernel(
     const T* __restrict__ y, const T* __restrict__ Wd, const int32_t* __restrict__ idx, const float* __restrict__ wts,
-    int top, int width, int ff, int ldw, float* __restrict__ out) {
+    int top, int width, int ff, int ldw, float* __restrict__ out, int E, const T* __restrict__ h, int h_row) {
     const int t = blockIdx.x;
     const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
     const bool vec = sizeof(T) == 2 && ff % 8 == 0 && ldw % 8 == 0 && ((uintptr_t)y % 16) == 0 && ((uintptr_t)Wd % 16) == 0;
@@ -221,7 +224,8 @@ __global__ __launch_bounds__(64 * EX_WAVES) void experts_down_kernel(
         float acc = 0.f;
         for (int k = 0; k < top; ++k) {
             const int e = idx[(size_t)t * top + k];
-            const float d = row_dot<T>(y + ((size_t)t * top + k) * ff, Wd + ((size_t)e * width + n) * ldw, ff, lane, vec);
+            const float d = e < E ? row_dot<T>(y + ((size_t)t * top + k) * ff, Wd + ((size_t)e * width + n) * ldw, ff, lane, vec)
+                                  : to_f32(h[(size_t)t * h_row + n]);
             acc = fmaf(wts ? wts[(size_t)t * top + k] : 1.0f, d, acc);
         }
         if (lane == 0) out[(size_t)t * width + n] = acc;
@@ -241,19 +245,22 @@ TFF_API int tff_experts_gate_up(const void* h, int h_row, const void* Wg, const 
     TFF_REQUIRE(grid.y <= 65535, "experts_gate_up: too many outputs");
     if (dtype == TFF_F32)
         experts_gate_up_kernel<float><<<grid, 64 * EX_WAVES, 0, s>>>((const float*)h, h_row, (const float*)Wg, (const float*)Wu,
-                                                                    idx, top, width, ff, ldw, limit, act_alpha, up_offset, in_wts, (float*)y);
+                                                                    idx, top, width, ff, ldw, limit, act_alpha, up_offset, in_wts, (float*)y, E);
     else if (dtype == TFF_BF16)
         experts_gate_up_kernel<bf16_t><<<grid, 64 * EX_WAVES, 0, s>>>((const bf16_t*)h, h_row, (const bf16_t*)Wg,
                                                                      (const bf16_t*)Wu, idx, top, width, ff, ldw, limit,
-                                                                     act_alpha, up_offset, in_wts, (bf16_t*)y);
+                                                                     act_alpha, up_offset, in_wts, (bf16_t*)y, E);
     else
         return tff_fail("experts_gate_up: unknown dtype %d", dtype);
     return tff_check_launch("experts_gate_up");
 }
 
+// h [T, width], rows h_row apart (may be null where every expert has matrices): what experts from number E on hand on.
 TFF_API int tff_experts_down(const void* y, const void* Wd, const int32_t* idx, const float* wts, int T, int top, int E,
-                             int width, int ff, int ldw, float* out, int dtype, tff_stream_t stream) {
+                             int width, int ff, int ldw, const void* h, int h_row, int identity, float* out, int dtype,
+                             tff_stream_t stream) {
     TFF_REQUIRE(y && Wd && idx && out, "experts_down: null pointer");      // (wts null: every pair counts 1)
+    TFF_REQUIRE(identity == 0 || (h && h_row >= width), "experts_down: experts without matrices need the rows they hand on");
     TFF_REQUIRE(T >= 0 && top > 0 && E > 0 && width > 0 && ff > 0 && ldw >= ff, "experts_down: bad sizes T=%d top=%d width=%d ff=%d",
                 T, top, width, ff);
     if (T == 0) return 0;
@@ -261,9 +268,9 @@ TFF_API int tff_experts_down(const void* y, const void* Wd, const int32_t* idx, 
     const dim3 grid(T, (width + EX_WAVES * EX_PER_WAVE - 1) / (EX_WAVES * EX_PER_WAVE));
     TFF_REQUIRE(grid.y <= 65535, "experts_down: too many outputs");
     if (dtype == TFF_F32)
-        experts_down_kernel<float><<<grid, 64 * EX_WAVES, 0, s>>>((const float*)y, (const float*)Wd, idx, wts, top, width, ff, ldw, out);
+        experts_down_kernel<float><<<grid, 64 * EX_WAVES, 0, s>>>((const float*)y, (const float*)Wd, idx, wts, top, width, ff, ldw, out, E, (const float*)h, h_row);
     else if (dtype == TFF_BF16)
-        experts_down_kernel<bf16_t><<<grid, 64 * EX_WAVES, 0, s>>>((const bf16_t*)y, (const bf16_t*)Wd, idx, wts, top, width, ff, ldw, out);
+        experts_down_kernel<bf16_t><<<grid, 64 * EX_WAVES, 0, s>>>((const bf16_t*)y, (const bf16_t*)Wd, idx, wts, top, width, ff, ldw, out, E, (const bf16_t*)h, h_row);
     else
         return tff_fail("experts_down: unknown dtype %d", dtype);
     return tff_check_launch("experts_down");
@@ -292,7 +299,8 @@ __global__ __launch_bounds__(1024) void experts_sort_kernel(const int32_t* __res
     const int tid = threadIdx.x;
     for (int e = tid; e < E; e += blockDim.x) count[e] = 0;
     __syncthreads();
-    for (int p = tid; p < pairs; p += blockDim.x) atomicAdd(&count[idx[p]], 1);
+    for (int p = tid; p < pairs; p += blockDim.x)
+        if (idx[p] < E) atomicAdd(&count[idx[p]], 1);       // (experts without matrices have no tiles)
     __syncthreads();
     if (tid == 0) {
         int t = 0;
@@ -313,6 +321,7 @@ __global__ __launch_bounds__(1024) void experts_sort_kernel(const int32_t* __res
     __syncthreads();
     for (int p = tid; p < pairs; p += blockDim.x) {
         const int e = idx[p];
+        if (e >= E) continue;
         const int at = atomicAdd(&count[e], 1);
         tile_rows[first[e] * rows + at] = p;
     }
@@ -472,6 +481,22 @@ __global__ __launch_bounds__(256) void experts_tiles_kernel(
     }
 }
 
+// The planes of the pairs whose expert has no matrices: out[k][t][:] = wts[t][k] * h[t][:].
+__global__ __launch_bounds__(256) void experts_identity_kernel(const bf16_t* __restrict__ h, int h_row,
+                                                               const int32_t* __restrict__ idx, const float* __restrict__ wts,
+                                                               int T, int top, int E, int width, float* __restrict__ out) {
+    const int p = blockIdx.x;
+    if (idx[p] < E) return;
+    const int t = p / top, k = p - t * top;
+    const float w = wts[p];
+    float* o = out + ((size_t)k * T + t) * width;
+    for (int e = threadIdx.x * 4; e < width; e += 1024) {       // (width is a multiple of 8 here)
+        union { uint2 u; bf16_t b[4]; } x;
+        x.u = *reinterpret_cast<const uint2*>(h + (size_t)t * h_row + e);
+        *reinterpret_cast<float4*>(o + e) = make_float4(w * (float)x.b[0], w * (float)x.b[1], w * (float)x.b[2], w * (float)x.b[3]);
+    }
+}
+
 TFF_API int tff_experts_tiles_supported(int width, int ff, int h_row) {
     return width % 8 == 0 && ff % 8 == 0 && h_row % 8 == 0;
 }
@@ -482,7 +507,7 @@ TFF_API int tff_experts_by_tiles(const void* h, int h_row, const void* Wg, const
                                  const int32_t* idx, const float* wts, int T, int top, int E, int width, int ff,
                                  int ldw_in, int ldw_down, float limit, float act_alpha, float up_offset, int32_t* tile_expert,
                                  int32_t* tile_rows, int32_t* num_tiles, int max_tiles, void* y, float* out,
-                                 int weight_input, tff_stream_t stream) {
+                                 int weight_input, int identity, tff_stream_t stream) {
     TFF_REQUIRE(h && Wu && Wd && idx && wts && tile_expert && tile_rows && num_tiles && y && out,
                 "experts_by_tiles: null pointer");
     TFF_REQUIRE(T >= 0 && top > 0 && E > 0 && E <= RT_MAX_E && width > 0 && ff > 0 && h_row >= width,
@@ -501,6 +526,10 @@ TFF_API int tff_experts_by_tiles(const void* h, int h_row, const void* Wg, const
     const int rows = tall ? 128 : 64;
     if (T == 0) return 0;
     hipStream_t s = (hipStream_t)stream;
+    if (identity > 0) {
+        experts_identity_kernel<<<T * top, 256, 0, s>>>((const bf16_t*)h, h_row, idx, wts, T, top, E, width, out);
+        if (int rc0 = tff_check_launch("experts_identity")) return rc0;
+    }
     experts_sort_kernel<<<1, 1024, 0, s>>>(idx, T * top, E, rows, tile_expert, tile_rows, num_tiles);
     int rc = tff_check_launch("experts_sort");
     if (rc) return rc;

@@ -40,6 +40,8 @@ TFF_API int tff_rmsnorm(const void* x, const float* weight, float eps, void* out
 // see tff_pack_weight).  glu_out > 0 (bfloat16 only): the 16-row groups of W
 // alternate between a gate and an up projection, N = 2 * ceil16(glu_out), and
 // C is [M, glu_out] = silu(gate) * up.
+// bias (may be null; bfloat16 only): ceil16(N) float32 numbers in the order of W's rows, added to the
+// product before the gate's activation.
 // workspace (may be null): device memory of tff_gemm_workspace_bytes() bytes the
 // product may keep partial sums in; with less it takes a path that needs none.
 // keep_partials (float32 result, no GLU): if the workspace is used, that is, if
@@ -48,7 +50,7 @@ TFF_API int tff_rmsnorm(const void* x, const float* weight, float eps, void* out
 // sums [bytes / (M * N * 4), M, N] are left there for the caller to add up
 // (tff_add_rmsnorm takes them as they are) and C is not written.
 TFF_API int tff_gemm(const void* A, const void* W, void* C, int M, int N, int K, int lda,
-                     int ab_dtype, int c_dtype, int w_packed, int glu_out, void* workspace,
+                     int ab_dtype, int c_dtype, int w_packed, int glu_out, const float* bias, void* workspace,
                      size_t workspace_bytes, int keep_partials, tff_stream_t stream);
 TFF_API size_t tff_gemm_workspace_bytes(int M, int N, int K, int ab_dtype, int glu, int keep_partials);
 // The bfloat16 product's plan for these sizes: rows and columns of a block tile (0: the
@@ -113,8 +115,8 @@ TFF_API int tff_attention_generic(const void* q, int q_stride, void* out,
                                   const int32_t* block_tables, int bt_stride,
                                   const int32_t* token_req, const int32_t* positions,
                                   int T, int nq, int nkv, int d, int page_size, int num_pages,
-                                  int window, float scale, const float* sinks, float softcap, int dtype, int cache_dtype,
-                                  tff_stream_t stream);
+                                  int window, float scale, const float* sinks, float softcap, const int32_t* pool_tables,
+                                  int pt_stride, int pool, int dtype, int cache_dtype, tff_stream_t stream);
 
 // bfloat16 attention on the matrix cores.  A wave works on `cols_per_wave` (16)
 // columns of one request and kv head; a column is a (token, q head of
@@ -139,7 +141,8 @@ TFF_API int tff_attention_mfma(const void* q, int q_stride, void* out, float* pa
                                const int32_t* block_items, int num_blocks,
                                int tiles_per_entry, int cols_per_wave, int key_groups, int splits, int T_total,
                                int nq, int nkv, int d, int page_size, int num_pages, int window,
-                               float scale, const float* sinks, float softcap, tff_stream_t stream);
+                               float scale, const float* sinks, float softcap, const int32_t* pool_tables, int pt_stride,
+                               int pool, tff_stream_t stream);
 // Decoding steps (every entry brings one token), bfloat16, from the fused projection's output:
 // row r of qkv ([R, (nq + 2 nkv) d], q heads first, then k, then v) is token r.  The kernel
 // does what tff_qk_norm_rope_kv and tff_attention_mfma do one after the other, in one pass:
@@ -305,7 +308,8 @@ TFF_API int tff_experts_gate_up(const void* h, int h_row, const void* Wg, const 
 // out[t, :] = sum_k wts[t, k] * Wd[idx[t, k]] y[(t, k), :]; Wd [E, width, ff], rows ldw elements apart; out float32.
 // wts null: every pair counts 1.
 TFF_API int tff_experts_down(const void* y, const void* Wd, const int32_t* idx, const float* wts, int T, int top, int E,
-                             int width, int ff, int ldw, float* out, int dtype, tff_stream_t stream);
+                             int width, int ff, int ldw, const void* h, int h_row, int identity, float* out, int dtype,
+                             tff_stream_t stream);
 
 // The same for steps of many tokens (bfloat16; width, ff and h_row multiples of 8): the (token, expert) pairs
 // are dealt to their experts in tiles of 64 or 128 rows and the two products run on the matrix cores.  out is
@@ -317,7 +321,7 @@ TFF_API int tff_experts_by_tiles(const void* h, int h_row, const void* Wg, const
                                  const int32_t* idx, const float* wts, int T, int top, int E, int width, int ff,
                                  int ldw_in, int ldw_down, float limit, float act_alpha, float up_offset, int32_t* tile_expert,
                                  int32_t* tile_rows, int32_t* num_tiles, int max_tiles, void* y, float* out,
-                                 int weight_input, tff_stream_t stream);
+                                 int weight_input, int identity, tff_stream_t stream);
 
 // ---- norms on a sublayer's output, sums over the model's depth (group_norm.hip) ----
 // y = delta row (planes added up first; row rows[r] where rows is given) cut into `groups` equal parts, each
@@ -412,11 +416,41 @@ TFF_API int tff_mixed_attention_q16(const void* q, const void* k_cache, const vo
                                     int window, int keep_first, int sink, void* out, int T, int H, int G, int D,
                                     int page_size, int splits, int tiles_per_split, float* workspace, tff_stream_t stream);
 
-TFF_API int tff_swiglu(const void* gu, void* out, int T, int I, int dtype, tff_stream_t stream);
+TFF_API int tff_swiglu(const void* gu, const float* bias, void* out, int T, int I, int dtype, tff_stream_t stream);
 
 // Element type conversion of n elements.
 TFF_API int tff_cast(const void* src, int src_dtype, void* dst, int dst_dtype, int64_t n,
                      tff_stream_t stream);
+
+// ---- norms before and after a sublayer, and the convolution of its input (sandwich_norm.hip) ----
+TFF_API int tff_add_layernorm(float* resid, const float* a, int planes_a, size_t plane_a, const float* b, int planes_b,
+                              size_t plane_b, const float* wa, const float* wb, float pair_eps, const float* bias,
+                              const float* nw, const float* nb, float n_eps, const float* scale, const float* w,
+                              const float* beta, float eps, void* out, const int32_t* rows, int n, int W, const float* conv_w,
+                              int taps, float* state, size_t state_row, size_t state_off, const int32_t* state_slots,
+                              int out_dtype, tff_stream_t stream);
+TFF_API int tff_input_conv_chunk(void);      // tokens an item of tff_input_conv holds at most
+TFF_API int tff_input_conv(const float* h, const float* w, int taps, float* state, size_t state_row, size_t state_off,
+                           const int32_t* items, int num_items, const int32_t* cu_tokens, const int32_t* state_slots, void* out,
+                           int W, int out_dtype, tff_stream_t stream);
+
+// ---- a linear recurrence with a fixed decay per head (lightning.hip) ----
+TFF_API int tff_lightning(const float* proj, size_t ldp, const float* decay, float* state, size_t state_row,
+                          const int32_t* cu_tokens, const int32_t* state_slots, float* o, int R, int H, int D, int E,
+                          int max_tokens, tff_stream_t stream);
+TFF_API int tff_row_norm_gate(const float* o, const float* g, size_t g_row, const float* w, float eps, void* out, int T, int N,
+                              int out_dtype, tff_stream_t stream);
+
+// ---- around a grouped attention with a query temperature and the mean keys of blocks (grouped_attention.hip) ----
+TFF_API int tff_grouped_qkv_store(const float* proj, size_t row, const float* cos_sin, int rot_dims, int pairing, int max_pos,
+                                  float temp_coef, int temp_every, const int32_t* positions, const int32_t* slots, void* q_out,
+                                  void* k_cache, void* v_cache, int page_size, int num_pages, int T, int H, int G, int D, int E,
+                                  int P, int store, int dtype, tff_stream_t stream);
+TFF_API int tff_pool_keys(void* k_cache, void* v_cache, const int32_t* block_tables, int bt_stride, const int32_t* pool_tables,
+                          int pt_stride, const int32_t* token_req, const int32_t* positions, const int32_t* slots, int page_size,
+                          int num_pages, int pool, int T, int G, int d, int dtype, tff_stream_t stream);
+TFF_API int tff_gate_heads(const void* o, size_t o_row, int P, const float* g, size_t g_row, void* out, int T, int H, int E,
+                           int dtype, tff_stream_t stream);
 
 // out[r] = lowest index among the maxima of logits[r, :].
 // workspace: tff_argmax_workspace_bytes(rows, V) bytes, 16-byte aligned (0: none needed), for the

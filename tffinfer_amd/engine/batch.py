@@ -28,10 +28,10 @@ class StepEntry:
 class KVView:
     """What a mixer sees of the cache in one layer call."""
     __slots__ = ("k_cache", "v_cache", "block_tables", "slot_mapping", "page_size", "group", "key_runs",
-                 "run_start", "runs_window", "runs_for_blocks", "runs_merge")
+                 "run_start", "runs_window", "runs_for_blocks", "runs_merge", "pool_tables")
 
     def __init__(self, k_cache, v_cache, block_tables, slot_mapping, page_size, group, key_runs=None,
-                 run_start=None, runs_window=0, runs_for_blocks=False, runs_merge=True):
+                 run_start=None, runs_window=0, runs_for_blocks=False, runs_merge=True, pool_tables=None):
         self.k_cache = k_cache
         self.v_cache = v_cache
         self.block_tables = block_tables
@@ -46,14 +46,15 @@ class KVView:
         self.runs_window = runs_window
         self.runs_for_blocks = runs_for_blocks
         self.runs_merge = runs_merge         # False: every request is one run, no result is partial
+        self.pool_tables = pool_tables or {}  # block size -> int32 [R, pages]: the pages of the blocks' mean keys
 
 
 class GroupTables:
     __slots__ = ("block_tables", "slot_mapping", "no_slot_mapping", "key_runs", "run_start", "runs_window",
-                 "runs_for_blocks", "runs_merge")
+                 "runs_for_blocks", "runs_merge", "pool_tables")
 
     def __init__(self, block_tables, slot_mapping, no_slot_mapping, key_runs=None, run_start=None, runs_window=0,
-                 runs_for_blocks=False, runs_merge=True):
+                 runs_for_blocks=False, runs_merge=True, pool_tables=None):
         self.block_tables = block_tables        # int32 [R, max_blocks]
         self.slot_mapping = slot_mapping        # int32 [T]: page * page_size + offset of each new token
         self.no_slot_mapping = no_slot_mapping  # int32 [T] of -1: for calls that only read a cache
@@ -62,6 +63,7 @@ class GroupTables:
         self.runs_window = runs_window
         self.runs_for_blocks = runs_for_blocks
         self.runs_merge = runs_merge            # False: the host knows that every request is one run
+        self.pool_tables = pool_tables or {}    # block size -> int32 [R, pages] (cache.manager: pools)
 
 
 class StepBatch:
@@ -161,6 +163,17 @@ def build_step_batch(entries, cache, device, pinned: PinnedTables | None = None)
             sections.append(dealt.runs.reshape(-1))
             sections.append(dealt.run_start)
             group_meta[-1] += (dealt.blocks, dealt.merge)
+    pool_meta = []      # (group, block size, section, width)
+    for gi, g in enumerate(cache.groups):
+        for which, p in enumerate(g.spec.pools):
+            tables = [cache.pool_table(gi, e.req, which) for e in entries]
+            width = max(1, max(len(t) for t in tables))
+            flat = []
+            for t in tables:
+                flat.extend(t)
+                flat.extend([0] * (width - len(t)))
+            pool_meta.append((gi, p, len(sections), width))
+            sections.append(flat)
     offs, total = [], 0
     for s in sections:
         offs.append(total)
@@ -191,6 +204,8 @@ def build_step_batch(entries, cache, device, pinned: PinnedTables | None = None)
             gt.runs_window = g.spec.window
             gt.runs_for_blocks, gt.runs_merge = dealt
         b.groups.append(gt)
+    for gi, p, si, width in pool_meta:
+        b.groups[gi].pool_tables[p] = dev[offs[si]:offs[si] + R * width].view(R, width)
     b.host_cu_tokens, b.host_start_pos, b.host_state_slots = cu, start, slots
     b.reqs = [e.req for e in entries]
     return b

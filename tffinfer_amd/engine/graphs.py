@@ -40,20 +40,28 @@ def _pad4(n: int) -> int:
     return (n + 3) & ~3
 
 
-def table_layout(bucket: int, widths: list[int], run_caps: list[int]) -> tuple[list[int], int]:
+def table_layout(bucket: int, widths: list[int], run_caps: list[int],
+                 pool_widths: list[int] = ()) -> tuple[list[int], int]:
     """Offsets of the sections of a decode step's packed tables (the order of
     build_step_batch) and their total length, for ``bucket`` rows; per cache group a block table
     of ``widths`` pages a row, the slots of the new tokens, ``run_caps`` runs of keys (four ints
-    each) and the rows' first runs."""
+    each) and the rows' first runs; then the tables of the groups' blocks, ``pool_widths`` pages a row."""
     B = bucket
     sizes = [B, B, B, B + 1, B, B, B, B, B]
     for w, cap in zip(widths, run_caps):
         sizes += [B * w, B, 4 * cap, B + 1]
+    sizes += [B * w for w in pool_widths]
     offs, total = [], 0
     for n in sizes:
         offs.append(total)
         total += _pad4(n)
     return offs, total
+
+
+def pool_table_widths(cache, max_model_len: int) -> list[tuple[int, int, int]]:
+    """(group, which of its block sizes, pages a row) of every table of blocks of a decode step."""
+    return [(gi, which, max(1, -(-(max_model_len // p) // cache.page_size)))
+            for gi, g in enumerate(cache.groups) for which, p in enumerate(g.spec.pools)]
 
 
 class DecodeTables:
@@ -75,7 +83,9 @@ class DecodeTables:
         ps = cache.page_size
         self.widths = [-(-max_model_len // ps) for _ in cache.groups]
         self.run_caps = [max_key_runs(B, g.spec.num_kv_heads) for g in cache.groups]
-        self.offs, self.total = table_layout(B, self.widths, self.run_caps)
+        #: (group, which of its block sizes, pages a row) of every table of blocks, behind the groups' sections
+        self.pools = pool_table_widths(cache, max_model_len)
+        self.offs, self.total = table_layout(B, self.widths, self.run_caps, [w for _, _, w in self.pools])
         if hv is None:
             hv = np.zeros(self.total, dtype=np.int32)
         if hv.dtype != np.int32 or hv.shape != (self.total,):
@@ -112,6 +122,11 @@ class DecodeTables:
             for r in range(first, B):
                 if self._row_state[r] is not None:
                     hv[o[9 + 4 * gi] + r * w:o[9 + 4 * gi] + (r + 1) * w] = 0
+        for k, (_, _, w) in enumerate(self.pools):
+            base = o[9 + 4 * len(self.widths) + k]
+            for r in range(first, B):
+                if self._row_state[r] is not None:
+                    hv[base + r * w:base + (r + 1) * w] = 0
         for r in range(first, B):
             self._row_state[r] = None
 
@@ -153,6 +168,16 @@ class DecodeTables:
                         hv[base + n:base + old] = 0
                 lens.append(n)
                 hv[o[10 + 4 * gi] + r] = table[P // ps] * ps + P % ps
+            for k, (gi, which, w) in enumerate(self.pools):
+                table = cache.pool_table(gi, e.req, which)
+                base = o[9 + 4 * len(self.widths) + k] + r * w
+                n, at = len(table), len(self.widths) + k
+                # (a table of the same stay in the cache only grows at its end; another's is written over, and
+                # pages behind a row's own are never read)
+                old = prev[2][at] if prev is not None and prev[0] == e.req and prev[1] == life and n >= prev[2][at] else 0
+                if n > old:
+                    hv[base + old:base + n] = table[old:]
+                lens.append(n)
             self._row_state[r] = (e.req, life, lens)
         self._pad_rows(R)
         self._deal_runs(R)
@@ -179,7 +204,8 @@ class DecodeGraph:
         self.B = B = int(bucket)
         cache = runner.cache
         widths = [-(-runner.max_model_len // cache.page_size) for _ in cache.groups]
-        _, total = table_layout(B, widths, [max_key_runs(B, g.spec.num_kv_heads) for g in cache.groups])
+        _, total = table_layout(B, widths, [max_key_runs(B, g.spec.num_kv_heads) for g in cache.groups],
+                                [w for _, _, w in pool_table_widths(cache, runner.max_model_len)])
         self.host = torch.zeros(total, dtype=torch.int32, pin_memory=True)
         self.tables = DecodeTables(cache, B, runner.max_model_len, self.host.numpy())
         self.widths = self.tables.widths
@@ -202,6 +228,9 @@ class DecodeGraph:
             b.groups.append(GroupTables(bt, sl(10 + 4 * gi, B), no_slot,
                                         sl(11 + 4 * gi, 4 * self.tables.run_caps[gi]).view(-1, 4),
                                         sl(12 + 4 * gi, B + 1), cache.groups[gi].spec.window))
+        for k, (gi, which, w) in enumerate(self.tables.pools):
+            base = o[9 + 4 * len(self.widths) + k]
+            b.groups[gi].pool_tables[cache.groups[gi].spec.pools[which]] = self.dev[base:base + B * w].view(B, w)
         b.host_cu_tokens = list(range(B + 1))
         b.host_start_pos = [0] * B
         b.host_state_slots = [cache.padding_slot] * B
@@ -317,7 +346,8 @@ class DecodeGraph:
         b.state_slots, b.logit_rows = g.state_slots[:R], g.logit_rows[:R]
         for gt in g.groups:
             # (no runs of keys: those of the graph's tables cover its padding rows too)
-            b.groups.append(GroupTables(gt.block_tables[:R], gt.slot_mapping[:R], gt.no_slot_mapping[:R]))
+            b.groups.append(GroupTables(gt.block_tables[:R], gt.slot_mapping[:R], gt.no_slot_mapping[:R],
+                                        pool_tables={p: t[:R] for p, t in gt.pool_tables.items()}))
         b.host_cu_tokens = list(range(R + 1))
         b.host_start_pos = list(t.host_start_pos)
         b.host_state_slots = list(t.host_state_slots)

@@ -13,6 +13,7 @@ import torch
 
 from ..cache.block_pool import OutOfPages
 from ..cache.manager import CacheManager
+from ..cache.sizing import state_id
 from ..kernels import ops as _ops
 from .batch import KVView, PinnedTables, StepBatch, StepEntry, build_step_batch
 from .graphs import DecodeGraph, graph_buckets
@@ -53,7 +54,7 @@ class StepContext(LayerContext):
             gt = self.batch.groups[group]
             c.kv = KVView(k, v, gt.block_tables, gt.slot_mapping if writes else gt.no_slot_mapping,
                           self._cache.page_size, group, gt.key_runs, gt.run_start, gt.runs_window,
-                          gt.runs_for_blocks, gt.runs_merge)
+                          gt.runs_for_blocks, gt.runs_merge, gt.pool_tables)
         c.state = state
         return c
 
@@ -76,12 +77,13 @@ class ModelRunner:
         self.cache = CacheManager(reqs, page_size, num_pages, max_seqs, dtype=self.act_dtype,
                                   device=self.device)
         self._calls = []
-        for cache_id, writes, kv_spec, state_spec in reqs:
+        for row in reqs:
+            cache_id, writes, kv_spec, state_spec = row[:4]
             group = self.cache.group_index(cache_id) if kv_spec is not None else None
             k = v = None
             if group is not None:
                 k, v = self.cache.kv_tensors(cache_id)
-            self._calls.append((cache_id, writes, group, k, v, self.cache.state_tensors.get(cache_id)))
+            self._calls.append((cache_id, writes, group, k, v, self.cache.state_tensors.get(state_id(row))))
         self._pinned = PinnedTables()     # the tables of steps that run eagerly leave through it
         # decode-only steps replay HIP graphs of the pieces of the model that can be captured
         self._graphs = {}

@@ -46,7 +46,7 @@ from collections import deque
 from dataclasses import dataclass, field
 
 from ..cache.manager import CacheManager
-from ..cache.sizing import min_window_pages
+from ..cache.sizing import request_pages
 from ..sampling.params import SamplingConfig
 
 
@@ -130,11 +130,10 @@ class Scheduler:
                 f"length limit of {self.max_model_len}")
         ps = self.cache.page_size
         # the last token chosen is never fed back, so total - 1 tokens reach the cache
-        pages = -(-(total - 1) // ps)
         for g in self.cache.groups:
             # a group with a window must hold what one more token touches; portions are cut to
             # what the free pages hold (_fit), so no larger bound is needed for the request to run
-            need = pages if g.spec.window <= 0 else min(pages, min_window_pages(g.spec.window, ps, g.spec.keep_first))
+            need = request_pages(g.spec, total - 1, ps)
             if need > g.pool.num_pages:
                 raise RequestRefused(
                     f"request {req.id!r} needs {need} cache pages, the pool has {g.pool.num_pages} in all")
@@ -161,13 +160,7 @@ class Scheduler:
     # ---- planning a step -------------------------------------------------
     def _fit(self, req: Request, want: int, free: list[int]) -> int:
         """Most tokens up to ``want`` whose pages the free counts allow."""
-        ps = self.cache.page_size
-        st_tokens = self.cache.num_tokens(req.id)
-        n = want
-        for gi, g in enumerate(self.cache.groups):
-            have = len(g.tables[req.id]) * ps - st_tokens
-            n = min(n, have + free[gi] * ps)
-        return max(0, n)
+        return self.cache.fit(req.id, want, free)
 
     def _take(self, req: Request, n: int, free: list[int]) -> None:
         need = self.cache.pages_needed(req.id, n)
@@ -233,8 +226,7 @@ class Scheduler:
                 and self.cache.slots.num_free > 0:
             req = self.waiting[0]
             want = min(req.num_pending, self.opt.prefill_chunk, budget)
-            ps = self.cache.page_size
-            n = min([want] + [f * ps for f in free])
+            n = self.cache.fit(None, want, free)
             if n < 1:
                 break
             self.waiting.popleft()

@@ -6,7 +6,7 @@ from ctypes import c_char_p, c_float, c_int, c_int64, c_size_t, c_void_p
 
 from .build import ensure_built
 
-ABI_VERSION = 34
+ABI_VERSION = 35
 
 
 class KernelLibraryError(RuntimeError):
@@ -23,7 +23,7 @@ _SIGNATURES = {
     "tff_embed": [_P, _P, _P, _I, _I, _I, _I, _P],
     "tff_add_rmsnorm": [_P, _P, _I, _Z, _P, _F, _P, _P, _I, _I, _I, _P],
     "tff_rmsnorm": [_P, _P, _F, _P, _I, _I, _I, _P],
-    "tff_gemm": [_P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _P, _Z, _I, _P],
+    "tff_gemm": [_P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _P, _P, _Z, _I, _P],
     "tff_gemm_workspace_bytes": [_I, _I, _I, _I, _I, _I],
     "tff_gemm_plan": [_I, _I, _I, _I, _I, _P, _P, _P],
     "tff_gemm_residual_prenorm": [_P, _P, _I, _I, _I, _I, _P, _P, _P, _P, _I, _P],
@@ -34,10 +34,10 @@ _SIGNATURES = {
     "tff_qk_norm_rope_kv": [_P, _I, _I, _I, _I, _P, _P, _F, _P, _I, _I, _I, _P, _P, _P, _P,
                             _I, _I, _I, _I, _P],
     "tff_attention_generic": [_P, _I, _P, _P, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _I,
-                              _F, _P, _F, _I, _I, _P],
+                              _F, _P, _F, _P, _I, _I, _I, _I, _P],
     "tff_attention_mfma_supported": [_I, _I],
     "tff_attention_mfma": [_P, _I, _P, _P, _P, _P, _P, _P, _I, _P, _P, _P, _I, _P, _I, _I, _I, _I, _I, _I,
-                           _I, _I, _I, _I, _I, _I, _F, _P, _F, _P],
+                           _I, _I, _I, _I, _I, _I, _F, _P, _F, _P, _I, _I, _P],
     "tff_attention_decode_fused": [_P, _I, _P, _P, _P, _P, _P, _P, _I, _P, _P, _P, _P, _P, _F, _P, _I, _I,
                                    _I, _I, _I, _I, _I, _I, _I, _I, _F, _P],
     "tff_attention_decode_runs": [_P, _I, _P, _P, _P, _P, _P, _P, _I, _P, _P, _P, _P, _P, _F, _P, _I, _I,
@@ -58,7 +58,7 @@ _SIGNATURES = {
     "tff_route_topk": [_P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _P, _P, _I, _P],
     "tff_experts_gate_up": [_P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _F, _F, _P, _P, _I, _P],
     "tff_experts_tiles_supported": [_I, _I, _I],
-    "tff_experts_by_tiles": [_P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _F, _F, _P, _P, _P, _I, _P, _P, _I, _P],
+    "tff_experts_by_tiles": [_P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _F, _F, _P, _P, _P, _I, _P, _P, _I, _I, _P],
     "tff_group_rmsnorm_add": [_P, _P, _I, _Z, _P, _P, _I, _F, _P, _I, _I, _I, _P],
     "tff_depth_average": [_P, _Z, _I, _P, _P, _P, _Z, _I, _P],
     "tff_scale_rows": [_P, _F, _Z, _P],
@@ -79,13 +79,22 @@ _SIGNATURES = {
     "tff_mixed_attention_workspace_bytes": [_I, _I, _I, _I],
     "tff_mixed_attention_q16_supported": [_I, _I, _I, _I],
     "tff_mixed_attention_q16": [_P, _P, _P, _P, _I, _P, _P, _P, _I, _P, _I, _P, _F, _F, _I, _I, _I, _P, _I, _I, _I, _I, _I, _I, _I, _P, _P],
-    "tff_experts_down": [_P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P, _I, _P],
-    "tff_swiglu": [_P, _P, _I, _I, _I, _P],
+    "tff_experts_down": [_P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P, _I, _I, _P, _I, _P],
+    "tff_swiglu": [_P, _P, _P, _I, _I, _I, _P],
     "tff_cast": [_P, _I, _P, _I, c_int64, _P],
     "tff_argmax_workspace_bytes": [_I, _I],
     "tff_argmax": [_P, _P, _I, _I, _P, _P],
     "tff_repetition_penalty": [_P, _I, _I, _P, _P, _P, _P],
     "tff_sample": [_P, _P, _I, _I, _P, _P, _P, _P, _P, _P, _P],
+    "tff_add_layernorm": [_P, _P, _I, _Z, _P, _I, _Z, _P, _P, _F, _P, _P, _P, _F, _P, _P, _P, _F, _P, _P, _I, _I, _P, _I, _P, _Z,
+                          _Z, _P, _I, _P],
+    "tff_input_conv_chunk": [],
+    "tff_input_conv": [_P, _P, _I, _P, _Z, _Z, _P, _I, _P, _P, _P, _I, _I, _P],
+    "tff_lightning": [_P, _Z, _P, _P, _Z, _P, _P, _P, _I, _I, _I, _I, _I, _P],
+    "tff_row_norm_gate": [_P, _P, _Z, _P, _F, _P, _I, _I, _I, _P],
+    "tff_grouped_qkv_store": [_P, _Z, _P, _I, _I, _I, _F, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _I, _I, _P],
+    "tff_pool_keys": [_P, _P, _P, _I, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P],
+    "tff_gate_heads": [_P, _Z, _I, _P, _Z, _P, _I, _I, _I, _I, _P],
     "tff_probe_stream_read": [_P, _Z, _P, _I, _P],
     "tff_probe_mfma": [_P, _I, _I, _I, _P],
 }

@@ -145,6 +145,17 @@ def pack_gate_up(gate: torch.Tensor, up: torch.Tensor) -> PackedWeight:
     return pw
 
 
+def pack_gate_up_bias(gate: torch.Tensor, up: torch.Tensor) -> torch.Tensor:
+    """Biases [I] of a gate and an up projection (float32, on the GPU) in the order of the rows of their
+    :func:`pack_gate_up` weight."""
+    I = gate.numel()
+    groups = -(-I // 16)
+    padded = torch.zeros(2, groups * 16, dtype=torch.float32, device=gate.device)
+    padded[0, :I] = gate
+    padded[1, :I] = up
+    return padded.view(2, groups, 16).permute(1, 0, 2).reshape(-1).contiguous()
+
+
 def embed(table, ids: torch.Tensor, out: torch.Tensor | None = None) -> torch.Tensor:
     """Rows of ``table`` [V, H] (a row-major tensor or a PackedWeight) for
     int32 ``ids`` [T] as float32 [T, H]."""
@@ -230,6 +241,8 @@ def as_tensor(t) -> torch.Tensor:
         return t.materialize()
     if isinstance(t, PendingTerms):
         return _as_tensor_terms(t)
+    if isinstance(t, OutputTerm):
+        return add_layernorm(None, t, None, None, 0.0, torch.float32)
     if isinstance(t, torch.Tensor) and t.dim() == 3:
         acc = t[0].clone()
         for part in t[1:]:
@@ -331,15 +344,23 @@ def _plan_tile(L, M: int, N: int, K: int) -> int:
 
 
 def linear(x: torch.Tensor, weight, out_dtype: torch.dtype | None = None,
-           out: torch.Tensor | None = None, partials: bool = False) -> torch.Tensor:
+           out: torch.Tensor | None = None, partials: bool = False, bias: torch.Tensor | None = None) -> torch.Tensor:
     """``x . weight^T`` for x [M, K] (rows may be strided) and weight [N, K]:
     a row-major float32 tensor, or a PackedWeight for bfloat16.
 
     ``partials=True`` (float32 result): where the product splits K over
     blocks, the partial sums are returned as they are, [S, M, N], for a
     consumer that adds them up anyway (``add_rmsnorm``); else the result is
-    [M, N] as always."""
+    [M, N] as always.
+
+    ``bias`` (a PackedWeight's product only): float32 [ceil16(N)] in the order of the weight's rows
+    (:func:`pack_gate_up_bias` for a gated one), added before the gate's activation."""
     packed = isinstance(weight, PackedWeight)
+    if bias is not None:
+        _req(bias, "linear bias", torch.float32, 1)
+        if not packed or partials or isinstance(x, ScaledRows) or bias.numel() != -(-weight.shape[0] // 16) * 16:
+            raise _lib.KernelError("linear: a bias goes with a packed weight, holds a number for each of its rows, rounded up "
+                                   "to 16, and its product is neither left in parts nor scaled by row")
     if isinstance(x, ScaledRows):
         if packed and out is None and not partials and x.shape[1] == weight.shape[1]:
             return _linear_row_scaled(x, weight, out_dtype or x.dtype)
@@ -385,7 +406,7 @@ def linear(x: torch.Tensor, weight, out_dtype: torch.dtype | None = None,
         if tuple(out.shape) != (M, n_out):
             raise _lib.KernelError(f"linear out: shape {tuple(out.shape)} is not {(M, n_out)}")
     _lib.check(L.tff_gemm(x.data_ptr(), weight.data_ptr(), out.data_ptr(), M, N, K, lda,
-                          dtype_code(x.dtype), dtype_code(out_dtype), 1 if packed else 0, glu_out,
+                          dtype_code(x.dtype), dtype_code(out_dtype), 1 if packed else 0, glu_out, _ptr(bias),
                           _ptr(ws), ws_bytes, 1 if keep else 0, _stream()))
     return out
 
@@ -445,10 +466,10 @@ def attention_generic(q: torch.Tensor, nq: int, nkv: int, d: int, k_cache: torch
                       v_cache: torch.Tensor, block_tables: torch.Tensor, token_req: torch.Tensor,
                       positions: torch.Tensor, window: int = 0, scale: float | None = None,
                       out: torch.Tensor | None = None, sinks: torch.Tensor | None = None,
-                      softcap: float = 0.0) -> torch.Tensor:
+                      softcap: float = 0.0, pool: int = 0, pool_tables: torch.Tensor | None = None) -> torch.Tensor:
     """Attention of each token over its request's pages; q is [T, >= nq*d]
     with the query heads at the start of each row.  Returns [T, nq*d].
-    ``sinks`` (float32 [nq]) and ``softcap``: see :func:`paged_attention`."""
+    ``sinks`` (float32 [nq]), ``softcap`` and ``pool``: see :func:`paged_attention`."""
     _req(q, "attention q", ndim=2)
     T = q.shape[0]
     if q.shape[1] < nq * d:
@@ -471,8 +492,19 @@ def attention_generic(q: torch.Tensor, nq: int, nkv: int, d: int, k_cache: torch
         q.data_ptr(), q.stride(0), out.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(),
         block_tables.data_ptr(), block_tables.stride(0), token_req.data_ptr(), positions.data_ptr(),
         T, nq, nkv, d, k_cache.shape[2], k_cache.shape[0], int(window), float(scale), _ptr(sinks), float(softcap or 0.0),
+        _ptr(pool_tables) if pool else None, pool_tables.stride(0) if pool else 0, int(pool),
         dtype_code(q.dtype), dtype_code(k_cache.dtype), _stream()))
     return out
+
+
+def _pool_table(kv, pool: int, window: int) -> torch.Tensor | None:
+    """The step's table of the pages that hold the mean keys of blocks of ``pool`` tokens."""
+    if not pool:
+        return None
+    t = kv.pool_tables.get(pool)
+    if t is None or window <= 0:
+        raise _lib.KernelError(f"attention: the cache keeps no keys of blocks of {pool} tokens before a window of {window}")
+    return _req(t, "pool tables", torch.int32, 2)
 
 
 def _check_sinks(sinks, nq: int) -> None:
@@ -525,7 +557,7 @@ def _num_cus(device) -> int:
 
 def _attention_block_work(batch, G: int, nkv: int, window: int, device, cols: int = 128,
                           bins: int | None = None, which: str = "all", key_groups: int | None = None,
-                          head_dim: int = 128, num_cus: int | None = None):
+                          head_dim: int = 128, num_cus: int | None = None, pool: int = 0):
     """Work table of the block kernel: items (entry, first column) of ``cols``
     columns, dealt to blocks so that every block goes through about the same
     number of 32-key slices (an item late in a long prompt sees many times the
@@ -537,7 +569,7 @@ def _attention_block_work(batch, G: int, nkv: int, window: int, device, cols: in
     cache = getattr(batch, "_attn_work", None)
     if cache is None:
         cache = batch._attn_work = {}
-    key = ("blocks", G, nkv, cols, window, bins, which, key_groups, head_dim, num_cus)
+    key = ("blocks", G, nkv, cols, window, bins, which, key_groups, head_dim, num_cus, pool)
     if key not in cache:
         cu, P = batch.host_cu_tokens, batch.host_start_pos
         items = []                       # (slices, entry, first column)
@@ -547,7 +579,8 @@ def _attention_block_work(batch, G: int, nkv: int, window: int, device, cols: in
                 first = P[r] + c0 // G
                 last = P[r] + (min(c0 + cols, ncols) - 1) // G
                 lo = max(0, first - window + 1) if window > 0 else 0
-                items.append((last // 32 - lo // 32 + 1, r, c0))
+                blocks = max(0, last - window + 1) // pool if pool else 0      # keys of blocks before the window
+                items.append((last // 32 - lo // 32 + 1 + -(-blocks // 32), r, c0))
         if num_cus is None:
             num_cus = _num_cus(device) if torch.device(device).type == "cuda" else 256
         per_cu = max(1, num_cus // max(1, nkv))
@@ -635,7 +668,7 @@ def attention_mfma(q: torch.Tensor, nq: int, nkv: int, d: int, kv, batch, window
                    scale: float | None = None, splits: int | None = None,
                    block_bins: int | None = None, key_groups: int | None = None,
                    block_cols: int | None = None, sinks: torch.Tensor | None = None,
-                   softcap: float = 0.0) -> torch.Tensor:
+                   softcap: float = 0.0, pool: int = 0) -> torch.Tensor:
     """bfloat16 attention of the step's tokens on the matrix cores; decode-only
     steps split each request's keys over several waves and merge them.
     ``splits``, ``block_bins`` (blocks per kv head that share the work of
@@ -663,6 +696,11 @@ def attention_mfma(q: torch.Tensor, nq: int, nkv: int, d: int, kv, batch, window
     out = torch.empty(T, nq * d, dtype=q.dtype, device=q.device)
     _check_sinks(sinks, nq)
     softcap = float(softcap or 0.0)
+    pt = _pool_table(kv, pool, int(window))
+    if pt is not None and pt.shape[0] != R:
+        raise _lib.KernelError("attention: the tables of blocks do not describe the step's requests")
+    # keys an entry can see at most (what the launch is sized for)
+    reach = batch.max_context if not pool else min(batch.max_context, int(window) + 32 + batch.max_context // pool)
     L = _lib.load()
     stream = _stream()
 
@@ -677,7 +715,7 @@ def attention_mfma(q: torch.Tensor, nq: int, nkv: int, d: int, kv, batch, window
             v_cache.data_ptr(), bt.data_ptr(), bt.stride(0), batch.cu_tokens.data_ptr(),
             batch.start_pos.data_ptr(), _ptr(work), num_work, _ptr(block_items), num_blocks, tiles, cols,
             groups, splits, R if splits > 1 else T, nq, nkv, d, k_cache.shape[2], k_cache.shape[0], int(window),
-            float(scale), _ptr(sinks), softcap, stream))
+            float(scale), _ptr(sinks), softcap, _ptr(pt), pt.stride(0) if pt is not None else 0, int(pool), stream))
         if splits > 1:
             _lib.check(L.tff_attention_split_reduce(
                 part_o.data_ptr(), part_ml.data_ptr(), out.data_ptr(), splits, R, nq, d, _ptr(rows),
@@ -686,7 +724,7 @@ def attention_mfma(q: torch.Tensor, nq: int, nkv: int, d: int, kv, batch, window
     if batch.max_new_tokens == 1:
         # decoding only: a wave per request, kv head and run of keys; sizes come from the tables
         tiles = -(-G // 16)
-        runs = getattr(kv, "key_runs", None)
+        runs = getattr(kv, "key_runs", None) if not pool else None      # (the runs deal tokens' keys only)
         if splits is None and runs is not None and kv.runs_window == int(window) and T == R:
             # (the keys dealt into runs by the step's tables; entry i's token is row i)
             part_o = torch.empty(runs.shape[0], nq, d, dtype=torch.float32, device=q.device)
@@ -699,7 +737,7 @@ def attention_mfma(q: torch.Tensor, nq: int, nkv: int, d: int, kv, batch, window
                 _ptr(sinks), softcap, stream))
             return out
         if splits is None:
-            splits = pick_splits(R * tiles * nkv, batch.max_context)
+            splits = pick_splits(R * tiles * nkv, reach)
         launch(None, R * tiles, None, 0, tiles, 16, splits)
         return out
     # long portions: blocks that share their keys through LDS (128 columns); short ones: a wave
@@ -715,7 +753,7 @@ def attention_mfma(q: torch.Tensor, nq: int, nkv: int, d: int, kv, batch, window
         cache = getattr(batch, "_attn_work", None)
         if cache is None:
             cache = batch._attn_work = {}
-        if splits is None and getattr(batch, "host_start_pos", None) is not None:
+        if splits is None and not pool and getattr(batch, "host_start_pos", None) is not None:
             # their keys dealt into runs of similar length, whatever the requests' lengths
             key = ("single_runs", nkv, int(window))
             if key not in cache:
@@ -740,10 +778,10 @@ def attention_mfma(q: torch.Tensor, nq: int, nkv: int, d: int, kv, batch, window
             if "single_rows" not in cache:
                 cu = batch.host_cu_tokens
                 cache["single_rows"] = _staging.send(q.device, [np.asarray([(r, cu[r]) for r in single], dtype=np.int32)])[0]
-            sp = splits if splits is not None else pick_splits(work.shape[0] * nkv, batch.max_context)
+            sp = splits if splits is not None else pick_splits(work.shape[0] * nkv, reach)
             launch(work, work.shape[0], None, 0, 1, 16, sp, cache["single_rows"])
     if cols == 128:
-        bcols = block_cols or _pick_block_cols(batch, G, nkv, int(window), q.device, which, d)
+        bcols = 128 if pool else block_cols or _pick_block_cols(batch, G, nkv, int(window), q.device, which, d)
         if bcols == 256:
             # long prompts: items of 256 columns for blocks whose waves take two column tiles
             # each (one block a CU, so one bin a CU and kv head)
@@ -754,7 +792,8 @@ def attention_mfma(q: torch.Tensor, nq: int, nkv: int, d: int, kv, batch, window
             launch(work, work.shape[0], block_items, num_blocks, 1, 256, 1, groups=1)
             return out
         work, block_items, num_blocks, groups = _attention_block_work(
-            batch, G, nkv, int(window), q.device, bins=block_bins, which=which, key_groups=key_groups, head_dim=d)
+            batch, G, nkv, int(window), q.device, bins=block_bins, which=which, key_groups=key_groups, head_dim=d,
+            pool=int(pool))
         launch(work, work.shape[0], block_items, num_blocks, 1, 128, 1, groups=groups)
     else:
         work = _attention_work(batch, G, cols, q.device, which)
@@ -891,19 +930,22 @@ def qkv_attention(qkv: torch.Tensor, nq: int, nkv: int, d: int, q_weight, k_weig
 
 def paged_attention(q: torch.Tensor, nq: int, nkv: int, d: int, kv, batch, window: int = 0,
                     scale: float | None = None, sinks: torch.Tensor | None = None,
-                    softcap: float = 0.0) -> torch.Tensor:
+                    softcap: float = 0.0, pool: int = 0) -> torch.Tensor:
     """Attention of a step's tokens over the cache view ``kv`` (k_cache,
     v_cache, block_tables) with the step's ``batch``.  bfloat16 with a head
     size the matrix-core kernel takes runs there; everything else (float32,
     other head sizes) on the general kernel.  ``sinks`` (float32 [nq]): a
     number per query head whose exponential is one more term of the softmax's
     denominator, with no key and no value, not scaled.  ``softcap`` c > 0: the
-    scaled scores are capped, s <- c tanh(s / c), before the mask."""
+    scaled scores are capped, s <- c tanh(s / c), before the mask.  ``pool`` P > 0 (with a window):
+    beside the window's keys a token sees the cache's mean keys and values of the whole blocks of P tokens
+    that lie before it (:func:`pool_keys` puts them there), in the same softmax."""
     # (the matrix-core kernels cap scores at head sizes up to 192)
     if mfma_attention_supported(q.dtype, d, kv.k_cache.shape[2]) and not (softcap and d > 192):
-        return attention_mfma(q, nq, nkv, d, kv, batch, window, scale, sinks=sinks, softcap=softcap)
+        return attention_mfma(q, nq, nkv, d, kv, batch, window, scale, sinks=sinks, softcap=softcap, pool=pool)
     return attention_generic(q, nq, nkv, d, kv.k_cache, kv.v_cache, kv.block_tables,
-                             batch.token_req, batch.positions, window, scale, sinks=sinks, softcap=softcap)
+                             batch.token_req, batch.positions, window, scale, sinks=sinks, softcap=softcap, pool=pool,
+                             pool_tables=_pool_table(kv, pool, int(window)))
 
 
 MFMA_HEAD_SIZES = tuple(range(16, 129, 16)) + (192, 256)
@@ -1117,12 +1159,14 @@ EXPERT_TILES_MIN_TOKENS = 32
 
 def routed_experts(h: torch.Tensor, w_gate: torch.Tensor, w_up: torch.Tensor, w_down: torch.Tensor,
                    idx: torch.Tensor, wts: torch.Tensor, limit: float, act_alpha: float,
-                   by_tiles: bool | None = None, up_offset: float = 1.0, weight_input: bool = False) -> torch.Tensor:
+                   by_tiles: bool | None = None, up_offset: float = 1.0, weight_input: bool = False,
+                   identity: int = 0) -> torch.Tensor:
     """The weighted sum of each token's chosen experts: y = g sigmoid(act_alpha g) (u + up_offset) with
     g = min(Wg h, limit), u = clamp(Wu h, -limit, limit); out = sum_k wts[:, k] Wd y.
     ``w_gate`` None: experts without a gate, y = max(Wu h, 0)^2.  ``weight_input``: a pair's weight multiplies
     what goes into its expert instead of what comes out, out = sum_k expert_k(wts[:, k] h); since W (w h) = w (W h)
     it is applied to both first products, before clamps and activation.
+    ``identity`` > 0: ``idx`` may name experts from the number of matrices on, which hand their input on.
     ``w_gate``, ``w_up`` [E, ff, >= width], ``w_down`` [E, width, >= ff] of h's type (the last
     dimension may be wider than what is multiplied: see :func:`pad_expert_rows`).  float32
     [T, width], or (many tokens in bfloat16, ``by_tiles``) [top, T, width]: the terms of the sum
@@ -1156,14 +1200,15 @@ def routed_experts(h: torch.Tensor, w_gate: torch.Tensor, w_up: torch.Tensor, w_
         _lib.check(L.tff_experts_by_tiles(
             h.data_ptr(), width, _ptr(w_gate), w_up.data_ptr(), w_down.data_ptr(), idx.data_ptr(), wts.data_ptr(),
             T, top, E, width, ff, ld_in, ld_down, float(limit), float(act_alpha), float(up_offset), tables.data_ptr(), tables[max_tiles:].data_ptr(),
-            tables[129 * max_tiles:].data_ptr(), max_tiles, y.data_ptr(), out.data_ptr(), 1 if weight_input else 0, _stream()))
+            tables[129 * max_tiles:].data_ptr(), max_tiles, y.data_ptr(), out.data_ptr(), 1 if weight_input else 0,
+            int(identity), _stream()))
         return out if top > 1 else out[0]
     _lib.check(L.tff_experts_gate_up(h.data_ptr(), width, _ptr(w_gate), w_up.data_ptr(), idx.data_ptr(), T, top, E,
                                      width, ff, ld_in, float(limit), float(act_alpha), float(up_offset),
                                      wts.data_ptr() if weight_input else None, y.data_ptr(), dtype_code(h.dtype), _stream()))
     out = torch.empty(T, width, dtype=torch.float32, device=h.device)
     _lib.check(L.tff_experts_down(y.data_ptr(), w_down.data_ptr(), idx.data_ptr(), None if weight_input else wts.data_ptr(), T, top, E, width, ff,
-                                  ld_down, out.data_ptr(), dtype_code(h.dtype), _stream()))
+                                  ld_down, h.data_ptr(), width, int(identity), out.data_ptr(), dtype_code(h.dtype), _stream()))
     return out
 
 
@@ -1486,6 +1531,199 @@ def add_rmsnorm_pair(resid: torch.Tensor, delta, bias: torch.Tensor | None, w1: 
     return out1, out2
 
 
+class OutputTerm:
+    """A sublayer's result on its way into the residual stream, with everything that happens to it there:
+
+        d = term + bias,   or with ``pair`` (b, wa, wb, eps)   d = (rms(term) * wa + rms(b) * wb) / 2
+        d <- layernorm(d) with ``norm`` (weight, bias, eps);   d <- d * scale
+
+    ``term`` and ``b`` are what ``linear`` may return with ``partials=True``.  ``add_layernorm`` adds it to the
+    stream in the kernel that norms the sum; ``as_tensor`` makes a tensor of it."""
+
+    def __init__(self, term, bias=None, pair=None, norm=None, scale=None):
+        self.term, self.bias, self.pair, self.norm, self.scale = term, bias, pair, norm, scale
+
+
+def output_term(delta, norm=None, scale=None) -> OutputTerm:
+    """What a mixer or feed-forward returned, with a norm and a scale on top."""
+    t = delta if isinstance(delta, OutputTerm) else OutputTerm(delta)
+    if t.norm is not None or t.scale is not None:
+        raise _lib.KernelError("output term: it has a norm already")
+    return OutputTerm(t.term, t.bias, t.pair, norm, scale)
+
+
+def _vec(t, n: int, what: str):
+    if t is None:
+        return None
+    _req(t, what, torch.float32, 1)
+    if t.numel() != n:
+        raise _lib.KernelError(f"{what}: {t.numel()} elements, rows have {n}")
+    return t
+
+
+def add_layernorm(resid: torch.Tensor | None, delta, weight, bias, eps: float, out_dtype: torch.dtype,
+                  rows: torch.Tensor | None = None, conv=None, batch=None) -> torch.Tensor:
+    """``resid += delta`` (None, an :class:`OutputTerm` or anything else a sublayer may return; not added when
+    ``rows`` is given) and the layer norm of the sum in ``out_dtype``; with ``rows`` (int32) of those rows only.
+    ``conv`` (weights float32 [taps, W], state float32 [slots, row], offset in a state row): the normed rows leave
+    with their causal convolution over time added, per request of ``batch``; the last taps - 1 normed
+    rows of each request are left in its state.  A step of one token per request is one kernel.
+    ``resid`` None and ``weight`` None: the term itself."""
+    term = delta if isinstance(delta, OutputTerm) else OutputTerm(delta)
+    if isinstance(term.term, PendingTerms):
+        term = OutputTerm(as_tensor(term.term), term.bias, term.pair, term.norm, term.scale)
+    shape = tuple(resid.shape) if resid is not None else tuple(term.term.shape[-2:])
+    W = shape[1]
+    if resid is not None:
+        _req(resid, "add_layernorm resid", torch.float32, 2)
+    dev = resid.device if resid is not None else term.term.device
+    a, pa, sa = _planes_of(term.term, shape, "add_layernorm term")
+    b, pb, sb, wa, wb, pair_eps = None, 0, 0, None, None, 0.0
+    if term.pair is not None:
+        b, wa, wb, pair_eps = term.pair
+        b, pb, sb = _planes_of(b, shape, "add_layernorm second term")
+    nw, nb, n_eps = term.norm if term.norm is not None else (None, None, 0.0)
+    vecs = [_vec(t, W, "add_layernorm " + n) for t, n in ((wa, "first weight"), (wb, "second weight"), (term.bias, "term's bias"),
+            (nw, "term's norm weight"), (nb, "term's norm bias"), (term.scale, "scale"), (weight, "weight"), (bias, "bias"))]
+    wa, wb, tb, nw, nb, sc, weight, bias = vecs
+    n = shape[0]
+    if rows is not None:
+        _req(rows, "add_layernorm rows", torch.int32, 1)
+        n = rows.numel()
+    one = conv is not None and batch.max_new_tokens == 1 and batch.num_reqs == n
+    cw, state, off, taps = None, None, 0, 0
+    if conv is not None:
+        cw, state, off = conv
+        _req(cw, "convolution weights", torch.float32, 2)
+        taps = cw.shape[0]
+        if cw.shape[1] != W or rows is not None or weight is None:
+            raise _lib.KernelError(f"add_layernorm: a convolution of {tuple(cw.shape)} on rows of {W}")
+        if taps > 1 and off + (taps - 1) * W > _state_rows(state, "convolution state"):
+            raise _lib.KernelError(f"add_layernorm: state rows of {state.shape[1]} do not hold {taps - 1} x {W} from {off}")
+        if batch.num_tokens != n or batch.cu_tokens.numel() != batch.num_reqs + 1:
+            raise _lib.KernelError("add_layernorm: the step's tables do not describe the rows")
+    split = conv is not None and not one
+    out = torch.empty(n, W, dtype=torch.float32 if split else out_dtype, device=dev)
+    L = _lib.load()
+    st = _ptr(state) if taps > 1 else None
+    st_row = state.stride(0) if taps > 1 else 0
+    slots = batch.state_slots.data_ptr() if conv is not None else None
+    _lib.check(L.tff_add_layernorm(
+        _ptr(resid), _ptr(a), pa, sa, _ptr(b), pb, sb, _ptr(wa), _ptr(wb), float(pair_eps), _ptr(tb), _ptr(nw), _ptr(nb),
+        float(n_eps), _ptr(sc), _ptr(weight), _ptr(bias), float(eps), out.data_ptr(), _ptr(rows), n, W,
+        _ptr(cw) if one else None, taps, st, st_row, off, slots, dtype_code(out.dtype), _stream()))
+    if not split:
+        return out
+    items = getattr(batch, "_conv_items", None)
+    if items is None:
+        cu, chunk = batch.host_cu_tokens, L.tff_input_conv_chunk()
+        flat = [(r, i) for r in range(len(cu) - 1) for i in range(0, cu[r + 1] - cu[r], chunk)]
+        items = batch._conv_items = _staging.send(dev, [np.asarray(flat, dtype=np.int32).reshape(-1, 2)])[0]
+    y = torch.empty(n, W, dtype=out_dtype, device=dev)
+    _lib.check(L.tff_input_conv(out.data_ptr(), cw.data_ptr(), taps, st, st_row, off, items.data_ptr(), items.shape[0],
+                                batch.cu_tokens.data_ptr(), slots, y.data_ptr(), W, dtype_code(out_dtype), _stream()))
+    return y
+
+
+def lightning(proj: torch.Tensor, decay: torch.Tensor, state: torch.Tensor, batch, H: int, D: int, E: int) -> torch.Tensor:
+    """The recurrence S <- decay_h S + k v^T, o = S^T q over each request's tokens of this step, per head; q [H, D],
+    k [H, D], v [H, E] are silu of the columns of ``proj`` (float32 [T, >= H (2 D + E)], rows may be strided);
+    S lies transposed, [H][E][D], at the start of the request's row of ``state``.  Returns o float32 [T, H E]."""
+    T = proj.shape[0]
+    ldp = _rows2(proj, "lightning proj", torch.float32, H * (2 * D + E))
+    _req(decay, "lightning decay", torch.float32, 1)
+    row = _state_rows(state, "lightning state")
+    if decay.numel() != H or H * E * D > row or batch.num_tokens != T:
+        raise _lib.KernelError(f"lightning: {decay.numel()} decays, state rows of {row}, {T} rows for {H} heads of {D} x {E} "
+                               f"and a step of {batch.num_tokens} tokens")
+    o = torch.empty(T, H * E, dtype=torch.float32, device=proj.device)
+    if T:
+        _lib.check(_lib.load().tff_lightning(proj.data_ptr(), ldp, decay.data_ptr(), state.data_ptr(), row,
+                                             batch.cu_tokens.data_ptr(), batch.state_slots.data_ptr(), o.data_ptr(),
+                                             batch.num_reqs, H, D, E, int(getattr(batch, "max_new_tokens", 0) or 0), _stream()))
+    return o
+
+
+def row_norm_gate(o: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, eps: float, out_dtype: torch.dtype) -> torch.Tensor:
+    """``o / sqrt(mean over the row of o^2 + eps) * weight * sigmoid(gate)`` for o float32 [T, N] and gate float32
+    [T, >= N] (rows may be strided)."""
+    _req(o, "row_norm_gate o", torch.float32, 2)
+    T, N = o.shape
+    _vec(weight, N, "row_norm_gate weight")
+    g_row = _rows2(gate, "row_norm_gate gate", torch.float32, N)
+    if gate.shape[0] != T:
+        raise _lib.KernelError("row_norm_gate: the gate needs one row per token")
+    out = torch.empty(T, N, dtype=out_dtype, device=o.device)
+    _lib.check(_lib.load().tff_row_norm_gate(o.data_ptr(), gate.data_ptr(), g_row, weight.data_ptr(), float(eps), out.data_ptr(), T,
+                                             N, dtype_code(out_dtype), _stream()))
+    return out
+
+
+def grouped_qkv_store(proj: torch.Tensor, H: int, G: int, D: int, E: int, cos_sin: torch.Tensor | None, pairing: int,
+                      temp: tuple, positions: torch.Tensor, kv, store: bool = True) -> torch.Tensor:
+    """Queries, keys and values of a grouped attention from their projections, ``proj`` float32 [T, >= H D (+ G D + G E
+    with ``store``)] (rows may be strided): the first ``2 * cos_sin.shape[1]`` elements of every head of q and k rotated,
+    q times 1 + coef ln(floor((p + 1) / every) + 1) for ``temp`` = (coef, every).  Returns q [T, H P] in the cache's type,
+    P the cache's head size, zeros behind a head's D elements; with ``store`` the token's key and value rows go to
+    its slot of ``kv``."""
+    cols = H * D + (G * (D + E) if store else 0)
+    T = proj.shape[0]
+    row = _rows2(proj, "grouped_qkv_store proj", torch.float32, cols)
+    k_cache, v_cache = kv.k_cache, kv.v_cache
+    _req(k_cache, "k cache", ndim=4)
+    _req(v_cache, "v cache", k_cache.dtype, 4)
+    P = k_cache.shape[3]
+    _check_cache(k_cache, v_cache, G, P, "grouped_qkv_store")
+    dims, max_pos = 0, 0
+    if cos_sin is not None:
+        _req(cos_sin, "rotation table", torch.float32, 3)
+        max_pos, dims = cos_sin.shape[0], 2 * cos_sin.shape[1]
+        if cos_sin.shape[2] != 2 or dims > D:
+            raise _lib.KernelError(f"rotation table {tuple(cos_sin.shape)} does not fit a head of {D}")
+    _req(positions, "positions", torch.int32, 1)
+    _req(kv.slot_mapping, "slot_mapping", torch.int32, 1)
+    if P < D or P < E or positions.numel() < T or kv.slot_mapping.numel() < T:
+        raise _lib.KernelError(f"grouped_qkv_store: a cache head of {P} for {D} and {E}, or fewer positions than tokens")
+    q = torch.empty(T, H * P, dtype=k_cache.dtype, device=proj.device)
+    _lib.check(_lib.load().tff_grouped_qkv_store(
+        proj.data_ptr(), row, _ptr(cos_sin), dims, int(pairing), max_pos, float(temp[0]), int(temp[1]), positions.data_ptr(),
+        kv.slot_mapping.data_ptr(), q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), k_cache.shape[2], k_cache.shape[0], T, H, G,
+        D, E, P, 1 if store else 0, dtype_code(k_cache.dtype), _stream()))
+    return q
+
+
+def pool_keys(kv, batch, pool: int) -> None:
+    """For every token of the step that ends a block of ``pool`` tokens: the means of the block's keys and of its values, as
+    the pages hold them, into the block's slot of ``kv``'s pages for blocks of that size."""
+    k_cache, v_cache = _req(kv.k_cache, "k cache", ndim=4), _req(kv.v_cache, "v cache", ndim=4)
+    pages, G, ps, d = k_cache.shape
+    _check_cache(k_cache, v_cache, G, d, "pool_keys")
+    bt, pt = _req(kv.block_tables, "block tables", torch.int32, 2), kv.pool_tables.get(pool)
+    if pt is None:
+        raise _lib.KernelError(f"pool_keys: the cache keeps no keys of blocks of {pool} tokens")
+    _req(pt, "pool tables", torch.int32, 2)
+    T = batch.num_tokens
+    if pt.shape[0] != bt.shape[0] or min(batch.token_req.numel(), batch.positions.numel(), kv.slot_mapping.numel()) < T:
+        raise _lib.KernelError("pool_keys: the step's tables do not describe the same requests and tokens")
+    _lib.check(_lib.load().tff_pool_keys(
+        k_cache.data_ptr(), v_cache.data_ptr(), bt.data_ptr(), bt.stride(0), pt.data_ptr(), pt.stride(0), batch.token_req.data_ptr(),
+        batch.positions.data_ptr(), kv.slot_mapping.data_ptr(), ps, pages, int(pool), T, G, d, dtype_code(k_cache.dtype), _stream()))
+
+
+def gate_heads(o: torch.Tensor, P: int, gate: torch.Tensor | None, H: int, E: int) -> torch.Tensor:
+    """The first E elements of every head of ``o`` (heads P apart) side by side, [T, H E], times sigmoid(gate[:, h])
+    (float32 [T, >= H], rows may be strided; None: as they are)."""
+    T = o.shape[0]
+    o_row = _rows2(o, "gate_heads o", o.dtype, H * P)
+    g_row = _rows2(gate, "gate_heads gate", torch.float32, H) if gate is not None else 0
+    if P < E or (gate is not None and gate.shape[0] != T):
+        raise _lib.KernelError("gate_heads: o and gate must have one row per token and heads that hold E elements")
+    out = torch.empty(T, H * E, dtype=o.dtype, device=o.device)
+    _lib.check(_lib.load().tff_gate_heads(o.data_ptr(), o_row, int(P), _ptr(gate), g_row, out.data_ptr(), T, H, E,
+                                          dtype_code(o.dtype), _stream()))
+    return out
+
+
 def softcap_(z: torch.Tensor, cap: float) -> torch.Tensor:
     """z <- cap * tanh(z / cap) in place on float32."""
     _req(z, "softcap", torch.float32)
@@ -1675,17 +1913,29 @@ def diff_combine(a: torch.Tensor, P: int, gate: torch.Tensor | None, lam: float,
     return out
 
 
-def swiglu(gate_up: torch.Tensor, out: torch.Tensor | None = None) -> torch.Tensor:
-    """``silu(gate) * up`` for gate_up [T, 2I] = [gate | up]."""
+def linear_swiglu_bias(x: torch.Tensor, weight, bias: torch.Tensor) -> torch.Tensor:
+    """silu(x Wg^T + bg) * (x Wu^T + bu).  bfloat16: ``weight`` and ``bias`` as :func:`pack_gate_up` and
+    :func:`pack_gate_up_bias` give them, one product; float32: ``weight`` [2I, H] and ``bias`` [2I] stacked."""
+    if isinstance(weight, PackedWeight):
+        return linear(x, weight, bias=bias)
+    return swiglu(linear(x, weight), bias=bias)
+
+
+def swiglu(gate_up: torch.Tensor, out: torch.Tensor | None = None, bias: torch.Tensor | None = None) -> torch.Tensor:
+    """``silu(gate) * up`` for gate_up [T, 2I] = [gate | up] (plus ``bias`` float32 [2I], if given)."""
     _req(gate_up, "swiglu input", ndim=2)
     T, two_i = gate_up.shape
     if two_i % 2:
         raise _lib.KernelError("swiglu: odd row width")
     I = two_i // 2
+    if bias is not None:
+        _req(bias, "swiglu bias", torch.float32, 1)
+        if bias.numel() != two_i:
+            raise _lib.KernelError(f"swiglu: a bias of {bias.numel()} for rows of {two_i}")
     if out is None:
         out = torch.empty(T, I, dtype=gate_up.dtype, device=gate_up.device)
     L = _lib.load()
-    _lib.check(L.tff_swiglu(gate_up.data_ptr(), out.data_ptr(), T, I, dtype_code(gate_up.dtype), _stream()))
+    _lib.check(L.tff_swiglu(gate_up.data_ptr(), _ptr(bias), out.data_ptr(), T, I, dtype_code(gate_up.dtype), _stream()))
     return out
 
 
@@ -1815,6 +2065,12 @@ OP_TABLE = {
     "add_dyt": add_dyt,
     "diff_qkv_store": diff_qkv_store,
     "diff_combine": diff_combine,
+    "add_layernorm": add_layernorm,
+    "lightning": lightning,
+    "row_norm_gate": row_norm_gate,
+    "grouped_qkv_store": grouped_qkv_store,
+    "pool_keys": pool_keys,
+    "gate_heads": gate_heads,
     "route_topk": route_topk,
     "routed_experts": routed_experts,
     "cast": cast,

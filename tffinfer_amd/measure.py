@@ -50,9 +50,12 @@ def prefill_flops(model, T: int) -> float:
         per_pair = mixer.flops_per_query_key_pair()
         if per_pair:
             spec = mixer.cache_spec()
-            w = spec.window if spec is not None and spec.window > 0 else T
+            w = getattr(mixer, "window", 0) or (spec.window if spec is not None and spec.window > 0 else T)
             w = min(w, T)
             pairs = w * (w + 1) / 2 + (T - w) * w      # token t reads min(t + 1, window) keys
+            pool = getattr(mixer, "pool", 0)
+            if pool and T > w:
+                pairs += (T - w) * (T - w) / (2 * pool)     # and the blocks before the window
             flops += per_pair * pairs
     return flops + 2.0 * cfg.hidden_size * cfg.vocab_size
 
@@ -69,9 +72,13 @@ def decode_bytes(model, batch: int, context: float, esz: int = 2) -> float:
         mixer = model.blocks[call.layer].mixer
         spec = mixer.cache_spec()
         if spec is not None:
-            keys = min(context, spec.window + spec.keep_first) if spec.window > 0 else context
+            window = getattr(mixer, "window", 0) or spec.window     # (a shared cache may hold more than this call reads)
+            keys = min(context, window + spec.keep_first) if window > 0 else context
+            pool = getattr(mixer, "pool", 0)
+            if pool and context > window:       # a key per whole block of tokens before the window
+                keys += (context - window) // pool
             kv += 2 * spec.num_kv_heads * spec.head_dim * esz * batch * keys
-        state = mixer.state_spec()
+        state = model.call_state(model.blocks[call.layer])
         if state is not None:       # (a request's state of fixed size is read whole at every token)
             kv += batch * math.prod(state.shape) * state.dtype.itemsize
     return weights + kv

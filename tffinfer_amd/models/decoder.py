@@ -13,7 +13,7 @@ from dataclasses import dataclass, field
 import torch
 
 from ..config.base import ModelConfig
-from ..parts.base import BLOCKS, FEED_FORWARDS, MIXERS, NORMS, Part, WeightSpec
+from ..parts.base import BLOCKS, FEED_FORWARDS, MIXERS, NORMS, Part, StateSpec, WeightSpec
 from ..parts.embedding import Embedding, OutputHead
 from ..weights.loader import check_weights, normalize_stored
 from ..weights.random_init import FLOAT32_INITS, random_tensor
@@ -199,12 +199,27 @@ class DecoderModel:
     # ---- cache needs -----------------------------------------------------
     def call_requirements(self):
         """For every entry of the run order: (cache id, writes, KVCacheSpec or
-        None, StateSpec or None)."""
+        None, StateSpec or None), and the state's id where it is not the cache's."""
         out = []
         for call in self.schedule:
-            mixer = self.blocks[call.layer].mixer
-            out.append((call.cache, call.writes_cache, mixer.cache_spec(), mixer.state_spec()))
+            block = self.blocks[call.layer]
+            row = (call.cache, call.writes_cache, block.mixer.cache_spec(), self.call_state(block))
+            out.append(row if call.state < 0 or call.state == call.cache else row + (call.state,))
         return out
+
+    @staticmethod
+    def call_state(block) -> StateSpec | None:
+        """The state of a layer call: the mixer's, with what the block itself carries behind it."""
+        mixer, own = block.mixer.state_spec(), block.state_spec()
+        if own is None:
+            return mixer
+        n = 0
+        if mixer is not None:
+            if len(mixer.shape) != 1 or mixer.dtype != own.dtype:
+                raise ValueError("a block with state of its own takes a mixer whose state is one row of the same type")
+            n = mixer.shape[0]
+        block.state_offset = n
+        return StateSpec((n + own.shape[0],), own.dtype)
 
     # ---- one step --------------------------------------------------------
     def forward(self, ctx) -> torch.Tensor:

@@ -329,3 +329,130 @@ class DifferentialAttention(Mixer):
         gate = proj[:, 2 * H * D + 2 * G * D + G * E:] if self.has_gate else None
         o = ops.diff_combine(a, P, gate, self.lam, self.norm_eps, 1.0 - self.diff, H, E)
         return ops.linear(o, self.w_o, out_dtype=torch.float32, partials=True)
+
+
+@register_mixer("grouped_attention")
+class GroupedAttention(Mixer):
+    """Grouped-query attention with queries, keys and values of sizes of their own, without a norm on them:
+
+        q_h = temp(p) rot(Wq x)_h,  k_g = rot(Wk x)_g  (heads of ``head_dim``),  v_g = (Wv x)_g  (``value_dim``)
+        temp(p) = 1 + q_temp_coef * ln(floor((p + 1) / q_temp_every) + 1)       (coef 0: 1)
+        y_h(i) = sum over what i sees of softmax(scale q_h(i) . key) value,   g = h // (heads / kv_heads)
+        out = Wo [y_h sigmoid(Wg x)_h]_h            (``head_gate``: one number per head; else no gate)
+
+    What position i sees: every j <= i; with a ``window`` the j with i - j < window; and with a ``pool`` P
+    beside them one key and one value per block of P tokens that lies wholly before the window: the means
+    of the block's keys and values as the cache holds them.  Tokens that left the window and whose block
+    is not seen yet are not seen at all; tokens and blocks share one softmax.
+
+    ``shared_cache``: the layer has no Wk and Wv; it reads the cache that another layer call fills (the run
+    order names it), with its own queries, window, pool and everything else.  ``cache_window`` and
+    ``cache_pools`` say what that cache keeps for all its readers (by default what this layer asks for).
+
+    The attention proper runs on the paged kernels with one head size for keys and values, the larger of the
+    two brought up to a size they take.  The projections' results stay float32 until temperature and
+    rotation are done (``ops.grouped_qkv_store``).  ``external``: the mixer is one of several that read the same
+    rows; whoever combines them forms all their projections in one product and calls ``forward_projected``.
+    """
+
+    graph_safe = True
+    input_goes_to_linear = True
+
+    def __init__(self, hidden_size: int, num_heads: int, num_kv_heads: int, head_dim: int, value_dim: int,
+                 position=None, scale: float | None = None, window: int = 0, pool: int = 0,
+                 cache_window: int | None = None, cache_pools: tuple | None = None, shared_cache: bool = False,
+                 head_gate: bool = False, q_temp_coef: float = 0.0, q_temp_every: int = 1, external: bool = False):
+        self.hidden_size = int(hidden_size)
+        self.num_heads = int(num_heads)
+        self.num_kv_heads = int(num_kv_heads)
+        self.head_dim = int(head_dim)
+        self.value_dim = int(value_dim)
+        if min(self.hidden_size, self.num_heads, self.num_kv_heads, self.head_dim, self.value_dim) <= 0:
+            raise ConfigError("grouped attention: sizes must be positive")
+        if self.num_heads % self.num_kv_heads:
+            raise ConfigError(f"grouped attention: {num_heads} heads are not a multiple of {num_kv_heads} kv heads")
+        self.scale = float(scale) if scale is not None else 1.0 / math.sqrt(self.head_dim)
+        self.window, self.pool = int(window or 0), int(pool or 0)
+        if self.window < 0 or self.pool < 0 or (self.pool and not self.window):
+            raise ConfigError(f"grouped attention: window {window} and pool {pool} (blocks are seen before a window)")
+        self.cache_window = self.window if cache_window is None else int(cache_window)
+        self.cache_pools = ((self.pool,) if self.pool else ()) if cache_pools is None else tuple(sorted(cache_pools))
+        if (self.pool and self.pool not in self.cache_pools) or (0 < self.cache_window < (self.window or self.cache_window + 1)):
+            raise ConfigError(f"grouped attention: a cache of window {self.cache_window} and blocks {self.cache_pools} does "
+                              f"not hold what a window of {self.window} and blocks of {self.pool} read")
+        self.shared_cache = bool(shared_cache)
+        self.has_gate = bool(head_gate)
+        self.q_temp_coef, self.q_temp_every = float(q_temp_coef), int(q_temp_every)
+        if self.q_temp_every <= 0:
+            raise ConfigError("grouped attention: the temperature's step must be positive")
+        if isinstance(position, PartSpec):
+            position = POSITION_ENCODINGS.build(position)
+        if position is not None and not isinstance(position, PositionEncoding):
+            raise ConfigError("grouped attention: 'position' must be a position encoding or its spec")
+        if position is not None and position.rotary_dim > self.head_dim:
+            raise ConfigError(f"grouped attention: {position.rotary_dim} rotated elements of a head of {self.head_dim}")
+        self.position = position
+        self.external = bool(external)
+        self._dtype = torch.bfloat16
+        self.w_in = self.w_o = None
+
+    # ---- sizes -----------------------------------------------------------
+    def padded_head_dim(self) -> int:
+        from ..kernels.ops import padded_head_size
+        return padded_head_size(max(self.head_dim, self.value_dim), self._dtype)
+
+    @property
+    def columns(self) -> int:
+        """Columns of the joint projection: q, then k and v (unless shared), then the gate."""
+        n = self.num_heads * self.head_dim + (self.num_heads if self.has_gate else 0)
+        return n + (0 if self.shared_cache else self.num_kv_heads * (self.head_dim + self.value_dim))
+
+    def cache_spec(self):
+        return KVCacheSpec(self.num_kv_heads, self.padded_head_dim(), self.cache_window, pools=self.cache_pools)
+
+    def flops_per_query_key_pair(self):
+        return 4 * self.num_heads * self.padded_head_dim()
+
+    def weight_specs(self):
+        W, H, G, D, E = self.hidden_size, self.num_heads, self.num_kv_heads, self.head_dim, self.value_dim
+        specs = {"q": WeightSpec((H * D, W))}
+        if not self.shared_cache:
+            specs |= {"k": WeightSpec((G * D, W)), "v": WeightSpec((G * E, W))}
+        if self.has_gate:
+            specs["g"] = WeightSpec((H, W))
+        specs["o"] = WeightSpec((W, H * E))
+        return specs
+
+    def stacked(self, weights) -> list:
+        """The projections' matrices in the order of the joint product's columns."""
+        return [weights[n] for n in ("q", "k", "v", "g") if n in weights]
+
+    def load_weights(self, weights, dtype, device):
+        self._dtype = dtype
+        if not self.external:
+            w = self.stacked(weights)
+            self.w_in = to_device(torch.cat([t.to(w[0].dtype) for t in w], 0), dtype, device)
+        self.w_o = to_device(weights["o"], dtype, device)
+
+    def forward_projected(self, ctx, proj):
+        """From the joint projection (float32 [T, >= columns], rows may be strided) to the mixer's output."""
+        ops, kv, b = ctx.ops, ctx.kv, ctx.batch
+        H, G, D, E = self.num_heads, self.num_kv_heads, self.head_dim, self.value_dim
+        P = kv.k_cache.shape[3]
+        table = self.position.cached_table(ctx.max_positions, proj.device) if self.position is not None else None
+        pairing = 1 if (self.position is not None and self.position.pairing == "interleaved") else 0
+        q = ops.grouped_qkv_store(proj, H, G, D, E, table, pairing, (self.q_temp_coef, self.q_temp_every), b.positions, kv,
+                                  store=not self.shared_cache)
+        if not self.shared_cache:
+            for p in self.cache_pools:
+                ops.pool_keys(kv, b, p)
+        o = ops.paged_attention(q, H, G, P, kv, b, self.window, self.scale, pool=self.pool)
+        gate = proj[:, self.columns - H:self.columns] if self.has_gate else None
+        if gate is not None or P != E:
+            o = ops.gate_heads(o, P, gate, H, E)
+        return ops.linear(o, self.w_o, out_dtype=torch.float32, partials=True)
+
+    def forward(self, ctx, x):
+        if self.external:
+            raise RuntimeError("grouped attention: its projections were left to a combining mixer")
+        return self.forward_projected(ctx, ctx.ops.linear(x, self.w_in, out_dtype=torch.float32))

@@ -45,11 +45,21 @@ class WeightSpec:
 class KVCacheSpec:
     """Cache need of a mixer that keeps keys and values per token.
     ``window`` 0: all tokens are kept; > 0: only the last ``window``, and the first
-    ``keep_first`` tokens of the request, which every later token goes on reading."""
+    ``keep_first`` tokens of the request, which every later token goes on reading.
+    ``pools``: block sizes in tokens, ascending; for each the cache also keeps, for good, one
+    key and one value per whole block of so many tokens (what the mixer makes of the block's
+    keys and values), and holds a block's tokens until it is whole."""
     num_kv_heads: int
     head_dim: int
     window: int = 0
     keep_first: int = 0
+    pools: tuple = ()
+
+    @property
+    def reach(self) -> int:
+        """Tokens before the next one that the cache holds at most beyond ``keep_first``: the window,
+        or an unfinished block where that is longer (0: all of them)."""
+        return max(self.window, *self.pools) if self.window > 0 and self.pools else self.window
 
 
 @dataclass(frozen=True)
@@ -164,6 +174,14 @@ class Block(Part):
 
     def __init__(self, mixer: Mixer, feed_forward: FeedForward, make_norm):
         raise NotImplementedError
+
+    def state_spec(self) -> StateSpec | None:
+        """State per request that the block itself carries from step to step, a row of floats: it lies
+        behind the mixer's own in the layer call's state (``state_offset`` floats from its start,
+        which the model sets)."""
+        return None
+
+    state_offset = 0
 
     def forward(self, ctx, resid: torch.Tensor, pending: torch.Tensor | None) -> torch.Tensor | None:
         """``resid`` is the float32 residual stream, ``pending`` a float32 term

@@ -216,3 +216,76 @@ class ParallelBlock(Block):
         if not self.has_ffn:
             return a
         return ops.PendingTerms([a, self.feed_forward.forward(ctx, h2)])
+
+
+@register_block("sandwich")
+class SandwichBlock(Block):
+    """x <- x + s1 * norm1_out(mixer(c1(norm1(x))));  x <- x + s2 * norm2_out(ffn(c2(norm2(x)))): a norm before and
+    after each sublayer.  ``layer_scale``: s1 and s2 are vectors (``ls1``, ``ls2``; else 1).  ``conv_taps`` K > 0:
+    c(h)_t = h_t + sum_j w[:, j] h_(t - K + 1 + j), a causal convolution over time on each channel added to
+    its input (``canon1``, ``canon2`` [hidden, K]; zeros before a request's start); the last K - 1 rows h of
+    both sublayers are the block's state.  A sublayer's result stays pending, with its norm and its scale, for
+    the norm before the next sublayer, whose kernel does everything from there to that sublayer's input.  A
+    layer without a feed-forward has no second half (its tensors may be left out)."""
+
+    graph_safe = True
+    MAX_TAPS = 32
+
+    def __init__(self, mixer, feed_forward, make_norm, hidden_size: int, conv_taps: int = 0, layer_scale: bool = False):
+        from ..config.base import ConfigError
+        self.hidden_size = int(hidden_size)
+        self.conv_taps = int(conv_taps)
+        self.layer_scale = bool(layer_scale)
+        if not 0 <= self.conv_taps <= self.MAX_TAPS:
+            raise ConfigError(f"sandwich block: a convolution of {conv_taps} taps (up to {self.MAX_TAPS})")
+        self.mixer, self.feed_forward = mixer, feed_forward
+        self.norm1, self.norm1_out, self.norm2, self.norm2_out = (make_norm() for _ in range(4))
+        for n in (self.norm1, self.norm1_out, self.norm2, self.norm2_out):
+            if not hasattr(n, "output_term"):
+                raise ConfigError("sandwich block: its norms are layer norms")
+        self.has_ffn = not getattr(feed_forward, "is_none", False)
+        if not self.has_ffn:
+            self.norm2.optional = self.norm2_out.optional = True
+        self.ls1 = self.ls2 = self.conv1 = self.conv2 = None
+
+    def children(self):
+        return {"norm1": self.norm1, "mixer": self.mixer, "norm1_out": self.norm1_out, "norm2": self.norm2,
+                "feed_forward": self.feed_forward, "norm2_out": self.norm2_out}
+
+    def weight_specs(self):
+        from .base import WeightSpec
+        W, K, late = self.hidden_size, self.conv_taps, not self.has_ffn
+        specs = {}
+        if self.layer_scale:
+            specs |= {"ls1": WeightSpec((W,), "norm"), "ls2": WeightSpec((W,), "norm", optional=late)}
+        if K:
+            specs |= {"canon1": WeightSpec((W, K), "vector"), "canon2": WeightSpec((W, K), "vector", optional=late)}
+        return specs
+
+    def load_weights(self, weights, dtype, device):
+        import torch
+        f32 = lambda t: t.to(torch.float32).contiguous().to(device)      # noqa: E731
+        get = lambda n: f32(weights[n]) if n in weights else None        # noqa: E731
+        self.ls1, self.ls2 = get("ls1"), get("ls2")
+        # tap by tap, so that neighbouring channels lie side by side
+        self.conv1, self.conv2 = (f32(weights[n].t()) if n in weights else None for n in ("canon1", "canon2"))
+
+    @property
+    def _conv_state(self) -> int:
+        return (self.conv_taps - 1) * self.hidden_size if self.conv_taps else 0
+
+    def state_spec(self):
+        from .base import StateSpec
+        n = self._conv_state * (2 if self.has_ffn else 1)
+        return StateSpec((n,)) if n else None
+
+    def _conv(self, ctx, w, which: int):
+        return (w, ctx.state, self.state_offset + which * self._conv_state) if self.conv_taps else None
+
+    def forward(self, ctx, resid, pending):
+        h = self.norm1.forward(ctx, resid, pending, conv=self._conv(ctx, self.conv1, 0))
+        a = self.norm1_out.output_term(ctx, self.mixer.forward(ctx, h), self.ls1)
+        if not self.has_ffn:
+            return a
+        z = self.norm2.forward(ctx, resid, a, conv=self._conv(ctx, self.conv2, 1))
+        return self.norm2_out.output_term(ctx, self.feed_forward.forward(ctx, z), self.ls2)

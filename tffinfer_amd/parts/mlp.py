@@ -13,6 +13,8 @@ class SwiGLU(FeedForward):
     Reference: src/core/model/base/ModelCreatorBase.cpp:51-94 (up, gate, the
     unary op with x1 = gate, x2 = up, down), src/kernel/cuda/unary.cu:10-27.
     Gate and up are put into one matrix at load so that one product streams both.
+    ``bias``: all three projections have one (``<name>.b``, float32 where it is added), f =
+    Wdown (silu(Wgate z + bg) * (Wup z + bu)) + bd; the last one is left to whoever adds f to the stream.
     """
 
     graph_safe = True
@@ -20,26 +22,41 @@ class SwiGLU(FeedForward):
     input_goes_to_linear = True
 
     def __init__(self, hidden_size: int, intermediate_size: int,
-                 names=("gate_proj.weight", "up_proj.weight", "down_proj.weight")):
+                 names=("gate_proj.weight", "up_proj.weight", "down_proj.weight"), bias: bool = False):
         self.hidden_size = int(hidden_size)
         self.intermediate_size = int(intermediate_size)
         self.names = tuple(names)       # how the files call gate, up and down
         if len(self.names) != 3:
             from ..config.base import ConfigError
             raise ConfigError("swiglu: 'names' are the names of gate, up and down")
+        self.has_bias = bool(bias)
         self.w_gate_up = None
         self.w_down = None
+        self.gate_up_bias = self.down_bias = None
 
     def weight_specs(self):
         H, I = self.hidden_size, self.intermediate_size
-        return {
+        specs = {
             self.names[0]: WeightSpec((I, H)),
             self.names[1]: WeightSpec((I, H)),
             self.names[2]: WeightSpec((H, I)),
         }
+        if self.has_bias:
+            for n, size in zip(self.names, (I, I, H)):
+                specs[n + ".b"] = WeightSpec((size,), "norm_offset")
+        return specs
 
     def load_weights(self, weights, dtype, device):
         gate, up = weights[self.names[0]], weights[self.names[1]]
+        if self.has_bias:
+            f32 = lambda t: t.to(torch.float32).contiguous().to(device)      # noqa: E731
+            gb, ub = (f32(weights[n + ".b"]) for n in self.names[:2])
+            if dtype == torch.bfloat16 and torch.device(device).type == "cuda":
+                from ..kernels import ops
+                self.gate_up_bias = ops.pack_gate_up_bias(gb, ub)       # in the order of the product's rows
+            else:
+                self.gate_up_bias = torch.cat([gb, ub], 0)
+            self.down_bias = f32(weights[self.names[2] + ".b"])
         if dtype == torch.bfloat16 and torch.device(device).type == "cuda":
             # bfloat16: gate and up rows interleaved in groups of 16 in one weight, so that one
             # product streams both and applies silu(gate) * up to its float32 accumulators
@@ -52,6 +69,10 @@ class SwiGLU(FeedForward):
         self.w_down = to_device(weights[self.names[2]], dtype, device)
 
     def forward(self, ctx, x):
+        if self.has_bias:
+            m = ctx.ops.linear_swiglu_bias(x, self.w_gate_up, self.gate_up_bias)
+            return ctx.ops.OutputTerm(ctx.ops.linear(m, self.w_down, out_dtype=torch.float32, partials=True),
+                                      bias=self.down_bias)
         gu = ctx.ops.linear(x, self.w_gate_up)
         m = gu if getattr(self.w_gate_up, "glu_out", 0) else ctx.ops.swiglu(gu)
         return ctx.ops.linear(m, self.w_down, out_dtype=torch.float32, partials=True)
@@ -120,6 +141,8 @@ class RoutedExperts(FeedForward):
     ``limit`` None: no clamp; ``up_offset`` 0 and ``act_alpha`` 1: y = silu(g) * u.
     ``weight_input``: the weight multiplies what goes into the expert, f = sum of expert_e(w_e z),
     instead of what comes out.
+    ``identity``: that many experts more, behind the others in the router's outputs, have no matrices and hand
+    their input on, f_e = z.
 
     The experts' matrices lie stacked, [experts, out, in], so that a kernel finds an expert's
     rows by its number."""
@@ -129,7 +152,8 @@ class RoutedExperts(FeedForward):
     def __init__(self, hidden_size: int, intermediate_size: int, num_experts: int, top: int,
                  limit: float | None, act_alpha: float = 1.702, correction: bool = True,
                  router_softmax: bool = False, up_offset: float = 1.0, normalize: bool = True,
-                 weight_input: bool = False):
+                 weight_input: bool = False, identity: int = 0):
+        self.identity = int(identity)
         self.router_softmax = bool(router_softmax)
         self.normalize = bool(normalize)
         self.weight_input = bool(weight_input)
@@ -141,16 +165,21 @@ class RoutedExperts(FeedForward):
         self.limit = float("inf") if limit is None else float(limit)
         self.act_alpha = float(act_alpha)
         self.has_correction = bool(correction)
-        if not 0 < self.top <= self.num_experts:
+        if self.identity < 0 or not 0 < self.top <= self.num_experts + self.identity or self.num_experts < 1:
             from ..config.base import ConfigError
-            raise ConfigError(f"routed experts: top={self.top} of {self.num_experts} experts")
+            raise ConfigError(f"routed experts: top={self.top} of {self.num_experts} experts"
+                              + (f" and {self.identity} that hand their input on" if self.identity else ""))
+        if self.identity and self.weight_input:
+            from ..config.base import ConfigError
+            raise ConfigError("routed experts: experts that hand their input on take the weight on their output")
         self.w_gate = self.w_up = self.w_down = self.router = self.router_w = self.correction = None
 
     def weight_specs(self):
         H, I = self.hidden_size, self.intermediate_size
-        specs = {"router": WeightSpec((self.num_experts, H))}
+        rows = self.num_experts + self.identity
+        specs = {"router": WeightSpec((rows, H))}
         if self.has_correction:
-            specs["correction"] = WeightSpec((self.num_experts,), "vector")
+            specs["correction"] = WeightSpec((rows,), "vector")
         for e in range(self.num_experts):
             specs[f"e{e}.gate"] = WeightSpec((I, H))
             specs[f"e{e}.up"] = WeightSpec((I, H))
@@ -160,13 +189,17 @@ class RoutedExperts(FeedForward):
     def active_matrix_elements(self) -> int:
         """Matrix elements a token multiplies with: the router and its ``top`` experts."""
         H, I = self.hidden_size, self.intermediate_size
-        return self.num_experts * H + self.top * 3 * H * I
+        # (on average over the experts, where some have no matrices)
+        share = self.num_experts / (self.num_experts + self.identity)
+        return (self.num_experts + self.identity) * H + round(self.top * share * 3 * H * I)
 
     def streamed_matrix_elements(self, rows: int) -> int:
         """Matrix elements a step of ``rows`` tokens reads at least: the router and as many
         experts as the tokens can choose between them."""
         H, I = self.hidden_size, self.intermediate_size
-        return self.num_experts * H + min(self.num_experts, rows * self.top) * 3 * H * I
+        share = self.num_experts / (self.num_experts + self.identity)
+        return ((self.num_experts + self.identity) * H
+                + round(min(self.num_experts, rows * self.top * share) * 3 * H * I))
 
     def load_weights(self, weights, dtype, device):
         E = self.num_experts
@@ -198,7 +231,8 @@ class RoutedExperts(FeedForward):
             idx, wts = ops.route_topk(x, self.router, self.correction, self.top, softmax=self.router_softmax,
                                       normalize=self.normalize)
         return ops.routed_experts(x, self.w_gate, self.w_up, self.w_down, idx, wts, self.limit, self.act_alpha,
-                                  up_offset=self.up_offset, weight_input=self.weight_input)
+                                  up_offset=self.up_offset, weight_input=self.weight_input,
+                                  **({"identity": self.identity} if self.identity else {}))
 
 
 @register_feed_forward("table_experts")
