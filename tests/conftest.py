@@ -53,6 +53,14 @@ def rutevik_dirs(tmp_path_factory):
     return {name: make_rutevik_dir(str(base / name), cfg, seed) for name, (cfg, seed) in RUTEVIK_CONFIGS.items()}
 
 
+@pytest.fixture(scope="session")
+def gopuzen_dirs(tmp_path_factory):
+    """Model folders of the tiny Gopuzen configurations (sharpened weights), once per session."""
+    from gopuzen_models import GOPUZEN_CONFIGS, make_gopuzen_dir
+    base = tmp_path_factory.mktemp("gopuzen")
+    return {name: make_gopuzen_dir(str(base / name), cfg, seed) for name, (cfg, seed) in GOPUZEN_CONFIGS.items()}
+
+
 @pytest.fixture(autouse=True)
 def _seeded():
     """Every test draws the same random inputs in every run."""

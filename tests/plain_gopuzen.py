@@ -2,8 +2,8 @@
 
 Whole sequences, no cache, no batching, one function per mechanism, float64.  It shares no code
 with the package: config.json is read with ``json``, the weights with the ``safetensors`` library,
-the recurrence goes token by token, and a window with pooled blocks is one softmax over a list of
-keys built anew for every position.
+the recurrence goes token by token, and a window with blocks before it is one softmax over all
+tokens and all blocks' means with what a position does not see masked out.
 """
 from __future__ import annotations
 
@@ -52,11 +52,10 @@ def with_input_conv(h: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
     """h plus a causal convolution of it over time, per channel: the last tap is the token itself."""
     T, taps = h.shape[0], w.shape[1]
     out = h.clone()
-    for t in range(T):
-        for j in range(taps):
-            s = t - taps + 1 + j
-            if s >= 0:
-                out[t] += w[:, j] * h[s]
+    for j in range(taps):
+        back = taps - 1 - j
+        if back < T:
+            out[back:] += w[:, j] * h[:T - back]
     return out
 
 
@@ -66,21 +65,21 @@ def query_temperature(T: int, coef: float, every: int) -> torch.Tensor:
     return torch.tensor([1.0 + coef * math.log((p + 1) // every + 1) for p in range(T)], dtype=torch.float64)
 
 
-def visible_keys(i: int, keys: torch.Tensor, values: torch.Tensor, size: int, pool: int):
-    """What position i sees of keys [T, D] and values [T, E]: the means of the whole blocks of ``pool``
-    tokens that lie before the window, then the window's own keys."""
-    ks, vs = [], []
-    if size and pool:
-        b = 0
-        while b * pool + pool - 1 <= i - size:
-            ks.append(keys[b * pool:(b + 1) * pool].mean(0))
-            vs.append(values[b * pool:(b + 1) * pool].mean(0))
-            b += 1
-    lo = max(0, i - size + 1) if size else 0
-    for j in range(lo, i + 1):
-        ks.append(keys[j])
-        vs.append(values[j])
-    return torch.stack(ks), torch.stack(vs)
+def block_means(x: torch.Tensor, pool: int) -> torch.Tensor:
+    """x [T, ...] -> the means over its whole blocks of ``pool`` rows, [T // pool, ...]."""
+    n = x.shape[0] // pool
+    return x[:n * pool].reshape(n, pool, *x.shape[1:]).mean(1)
+
+
+def visible(T: int, size: int, pool: int):
+    """(what position i sees of the tokens [T, T], of the blocks [T, T // pool]): tokens j <= i with
+    i - j < size; blocks whose last token lies before that window.  size 0: every token j <= i."""
+    i, j = torch.arange(T)[:, None], torch.arange(T)[None, :]
+    tokens = (j <= i) & ((i - j < size) if size else True)
+    if not (size and pool):
+        return tokens, torch.zeros(T, 0, dtype=torch.bool)
+    last = torch.arange(T // pool)[None, :] * pool + pool - 1
+    return tokens, last <= i - size
 
 
 def grouped_attention(q, k, v, scale: float, size: int = 0, pool: int = 0) -> torch.Tensor:
@@ -88,13 +87,14 @@ def grouped_attention(q, k, v, scale: float, size: int = 0, pool: int = 0) -> to
     everything that is visible."""
     T, H, _ = q.shape
     G, E = k.shape[1], v.shape[2]
+    sees = torch.cat(visible(T, size, pool), 1)
+    if size and pool:
+        k, v = torch.cat([k, block_means(k, pool)]), torch.cat([v, block_means(v, pool)])
     out = torch.zeros(T, H, E, dtype=q.dtype)
-    for g in range(G):
-        heads = range(g * (H // G), (g + 1) * (H // G))
-        for i in range(T):
-            ks, vs = visible_keys(i, k[:, g], v[:, g], size, pool)
-            for a in heads:
-                out[i, a] = torch.softmax((ks @ q[i, a]) * scale, 0) @ vs
+    for a in range(H):
+        g = a // (H // G)
+        s = (q[:, a] @ k[:, g].T) * scale
+        out[:, a] = torch.softmax(s.masked_fill(~sees, -math.inf), -1) @ v[:, g]
     return out
 
 
