@@ -142,8 +142,44 @@ RUTEVIK_SHAPES = {
                       diff_dim=64, diff_vdim=128, dense_ff=18432, experts=32, top=4, expert_ff=1536)),
 }
 
+def gopuzen_shape(width, heads, kv_heads, dim, window, pool, left_heads, left_kv_heads, left_dim, left_vdim, right_heads, right_dim,
+                  right_vdim, dense_ff, experts, identity, top, expert_ff, layers, vocab=151936):
+    """A Gopuzen configuration of ``layers`` layers: a windowed attention with the keys of blocks before its window that
+    fills its cache, two layers of an attention beside a recurrence, a windowed attention that reads the first one's
+    cache, and so on; dense feed-forwards and mixtures of experts in turn."""
+    def window_layer(source):
+        m = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5,
+             "mask": {"size": window, "pool": pool}, "rot": {"base": 10000.0, "dims": dim}}
+        if source is not None:
+            m["kv_from"] = source
+        return {"type": "attention", "mixer": m}
+    par = {"type": "parallel", "mixer": {
+        "left": {"heads": left_heads, "kv_heads": left_kv_heads, "dim": left_dim, "vdim": left_vdim, "scale": left_dim ** -0.5,
+                 "q_temp": {"coef": 0.1, "every": 1024}},
+        "right": {"heads": right_heads, "dim": right_dim, "vdim": right_vdim,
+                  "decay": [1.0 - 0.5 ** (1 + 8.0 * i / right_heads) for i in range(right_heads)]}}}
+    mlps = [{"kind": "dense", "ff": dense_ff},
+            {"kind": "moe", "expert": {"ff": expert_ff}, "router": {"experts": experts, "identity": identity, "top": top}}]
+    kinds = [window_layer(None if i % 6 == 0 else i - 3) if i % 3 == 0 else par for i in range(layers)]
+    return {"architecture": "Gopuzen", "width": width, "vocab": vocab, "norm": {"eps": 1e-6}, "canon": {"taps": 4},
+            "embedding": {"scale": 1.0}, "layers": [dict(kinds[i], mlp=mlps[i % 2]) for i in range(layers)]}
+
+
+# Gopuzen at sizes that resemble a real model's layers, beside the Qwen3 shape of the same width (the same gated
+# feed-forward) and, with --design-beside sipilorn, beside the design whose layers are closest: an attention beside a
+# recurrence with a matrix of state per head, a windowed attention, routed experts
+GOPUZEN_SHAPES = {
+    "2k": ("1.7b", dict(width=2048, heads=16, kv_heads=4, dim=128, window=1024, pool=16, left_heads=16, left_kv_heads=4, left_dim=128,
+                        left_vdim=128, right_heads=8, right_dim=128, right_vdim=128, dense_ff=6144, experts=16, identity=4, top=2,
+                        expert_ff=1536)),
+    "4k": ("8b", dict(width=4096, heads=32, kv_heads=8, dim=128, window=1024, pool=16, left_heads=32, left_kv_heads=8, left_dim=128,
+                      left_vdim=128, right_heads=16, right_dim=128, right_vdim=128, dense_ff=12288, experts=32, identity=8, top=4,
+                      expert_ff=1536)),
+}
+
 DESIGNS = {"disunex": ("Disunex", DISUNEX_SHAPES, disunex_shape), "netovik": ("Netovik", NETOVIK_SHAPES, netovik_shape),
-           "sipilorn": ("Sipilorn", SIPILORN_SHAPES, sipilorn_shape), "rutevik": ("Rutevik", RUTEVIK_SHAPES, rutevik_shape)}
+           "sipilorn": ("Sipilorn", SIPILORN_SHAPES, sipilorn_shape), "rutevik": ("Rutevik", RUTEVIK_SHAPES, rutevik_shape),
+           "gopuzen": ("Gopuzen", GOPUZEN_SHAPES, gopuzen_shape)}
 
 
 def design_points(args):

@@ -88,6 +88,10 @@ __global__ __launch_bounds__(NT) void add_layernorm_kernel(float* __restrict__ r
     const int i = blockIdx.x, tid = threadIdx.x;
     const size_t row = rows ? (size_t)rows[i] : (size_t)i;
     const float inv_w = 1.0f / (float)W;
+    const size_t at = row * W;
+    float* const xr = resid ? resid + at : nullptr;
+    const float* const ar = tm.a ? tm.a + at : nullptr;
+    const float* const br = tm.b ? tm.b + at : nullptr;
     float x[IT][VEC], d[IT][VEC], p2[IT][VEC];
 #pragma unroll
     for (int it = 0; it < IT; ++it) {
@@ -95,12 +99,12 @@ __global__ __launch_bounds__(NT) void add_layernorm_kernel(float* __restrict__ r
 #pragma unroll
         for (int u = 0; u < VEC; ++u) x[it][u] = d[it][u] = p2[it][u] = 0.f;
         if (e < W) {
-            if (resid) sn_load<VEC>(x[it], resid + row * W + e);
+            if (xr) sn_load<VEC>(x[it], xr + e);
             if (tm.a) {
-                sn_load<VEC>(d[it], tm.a + row * W + e);
+                sn_load<VEC>(d[it], ar + e);
                 for (int p = 1; p < tm.planes_a; ++p) {
                     float t[VEC];
-                    sn_load<VEC>(t, tm.a + p * tm.plane_a + row * W + e);
+                    sn_load<VEC>(t, ar + p * tm.plane_a + e);
 #pragma unroll
                     for (int u = 0; u < VEC; ++u) d[it][u] += t[u];
                 }
@@ -112,10 +116,10 @@ __global__ __launch_bounds__(NT) void add_layernorm_kernel(float* __restrict__ r
                 }
             }
             if (tm.b) {
-                sn_load<VEC>(p2[it], tm.b + row * W + e);
+                sn_load<VEC>(p2[it], br + e);
                 for (int p = 1; p < tm.planes_b; ++p) {
                     float t[VEC];
-                    sn_load<VEC>(t, tm.b + p * tm.plane_b + row * W + e);
+                    sn_load<VEC>(t, br + p * tm.plane_b + e);
 #pragma unroll
                     for (int u = 0; u < VEC; ++u) p2[it][u] += t[u];
                 }
@@ -195,7 +199,7 @@ __global__ __launch_bounds__(NT) void add_layernorm_kernel(float* __restrict__ r
                 }
 #pragma unroll
                 for (int u = 0; u < VEC; ++u) x[it][u] += d[it][u];
-                if (resid && !rows) sn_store<VEC, float>(resid + row * W + e, x[it]);
+                if (xr && !rows) sn_store<VEC, float>(xr + e, x[it]);
             }
         }
     }
@@ -228,10 +232,11 @@ __global__ __launch_bounds__(NT) void add_layernorm_kernel(float* __restrict__ r
             }
         }
     }
+    TO* const orow = out + (size_t)i * W;
 #pragma unroll
     for (int it = 0; it < IT; ++it) {
         const int e = (it * NT + tid) * VEC;
-        if (e < W) sn_store<VEC, TO>(out + (size_t)i * W + e, x[it]);
+        if (e < W) sn_store<VEC, TO>(orow + e, x[it]);
     }
 }
 
@@ -256,13 +261,14 @@ TFF_API int tff_add_layernorm(float* resid, const float* a, int planes_a, size_t
     auto ok16 = [](const void* p) { return ((uintptr_t)p % 16) == 0; };
     const bool vec = W % 4 == 0 && plane_a % 4 == 0 && plane_b % 4 == 0 && ok16(resid) && ok16(a) && ok16(b) && ok16(wa) && ok16(wb) &&
                      ok16(bias) && ok16(nw) && ok16(nb) && ok16(scale) && ok16(w) && ok16(beta) && ok16(out) && ok16(conv_w);
+    TFF_REQUIRE(vec || W <= 8192, "add_layernorm: rows of %d (more than 8192) must be a multiple of 4 wide and 16-byte aligned", W);
 #define SN_LAUNCH(TO, NT, VPT, VEC) add_layernorm_kernel<TO, NT, VPT, VEC><<<n, NT, 0, s>>>(resid, tm, w, beta, eps, (TO*)out, rows, W, cv)
 #define SN_SIZES(TO)                                                                         \
     do {                                                                                     \
         if (!vec) {                                                                          \
             if (W <= 1024) SN_LAUNCH(TO, 256, 4, 1);                                         \
             else if (W <= 4096) SN_LAUNCH(TO, 1024, 4, 1);                                   \
-            else SN_LAUNCH(TO, 1024, 16, 1);                                                 \
+            else SN_LAUNCH(TO, 1024, 8, 1);                                                  \
         } else if (W <= 1024) SN_LAUNCH(TO, 256, 4, 4);                                      \
         else if (W <= 4096 && n <= 256) SN_LAUNCH(TO, 1024, 4, 4);                           \
         else if (W <= 2048) SN_LAUNCH(TO, 256, 8, 4);                                        \

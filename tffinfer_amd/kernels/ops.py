@@ -569,7 +569,7 @@ def _attention_block_work(batch, G: int, nkv: int, window: int, device, cols: in
     cache = getattr(batch, "_attn_work", None)
     if cache is None:
         cache = batch._attn_work = {}
-    key = ("blocks", G, nkv, cols, window, bins, which, key_groups, head_dim, num_cus, pool)
+    key = ("blocks", G, nkv, cols, window, bins, which, key_groups, head_dim, num_cus) + ((pool,) if pool else ())
     if key not in cache:
         cu, P = batch.host_cu_tokens, batch.host_start_pos
         items = []                       # (slices, entry, first column)
