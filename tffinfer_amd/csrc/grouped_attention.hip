@@ -101,7 +101,9 @@ TFF_API int tff_grouped_qkv_store(const float* proj, size_t row, const float* co
 }
 
 // Blocks (token, kv head).  The sum runs over the block's tokens in their order; a thread takes elements tid, tid + 128, ...
+// Where the tokens' keys and values lie is worked out by the threads side by side, PK_RUN tokens at a time.
 #define PK_THREADS 128
+#define PK_RUN 64
 
 template <typename TC>
 __global__ __launch_bounds__(PK_THREADS) void pool_keys_kernel(TC* __restrict__ k_cache, TC* __restrict__ v_cache,
@@ -111,25 +113,38 @@ __global__ __launch_bounds__(PK_THREADS) void pool_keys_kernel(TC* __restrict__ 
                                                                const int32_t* __restrict__ positions,
                                                                const int32_t* __restrict__ slots, int page_size, int pool, int G,
                                                                int d) {
-    const int t = blockIdx.x, g = blockIdx.y;
+    __shared__ size_t koff[PK_RUN], voff[PK_RUN];
+    const int t = blockIdx.x, g = blockIdx.y, tid = threadIdx.x;
     const int pos = positions[t];
     if (slots[t] < 0 || (pos + 1) % pool) return;      // (the whole block)
     const int r = token_req[t], blk = pos / pool, first = pos + 1 - pool;
     const int32_t* bt = block_tables + (size_t)r * bt_stride;
     const int dpage = pool_tables[(size_t)r * pt_stride + blk / page_size], dslot = blk % page_size;
     const float f = 1.0f / (float)pool;
-    for (int e = threadIdx.x; e < d; e += PK_THREADS) {
+    const size_t dhead = ((size_t)dpage * G + g) * page_size * d;
+    for (int e0 = 0; e0 < d; e0 += PK_THREADS) {
+        const int e = min(e0 + tid, d - 1);
         float ks = 0.f, vs = 0.f;
-#pragma unroll 4
-        for (int i = 0; i < pool; ++i) {
-            const int j = first + i, slot = j % page_size;
-            const size_t head = ((size_t)bt[j / page_size] * G + g) * page_size * d;
-            ks += to_f32(k_cache[head + (size_t)slot * d + e]);
-            vs += to_f32(v_cache[head + (size_t)e * page_size + slot]);
+        for (int i0 = 0; i0 < pool; i0 += PK_RUN) {
+            const int cnt = min(PK_RUN, pool - i0);
+            if (i0 || e0) __syncthreads();             // the run before is read
+            if (tid < cnt) {
+                const int j = first + i0 + tid, slot = j % page_size;
+                const size_t head = ((size_t)bt[j / page_size] * G + g) * page_size * d;
+                koff[tid] = head + (size_t)slot * d;
+                voff[tid] = head + slot;
+            }
+            __syncthreads();
+#pragma unroll 8
+            for (int i = 0; i < cnt; ++i) {
+                ks += to_f32(k_cache[koff[i] + e]);
+                vs += to_f32(v_cache[voff[i] + (size_t)e * page_size]);
+            }
         }
-        const size_t head = ((size_t)dpage * G + g) * page_size * d;
-        k_cache[head + (size_t)dslot * d + e] = from_f32<TC>(ks * f);
-        v_cache[head + (size_t)e * page_size + dslot] = from_f32<TC>(vs * f);
+        if (e0 + tid < d) {
+            k_cache[dhead + (size_t)dslot * d + e] = from_f32<TC>(ks * f);
+            v_cache[dhead + (size_t)e * page_size + dslot] = from_f32<TC>(vs * f);
+        }
     }
 }
 
@@ -165,6 +180,21 @@ __global__ __launch_bounds__(256) void gate_heads_kernel(const T* __restrict__ o
     out[t * HE + c] = from_f32<T>(to_f32(o[t * o_row + (size_t)h * P + e]) * f);
 }
 
+// The same, eight neighbouring elements a thread (E, P and the rows' strides multiples of 8).
+__global__ __launch_bounds__(256) void gate_heads8_kernel(const bf16_t* __restrict__ o, size_t o_row, int P, const float* __restrict__ g,
+                                                          size_t g_row, bf16_t* __restrict__ out, int HE8, int E8, size_t count) {
+    const size_t id = (size_t)blockIdx.x * 256 + threadIdx.x;
+    if (id >= count) return;
+    const size_t t = id / HE8;
+    const int c = (int)(id - t * HE8), h = c / E8, e = c - h * E8;
+    const float f = g ? 1.0f / (1.0f + expf(-g[t * g_row + h])) : 1.0f;
+    union { uint4 u; bf16_t b[8]; } x;
+    x.u = *reinterpret_cast<const uint4*>(o + t * o_row + (size_t)h * P + e * 8);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) x.b[i] = (bf16_t)((float)x.b[i] * f);
+    *reinterpret_cast<uint4*>(out + (t * HE8 + c) * 8) = x.u;
+}
+
 TFF_API int tff_gate_heads(const void* o, size_t o_row, int P, const float* g, size_t g_row, void* out, int T, int H, int E,
                            int dtype, tff_stream_t stream) {
     TFF_REQUIRE(o && out, "gate_heads: null pointer");
@@ -173,6 +203,11 @@ TFF_API int tff_gate_heads(const void* o, size_t o_row, int P, const float* g, s
     hipStream_t s = (hipStream_t)stream;
     const size_t count = (size_t)T * H * E;
     const unsigned blocks = (unsigned)((count + 255) / 256);
+    if (dtype == TFF_BF16 && E % 8 == 0 && P % 8 == 0 && o_row % 8 == 0 && ((uintptr_t)o % 16) == 0 && ((uintptr_t)out % 16) == 0) {
+        gate_heads8_kernel<<<(unsigned)((count / 8 + 255) / 256), 256, 0, s>>>((const bf16_t*)o, o_row, P, g, g_row, (bf16_t*)out, H * E / 8,
+                                                                               E / 8, count / 8);
+        return tff_check_launch("gate_heads");
+    }
     if (dtype == TFF_F32)
         gate_heads_kernel<float><<<blocks, 256, 0, s>>>((const float*)o, o_row, P, g, g_row, (float*)out, H * E, E, count);
     else if (dtype == TFF_BF16)

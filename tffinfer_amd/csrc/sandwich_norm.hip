@@ -283,21 +283,20 @@ TFF_API int tff_add_layernorm(float* resid, const float* a, int planes_a, size_t
     return tff_check_launch("add_layernorm");
 }
 
-// Items (row of the step's tables, first place in the request's portion) of up to SC_CHUNK tokens; a thread takes
+// Items (row of the step's tables, first place in the request's portion) of up to `chunk` tokens; a thread takes
 // VEC neighbouring channels through an item's tokens, the taps' inputs in registers.  The first item of a portion
-// alone reads the state (SC_CHUNK >= taps - 1) and alone leaves the new one there, each thread its own channels.
-#define SC_CHUNK 32
+// alone reads the state (chunk >= taps - 1) and alone leaves the new one there, each thread its own channels.
 
 template <typename TO, int TAPS, int VEC>
 __global__ __launch_bounds__(256) void input_conv_kernel(const float* __restrict__ h, const float* __restrict__ w, int taps_any,
                                                          float* __restrict__ state, size_t state_row, size_t off,
-                                                         const int32_t* __restrict__ items, const int32_t* __restrict__ cu_tokens,
+                                                         const int32_t* __restrict__ items, int chunk, const int32_t* __restrict__ cu_tokens,
                                                          const int32_t* __restrict__ slots, TO* __restrict__ out, int W) {
     const int e = (blockIdx.y * 256 + threadIdx.x) * VEC;
     if (e >= W) return;
     const int r = items[2 * blockIdx.x], i0 = items[2 * blockIdx.x + 1];
     const int t0 = cu_tokens[r], n = cu_tokens[r + 1] - t0;
-    const int i1 = min(n, i0 + SC_CHUNK);
+    const int i1 = min(n, i0 + chunk);
     const int taps = TAPS ? TAPS : taps_any;
     float* st = state ? state + (size_t)slots[r] * state_row + off : nullptr;
     const float* base = h + (size_t)t0 * W + e;
@@ -358,14 +357,12 @@ __global__ __launch_bounds__(256) void input_conv_kernel(const float* __restrict
     }
 }
 
-TFF_API int tff_input_conv_chunk(void) { return SC_CHUNK; }
-
 TFF_API int tff_input_conv(const float* h, const float* w, int taps, float* state, size_t state_row, size_t state_off,
-                           const int32_t* items, int num_items, const int32_t* cu_tokens, const int32_t* state_slots, void* out,
-                           int W, int out_dtype, tff_stream_t stream) {
+                           const int32_t* items, int num_items, int chunk, const int32_t* cu_tokens, const int32_t* state_slots,
+                           void* out, int W, int out_dtype, tff_stream_t stream) {
     TFF_REQUIRE(h && w && items && cu_tokens && out, "input_conv: null pointer");
-    TFF_REQUIRE(num_items >= 0 && W > 0 && taps >= 1 && taps <= SN_MAX_TAPS && SC_CHUNK >= SN_MAX_TAPS - 1,
-                "input_conv: rows of %d, %d taps (up to %d)", W, taps, SN_MAX_TAPS);
+    TFF_REQUIRE(num_items >= 0 && W > 0 && taps >= 1 && taps <= SN_MAX_TAPS && chunk >= 1 && chunk >= taps - 1,
+                "input_conv: rows of %d, %d taps (up to %d), items of %d tokens", W, taps, SN_MAX_TAPS, chunk);
     TFF_REQUIRE(taps == 1 || (state && state_slots && state_off + (size_t)(taps - 1) * W <= state_row),
                 "input_conv: state rows of %zu do not hold %d rows of %d", state_row, taps - 1, W);
     if (num_items == 0) return 0;
@@ -374,7 +371,7 @@ TFF_API int tff_input_conv(const float* h, const float* w, int taps, float* stat
     const int per = vec ? 1024 : 256;
     const dim3 grid(num_items, (W + per - 1) / per);
     if (taps == 1) state = nullptr;
-#define SC_GO(TO, TAPS, VEC) input_conv_kernel<TO, TAPS, VEC><<<grid, 256, 0, s>>>(h, w, taps, state, state_row, state_off, items, \
+#define SC_GO(TO, TAPS, VEC) input_conv_kernel<TO, TAPS, VEC><<<grid, 256, 0, s>>>(h, w, taps, state, state_row, state_off, items, chunk, \
                                                                                   cu_tokens, state_slots, (TO*)out, W)
 #define SC_TAPS(TO)                                                                               \
     do {                                                                                          \

@@ -429,15 +429,21 @@ TFF_API int tff_add_layernorm(float* resid, const float* a, int planes_a, size_t
                               const float* beta, float eps, void* out, const int32_t* rows, int n, int W, const float* conv_w,
                               int taps, float* state, size_t state_row, size_t state_off, const int32_t* state_slots,
                               int out_dtype, tff_stream_t stream);
-TFF_API int tff_input_conv_chunk(void);      // tokens an item of tff_input_conv holds at most
+// items of up to `chunk` tokens (row of the step's tables, first place in its portion), chunk >= taps - 1
 TFF_API int tff_input_conv(const float* h, const float* w, int taps, float* state, size_t state_row, size_t state_off,
-                           const int32_t* items, int num_items, const int32_t* cu_tokens, const int32_t* state_slots, void* out,
+                           const int32_t* items, int num_items, int chunk, const int32_t* cu_tokens, const int32_t* state_slots, void* out,
                            int W, int out_dtype, tff_stream_t stream);
 
 // ---- a linear recurrence with a fixed decay per head (lightning.hip) ----
 TFF_API int tff_lightning(const float* proj, size_t ldp, const float* decay, float* state, size_t state_row,
                           const int32_t* cu_tokens, const int32_t* state_slots, float* o, int R, int H, int D, int E,
-                          int max_tokens, tff_stream_t stream);
+                          tff_stream_t stream);
+TFF_API int tff_lightning_chunk(void);       // tokens an item of tff_lightning_chunks holds at most
+// items [num_items][2]: (row of the step's tables, first place in its portion); item_start [R + 1]: a row's items, in
+// order; sums: float32 [num_items][H][E][D] of workspace; decays must not be negative.
+TFF_API int tff_lightning_chunks(const float* proj, size_t ldp, const float* decay, float* state, size_t state_row,
+                                 const int32_t* items, const int32_t* item_start, int num_items, const int32_t* cu_tokens,
+                                 const int32_t* state_slots, float* sums, float* o, int R, int H, int D, int E, tff_stream_t stream);
 TFF_API int tff_row_norm_gate(const float* o, const float* g, size_t g_row, const float* w, float eps, void* out, int T, int N,
                               int out_dtype, tff_stream_t stream);
 

@@ -88,9 +88,10 @@ _SIGNATURES = {
     "tff_sample": [_P, _P, _I, _I, _P, _P, _P, _P, _P, _P, _P],
     "tff_add_layernorm": [_P, _P, _I, _Z, _P, _I, _Z, _P, _P, _F, _P, _P, _P, _F, _P, _P, _P, _F, _P, _P, _I, _I, _P, _I, _P, _Z,
                           _Z, _P, _I, _P],
-    "tff_input_conv_chunk": [],
-    "tff_input_conv": [_P, _P, _I, _P, _Z, _Z, _P, _I, _P, _P, _P, _I, _I, _P],
-    "tff_lightning": [_P, _Z, _P, _P, _Z, _P, _P, _P, _I, _I, _I, _I, _I, _P],
+    "tff_input_conv": [_P, _P, _I, _P, _Z, _Z, _P, _I, _I, _P, _P, _P, _I, _I, _P],
+    "tff_lightning": [_P, _Z, _P, _P, _Z, _P, _P, _P, _I, _I, _I, _I, _P],
+    "tff_lightning_chunk": [],
+    "tff_lightning_chunks": [_P, _Z, _P, _P, _Z, _P, _P, _I, _P, _P, _P, _P, _I, _I, _I, _I, _P],
     "tff_row_norm_gate": [_P, _P, _Z, _P, _F, _P, _I, _I, _I, _P],
     "tff_grouped_qkv_store": [_P, _Z, _P, _I, _I, _I, _F, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _I, _I, _P],
     "tff_pool_keys": [_P, _P, _P, _I, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P],

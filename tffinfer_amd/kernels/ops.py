@@ -1561,6 +1561,25 @@ def _vec(t, n: int, what: str):
     return t
 
 
+#: tokens an item of the convolution over time holds: short runs, so that a prompt's channels fill the GPU
+CONV_CHUNK = 8
+
+
+def _token_items(batch, chunk: int, device):
+    """The step's entries cut into items of up to ``chunk`` tokens: (int32 [items, 2] of (row of the step's tables, first
+    place in the entry's portion), int32 [rows + 1]: a row's first item), made once a step."""
+    cache = getattr(batch, "_token_items", None)
+    if cache is None:
+        cache = batch._token_items = {}
+    if chunk not in cache:
+        cu = batch.host_cu_tokens
+        counts = [-(-(cu[r + 1] - cu[r]) // chunk) for r in range(len(cu) - 1)]
+        flat = [(r, i * chunk) for r, n in enumerate(counts) for i in range(n)]
+        cache[chunk] = _staging.send(device, [np.asarray(flat, dtype=np.int32).reshape(-1, 2),
+                                              np.cumsum([0] + counts).astype(np.int32)])
+    return cache[chunk]
+
+
 def add_layernorm(resid: torch.Tensor | None, delta, weight, bias, eps: float, out_dtype: torch.dtype,
                   rows: torch.Tensor | None = None, conv=None, batch=None) -> torch.Tensor:
     """``resid += delta`` (None, an :class:`OutputTerm` or anything else a sublayer may return; not added when
@@ -1614,21 +1633,25 @@ def add_layernorm(resid: torch.Tensor | None, delta, weight, bias, eps: float, o
         _ptr(cw) if one else None, taps, st, st_row, off, slots, dtype_code(out.dtype), _stream()))
     if not split:
         return out
-    items = getattr(batch, "_conv_items", None)
-    if items is None:
-        cu, chunk = batch.host_cu_tokens, L.tff_input_conv_chunk()
-        flat = [(r, i) for r in range(len(cu) - 1) for i in range(0, cu[r + 1] - cu[r], chunk)]
-        items = batch._conv_items = _staging.send(dev, [np.asarray(flat, dtype=np.int32).reshape(-1, 2)])[0]
+    chunk = CONV_CHUNK if taps - 1 <= CONV_CHUNK else 32
+    items, _ = _token_items(batch, chunk, dev)
     y = torch.empty(n, W, dtype=out_dtype, device=dev)
-    _lib.check(L.tff_input_conv(out.data_ptr(), cw.data_ptr(), taps, st, st_row, off, items.data_ptr(), items.shape[0],
+    _lib.check(L.tff_input_conv(out.data_ptr(), cw.data_ptr(), taps, st, st_row, off, items.data_ptr(), items.shape[0], chunk,
                                 batch.cu_tokens.data_ptr(), slots, y.data_ptr(), W, dtype_code(out_dtype), _stream()))
     return y
 
 
-def lightning(proj: torch.Tensor, decay: torch.Tensor, state: torch.Tensor, batch, H: int, D: int, E: int) -> torch.Tensor:
+#: tokens of a step's longest entry from which the recurrence runs in chunks on the matrix cores
+LIGHTNING_LONG_PORTION = 12
+
+
+def lightning(proj: torch.Tensor, decay: torch.Tensor, state: torch.Tensor, batch, H: int, D: int, E: int,
+              chunked: bool | None = None) -> torch.Tensor:
     """The recurrence S <- decay_h S + k v^T, o = S^T q over each request's tokens of this step, per head; q [H, D],
     k [H, D], v [H, E] are silu of the columns of ``proj`` (float32 [T, >= H (2 D + E)], rows may be strided);
-    S lies transposed, [H][E][D], at the start of the request's row of ``state``.  Returns o float32 [T, H E]."""
+    S lies transposed, [H][E][D], at the start of the request's row of ``state``.  Returns o float32 [T, H E].
+    ``chunked``: in chunks of 64 tokens instead of token by token (None: by the step's longest entry; the decays must
+    not be negative then)."""
     T = proj.shape[0]
     ldp = _rows2(proj, "lightning proj", torch.float32, H * (2 * D + E))
     _req(decay, "lightning decay", torch.float32, 1)
@@ -1637,10 +1660,21 @@ def lightning(proj: torch.Tensor, decay: torch.Tensor, state: torch.Tensor, batc
         raise _lib.KernelError(f"lightning: {decay.numel()} decays, state rows of {row}, {T} rows for {H} heads of {D} x {E} "
                                f"and a step of {batch.num_tokens} tokens")
     o = torch.empty(T, H * E, dtype=torch.float32, device=proj.device)
-    if T:
-        _lib.check(_lib.load().tff_lightning(proj.data_ptr(), ldp, decay.data_ptr(), state.data_ptr(), row,
-                                             batch.cu_tokens.data_ptr(), batch.state_slots.data_ptr(), o.data_ptr(),
-                                             batch.num_reqs, H, D, E, int(getattr(batch, "max_new_tokens", 0) or 0), _stream()))
+    if T == 0:
+        return o
+    L = _lib.load()
+    if chunked is None:
+        chunked = batch.max_new_tokens >= LIGHTNING_LONG_PORTION
+    if chunked:
+        items, start = _token_items(batch, L.tff_lightning_chunk(), proj.device)
+        sums = torch.empty(items.shape[0], H, E, D, dtype=torch.float32, device=proj.device)
+        _lib.check(L.tff_lightning_chunks(proj.data_ptr(), ldp, decay.data_ptr(), state.data_ptr(), row, items.data_ptr(),
+                                          start.data_ptr(), items.shape[0], batch.cu_tokens.data_ptr(),
+                                          batch.state_slots.data_ptr(), sums.data_ptr(), o.data_ptr(), batch.num_reqs, H, D, E,
+                                          _stream()))
+        return o
+    _lib.check(L.tff_lightning(proj.data_ptr(), ldp, decay.data_ptr(), state.data_ptr(), row, batch.cu_tokens.data_ptr(),
+                               batch.state_slots.data_ptr(), o.data_ptr(), batch.num_reqs, H, D, E, _stream()))
     return o
 
 

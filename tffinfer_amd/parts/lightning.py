@@ -66,7 +66,7 @@ class LightningMixer(Mixer):
     def forward_projected(self, ctx, proj):
         ops = ctx.ops
         H, D, E = self.num_heads, self.head_dim, self.value_dim
-        o = ops.lightning(proj, self.decay, ctx.state, ctx.batch, H, D, E)
+        o = ops.lightning(proj, self.decay, ctx.state, ctx.batch, H, D, E, chunked=False if min(self.decay_list) < 0 else None)
         gate = proj[:, H * (2 * D + E):self.columns]
         y = ops.row_norm_gate(o, gate, self.norm, self.norm_eps, ctx.act_dtype)
         return ops.linear(y, self.w_o, out_dtype=torch.float32, partials=True)
