@@ -476,6 +476,33 @@ def test_batches_of_unequal_requests_share_a_window_with_blocks():
     assert cache.groups[0].pool.num_used == 0
 
 
+@pytest.mark.parametrize("dtype,limit", [(torch.float32, 3e-5), (torch.bfloat16, 3e-2)])
+def test_long_contexts_decode_beside_a_portion(dtype, limit):
+    """Requests of 300 to 900 tokens that decode beside another's portion get the kernel that splits keys among waves,
+    those of the blocks before the window among them."""
+    from tffinfer_amd.cache import CacheManager
+    W, page = 40, 16
+    att, m, P = _attention(W, 8, 2, 64, 64, 0.04, (70, 4), (64, 1000.0), dtype, 41)
+    lengths = {"a": 901, "b": 302, "c": 90}
+    xs = {r: _rand(n, W, seed=n).to(BF).float() for r, n in lengths.items()}
+    refs = {r: plain.window_attention(m, P, x.double(), plain.attention_cache(m, P, x.double())) for r, x in xs.items()}
+    cache = CacheManager([(0, True, att.cache_spec(), None)], page, 90, 3, dtype=dtype, device=DEV)
+    plan = [[("a", 899), ("b", 300)], [("a", 1), ("b", 1), ("c", 80)], [("b", 1), ("c", 9)], [("a", 1), ("c", 1)]]
+    at = dict.fromkeys("abc", 0)
+    for parts, batch in zip(plan, _steps(cache, plan)):
+        ctx = _ctx(batch, dtype)
+        ctx.kv = _view(cache, batch, 0)
+        rows = torch.cat([xs[r][at[r]:at[r] + n] for r, n in parts]).to(dtype).to(DEV)
+        out = _ops().as_tensor(att.forward(ctx, rows))
+        assert _err(out, torch.cat([refs[r][at[r]:at[r] + n] for r, n in parts])) < limit, parts
+        for r, n in parts:
+            at[r] += n
+    # the blocks matter: without them the last rows are others
+    bare = dict(m, mask={"size": 70, "pool": 0})
+    lost = plain.window_attention(bare, P, xs["a"].double(), plain.attention_cache(bare, P, xs["a"].double()))
+    assert _err(lost[-1], refs["a"][-1]) > 0.1
+
+
 # ---------------------------------------------------------------------- whole models ---
 
 def requests_for(name, model_dir):

@@ -100,7 +100,8 @@ TFF_API int tff_grouped_qkv_store(const float* proj, size_t row, const float* co
     return tff_check_launch("grouped_qkv_store");
 }
 
-// Blocks (token, kv head).  The sum runs over the block's tokens in their order; a thread takes elements tid, tid + 128, ...
+// Blocks (token, kv head); the tokens are those that `tokens` lists, or all of the step's, of which those that end no
+// block leave at once.  The sum runs over the block's tokens in their order; a thread takes elements tid, tid + 128, ...
 // Where the tokens' keys and values lie is worked out by the threads side by side, PK_RUN tokens at a time.
 #define PK_THREADS 128
 #define PK_RUN 64
@@ -111,10 +112,11 @@ __global__ __launch_bounds__(PK_THREADS) void pool_keys_kernel(TC* __restrict__ 
                                                                const int32_t* __restrict__ pool_tables, int pt_stride,
                                                                const int32_t* __restrict__ token_req,
                                                                const int32_t* __restrict__ positions,
-                                                               const int32_t* __restrict__ slots, int page_size, int pool, int G,
+                                                               const int32_t* __restrict__ slots,
+                                                               const int32_t* __restrict__ tokens, int page_size, int pool, int G,
                                                                int d) {
     __shared__ size_t koff[PK_RUN], voff[PK_RUN];
-    const int t = blockIdx.x, g = blockIdx.y, tid = threadIdx.x;
+    const int t = tokens ? tokens[blockIdx.x] : (int)blockIdx.x, g = blockIdx.y, tid = threadIdx.x;
     const int pos = positions[t];
     if (slots[t] < 0 || (pos + 1) % pool) return;      // (the whole block)
     const int r = token_req[t], blk = pos / pool, first = pos + 1 - pool;
@@ -149,8 +151,8 @@ __global__ __launch_bounds__(PK_THREADS) void pool_keys_kernel(TC* __restrict__ 
 }
 
 TFF_API int tff_pool_keys(void* k_cache, void* v_cache, const int32_t* block_tables, int bt_stride, const int32_t* pool_tables,
-                          int pt_stride, const int32_t* token_req, const int32_t* positions, const int32_t* slots, int page_size,
-                          int num_pages, int pool, int T, int G, int d, int dtype, tff_stream_t stream) {
+                          int pt_stride, const int32_t* token_req, const int32_t* positions, const int32_t* slots,
+                          const int32_t* tokens, int page_size, int num_pages, int pool, int T, int G, int d, int dtype, tff_stream_t stream) {
     TFF_REQUIRE(k_cache && v_cache && block_tables && pool_tables && token_req && positions && slots, "pool_keys: null pointer");
     TFF_REQUIRE(T >= 0 && G > 0 && G <= 65535 && d > 0 && pool > 0 && page_size > 0 && num_pages > 0 && bt_stride > 0 && pt_stride > 0,
                 "pool_keys: bad sizes");
@@ -159,10 +161,10 @@ TFF_API int tff_pool_keys(void* k_cache, void* v_cache, const int32_t* block_tab
     const dim3 grid(T, G);
     if (dtype == TFF_F32)
         pool_keys_kernel<float><<<grid, PK_THREADS, 0, s>>>((float*)k_cache, (float*)v_cache, block_tables, bt_stride, pool_tables, pt_stride,
-                                                            token_req, positions, slots, page_size, pool, G, d);
+                                                            token_req, positions, slots, tokens, page_size, pool, G, d);
     else if (dtype == TFF_BF16)
         pool_keys_kernel<bf16_t><<<grid, PK_THREADS, 0, s>>>((bf16_t*)k_cache, (bf16_t*)v_cache, block_tables, bt_stride, pool_tables,
-                                                             pt_stride, token_req, positions, slots, page_size, pool, G, d);
+                                                             pt_stride, token_req, positions, slots, tokens, page_size, pool, G, d);
     else
         return tff_fail("pool_keys: unknown dtype %d", dtype);
     return tff_check_launch("pool_keys");

@@ -15,7 +15,8 @@
 #include "common.h"
 #include "tffinfer_kernels.h"
 
-__device__ __forceinline__ float lt_silu(float z) { return z / (1.0f + expf(-z)); }
+// (the hardware's exponential and reciprocal: a few units in the last place of float32)
+__device__ __forceinline__ float lt_silu(float z) { return z * __builtin_amdgcn_rcpf(1.0f + __expf(-z)); }
 
 // Block: sixteen value channels of one head of one request; a row of sixteen lanes shares a value channel, lane s
 // holding the key channels s, s + 16, ...  No LDS and no barrier: for steps of a few tokens a request.
@@ -31,21 +32,33 @@ __global__ __launch_bounds__(256) void lightning_few_kernel(const float* __restr
     const bool live = j < E;
     const float g = decay[h];
     float* sp = state + (size_t)state_slots[r] * state_row + ((size_t)h * E + jc) * D + s;
-    float S[KPL];
-#pragma unroll
-    for (int m = 0; m < KPL; ++m) S[m] = (live && s + 16 * m < D) ? sp[16 * m] : 0.f;
-    for (int t = 0; t < n; ++t) {
-        const float* p = proj + (size_t)(t0 + t) * ldp;
-        const float* pq = p + (size_t)h * D + s;
-        const float* pk = pq + (size_t)H * D;
-        float kk[KPL], qq[KPL];
+    if (n <= 0) return;
+    // a token's projections are asked for while the token before is worked on, the first one's with the state
+    float S[KPL], qn[KPL], kn[KPL], vn;
+    const float* p = proj + (size_t)t0 * ldp;
+    const size_t oq = (size_t)h * D + s, ok = oq + (size_t)H * D, ov = 2 * (size_t)H * D + (size_t)h * E + jc;
+    auto ask = [&](const float* row) {
 #pragma unroll
         for (int m = 0; m < KPL; ++m) {
             const bool in = s + 16 * m < D;
-            qq[m] = in ? lt_silu(pq[16 * m]) : 0.f;
-            kk[m] = in ? lt_silu(pk[16 * m]) : 0.f;
+            qn[m] = in ? row[oq + 16 * m] : 0.f;
+            kn[m] = in ? row[ok + 16 * m] : 0.f;
         }
-        const float v = lt_silu(p[2 * (size_t)H * D + (size_t)h * E + jc]);
+        vn = row[ov];
+    };
+    ask(p);
+#pragma unroll
+    for (int m = 0; m < KPL; ++m) S[m] = (live && s + 16 * m < D) ? sp[16 * m] : 0.f;
+    for (int t = 0; t < n; ++t) {
+        float kk[KPL], qq[KPL];
+#pragma unroll
+        for (int m = 0; m < KPL; ++m) {
+            qq[m] = lt_silu(qn[m]);         // (silu(0) = 0)
+            kk[m] = lt_silu(kn[m]);
+        }
+        const float v = lt_silu(vn);
+        p += ldp;
+        if (t + 1 < n) ask(p);
         float a = 0.f;
 #pragma unroll
         for (int m = 0; m < KPL; ++m) {

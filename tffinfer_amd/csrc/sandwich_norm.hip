@@ -78,12 +78,44 @@ __device__ __forceinline__ void sn_store(TO* p, const float (&v)[VEC]) {
     }
 }
 
+// What a thread needs of the vectors as long as a row (weights, biases, the convolution's taps and state).  With few
+// elements a thread (EARLY) everything is asked for at the start, so that a step of few rows, which nothing else
+// hides, waits for memory once; with many it is fetched where it is used.
+#define SN_EARLY_TAPS 4
+
+template <int IT, int VEC, bool EARLY>
+struct SandwichVector {
+    float v[EARLY ? IT : 1][VEC];
+    const float* p;
+    __device__ __forceinline__ void ask(const float* src, int W, int tid, int nt) {
+        p = src;
+        if constexpr (EARLY) {
+#pragma unroll
+            for (int it = 0; it < IT; ++it) {
+#pragma unroll
+                for (int u = 0; u < VEC; ++u) v[it][u] = 0.f;
+                const int e = (it * nt + tid) * VEC;
+                if (src && e < W) sn_load<VEC>(v[it], src + e);
+            }
+        }
+    }
+    __device__ __forceinline__ void take(float (&out)[VEC], int it, int e) const {
+        if constexpr (EARLY) {
+#pragma unroll
+            for (int u = 0; u < VEC; ++u) out[u] = v[it][u];
+        } else {
+            sn_load<VEC>(out, p + e);
+        }
+    }
+};
+
 template <typename TO, int NT, int VPT, int VEC>
 __global__ __launch_bounds__(NT) void add_layernorm_kernel(float* __restrict__ resid, const SandwichTerm tm,
                                                            const float* __restrict__ w, const float* __restrict__ b, float eps,
                                                            TO* __restrict__ out, const int32_t* __restrict__ rows, int W,
                                                            const SandwichConv cv) {
     constexpr int IT = VPT / VEC;
+    constexpr bool EARLY = VPT <= 4;
     __shared__ float red[6][NT / 64];
     const int i = blockIdx.x, tid = threadIdx.x;
     const size_t row = rows ? (size_t)rows[i] : (size_t)i;
@@ -92,6 +124,7 @@ __global__ __launch_bounds__(NT) void add_layernorm_kernel(float* __restrict__ r
     float* const xr = resid ? resid + at : nullptr;
     const float* const ar = tm.a ? tm.a + at : nullptr;
     const float* const br = tm.b ? tm.b + at : nullptr;
+    const int slot = cv.w ? cv.slots[i] : 0;
     float x[IT][VEC], d[IT][VEC], p2[IT][VEC];
 #pragma unroll
     for (int it = 0; it < IT; ++it) {
@@ -100,34 +133,65 @@ __global__ __launch_bounds__(NT) void add_layernorm_kernel(float* __restrict__ r
         for (int u = 0; u < VEC; ++u) x[it][u] = d[it][u] = p2[it][u] = 0.f;
         if (e < W) {
             if (xr) sn_load<VEC>(x[it], xr + e);
-            if (tm.a) {
-                sn_load<VEC>(d[it], ar + e);
-                for (int p = 1; p < tm.planes_a; ++p) {
-                    float t[VEC];
-                    sn_load<VEC>(t, ar + p * tm.plane_a + e);
+            if (ar) sn_load<VEC>(d[it], ar + e);
+            if (br) sn_load<VEC>(p2[it], br + e);
+        }
+    }
+    SandwichVector<IT, VEC, EARLY> vbias, vwa, vwb, vnw, vnb, vsc, vw, vb;
+    vbias.ask(tm.bias, W, tid, NT);
+    vwa.ask(tm.wa, W, tid, NT);
+    vwb.ask(tm.wb, W, tid, NT);
+    vnw.ask(tm.nw, W, tid, NT);
+    vnb.ask(tm.nb, W, tid, NT);
+    vsc.ask(tm.scale, W, tid, NT);
+    vw.ask(w, W, tid, NT);
+    vb.ask(b, W, tid, NT);
+    float* const st = cv.w && cv.taps > 1 ? cv.state + (size_t)slot * cv.state_row + cv.off : nullptr;
+    float cw[EARLY ? SN_EARLY_TAPS : 1][EARLY ? IT : 1][VEC], cs[EARLY ? SN_EARLY_TAPS : 1][EARLY ? IT : 1][VEC];
+    const bool early_conv = EARLY && cv.w && cv.taps <= SN_EARLY_TAPS;
+    if constexpr (EARLY) {
+        if (early_conv) {
 #pragma unroll
-                    for (int u = 0; u < VEC; ++u) d[it][u] += t[u];
-                }
-                if (tm.bias) {
-                    float t[VEC];
-                    sn_load<VEC>(t, tm.bias + e);
+            for (int j = 0; j < SN_EARLY_TAPS; ++j)
 #pragma unroll
-                    for (int u = 0; u < VEC; ++u) d[it][u] += t[u];
+                for (int it = 0; it < IT; ++it) {
+                    const int e = (it * NT + tid) * VEC;
+#pragma unroll
+                    for (int u = 0; u < VEC; ++u) cw[j][it][u] = cs[j][it][u] = 0.f;
+                    if (j < cv.taps && e < W) {
+                        sn_load<VEC>(cw[j][it], cv.w + (size_t)j * W + e);
+                        if (j < cv.taps - 1) {
+#pragma unroll
+                            for (int u = 0; u < VEC; ++u) cs[j][it][u] = st[(size_t)j * W + e + u];
+                        }
+                    }
                 }
+        }
+    }
+#pragma unroll
+    for (int it = 0; it < IT; ++it) {
+        const int e = (it * NT + tid) * VEC;
+        if (e < W) {
+            float t[VEC];
+            for (int p = 1; p < tm.planes_a; ++p) {
+                sn_load<VEC>(t, ar + p * tm.plane_a + e);
+#pragma unroll
+                for (int u = 0; u < VEC; ++u) d[it][u] += t[u];
             }
-            if (tm.b) {
-                sn_load<VEC>(p2[it], br + e);
-                for (int p = 1; p < tm.planes_b; ++p) {
-                    float t[VEC];
-                    sn_load<VEC>(t, br + p * tm.plane_b + e);
+            for (int p = 1; p < tm.planes_b; ++p) {
+                sn_load<VEC>(t, br + p * tm.plane_b + e);
 #pragma unroll
-                    for (int u = 0; u < VEC; ++u) p2[it][u] += t[u];
-                }
+                for (int u = 0; u < VEC; ++u) p2[it][u] += t[u];
+            }
+            if (tm.bias) {
+                vbias.take(t, it, e);
+#pragma unroll
+                for (int u = 0; u < VEC; ++u) d[it][u] += t[u];
             }
         }
     }
     // v <- (v - mean) / sqrt(variance + eps) * lw + lb, elements past the row left at what they are
-    auto layernorm = [&](float (&v)[IT][VEC], const float* lw, const float* lb, float le, float* r0, float* r1) {
+    auto layernorm = [&](float (&v)[IT][VEC], const auto& lw, const auto& lb, float le, float* r0, float* r1) {
         float s = 0.f;
 #pragma unroll
         for (int it = 0; it < IT; ++it)
@@ -149,14 +213,14 @@ __global__ __launch_bounds__(NT) void add_layernorm_kernel(float* __restrict__ r
             const int e = (it * NT + tid) * VEC;
             if (e < W) {
                 float a[VEC], c[VEC];
-                sn_load<VEC>(a, lw + e);
-                sn_load<VEC>(c, lb + e);
+                lw.take(a, it, e);
+                lb.take(c, it, e);
 #pragma unroll
                 for (int u = 0; u < VEC; ++u) v[it][u] = fmaf(v[it][u] * rr, a[u], c[u]);
             }
         }
     };
-    if (tm.b) {
+    if (br) {
         float s0 = 0.f, s1 = 0.f;
 #pragma unroll
         for (int it = 0; it < IT; ++it)
@@ -178,22 +242,22 @@ __global__ __launch_bounds__(NT) void add_layernorm_kernel(float* __restrict__ r
             const int e = (it * NT + tid) * VEC;
             if (e < W) {
                 float a[VEC], c[VEC];
-                sn_load<VEC>(a, tm.wa + e);
-                sn_load<VEC>(c, tm.wb + e);
+                vwa.take(a, it, e);
+                vwb.take(c, it, e);
 #pragma unroll
                 for (int u = 0; u < VEC; ++u) d[it][u] = d[it][u] * fa * a[u] + p2[it][u] * fb * c[u];
             }
         }
     }
-    if (tm.a) {
-        if (tm.nw) layernorm(d, tm.nw, tm.nb, tm.n_eps, red[0], red[1]);
+    if (ar) {
+        if (tm.nw) layernorm(d, vnw, vnb, tm.n_eps, red[0], red[1]);
 #pragma unroll
         for (int it = 0; it < IT; ++it) {
             const int e = (it * NT + tid) * VEC;
             if (e < W) {
                 if (tm.scale) {
                     float c[VEC];
-                    sn_load<VEC>(c, tm.scale + e);
+                    vsc.take(c, it, e);
 #pragma unroll
                     for (int u = 0; u < VEC; ++u) d[it][u] *= c[u];
                 }
@@ -203,32 +267,47 @@ __global__ __launch_bounds__(NT) void add_layernorm_kernel(float* __restrict__ r
             }
         }
     }
-    if (w) layernorm(x, w, b, eps, red[2], red[3]);
+    if (w) layernorm(x, vw, vb, eps, red[2], red[3]);
     if (cv.w) {
-        float* st = cv.state + (size_t)cv.slots[i] * cv.state_row + cv.off;
 #pragma unroll
         for (int it = 0; it < IT; ++it) {
             const int e = (it * NT + tid) * VEC;
             if (e < W) {
-                float y[VEC], c[VEC];
+                float y[VEC];
 #pragma unroll
                 for (int u = 0; u < VEC; ++u) y[u] = 0.f;
-                for (int j = 0; j < cv.taps - 1; ++j) {
-                    sn_load<VEC>(c, cv.w + (size_t)j * W + e);
+                bool done = false;
+                if constexpr (EARLY) {
+                    if (early_conv) {
+                        done = true;
 #pragma unroll
-                    for (int u = 0; u < VEC; ++u) {
-                        const float s = st[(size_t)j * W + e + u];
-                        y[u] = fmaf(c[u], s, y[u]);
-                        if (j > 0) st[(size_t)(j - 1) * W + e + u] = s;
+                        for (int j = 0; j < SN_EARLY_TAPS; ++j) {
+                            const bool last = j == cv.taps - 1;
+                            if (j < cv.taps) {
+#pragma unroll
+                                for (int u = 0; u < VEC; ++u) {
+                                    y[u] = fmaf(cw[j][it][u], last ? x[it][u] : cs[j][it][u], y[u]);
+                                    if (j > 0) st[(size_t)(j - 1) * W + e + u] = last ? x[it][u] : cs[j][it][u];
+                                }
+                            }
+                        }
                     }
                 }
-                sn_load<VEC>(c, cv.w + (size_t)(cv.taps - 1) * W + e);
+                if (!done) {
+                    for (int j = 0; j < cv.taps; ++j) {
+                        float c[VEC];
+                        sn_load<VEC>(c, cv.w + (size_t)j * W + e);
+                        const bool last = j == cv.taps - 1;
 #pragma unroll
-                for (int u = 0; u < VEC; ++u) {
-                    if (cv.taps > 1) st[(size_t)(cv.taps - 2) * W + e + u] = x[it][u];
-                    y[u] = fmaf(c[u], x[it][u], y[u]);
-                    x[it][u] += y[u];
+                        for (int u = 0; u < VEC; ++u) {
+                            const float h = last ? x[it][u] : st[(size_t)j * W + e + u];
+                            y[u] = fmaf(c[u], h, y[u]);
+                            if (j > 0) st[(size_t)(j - 1) * W + e + u] = h;
+                        }
+                    }
                 }
+#pragma unroll
+                for (int u = 0; u < VEC; ++u) x[it][u] += y[u];
             }
         }
     }

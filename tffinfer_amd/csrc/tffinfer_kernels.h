@@ -452,9 +452,10 @@ TFF_API int tff_grouped_qkv_store(const float* proj, size_t row, const float* co
                                   float temp_coef, int temp_every, const int32_t* positions, const int32_t* slots, void* q_out,
                                   void* k_cache, void* v_cache, int page_size, int num_pages, int T, int H, int G, int D, int E,
                                   int P, int store, int dtype, tff_stream_t stream);
+// tokens [T] (may be null: tokens 0 .. T - 1): the step's tokens to look at; those that end no block are left out.
 TFF_API int tff_pool_keys(void* k_cache, void* v_cache, const int32_t* block_tables, int bt_stride, const int32_t* pool_tables,
-                          int pt_stride, const int32_t* token_req, const int32_t* positions, const int32_t* slots, int page_size,
-                          int num_pages, int pool, int T, int G, int d, int dtype, tff_stream_t stream);
+                          int pt_stride, const int32_t* token_req, const int32_t* positions, const int32_t* slots,
+                          const int32_t* tokens, int page_size, int num_pages, int pool, int T, int G, int d, int dtype, tff_stream_t stream);
 TFF_API int tff_gate_heads(const void* o, size_t o_row, int P, const float* g, size_t g_row, void* out, int T, int H, int E,
                            int dtype, tff_stream_t stream);
 

@@ -94,7 +94,7 @@ _SIGNATURES = {
     "tff_lightning_chunks": [_P, _Z, _P, _P, _Z, _P, _P, _I, _P, _P, _P, _P, _I, _I, _I, _I, _P],
     "tff_row_norm_gate": [_P, _P, _Z, _P, _F, _P, _I, _I, _I, _P],
     "tff_grouped_qkv_store": [_P, _Z, _P, _I, _I, _I, _F, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _I, _I, _P],
-    "tff_pool_keys": [_P, _P, _P, _I, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P],
+    "tff_pool_keys": [_P, _P, _P, _I, _P, _I, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P],
     "tff_gate_heads": [_P, _Z, _I, _P, _Z, _P, _I, _I, _I, _I, _P],
     "tff_probe_stream_read": [_P, _Z, _P, _I, _P],
     "tff_probe_mfma": [_P, _I, _I, _I, _P],

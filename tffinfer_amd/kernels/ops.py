@@ -1739,9 +1739,22 @@ def pool_keys(kv, batch, pool: int) -> None:
     T = batch.num_tokens
     if pt.shape[0] != bt.shape[0] or min(batch.token_req.numel(), batch.positions.numel(), kv.slot_mapping.numel()) < T:
         raise _lib.KernelError("pool_keys: the step's tables do not describe the same requests and tokens")
+    tokens = None
+    if batch.max_new_tokens > 1:        # (the host knows which tokens end a block; a captured step looks at every row)
+        cache = getattr(batch, "_block_ends", None)
+        if cache is None:
+            cache = batch._block_ends = {}
+        if pool not in cache:
+            cu, start = batch.host_cu_tokens, batch.host_start_pos
+            flat = [t for r in range(len(cu) - 1) for t in range(cu[r] + (-start[r] - 1) % pool, cu[r + 1], pool)]
+            cache[pool] = _staging.send(k_cache.device, [np.asarray(flat, dtype=np.int32)])[0] if flat else None
+        tokens = cache[pool]
+        if tokens is None:
+            return
+        T = tokens.numel()
     _lib.check(_lib.load().tff_pool_keys(
         k_cache.data_ptr(), v_cache.data_ptr(), bt.data_ptr(), bt.stride(0), pt.data_ptr(), pt.stride(0), batch.token_req.data_ptr(),
-        batch.positions.data_ptr(), kv.slot_mapping.data_ptr(), ps, pages, int(pool), T, G, d, dtype_code(k_cache.dtype), _stream()))
+        batch.positions.data_ptr(), kv.slot_mapping.data_ptr(), _ptr(tokens), ps, pages, int(pool), T, G, d, dtype_code(k_cache.dtype), _stream()))
 
 
 def gate_heads(o: torch.Tensor, P: int, gate: torch.Tensor | None, H: int, E: int) -> torch.Tensor:
