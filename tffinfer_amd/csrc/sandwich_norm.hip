@@ -10,8 +10,9 @@
 //   h from the request's state row, which moves on by one
 // Every part is optional: without a term the stream is only normed; with `rows` the norm of those rows leaves
 // and resid stays as it is; without resid out is y itself.
-// A layer norm's variance is the mean of the squared deviations from the mean (two sums, not the difference of
-// moments).  Everything is float32; one block a row, the row in registers, a reduction costs one barrier.
+// A layer norm takes two passes over its row's registers: the mean first, then the squares of what is left after
+// subtracting it (no difference of moments).  Everything is float32; one block a row, the row in registers, a
+// reduction costs one barrier.
 //
 // tff_input_conv: the same convolution for portions of any length: out = h + conv(h) over each request's tokens of
 // the step, inputs before the portion from the state, the last taps - 1 inputs left there.

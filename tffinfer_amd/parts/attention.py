@@ -342,8 +342,8 @@ class GroupedAttention(Mixer):
 
     What position i sees: every j <= i; with a ``window`` the j with i - j < window; and with a ``pool`` P
     beside them one key and one value per block of P tokens that lies wholly before the window: the means
-    of the block's keys and values as the cache holds them.  Tokens that left the window and whose block
-    is not seen yet are not seen at all; tokens and blocks share one softmax.
+    of the block's keys and values as the cache holds them.  Between the two may lie tokens that neither
+    covers (a block that reaches into the window does not count).  The softmax runs over the union.
 
     ``shared_cache``: the layer has no Wk and Wv; it reads the cache that another layer call fills (the run
     order names it), with its own queries, window, pool and everything else.  ``cache_window`` and

@@ -222,8 +222,8 @@ class ParallelBlock(Block):
 class SandwichBlock(Block):
     """x <- x + s1 * norm1_out(mixer(c1(norm1(x))));  x <- x + s2 * norm2_out(ffn(c2(norm2(x)))): a norm before and
     after each sublayer.  ``layer_scale``: s1 and s2 are vectors (``ls1``, ``ls2``; else 1).  ``conv_taps`` K > 0:
-    c(h)_t = h_t + sum_j w[:, j] h_(t - K + 1 + j), a causal convolution over time on each channel added to
-    its input (``canon1``, ``canon2`` [hidden, K]; zeros before a request's start); the last K - 1 rows h of
+    c(h)_t = h_t + sum_j w[:, j] h_(t - K + 1 + j), every channel filtered along its own past and added to
+    itself (``canon1``, ``canon2`` [hidden, K]; zeros before a request's start); the last K - 1 rows h of
     both sublayers are the block's state.  A sublayer's result stays pending, with its norm and its scale, for
     the norm before the next sublayer, whose kernel does everything from there to that sublayer's input.  A
     layer without a feed-forward has no second half (its tensors may be left out)."""
