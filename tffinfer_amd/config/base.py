@@ -49,12 +49,15 @@ class LayerCall:
     (``ModelConfig.stream_offset_rows``) is added to the stream before the call.
     ``state`` >= 0: the state this call works on, where it is not the one of the
     cache's number (a call that borrows keys and values and has a state of its own).
+    ``add_embedding``: the embedding's output (the stream as it was before the first call) is added to
+    the stream before the call.
     """
     layer: int
     cache: int
     writes_cache: bool = True
     offset: int = -1
     state: int = -1
+    add_embedding: bool = False
 
 
 class ModelConfig:
@@ -98,6 +101,11 @@ class ModelConfig:
 
     def embedding_norm_spec(self) -> PartSpec | None:
         """A norm right after the embedding, or None."""
+        return None
+
+    def bigram_spec(self) -> dict | None:
+        """A table of rows for pairs of neighbouring tokens beside the embedding's (``parts.BigramTable``: buckets,
+        mul_prev, mul_cur), or None."""
         return None
 
     def stream_offset_rows(self) -> int:

@@ -11,6 +11,16 @@ enum { TFF_F32 = 0, TFF_BF16 = 1 };
 
 #define TFF_WAVE 64
 
+// How a gated feed-forward joins its two projections: silu(g) u (plain), or with constants
+// a sigmoid(alpha a) (b + up_offset), a = min(g, limit), b = clamp(u, -limit, limit).
+struct GluAct {
+    int plain;
+    float limit, alpha, up_offset;
+};
+static inline GluAct glu_act(float limit, float alpha, float up_offset) {
+    return GluAct{limit == __builtin_inff() && alpha == 1.0f && up_offset == 0.0f ? 1 : 0, limit, alpha, up_offset};
+}
+
 __device__ __forceinline__ float to_f32(float v) { return v; }
 __device__ __forceinline__ float to_f32(bf16_t v) { return (float)v; }
 template <typename T> __device__ __forceinline__ T from_f32(float v);

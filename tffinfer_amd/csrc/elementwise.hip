@@ -23,7 +23,7 @@ int tff_check_launch(const char* what) {
     return 0;
 }
 TFF_API const char* tff_last_error() { return g_error; }
-TFF_API int tff_abi_version() { return 35; }
+TFF_API int tff_abi_version() { return 36; }
 
 // ----------------------------------------------------------------- embed ---
 // x[t, :] = E[token[t], :]   (reference: src/kernel/cpu/embedding.cpp:34-49,
@@ -610,30 +610,39 @@ TFF_API int tff_qk_norm_rope_kv(void* qkv, int T, int nq, int nkv, int d, const 
 
 // ---------------------------------------------------------------- swiglu ---
 // m = silu(g) * u, silu(x) = x / (1 + exp(-x))  (reference:
-// src/kernel/cuda/unary.cu:10-27, x1 = gate, x2 = up).
+// src/kernel/cuda/unary.cu:10-27, x1 = gate, x2 = up); or the form with constants (GluAct).
 template <typename T>
-__global__ void swiglu_kernel(const T* __restrict__ gu, const float* __restrict__ bias, T* __restrict__ out, int64_t total, int I) {
+__global__ void swiglu_kernel(const T* __restrict__ gu, const float* __restrict__ bias, T* __restrict__ out, int64_t total, int I,
+                              GluAct act) {
     const int64_t idx = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (idx >= total) return;
     const int64_t t = idx / I;
     const int i = (int)(idx - t * I);
-    const float g = to_f32(gu[t * 2 * I + i]) + (bias ? bias[i] : 0.f);
-    const float u = to_f32(gu[t * 2 * I + I + i]) + (bias ? bias[I + i] : 0.f);
-    out[idx] = from_f32<T>(g / (1.0f + expf(-g)) * u);
+    float g = to_f32(gu[t * 2 * I + i]) + (bias ? bias[i] : 0.f);
+    float u = to_f32(gu[t * 2 * I + I + i]) + (bias ? bias[I + i] : 0.f);
+    if (act.plain) {
+        out[idx] = from_f32<T>(g / (1.0f + expf(-g)) * u);
+    } else {
+        g = fminf(g, act.limit);
+        u = fminf(fmaxf(u, -act.limit), act.limit);
+        out[idx] = from_f32<T>(g / (1.0f + expf(-act.alpha * g)) * (u + act.up_offset));
+    }
 }
 
-TFF_API int tff_swiglu(const void* gu, const float* bias, void* out, int T, int I, int dtype, tff_stream_t stream) {
+TFF_API int tff_swiglu(const void* gu, const float* bias, void* out, int T, int I, float limit, float alpha, float up_offset, int dtype,
+                       tff_stream_t stream) {
     TFF_REQUIRE(gu && out, "swiglu: null pointer");
     TFF_REQUIRE(T >= 0 && I > 0, "swiglu: bad sizes T=%d I=%d", T, I);
     if (T == 0) return 0;
+    const GluAct act = glu_act(limit, alpha, up_offset);
     const int64_t total = (int64_t)T * I;
     const int64_t blocks = (total + 255) / 256;
     TFF_REQUIRE(blocks < 2147483647LL, "swiglu: too many elements");
     hipStream_t s = (hipStream_t)stream;
     if (dtype == TFF_F32)
-        swiglu_kernel<float><<<(unsigned)blocks, 256, 0, s>>>((const float*)gu, bias, (float*)out, total, I);
+        swiglu_kernel<float><<<(unsigned)blocks, 256, 0, s>>>((const float*)gu, bias, (float*)out, total, I, act);
     else if (dtype == TFF_BF16)
-        swiglu_kernel<bf16_t><<<(unsigned)blocks, 256, 0, s>>>((const bf16_t*)gu, bias, (bf16_t*)out, total, I);
+        swiglu_kernel<bf16_t><<<(unsigned)blocks, 256, 0, s>>>((const bf16_t*)gu, bias, (bf16_t*)out, total, I, act);
     else
         return tff_fail("swiglu: unknown dtype %d", dtype);
     return tff_check_launch("swiglu");

@@ -40,12 +40,28 @@ __device__ __forceinline__ void store4(TC* dst, const floatx4& v, int n, int N, 
     }
 }
 
+// What a product takes besides its operands: a bias (float32, in the order of W's rows, ceil16(N) numbers) or null,
+// and how a gated product joins gate and up.
+struct GemmExtra {
+    const float* bias;
+    GluAct act;
+};
+
 // GLU: the 16-row groups of W alternate between a gate and an up projection
-// (group 2p gate, group 2p+1 up); the epilogue writes silu(gate) * up, N / 2 columns.
-__device__ __forceinline__ floatx4 silu_mul(const floatx4& g, const floatx4& u) {
+// (group 2p gate, group 2p+1 up); the epilogue writes act(gate, up), N / 2 columns: silu(gate) * up, or in the form
+// with constants g sigmoid(alpha g) (u + up_offset), g = min(gate, limit), u = clamp(up, -limit, limit).
+__device__ __forceinline__ floatx4 glu4(const floatx4& g, const floatx4& u, const GluAct& act) {
     floatx4 o;
+    if (act.plain) {
 #pragma unroll
-    for (int e = 0; e < 4; ++e) o[e] = g[e] / (1.0f + __expf(-g[e])) * u[e];
+        for (int e = 0; e < 4; ++e) o[e] = g[e] / (1.0f + __expf(-g[e])) * u[e];
+    } else {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            const float a = fminf(g[e], act.limit), b = fminf(fmaxf(u[e], -act.limit), act.limit);
+            o[e] = a / (1.0f + __expf(-act.alpha * a)) * (b + act.up_offset);
+        }
+    }
     return o;
 }
 
@@ -75,7 +91,8 @@ constexpr int vmcnt_imm(int v) { return (v & 15) | (7 << 4) | (15 << 8) | ((v >>
 template <int WGM, int WGN, int WTM, int WTN, int STAGES, bool GLU, typename TC, int KPS = 2, bool EARLY = false>
 __global__ __launch_bounds__(64 * WGM * WGN) void gemm_bf16_async_kernel(
     const bf16_t* __restrict__ A, const bf16_t* __restrict__ Wp, TC* __restrict__ C, int M, int N,
-    int K, int lda, int KB, int n_out, float* __restrict__ part, const float* __restrict__ bias) {
+    int K, int lda, int KB, int n_out, float* __restrict__ part, const GemmExtra ex) {
+    const float* __restrict__ const bias = ex.bias;
     // WGM x WGN waves, each WTM x WTN MFMA tiles of 16 x 16
     constexpr int NW = WGM * WGN;
     constexpr int BM = WGM * WTM * 16, BN = WGN * WTN * 16;
@@ -250,7 +267,7 @@ __global__ __launch_bounds__(64 * WGM * WGN) void gemm_bf16_async_kernel(
             for (int j = 0; j < WTM; ++j) {
                 const int m = m0 + (wm * WTM + j) * 16 + fr;
                 if (m < M && n < n_out)
-                    store4<TC>(C + (size_t)m * n_out + n, silu_mul(acc[i][j], acc[i + 1][j]), n, n_out, vec);
+                    store4<TC>(C + (size_t)m * n_out + n, glu4(acc[i][j], acc[i + 1][j], ex.act), n, n_out, vec);
             }
         }
     } else {
@@ -273,7 +290,7 @@ __global__ __launch_bounds__(64 * WGM * WGN) void gemm_bf16_async_kernel(
 template <bool GLU, typename TC>
 __global__ __launch_bounds__(256) void gemm_splitk_reduce_kernel(const float* __restrict__ part, int S,
                                                                   int M, int N, TC* __restrict__ C,
-                                                                  int n_out) {
+                                                                  int n_out, GluAct act) {
     const int per_row = (n_out + 3) / 4;
     const long idx = (long)blockIdx.x * blockDim.x + threadIdx.x;
     if (idx >= (long)M * per_row) return;
@@ -289,7 +306,7 @@ __global__ __launch_bounds__(256) void gemm_splitk_reduce_kernel(const float* __
             a[0] += g.x; a[1] += g.y; a[2] += g.z; a[3] += g.w;
             b[0] += u.x; b[1] += u.y; b[2] += u.z; b[3] += u.w;
         }
-        a = silu_mul(a, b);
+        a = glu4(a, b, act);
     } else {
         const float* p = part + (size_t)m * N + j;
         const bool vec = (N % 4) == 0;
@@ -310,7 +327,7 @@ __global__ __launch_bounds__(256) void gemm_splitk_reduce_kernel(const float* __
 // splits > 1: the blocks of a tile split K among them; part holds splits * M * N floats
 template <int WGM, int WGN, int WTM, int WTN, int STAGES, bool GLU = false, int KPS = 2, bool EARLY = false>
 static int launch_async_g(const bf16_t* A, const bf16_t* Wp, void* C, int M, int N, int K, int lda,
-                          const float* bias, int c_dtype, int n_out, hipStream_t s, int splits = 1, float* part = nullptr,
+                          const GemmExtra ex, int c_dtype, int n_out, hipStream_t s, int splits = 1, float* part = nullptr,
                           bool reduce = true) {
     const int KB = (K + 31) / 32;
     constexpr int BM = WGM * WTM * 16, BN = WGN * WTN * 16;
@@ -321,19 +338,19 @@ static int launch_async_g(const bf16_t* A, const bf16_t* Wp, void* C, int M, int
     const dim3 grid((unsigned)tiles, 1, splits);
     if (c_dtype == TFF_F32)
         gemm_bf16_async_kernel<WGM, WGN, WTM, WTN, STAGES, GLU, float, KPS, EARLY>
-            <<<grid, 64 * WGM * WGN, 0, s>>>(A, Wp, (float*)C, M, N, K, lda, KB, n_out, part, bias);
+            <<<grid, 64 * WGM * WGN, 0, s>>>(A, Wp, (float*)C, M, N, K, lda, KB, n_out, part, ex);
     else
         gemm_bf16_async_kernel<WGM, WGN, WTM, WTN, STAGES, GLU, bf16_t, KPS, EARLY>
-            <<<grid, 64 * WGM * WGN, 0, s>>>(A, Wp, (bf16_t*)C, M, N, K, lda, KB, n_out, part, bias);
+            <<<grid, 64 * WGM * WGN, 0, s>>>(A, Wp, (bf16_t*)C, M, N, K, lda, KB, n_out, part, ex);
     if (int rc = tff_check_launch("gemm_bf16_async")) return rc;
     if (splits > 1 && reduce) {
         const int No = GLU ? n_out : N;
         const long threads = (long)M * ((No + 3) / 4);
         const int blocks = (int)((threads + 255) / 256);
         if (c_dtype == TFF_F32)
-            gemm_splitk_reduce_kernel<GLU, float><<<blocks, 256, 0, s>>>(part, splits, M, N, (float*)C, No);
+            gemm_splitk_reduce_kernel<GLU, float><<<blocks, 256, 0, s>>>(part, splits, M, N, (float*)C, No, ex.act);
         else
-            gemm_splitk_reduce_kernel<GLU, bf16_t><<<blocks, 256, 0, s>>>(part, splits, M, N, (bf16_t*)C, No);
+            gemm_splitk_reduce_kernel<GLU, bf16_t><<<blocks, 256, 0, s>>>(part, splits, M, N, (bf16_t*)C, No, ex.act);
         return tff_check_launch("gemm_splitk_reduce");
     }
     return 0;
@@ -460,7 +477,8 @@ struct W4Scale {
 template <int WTN, int NWS, bool GLU, typename TC, int WGM = 2, bool SCALE = false, int WTM = 8>
 __global__ __launch_bounds__(256) void gemm_bf16_w4_kernel(
     const bf16_t* __restrict__ A, const bf16_t* __restrict__ Wp, TC* __restrict__ C, int M, int N,
-    int K, int lda, int KB, int n_out, W4Scale sc, const float* __restrict__ bias) {
+    int K, int lda, int KB, int n_out, W4Scale sc, const GemmExtra ex) {
+    const float* __restrict__ const bias = ex.bias;
     static_assert(!SCALE || WGM == 1, "rows that lack their norm's factor: up to 16, one row tile");
     // WGM: waves along the rows, 2 (a block tile of 256 rows, two waves side by side) or 1 (128 rows, four side by side)
     // WTM: row groups of 16 a wave, 8, or with the waves side by side 4 or 2 (a block tile of 64 or 32 rows)
@@ -680,7 +698,7 @@ __global__ __launch_bounds__(256) void gemm_bf16_w4_kernel(
     };
     if constexpr (GLU) {
         static_assert(WTN % 2 == 0, "gate and up groups come in pairs");
-        w4_store_rows<WTN / 2, REGION, TC, WTM>(region, [&](int i, int jj) { return silu_mul(scaled(acc[2 * i][jj]), scaled(acc[2 * i + 1][jj])); },
+        w4_store_rows<WTN / 2, REGION, TC, WTM>(region, [&](int i, int jj) { return glu4(scaled(acc[2 * i][jj]), scaled(acc[2 * i + 1][jj]), ex.act); },
                                            C, (size_t)n_out, mw, (n0 + wn * WTN * 16) / 2, M, n_out, lane_out,
                                            n_out % E == 0);
     } else {
@@ -693,7 +711,7 @@ __global__ __launch_bounds__(256) void gemm_bf16_w4_kernel(
 
 // splits > 1: the blocks of a tile split K among them in units of 64; part holds splits * M * N floats
 template <int WTN, int NWS, bool GLU = false, int WGM = 2, bool SCALE = false, int WTM = 8>
-static int launch_w4(const bf16_t* A, const bf16_t* Wp, void* C, int M, int N, int K, int lda, const float* bias, int c_dtype,
+static int launch_w4(const bf16_t* A, const bf16_t* Wp, void* C, int M, int N, int K, int lda, const GemmExtra ex, int c_dtype,
                      int n_out, hipStream_t s, int splits = 1, float* part = nullptr, bool reduce = true,
                      W4Scale sc = W4Scale{nullptr, 0, 0, 0.f, 0.f}) {
     TFF_REQUIRE(!SCALE || (M <= 16 && sc.ss && (splits <= 1 || !part)),
@@ -710,20 +728,20 @@ static int launch_w4(const bf16_t* A, const bf16_t* Wp, void* C, int M, int N, i
     const dim3 grid((unsigned)tiles, 1, splits);
     // the blocks of a split K leave plain float32 sums, plane by plane; a gate is applied when they are added up
     if (splits > 1)
-        gemm_bf16_w4_kernel<WTN, NWS, false, float, WGM, false, WTM><<<grid, 256, 0, s>>>(A, Wp, part, M, N, K, lda, KB, 0, sc, bias);
+        gemm_bf16_w4_kernel<WTN, NWS, false, float, WGM, false, WTM><<<grid, 256, 0, s>>>(A, Wp, part, M, N, K, lda, KB, 0, sc, ex);
     else if (c_dtype == TFF_F32)
-        gemm_bf16_w4_kernel<WTN, NWS, GLU, float, WGM, SCALE, WTM><<<grid, 256, 0, s>>>(A, Wp, (float*)C, M, N, K, lda, KB, n_out, sc, bias);
+        gemm_bf16_w4_kernel<WTN, NWS, GLU, float, WGM, SCALE, WTM><<<grid, 256, 0, s>>>(A, Wp, (float*)C, M, N, K, lda, KB, n_out, sc, ex);
     else
-        gemm_bf16_w4_kernel<WTN, NWS, GLU, bf16_t, WGM, SCALE, WTM><<<grid, 256, 0, s>>>(A, Wp, (bf16_t*)C, M, N, K, lda, KB, n_out, sc, bias);
+        gemm_bf16_w4_kernel<WTN, NWS, GLU, bf16_t, WGM, SCALE, WTM><<<grid, 256, 0, s>>>(A, Wp, (bf16_t*)C, M, N, K, lda, KB, n_out, sc, ex);
     if (int rc = tff_check_launch("gemm_bf16_w4")) return rc;
     if (splits > 1 && reduce) {
         const int No = GLU ? n_out : N;
         const long threads = (long)M * ((No + 3) / 4);
         const int blocks = (int)((threads + 255) / 256);
         if (c_dtype == TFF_F32)
-            gemm_splitk_reduce_kernel<GLU, float><<<blocks, 256, 0, s>>>(part, splits, M, N, (float*)C, No);
+            gemm_splitk_reduce_kernel<GLU, float><<<blocks, 256, 0, s>>>(part, splits, M, N, (float*)C, No, ex.act);
         else
-            gemm_splitk_reduce_kernel<GLU, bf16_t><<<blocks, 256, 0, s>>>(part, splits, M, N, (bf16_t*)C, No);
+            gemm_splitk_reduce_kernel<GLU, bf16_t><<<blocks, 256, 0, s>>>(part, splits, M, N, (bf16_t*)C, No, ex.act);
         return tff_check_launch("gemm_splitk_reduce");
     }
     return 0;
@@ -776,7 +794,8 @@ struct SkinnyFuse {
 template <int MT, int R, int UNROLL, int KSPLIT, int NSETS, bool GLU, typename TC, bool RING = false, int EPI = 0>
 __global__ __launch_bounds__(64 * KSPLIT * NSETS) void gemm_bf16_skinny_kernel(
     const bf16_t* __restrict__ A, const bf16_t* __restrict__ Wp, TC* __restrict__ C, int M, int N,
-    int K, int lda, int KB, int n_out, SkinnyFuse fz, const float* __restrict__ bias) {
+    int K, int lda, int KB, int n_out, SkinnyFuse fz, const GemmExtra ex) {
+    const float* __restrict__ const bias = ex.bias;
     static_assert(EPI == 0 || MT == 1, "the fused norm is for up to 16 rows");
     static_assert(EPI < 2 || !GLU, "the product before a norm has a plain float32 result");
     constexpr int SK_WAVES = KSPLIT * NSETS;
@@ -976,7 +995,7 @@ __global__ __launch_bounds__(64 * KSPLIT * NSETS) void gemm_bf16_skinny_kernel(
                     }
                     const int n = (nb0 >> 1) * 16 + fg * 4;
                     const int m = t * 16 + fr;
-                    if (m < M && n < n_out) store4<TC>(C + (size_t)m * n_out + n, silu_mul(g, u), n, n_out, vec);
+                    if (m < M && n < n_out) store4<TC>(C + (size_t)m * n_out + n, glu4(g, u, ex.act), n, n_out, vec);
                 }
             }
         } else {
@@ -1036,17 +1055,17 @@ __global__ __launch_bounds__(64 * KSPLIT * NSETS) void gemm_bf16_skinny_kernel(
 
 template <int MT, int R, int UNROLL, int KSPLIT, int NSETS = 1, bool GLU = false, bool RING = false, int EPI = 0>
 static int launch_skinny(const bf16_t* A, const bf16_t* Wp, void* C, int M, int N, int K, int lda,
-                         const float* bias, int c_dtype, int n_out, hipStream_t s, const SkinnyFuse* fuse = nullptr) {
+                         const GemmExtra ex, int c_dtype, int n_out, hipStream_t s, const SkinnyFuse* fuse = nullptr) {
     const int NB = (N + 15) / 16, KB = (K + 31) / 32;
     const int per_block = NSETS * R;
     const dim3 grid((NB + per_block - 1) / per_block);
     const SkinnyFuse fz = fuse ? *fuse : SkinnyFuse{nullptr, 0, 0, 0.f, 0.f, nullptr, nullptr, nullptr, nullptr, 0, nullptr, 0.f};
     if (c_dtype == TFF_F32)
         gemm_bf16_skinny_kernel<MT, R, UNROLL, KSPLIT, NSETS, GLU, float, RING, EPI>
-            <<<grid, 64 * KSPLIT * NSETS, 0, s>>>(A, Wp, (float*)C, M, N, K, lda, KB, n_out, fz, bias);
+            <<<grid, 64 * KSPLIT * NSETS, 0, s>>>(A, Wp, (float*)C, M, N, K, lda, KB, n_out, fz, ex);
     else if constexpr (EPI < 2)
         gemm_bf16_skinny_kernel<MT, R, UNROLL, KSPLIT, NSETS, GLU, bf16_t, RING, EPI>
-            <<<grid, 64 * KSPLIT * NSETS, 0, s>>>(A, Wp, (bf16_t*)C, M, N, K, lda, KB, n_out, fz, bias);
+            <<<grid, 64 * KSPLIT * NSETS, 0, s>>>(A, Wp, (bf16_t*)C, M, N, K, lda, KB, n_out, fz, ex);
     else
         return tff_fail("gemm: the product before a norm has a float32 result");
     return tff_check_launch("gemm_bf16_skinny");
@@ -1232,19 +1251,19 @@ TFF_API int tff_gemm_plan(int M, int N, int K, int glu, int keep_partials, int* 
 // a group's whole K through a ring (384 such waves, at N = 6,144, are too few: 3 % slower).  Plain: more waves per block where there are few blocks
 // (small N) or long rows (large K), fewer and deeper ones in between.
 template <int EPI>
-static int skinny_for(const bf16_t* A, const bf16_t* Wp, void* C, int M, int N, int K, int lda, const float* bias, int c_dtype,
+static int skinny_for(const bf16_t* A, const bf16_t* Wp, void* C, int M, int N, int K, int lda, const GemmExtra ex, int c_dtype,
                       int glu_out, hipStream_t s, const SkinnyFuse* fuse) {
     if (glu_out > 0) {
         if constexpr (EPI < 2) {
             if (N >= 8 * 1024)
-                return launch_skinny<1, 1, 8, 1, 2, true, true, EPI>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, fuse);
+                return launch_skinny<1, 1, 8, 1, 2, true, true, EPI>(A, Wp, C, M, N, K, lda, ex, c_dtype, glu_out, s, fuse);
             // A wave takes a quarter of K in groups of k-steps whose loads are issued together, and
             // the steps that are left when a group is not full go one at a time: groups of eight
             // where a quarter of K is fewer than 32 steps, of 32 (with the norm's factor taken in,
             // which needs registers of its own, 24) otherwise.
             if (K < 4096)
-                return launch_skinny<1, 1, 8, 4, 2, true, false, EPI>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, fuse);
-            return launch_skinny<1, 1, (EPI == 1 ? 24 : 32), 4, 2, true, false, EPI>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, fuse);
+                return launch_skinny<1, 1, 8, 4, 2, true, false, EPI>(A, Wp, C, M, N, K, lda, ex, c_dtype, glu_out, s, fuse);
+            return launch_skinny<1, 1, (EPI == 1 ? 24 : 32), 4, 2, true, false, EPI>(A, Wp, C, M, N, K, lda, ex, c_dtype, glu_out, s, fuse);
         } else {
             return tff_fail("gemm: a gated product does not come before a norm");
         }
@@ -1258,7 +1277,7 @@ static int skinny_for(const bf16_t* A, const bf16_t* Wp, void* C, int M, int N, 
     // 39.8 against 42.9 / 42.8 at 1 / 8 rows (at 16 rows the tiles are ahead, see plan_for).  Not for
     // the product after a norm: the row factors' registers do not fit beside two row groups.
     if constexpr (EPI != 1) {
-        if (two_row_groups(N)) return launch_skinny<1, 2, 4, 16, 1, false, false, EPI>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, fuse);
+        if (two_row_groups(N)) return launch_skinny<1, 2, 4, 16, 1, false, false, EPI>(A, Wp, C, M, N, K, lda, ex, c_dtype, 0, s, fuse);
     }
     // A very wide product (an output head) has thousands of blocks, each of which fetches all of A's
     // rows: with many rows and a long K that traffic shows (152k columns, K = 4,096: 196 / 217 / 281 us
@@ -1266,14 +1285,14 @@ static int skinny_for(const bf16_t* A, const bf16_t* Wp, void* C, int M, int N, 
     // 8 / 16 rows 264 / 303 us against 278 / 366; with fewer rows one group a block stays ahead.
     if constexpr (EPI == 0) {
         if (N >= 32 * 1024 && (long)M * K >= 40000)
-            return launch_skinny<1, 2, 4, 8, 1, false, false, 0>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, fuse);
+            return launch_skinny<1, 2, 4, 8, 1, false, false, 0>(A, Wp, C, M, N, K, lda, ex, c_dtype, 0, s, fuse);
     }
     // (K up to 1,024: sixteen waves would have two k-steps each, less than a group of four)
     if (N >= 32 * 1024 || K <= 1024)
-        return launch_skinny<1, 1, 4, 8, 1, false, false, EPI>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, fuse);
+        return launch_skinny<1, 1, 4, 8, 1, false, false, EPI>(A, Wp, C, M, N, K, lda, ex, c_dtype, 0, s, fuse);
     if (K >= 8192 || N <= 4096)
-        return launch_skinny<1, 1, 4, 16, 1, false, false, EPI>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, fuse);
-    return launch_skinny<1, 1, 8, 4, 1, false, false, EPI>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, fuse);
+        return launch_skinny<1, 1, 4, 16, 1, false, false, EPI>(A, Wp, C, M, N, K, lda, ex, c_dtype, 0, s, fuse);
+    return launch_skinny<1, 1, 8, 4, 1, false, false, EPI>(A, Wp, C, M, N, K, lda, ex, c_dtype, 0, s, fuse);
 }
 
 // glu_out > 0: W holds gate and up groups in turn (N = 2 * ceil16(glu_out) rows) and C is
@@ -1284,7 +1303,7 @@ static int skinny_for(const bf16_t* A, const bf16_t* Wp, void* C, int M, int N, 
 // keep_partials: where the plan splits K, the partial sums stay in the workspace
 // ([splits, M, N] float32) for the caller to add up, and C is not written.
 int tff_gemm_bf16(const bf16_t* A, const bf16_t* Wp, void* C, int M, int N, int K, int lda,
-                  const float* bias, int c_dtype, int glu_out, float* workspace, size_t workspace_bytes,
+                  const GemmExtra ex, int c_dtype, int glu_out, float* workspace, size_t workspace_bytes,
                   int keep_partials, hipStream_t s) {
     TFF_REQUIRE(K % 8 == 0 && lda % 8 == 0,
                 "gemm: the bfloat16 product needs the inner size (K=%d, row stride %d) to be a multiple of 8",
@@ -1302,64 +1321,64 @@ int tff_gemm_bf16(const bf16_t* A, const bf16_t* Wp, void* C, int M, int N, int 
     if (glu_out > 0) {
         TFF_REQUIRE(N % 32 == 0 && glu_out <= N / 2 && glu_out > N / 2 - 16,
                     "gemm: a gated weight of %d rows does not fit %d output columns", N, glu_out);
-        if (plan.tile == 0) return skinny_for<0>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, nullptr);
+        if (plan.tile == 0) return skinny_for<0>(A, Wp, C, M, N, K, lda, ex, c_dtype, glu_out, s, nullptr);
         if (plan.tile <= 64 && K % 64 == 0) {                // the four waves side by side on 64 or 32 rows
-            if (plan.tile == 32 && plan.bn == 128) return launch_w4<2, 5, true, 1, false, 2>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, S, workspace);
-            if (plan.tile == 32) return launch_w4<4, 5, true, 1, false, 2>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, S, workspace);
-            if (plan.bn == 128) return launch_w4<2, 5, true, 1, false, 4>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, S, workspace);
-            return launch_w4<4, 5, true, 1, false, 4>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, S, workspace);
+            if (plan.tile == 32 && plan.bn == 128) return launch_w4<2, 5, true, 1, false, 2>(A, Wp, C, M, N, K, lda, ex, c_dtype, glu_out, s, S, workspace);
+            if (plan.tile == 32) return launch_w4<4, 5, true, 1, false, 2>(A, Wp, C, M, N, K, lda, ex, c_dtype, glu_out, s, S, workspace);
+            if (plan.bn == 128) return launch_w4<2, 5, true, 1, false, 4>(A, Wp, C, M, N, K, lda, ex, c_dtype, glu_out, s, S, workspace);
+            return launch_w4<4, 5, true, 1, false, 4>(A, Wp, C, M, N, K, lda, ex, c_dtype, glu_out, s, S, workspace);
         }
         if (plan.tile == 64)
-            return launch_async_g<2, 2, 2, 4, 3, true>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, S, workspace);
+            return launch_async_g<2, 2, 2, 4, 3, true>(A, Wp, C, M, N, K, lda, ex, c_dtype, glu_out, s, S, workspace);
         if (K % 64 == 0) {
             if (plan.tile == 128) {
-                if (plan.bn == 128) return launch_w4<2, 5, true, 1>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, S, workspace);
-                if (plan.bn == 256) return launch_w4<4, 5, true, 1>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, S, workspace);
-                return launch_w4<6, 4, true, 1>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, S, workspace);
+                if (plan.bn == 128) return launch_w4<2, 5, true, 1>(A, Wp, C, M, N, K, lda, ex, c_dtype, glu_out, s, S, workspace);
+                if (plan.bn == 256) return launch_w4<4, 5, true, 1>(A, Wp, C, M, N, K, lda, ex, c_dtype, glu_out, s, S, workspace);
+                return launch_w4<6, 4, true, 1>(A, Wp, C, M, N, K, lda, ex, c_dtype, glu_out, s, S, workspace);
             }
-            if (plan.bn == 128) return launch_w4<4, 5, true>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, S, workspace);
-            if (plan.bn == 192) return launch_w4<6, 5, true>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, S, workspace);
-            return launch_w4<8, 4, true>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, S, workspace);
+            if (plan.bn == 128) return launch_w4<4, 5, true>(A, Wp, C, M, N, K, lda, ex, c_dtype, glu_out, s, S, workspace);
+            if (plan.bn == 192) return launch_w4<6, 5, true>(A, Wp, C, M, N, K, lda, ex, c_dtype, glu_out, s, S, workspace);
+            return launch_w4<8, 4, true>(A, Wp, C, M, N, K, lda, ex, c_dtype, glu_out, s, S, workspace);
         }
         if (plan.tile == 128 && plan.bn == 128)
-            return launch_async_g<2, 2, 4, 4, 3, true>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, S, workspace);
+            return launch_async_g<2, 2, 4, 4, 3, true>(A, Wp, C, M, N, K, lda, ex, c_dtype, glu_out, s, S, workspace);
         if (plan.tile == 128)
-            return launch_async_g<2, 4, 4, 4, 3, true>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, S, workspace);
-        return launch_async_g<4, 4, 4, 4, 5, true, 1, true>(A, Wp, C, M, N, K, lda, bias, c_dtype, glu_out, s, S, workspace);
+            return launch_async_g<2, 4, 4, 4, 3, true>(A, Wp, C, M, N, K, lda, ex, c_dtype, glu_out, s, S, workspace);
+        return launch_async_g<4, 4, 4, 4, 5, true, 1, true>(A, Wp, C, M, N, K, lda, ex, c_dtype, glu_out, s, S, workspace);
     }
-    if (plan.tile == 0) return skinny_for<0>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, nullptr);
+    if (plan.tile == 0) return skinny_for<0>(A, Wp, C, M, N, K, lda, ex, c_dtype, 0, s, nullptr);
     if (plan.tile == 64 || plan.tile == 32) {
         // few columns and no room for partial sums: the streaming kernel, whose blocks split K
         // among their waves
         if (S == 1 && planned_splits > 1 && M <= 64) {
-            if (M <= 32) return launch_skinny<2, 2, 4, 8>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s);
-            return launch_skinny<4, 2, 4, 8>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s);
+            if (M <= 32) return launch_skinny<2, 2, 4, 8>(A, Wp, C, M, N, K, lda, ex, c_dtype, 0, s);
+            return launch_skinny<4, 2, 4, 8>(A, Wp, C, M, N, K, lda, ex, c_dtype, 0, s);
         }
         if (K % 64 == 0) {                                   // the four waves side by side on 64 or 32 rows
-            if (plan.tile == 32 && plan.bn == 128) return launch_w4<2, 5, false, 1, false, 2>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, S, workspace, red);
-            if (plan.tile == 32) return launch_w4<4, 5, false, 1, false, 2>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, S, workspace, red);
-            if (plan.bn == 128) return launch_w4<2, 5, false, 1, false, 4>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, S, workspace, red);
-            return launch_w4<4, 5, false, 1, false, 4>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, S, workspace, red);
+            if (plan.tile == 32 && plan.bn == 128) return launch_w4<2, 5, false, 1, false, 2>(A, Wp, C, M, N, K, lda, ex, c_dtype, 0, s, S, workspace, red);
+            if (plan.tile == 32) return launch_w4<4, 5, false, 1, false, 2>(A, Wp, C, M, N, K, lda, ex, c_dtype, 0, s, S, workspace, red);
+            if (plan.bn == 128) return launch_w4<2, 5, false, 1, false, 4>(A, Wp, C, M, N, K, lda, ex, c_dtype, 0, s, S, workspace, red);
+            return launch_w4<4, 5, false, 1, false, 4>(A, Wp, C, M, N, K, lda, ex, c_dtype, 0, s, S, workspace, red);
         }
-        return launch_async_g<2, 2, 2, 4, 3>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, S, workspace, red);
+        return launch_async_g<2, 2, 2, 4, 3>(A, Wp, C, M, N, K, lda, ex, c_dtype, 0, s, S, workspace, red);
     }
     if (K % 64 == 0) {
         if (plan.tile == 128) {
-            if (plan.bn == 128) return launch_w4<2, 5, false, 1>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, S, workspace, red);
-            if (plan.bn == 256) return launch_w4<4, 5, false, 1>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, S, workspace, red);
-            return launch_w4<6, 4, false, 1>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, S, workspace, red);
+            if (plan.bn == 128) return launch_w4<2, 5, false, 1>(A, Wp, C, M, N, K, lda, ex, c_dtype, 0, s, S, workspace, red);
+            if (plan.bn == 256) return launch_w4<4, 5, false, 1>(A, Wp, C, M, N, K, lda, ex, c_dtype, 0, s, S, workspace, red);
+            return launch_w4<6, 4, false, 1>(A, Wp, C, M, N, K, lda, ex, c_dtype, 0, s, S, workspace, red);
         }
-        if (plan.bn == 128) return launch_w4<4, 5>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, S, workspace, red);
-        if (plan.bn == 192) return launch_w4<6, 5>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, S, workspace, red);
-        return launch_w4<8, 4>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, S, workspace, red);
+        if (plan.bn == 128) return launch_w4<4, 5>(A, Wp, C, M, N, K, lda, ex, c_dtype, 0, s, S, workspace, red);
+        if (plan.bn == 192) return launch_w4<6, 5>(A, Wp, C, M, N, K, lda, ex, c_dtype, 0, s, S, workspace, red);
+        return launch_w4<8, 4>(A, Wp, C, M, N, K, lda, ex, c_dtype, 0, s, S, workspace, red);
     }
     if (plan.tile == 128 && plan.bn == 128)
-        return launch_async_g<2, 2, 4, 4, 3>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, S, workspace, red);
+        return launch_async_g<2, 2, 4, 4, 3>(A, Wp, C, M, N, K, lda, ex, c_dtype, 0, s, S, workspace, red);
     if (plan.tile == 128)
-        return launch_async_g<2, 4, 4, 4, 3>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, S, workspace, red);
+        return launch_async_g<2, 4, 4, 4, 3>(A, Wp, C, M, N, K, lda, ex, c_dtype, 0, s, S, workspace, red);
     if (plan.bn == 192)
-        return launch_async_g<4, 4, 4, 3, 5, false, 1, true>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, S, workspace, red);
-    return launch_async_g<4, 4, 4, 4, 5, false, 1, true>(A, Wp, C, M, N, K, lda, bias, c_dtype, 0, s, S, workspace, red);
+        return launch_async_g<4, 4, 4, 3, 5, false, 1, true>(A, Wp, C, M, N, K, lda, ex, c_dtype, 0, s, S, workspace, red);
+    return launch_async_g<4, 4, 4, 4, 5, false, 1, true>(A, Wp, C, M, N, K, lda, ex, c_dtype, 0, s, S, workspace, red);
 }
 
 // ---- the norm between two products of up to 16 rows, taken into them ----
@@ -1386,7 +1405,7 @@ TFF_API int tff_gemm_residual_prenorm(const void* A, const void* Wp, int M, int 
     TFF_REQUIRE(((uintptr_t)resid % 16) == 0 && ((uintptr_t)norm_w % 16) == 0 && ((uintptr_t)x_out % 8) == 0,
                 "gemm_residual_prenorm: operands must be 16-byte aligned");
     SkinnyFuse fz{nullptr, 0, 0, 0.f, 0.f, resid, norm_w, (bf16_t*)x_out, ss_out, ss_stride, nullptr, 0.f};
-    return skinny_for<2>((const bf16_t*)A, (const bf16_t*)Wp, resid, M, N, K, lda, nullptr, TFF_F32, 0, (hipStream_t)stream, &fz);
+    return skinny_for<2>((const bf16_t*)A, (const bf16_t*)Wp, resid, M, N, K, lda, GemmExtra{nullptr, glu_act(__builtin_inff(), 1.0f, 0.0f)}, TFF_F32, 0, (hipStream_t)stream, &fz);
 }
 
 // resid[M, N] += A . W^T (bfloat16 A and packed W, float32 sums); x_out[M, N] = bfloat16 of
@@ -1400,14 +1419,15 @@ TFF_API int tff_gemm_residual_dyt(const void* A, const void* Wp, int M, int N, i
     TFF_REQUIRE(((uintptr_t)resid % 16) == 0 && ((uintptr_t)norm_w % 16) == 0 && ((uintptr_t)bias % 16) == 0 &&
                 ((uintptr_t)x_out % 8) == 0, "gemm_residual_dyt: operands must be 16-byte aligned");
     SkinnyFuse fz{nullptr, 0, 0, 0.f, 0.f, resid, norm_w, (bf16_t*)x_out, nullptr, 0, bias, alpha};
-    return skinny_for<3>((const bf16_t*)A, (const bf16_t*)Wp, resid, M, N, K, lda, nullptr, TFF_F32, 0, (hipStream_t)stream, &fz);
+    return skinny_for<3>((const bf16_t*)A, (const bf16_t*)Wp, resid, M, N, K, lda, GemmExtra{nullptr, glu_act(__builtin_inff(), 1.0f, 0.0f)}, TFF_F32, 0, (hipStream_t)stream, &fz);
 }
 
 // C = rstd[m] * (A . W^T) with rstd[m] = rsqrt(sum_g ss[m][g] / dim + eps), g < ss_count: the product
 // after tff_gemm_residual_prenorm (A = its x_out, ss = its ss_out, dim = its N).  glu_out as in tff_gemm.
 TFF_API int tff_gemm_row_scaled(const void* A, const void* Wp, void* C, int M, int N, int K, int lda, int c_dtype,
                                 int glu_out, const float* ss, int ss_stride, int ss_count, int dim, float eps,
-                                tff_stream_t stream) {
+                                float glu_limit, float glu_alpha, float glu_up_offset, tff_stream_t stream) {
+    const GemmExtra ex{nullptr, glu_act(glu_limit, glu_alpha, glu_up_offset)};
     if (int rc = check_fused_operands("gemm_row_scaled", A, Wp, M, N, K, lda)) return rc;
     TFF_REQUIRE(C && ss && ((uintptr_t)C % 16) == 0 && ((uintptr_t)ss % 16) == 0, "gemm_row_scaled: null or unaligned pointer");
     TFF_REQUIRE(c_dtype == TFF_F32 || c_dtype == TFF_BF16, "gemm_row_scaled: unknown output type %d", c_dtype);
@@ -1424,19 +1444,20 @@ TFF_API int tff_gemm_row_scaled(const void* A, const void* Wp, void* C, int M, i
         const bf16_t* w = (const bf16_t*)Wp;
         hipStream_t s = (hipStream_t)stream;
         if (plan_rows32(N, K) == 128)
-            return launch_w4<2, 5, true, 1, true, 2>(a, w, C, M, N, K, lda, nullptr, c_dtype, glu_out, s, 1, nullptr, true, sc);
-        return launch_w4<4, 5, true, 1, true, 2>(a, w, C, M, N, K, lda, nullptr, c_dtype, glu_out, s, 1, nullptr, true, sc);
+            return launch_w4<2, 5, true, 1, true, 2>(a, w, C, M, N, K, lda, ex, c_dtype, glu_out, s, 1, nullptr, true, sc);
+        return launch_w4<4, 5, true, 1, true, 2>(a, w, C, M, N, K, lda, ex, c_dtype, glu_out, s, 1, nullptr, true, sc);
     }
     SkinnyFuse fz{ss, ss_stride, ss_count, 1.0f / (float)dim, eps, nullptr, nullptr, nullptr, nullptr, 0, nullptr, 0.f};
-    return skinny_for<1>((const bf16_t*)A, (const bf16_t*)Wp, C, M, N, K, lda, nullptr, c_dtype, glu_out, (hipStream_t)stream, &fz);
+    return skinny_for<1>((const bf16_t*)A, (const bf16_t*)Wp, C, M, N, K, lda, ex, c_dtype, glu_out, (hipStream_t)stream, &fz);
 }
 
 int tff_gemm_f32(const float* A, const float* W, void* C, int M, int N, int K, int lda,
                  int c_dtype, hipStream_t s);
 
 TFF_API int tff_gemm(const void* A, const void* W, void* C, int M, int N, int K, int lda,
-                     int ab_dtype, int c_dtype, int w_packed, int glu_out, const float* bias, void* workspace,
-                     size_t workspace_bytes, int keep_partials, tff_stream_t stream) {
+                     int ab_dtype, int c_dtype, int w_packed, int glu_out, const float* bias, float glu_limit,
+                     float glu_alpha, float glu_up_offset, void* workspace, size_t workspace_bytes, int keep_partials,
+                     tff_stream_t stream) {
     TFF_REQUIRE(A && W && C, "gemm: null pointer");
     TFF_REQUIRE(M >= 0 && N > 0 && K > 0 && lda >= K, "gemm: bad sizes M=%d N=%d K=%d lda=%d", M, N, K, lda);
     if (M == 0) return 0;
@@ -1450,7 +1471,8 @@ TFF_API int tff_gemm(const void* A, const void* W, void* C, int M, int N, int K,
         TFF_REQUIRE(w_packed, "gemm: the bfloat16 product takes a weight in fragment order");
         TFF_REQUIRE(((uintptr_t)workspace % 16) == 0, "gemm: the workspace must be 16-byte aligned");
         TFF_REQUIRE(((uintptr_t)bias % 16) == 0, "gemm: the bias must be 16-byte aligned");
-        return tff_gemm_bf16((const bf16_t*)A, (const bf16_t*)W, C, M, N, K, lda, bias, c_dtype, glu_out,
+        return tff_gemm_bf16((const bf16_t*)A, (const bf16_t*)W, C, M, N, K, lda,
+                             GemmExtra{bias, glu_act(glu_limit, glu_alpha, glu_up_offset)}, c_dtype, glu_out,
                              (float*)workspace, workspace ? workspace_bytes : 0, keep_partials, s);
     }
     return tff_fail("gemm: unknown operand type %d", ab_dtype);

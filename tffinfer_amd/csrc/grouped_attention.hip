@@ -1,11 +1,12 @@
 // What stands around the paged attention kernels in a grouped attention whose queries carry a temperature that grows
 // with the position and whose window has the mean keys of whole blocks of tokens before it.
 //
-// tff_grouped_qkv_store:  from the joint projection (float32): rotation of q and k, the temperature on q, q laid out
-//                         with the cache's head size, the token's key and value into its slot.
+// tff_grouped_qkv_store:  from the joint projection (float32): biases, an RMS norm over all of a token's q (and of its k)
+//                         at once, rotation of q and k, the temperature on q, q laid out with the cache's head size, the
+//                         token's key and value into its slot.
 // tff_pool_keys:          for every token of the step that ends a block of P tokens: the means of the block's P keys and
 //                         values, as the pages hold them, into the block's slot.
-// tff_gate_heads:         a head's output times one gate per head, heads brought together.
+// tff_gate_heads:         a head's output times one gate per head and a scale, heads brought together.
 #include "common.h"
 #include "tffinfer_kernels.h"
 
@@ -15,8 +16,10 @@ struct GroupedRot {
     int pairing;         // 0: (i, i + dims/2), 1: (2i, 2i+1)
 };
 
-__device__ __forceinline__ float grouped_rotated(const float* __restrict__ x, int e, const GroupedRot r) {
-    const float v = x[e];
+// Element e of a head whose elements are value(0), value(1), ...
+template <typename F>
+__device__ __forceinline__ float grouped_rotated(F value, int e, const GroupedRot r) {
+    const float v = value(e);
     if (!r.cs || e >= r.dims) return v;
     int i, other;
     bool first;
@@ -30,53 +33,95 @@ __device__ __forceinline__ float grouped_rotated(const float* __restrict__ x, in
         i = e >> 1;
         other = e ^ 1;
     }
-    const float o = x[other], c = r.cs[2 * i], s = r.cs[2 * i + 1];
+    const float o = value(other), c = r.cs[2 * i], s = r.cs[2 * i + 1];
     // the pair (u, w) becomes (u c - w s, w c + u s)
     return first ? fmaf(v, c, -(o * s)) : fmaf(v, c, o * s);
 }
 
+// What happens to the projections before rotation.
+struct GroupedPre {
+    const float* bias;                 // [H D + G D + G E] in the projection's column order, or null
+    const float *q_norm, *k_norm;      // [H D], [G D]: RMS norms over the whole of q and of k, or null
+    float eps;
+};
+
 // Blocks (token, y): y < q_blocks works through GQ_HEADS query heads; the others are one kv head each: its key row and
-// its value row into the token's slot.  Elements past a head's own size are zeros.
+// its value row into the token's slot.  Elements past a head's own size are zeros.  With a norm every block forms the
+// sum of squares it needs by itself, always in the same order.
 #define GQ_THREADS 128
 #define GQ_HEADS 8
+
+// 1 / sqrt(mean over x[0 .. n) of (x + bias)^2 + eps), the result in every thread of the block
+__device__ __forceinline__ float grouped_rms(const float* __restrict__ x, const float* __restrict__ bias, int n, float eps, float* red) {
+    float ss = 0.f;
+    for (int c = threadIdx.x; c < n; c += GQ_THREADS) {
+        const float v = x[c] + (bias ? bias[c] : 0.f);
+        ss = fmaf(v, v, ss);
+    }
+    ss = rows_sum(row16_sum(ss));
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = ss;
+    __syncthreads();
+    ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < GQ_THREADS / 64; ++i) ss += red[i];
+    return 1.0f / sqrtf(ss / (float)n + eps);
+}
 
 template <typename TC>
 __global__ __launch_bounds__(GQ_THREADS) void grouped_qkv_store_kernel(
     const float* __restrict__ proj, size_t row, const float* __restrict__ cos_sin, int rot_dims, int pairing, int max_pos,
-    float temp_coef, int temp_every, const int32_t* __restrict__ positions, const int32_t* __restrict__ slots,
+    float temp_coef, int temp_every, const GroupedPre pre, const int32_t* __restrict__ positions, const int32_t* __restrict__ slots,
     TC* __restrict__ q_out, TC* __restrict__ k_cache, TC* __restrict__ v_cache, int page_size, int H, int G, int D, int E, int P,
     int q_blocks) {
+    __shared__ float red[GQ_THREADS / 64];
     const int t = blockIdx.x, y = blockIdx.y, tid = threadIdx.x;
     const float* x = proj + (size_t)t * row;
     const int pos = max(positions[t], 0), tpos = min(pos, max(max_pos - 1, 0));
     const GroupedRot rot{(cos_sin && rot_dims) ? cos_sin + (size_t)tpos * rot_dims : nullptr, rot_dims, pairing};
     if (y < q_blocks) {
         const float temp = temp_coef != 0.f ? 1.0f + temp_coef * logf((float)((pos + 1) / temp_every + 1)) : 1.0f;
+        const float rr = pre.q_norm ? grouped_rms(x, pre.bias, H * D, pre.eps, red) : 1.0f;
         TC* qo = q_out + (size_t)t * H * P;
         const int h0 = y * GQ_HEADS, h1 = min(H, h0 + GQ_HEADS);
-        for (int h = h0; h < h1; ++h)
+        for (int h = h0; h < h1; ++h) {
+            const int c0 = h * D;
+            auto value = [&](int e) {
+                float v = x[c0 + e];
+                if (pre.bias) v += pre.bias[c0 + e];
+                return pre.q_norm ? v * rr * pre.q_norm[c0 + e] : v;
+            };
             for (int e = tid; e < P; e += GQ_THREADS)
-                qo[(size_t)h * P + e] = from_f32<TC>(e < D ? grouped_rotated(x + (size_t)h * D, e, rot) * temp : 0.f);
+                qo[(size_t)h * P + e] = from_f32<TC>(e < D ? grouped_rotated(value, e, rot) * temp : 0.f);
+        }
         return;
     }
     const int slot = slots[t];
     if (slot < 0) return;      // (the whole block: a token that writes no key)
     const int g = y - q_blocks;
     const int page = slot / page_size, off = slot - page * page_size;
-    const float* xk = x + (size_t)H * D + (size_t)g * D;
-    const float* xv = x + (size_t)H * D + (size_t)G * D + (size_t)g * E;
+    const size_t ck = (size_t)H * D, cv = ck + (size_t)G * D + (size_t)g * E;
+    const float* xk = x + ck;
+    const float* bk = pre.bias ? pre.bias + ck : nullptr;
+    const float rr = pre.k_norm ? grouped_rms(xk, bk, G * D, pre.eps, red) : 1.0f;
+    const int c0 = g * D;
+    auto value = [&](int e) {
+        float v = xk[c0 + e];
+        if (bk) v += bk[c0 + e];
+        return pre.k_norm ? v * rr * pre.k_norm[c0 + e] : v;
+    };
     TC* kd = k_cache + (((size_t)page * G + g) * page_size + off) * P;
     TC* vd = v_cache + ((size_t)page * G + g) * P * page_size + off;
     for (int e = tid; e < P; e += GQ_THREADS) {
-        kd[e] = from_f32<TC>(e < D ? grouped_rotated(xk, e, rot) : 0.f);
-        vd[(size_t)e * page_size] = from_f32<TC>(e < E ? xv[e] : 0.f);
+        kd[e] = from_f32<TC>(e < D ? grouped_rotated(value, e, rot) : 0.f);
+        vd[(size_t)e * page_size] = from_f32<TC>(e < E ? x[cv + e] + (pre.bias ? pre.bias[cv + e] : 0.f) : 0.f);
     }
 }
 
 TFF_API int tff_grouped_qkv_store(const float* proj, size_t row, const float* cos_sin, int rot_dims, int pairing, int max_pos,
-                                  float temp_coef, int temp_every, const int32_t* positions, const int32_t* slots, void* q_out,
-                                  void* k_cache, void* v_cache, int page_size, int num_pages, int T, int H, int G, int D, int E,
-                                  int P, int store, int dtype, tff_stream_t stream) {
+                                  float temp_coef, int temp_every, const float* bias, const float* q_norm, const float* k_norm,
+                                  float norm_eps, const int32_t* positions, const int32_t* slots, void* q_out, void* k_cache,
+                                  void* v_cache, int page_size, int num_pages, int T, int H, int G, int D, int E, int P, int store,
+                                  int dtype, tff_stream_t stream) {
     TFF_REQUIRE(proj && positions && q_out && (!store || (slots && k_cache && v_cache)), "grouped_qkv_store: null pointer");
     TFF_REQUIRE(T >= 0 && H > 0 && G > 0 && H % G == 0 && D > 0 && E > 0 && P >= D && P >= E && temp_every > 0,
                 "grouped_qkv_store: bad sizes H=%d G=%d D=%d E=%d P=%d", H, G, D, E, P);
@@ -91,7 +136,7 @@ TFF_API int tff_grouped_qkv_store(const float* proj, size_t row, const float* co
     const dim3 grid(T, q_blocks + kv_blocks);
 #define GQ_LAUNCH(TC)                                                                                                          \
     grouped_qkv_store_kernel<TC><<<grid, GQ_THREADS, 0, s>>>(proj, row, cos_sin, rot_dims, pairing, max_pos, temp_coef, temp_every, \
-                                                             positions, slots, (TC*)q_out, (TC*)k_cache, (TC*)v_cache, page_size, H, \
+                                                             GroupedPre{bias, q_norm, k_norm, norm_eps}, positions, slots, (TC*)q_out, (TC*)k_cache, (TC*)v_cache, page_size, H, \
                                                              G, D, E, P, q_blocks)
     if (dtype == TFF_F32) GQ_LAUNCH(float);
     else if (dtype == TFF_BF16) GQ_LAUNCH(bf16_t);
@@ -170,50 +215,54 @@ TFF_API int tff_pool_keys(void* k_cache, void* v_cache, const int32_t* block_tab
     return tff_check_launch("pool_keys");
 }
 
-// out[t, h E + e] = o[t, h P + e] * sigmoid(g[t, h])      (g null: the heads brought together only)
+// out[t, h E + e] = o[t, h P + e] * sigmoid(g[t, h]) * scale      (g null: no gate); rows of out out_row apart
 template <typename T>
 __global__ __launch_bounds__(256) void gate_heads_kernel(const T* __restrict__ o, size_t o_row, int P, const float* __restrict__ g,
-                                                         size_t g_row, T* __restrict__ out, int HE, int E, size_t count) {
+                                                         size_t g_row, float scale, T* __restrict__ out, size_t out_row, int HE, int E,
+                                                         size_t count) {
     const size_t id = (size_t)blockIdx.x * 256 + threadIdx.x;
     if (id >= count) return;
     const size_t t = id / HE;
     const int c = (int)(id - t * HE), h = c / E, e = c - h * E;
-    const float f = g ? 1.0f / (1.0f + expf(-g[t * g_row + h])) : 1.0f;
-    out[t * HE + c] = from_f32<T>(to_f32(o[t * o_row + (size_t)h * P + e]) * f);
+    const float f = g ? scale / (1.0f + expf(-g[t * g_row + h])) : scale;
+    out[t * out_row + c] = from_f32<T>(to_f32(o[t * o_row + (size_t)h * P + e]) * f);
 }
 
 // The same, eight neighbouring elements a thread (E, P and the rows' strides multiples of 8).
 __global__ __launch_bounds__(256) void gate_heads8_kernel(const bf16_t* __restrict__ o, size_t o_row, int P, const float* __restrict__ g,
-                                                          size_t g_row, bf16_t* __restrict__ out, int HE8, int E8, size_t count) {
+                                                          size_t g_row, float scale, bf16_t* __restrict__ out, size_t out_row, int HE8,
+                                                          int E8, size_t count) {
     const size_t id = (size_t)blockIdx.x * 256 + threadIdx.x;
     if (id >= count) return;
     const size_t t = id / HE8;
     const int c = (int)(id - t * HE8), h = c / E8, e = c - h * E8;
-    const float f = g ? 1.0f / (1.0f + expf(-g[t * g_row + h])) : 1.0f;
+    const float f = g ? scale / (1.0f + expf(-g[t * g_row + h])) : scale;
     union { uint4 u; bf16_t b[8]; } x;
     x.u = *reinterpret_cast<const uint4*>(o + t * o_row + (size_t)h * P + e * 8);
 #pragma unroll
     for (int i = 0; i < 8; ++i) x.b[i] = (bf16_t)((float)x.b[i] * f);
-    *reinterpret_cast<uint4*>(out + (t * HE8 + c) * 8) = x.u;
+    *reinterpret_cast<uint4*>(out + t * out_row + (size_t)c * 8) = x.u;
 }
 
-TFF_API int tff_gate_heads(const void* o, size_t o_row, int P, const float* g, size_t g_row, void* out, int T, int H, int E,
-                           int dtype, tff_stream_t stream) {
+TFF_API int tff_gate_heads(const void* o, size_t o_row, int P, const float* g, size_t g_row, float scale, void* out, size_t out_row,
+                           int T, int H, int E, int dtype, tff_stream_t stream) {
     TFF_REQUIRE(o && out, "gate_heads: null pointer");
-    TFF_REQUIRE(T >= 0 && H > 0 && E > 0 && P >= E && o_row >= (size_t)H * P && (!g || g_row >= (size_t)H), "gate_heads: bad sizes");
+    TFF_REQUIRE(T >= 0 && H > 0 && E > 0 && P >= E && o_row >= (size_t)H * P && out_row >= (size_t)H * E && (!g || g_row >= (size_t)H),
+                "gate_heads: bad sizes");
     if (T == 0) return 0;
     hipStream_t s = (hipStream_t)stream;
     const size_t count = (size_t)T * H * E;
     const unsigned blocks = (unsigned)((count + 255) / 256);
-    if (dtype == TFF_BF16 && E % 8 == 0 && P % 8 == 0 && o_row % 8 == 0 && ((uintptr_t)o % 16) == 0 && ((uintptr_t)out % 16) == 0) {
-        gate_heads8_kernel<<<(unsigned)((count / 8 + 255) / 256), 256, 0, s>>>((const bf16_t*)o, o_row, P, g, g_row, (bf16_t*)out, H * E / 8,
-                                                                               E / 8, count / 8);
+    if (dtype == TFF_BF16 && E % 8 == 0 && P % 8 == 0 && o_row % 8 == 0 && out_row % 8 == 0 && ((uintptr_t)o % 16) == 0 &&
+        ((uintptr_t)out % 16) == 0) {
+        gate_heads8_kernel<<<(unsigned)((count / 8 + 255) / 256), 256, 0, s>>>((const bf16_t*)o, o_row, P, g, g_row, scale, (bf16_t*)out,
+                                                                               out_row, H * E / 8, E / 8, count / 8);
         return tff_check_launch("gate_heads");
     }
     if (dtype == TFF_F32)
-        gate_heads_kernel<float><<<blocks, 256, 0, s>>>((const float*)o, o_row, P, g, g_row, (float*)out, H * E, E, count);
+        gate_heads_kernel<float><<<blocks, 256, 0, s>>>((const float*)o, o_row, P, g, g_row, scale, (float*)out, out_row, H * E, E, count);
     else if (dtype == TFF_BF16)
-        gate_heads_kernel<bf16_t><<<blocks, 256, 0, s>>>((const bf16_t*)o, o_row, P, g, g_row, (bf16_t*)out, H * E, E, count);
+        gate_heads_kernel<bf16_t><<<blocks, 256, 0, s>>>((const bf16_t*)o, o_row, P, g, g_row, scale, (bf16_t*)out, out_row, H * E, E, count);
     else
         return tff_fail("gate_heads: unknown dtype %d", dtype);
     return tff_check_launch("gate_heads");

@@ -4,6 +4,10 @@
 //                   s + bias are chosen (the lowest index among equals), their weights are
 //                   s / (sum of the chosen s + 1e-20): the bias moves the choice only.  With `softmax`,
 //                   s = softmax(z) over all experts and the weights are the chosen s as they are.
+//                   With `groups`, E / groups neighbours form a group whose score is the sum of its two
+//                   largest s + bias, and only experts of the best `keep` groups can be chosen.  The weights
+//                   are multiplied by `scale`.  With `shared`, every token also gets the experts E .. E + shared - 1,
+//                   each with the weight sigmoid(row E of z).
 // tff_experts_gate_up: for every (token, chosen expert): g = min(Wg h, limit),
 //                   u = clamp(Wu h, -limit, limit), y = g * sigmoid(act_alpha * g) * (u + up_offset)
 //                   (limit = infinity, act_alpha = 1, up_offset = 0: silu(g) * u).
@@ -60,17 +64,20 @@ __global__ __launch_bounds__(64 * RT_WAVES) void route_topk_kernel(const T* __re
                                                                    const float* __restrict__ Wr,
                                                                    const float* __restrict__ logits,
                                                                    const float* __restrict__ bias, int width, int E,
-                                                                   int top, int softmax, int32_t* __restrict__ idx,
+                                                                   int top, int softmax, int groups, int keep, float scale,
+                                                                   int shared, int32_t* __restrict__ idx,
                                                                    float* __restrict__ wts) {
-    __shared__ float s_all[RT_MAX_E];
+    __shared__ float s_all[RT_MAX_E + 1];
     __shared__ float c_all[RT_MAX_E];
+    __shared__ float g_all[RT_MAX_E];       // a group's score; of the chosen groups -infinity
     __shared__ int chosen[64];
     const int t = blockIdx.x, lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
+    const int rows = E + (shared > 0 ? 1 : 0), out_cols = top + shared;
     if (logits) {
-        for (int e = threadIdx.x; e < E; e += blockDim.x) s_all[e] = logits[(size_t)t * E + e];
+        for (int e = threadIdx.x; e < rows; e += blockDim.x) s_all[e] = logits[(size_t)t * rows + e];
     } else {
         const T* hr = h + (size_t)t * h_row;
-        for (int e = wv; e < E; e += RT_WAVES) {
+        for (int e = wv; e < rows; e += RT_WAVES) {
             const float z = wave_dot(hr, Wr + (size_t)e * width, width, lane);
             if (lane == 0) s_all[e] = z;
         }
@@ -104,12 +111,12 @@ __global__ __launch_bounds__(64 * RT_WAVES) void route_topk_kernel(const T* __re
     }
     __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "workgroup");
     __builtin_amdgcn_wave_barrier();
-    float sum = 0.f;
-    for (int k = 0; k < top; ++k) {
+    // the first of the largest of n numbers in LDS
+    auto largest = [&](const float* v, int n) {
         float best = -INFINITY;
         int bi = 0x7fffffff;
-        for (int e = lane; e < E; e += 64) {
-            const float c = c_all[e];
+        for (int e = lane; e < n; e += 64) {
+            const float c = v[e];
             if (c > best) { best = c; bi = e; }      // (ascending e: the first of equals stays)
         }
 #pragma unroll
@@ -118,9 +125,38 @@ __global__ __launch_bounds__(64 * RT_WAVES) void route_topk_kernel(const T* __re
             const int oi = __shfl_xor(bi, o, 64);
             if (ob > best || (ob == best && oi < bi)) { best = ob; bi = oi; }
         }
+        return min(bi, n - 1);
+    };
+    if (keep < groups) {
+        const int size = E / groups;
+        for (int g = lane; g < groups; g += 64) {
+            float a = -INFINITY, b = -INFINITY;      // the two largest
+            for (int j = 0; j < size; ++j) {
+                const float c = c_all[g * size + j];
+                b = fmaxf(b, fminf(a, c));
+                a = fmaxf(a, c);
+            }
+            g_all[g] = size > 1 ? a + b : a;
+        }
+        __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "workgroup");
+        __builtin_amdgcn_wave_barrier();
+        for (int k = 0; k < keep; ++k) {
+            const int g = largest(g_all, groups);
+            if (lane == 0) g_all[g] = -INFINITY;
+            __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "workgroup");
+            __builtin_amdgcn_wave_barrier();
+        }
+        for (int e = lane; e < E; e += 64)
+            if (g_all[e / size] != -INFINITY) c_all[e] = -INFINITY;
+        __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "workgroup");
+        __builtin_amdgcn_wave_barrier();
+    }
+    float sum = 0.f;
+    for (int k = 0; k < top; ++k) {
+        const int bi = largest(c_all, E);
         // (one wave from here on: LDS works through its accesses in order)
         if (lane == 0) {
-            idx[(size_t)t * top + k] = bi;
+            idx[(size_t)t * out_cols + k] = bi;
             chosen[k] = bi;
             c_all[bi] = -INFINITY;
         }
@@ -129,21 +165,31 @@ __global__ __launch_bounds__(64 * RT_WAVES) void route_topk_kernel(const T* __re
         __builtin_amdgcn_wave_barrier();
     }
     const float inv = softmax ? 1.0f : 1.0f / (sum + 1e-20f);      // (mode 2: sigmoid scores as they are)
-    if (lane < top) wts[(size_t)t * top + lane] = s_all[chosen[lane]] * inv;
+    if (lane < top) {
+        wts[(size_t)t * out_cols + lane] = s_all[chosen[lane]] * inv * scale;
+    } else if (lane < out_cols) {
+        idx[(size_t)t * out_cols + lane] = E + lane - top;
+        wts[(size_t)t * out_cols + lane] = 1.0f / (1.0f + expf(-s_all[E]));
+    }
 }
 
 TFF_API int tff_route_topk(const void* h, int h_row, const float* Wr, const float* logits, const float* bias, int T,
-                           int width, int E, int top, int softmax, int32_t* idx, float* wts, int dtype, tff_stream_t stream) {
+                           int width, int E, int top, int softmax, int groups, int keep, float scale, int shared, int32_t* idx,
+                           float* wts, int dtype, tff_stream_t stream) {
     TFF_REQUIRE(idx && wts && (logits || (h && Wr)), "route_topk: null pointer");
     TFF_REQUIRE(T >= 0 && (logits || (width > 0 && h_row >= width)), "route_topk: bad sizes T=%d width=%d row=%d", T, width, h_row);
-    TFF_REQUIRE(E > 0 && E <= RT_MAX_E && top > 0 && top <= E && top <= 64,
-                "route_topk: %d of %d experts (up to 64 of up to %d)", top, E, RT_MAX_E);
+    TFF_REQUIRE(E > 0 && E <= RT_MAX_E && top > 0 && top <= E && shared >= 0 && top + shared <= 64,
+                "route_topk: %d of %d experts and %d for every token (up to 64 of up to %d)", top, E, shared, RT_MAX_E);
+    TFF_REQUIRE(groups >= 1 && E % groups == 0 && keep >= 1 && keep <= groups && top <= keep * (E / groups),
+                "route_topk: %d of %d experts from %d of %d groups", top, E, keep, groups);
     if (T == 0) return 0;
     hipStream_t s = (hipStream_t)stream;
     if (dtype == TFF_F32)
-        route_topk_kernel<float><<<T, 64 * RT_WAVES, 0, s>>>((const float*)h, h_row, Wr, logits, bias, width, E, top, softmax, idx, wts);
+        route_topk_kernel<float><<<T, 64 * RT_WAVES, 0, s>>>((const float*)h, h_row, Wr, logits, bias, width, E, top, softmax,
+                                                                groups, keep, scale, shared, idx, wts);
     else if (dtype == TFF_BF16)
-        route_topk_kernel<bf16_t><<<T, 64 * RT_WAVES, 0, s>>>((const bf16_t*)h, h_row, Wr, logits, bias, width, E, top, softmax, idx, wts);
+        route_topk_kernel<bf16_t><<<T, 64 * RT_WAVES, 0, s>>>((const bf16_t*)h, h_row, Wr, logits, bias, width, E, top, softmax,
+                                                                groups, keep, scale, shared, idx, wts);
     else
         return tff_fail("route_topk: unknown dtype %d", dtype);
     return tff_check_launch("route_topk");

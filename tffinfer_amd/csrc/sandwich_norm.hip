@@ -5,7 +5,8 @@
 //   d = (planes of a, in order) + bias                                       one sublayer's result, or
 //   d = (rms(a) * wa + rms(b) * wb) / 2                                      two normed results side by side
 //   y = layernorm(d; nw, nb) * scale                                         (nw null: y = d; scale null: 1)
-//   resid <- resid + y;   h = layernorm(resid; w, b)                         -> out
+//   resid <- resid + y + extra;   h = layernorm(resid; w, b)                 -> out
+//   (extra: a row for every row of the step, or one row for all; a layer norm's bias may be null)
 //   with a convolution (steps of one token a request):  h <- h + sum_j cw[j] h_(t - taps + 1 + j), the earlier
 //   h from the request's state row, which moves on by one
 // Every part is optional: without a term the stream is only normed; with `rows` the norm of those rows leaves
@@ -32,6 +33,8 @@ struct SandwichTerm {
     size_t plane_a, plane_b;
     int planes_a, planes_b;
     float pair_eps, n_eps;
+    const float* extra;        // added to the stream beside the term, rows extra_row apart (0: one row for all), or null
+    size_t extra_row;
 };
 
 struct SandwichConv {
@@ -104,8 +107,11 @@ struct SandwichVector {
         if constexpr (EARLY) {
 #pragma unroll
             for (int u = 0; u < VEC; ++u) out[u] = v[it][u];
-        } else {
+        } else if (p) {
             sn_load<VEC>(out, p + e);
+        } else {
+#pragma unroll
+            for (int u = 0; u < VEC; ++u) out[u] = 0.f;
         }
     }
 };
@@ -136,6 +142,12 @@ __global__ __launch_bounds__(NT) void add_layernorm_kernel(float* __restrict__ r
             if (xr) sn_load<VEC>(x[it], xr + e);
             if (ar) sn_load<VEC>(d[it], ar + e);
             if (br) sn_load<VEC>(p2[it], br + e);
+            if (tm.extra) {
+                float t[VEC];
+                sn_load<VEC>(t, tm.extra + row * tm.extra_row + e);
+#pragma unroll
+                for (int u = 0; u < VEC; ++u) x[it][u] += t[u];
+            }
         }
     }
     SandwichVector<IT, VEC, EARLY> vbias, vwa, vwb, vnw, vnb, vsc, vw, vb;
@@ -264,8 +276,14 @@ __global__ __launch_bounds__(NT) void add_layernorm_kernel(float* __restrict__ r
                 }
 #pragma unroll
                 for (int u = 0; u < VEC; ++u) x[it][u] += d[it][u];
-                if (xr && !rows) sn_store<VEC, float>(xr + e, x[it]);
             }
+        }
+    }
+    if ((ar || tm.extra) && xr && !rows) {
+#pragma unroll
+        for (int it = 0; it < IT; ++it) {
+            const int e = (it * NT + tid) * VEC;
+            if (e < W) sn_store<VEC, float>(xr + e, x[it]);
         }
     }
     if (w) layernorm(x, vw, vb, eps, red[2], red[3]);
@@ -325,22 +343,23 @@ TFF_API int tff_add_layernorm(float* resid, const float* a, int planes_a, size_t
                               const float* nw, const float* nb, float n_eps, const float* scale, const float* w,
                               const float* beta, float eps, void* out, const int32_t* rows, int n, int W, const float* conv_w,
                               int taps, float* state, size_t state_row, size_t state_off, const int32_t* state_slots,
-                              int out_dtype, tff_stream_t stream) {
+                              const float* extra, size_t extra_row, int out_dtype, tff_stream_t stream) {
     TFF_REQUIRE((resid || a) && out, "add_layernorm: null pointer");
     TFF_REQUIRE(n >= 0 && W > 0 && W <= SN_MAX_W, "add_layernorm: rows of %d (up to %d)", W, SN_MAX_W);
     TFF_REQUIRE(!a || planes_a >= 1, "add_layernorm: a term without planes");
     TFF_REQUIRE(!b || (a && wa && wb && planes_b >= 1), "add_layernorm: the second of two results needs the first and both weights");
-    TFF_REQUIRE((!nw) == (!nb) && (!w) == (!beta) && (!nw || a), "add_layernorm: a norm takes a weight and a bias");
+    TFF_REQUIRE((nw || !nb) && (w || !beta) && (!nw || a), "add_layernorm: a norm takes a weight, and a bias or none");
+    TFF_REQUIRE(!extra || (resid && (extra_row == 0 || extra_row >= (size_t)W)), "add_layernorm: rows of %zu to add to a stream of %d", extra_row, W);
     TFF_REQUIRE(!rows || resid, "add_layernorm: chosen rows of no stream");
     TFF_REQUIRE(!conv_w || (taps >= 1 && taps <= SN_MAX_TAPS && !rows && (taps == 1 || (state && state_slots &&
                 state_off + (size_t)(taps - 1) * W <= state_row))), "add_layernorm: a convolution of %d taps (up to %d) needs its state", taps, SN_MAX_TAPS);
     if (n == 0) return 0;
-    const SandwichTerm tm{a, b, wa, wb, bias, nw, nb, scale, plane_a, plane_b, planes_a, planes_b, pair_eps, n_eps};
+    const SandwichTerm tm{a, b, wa, wb, bias, nw, nb, scale, plane_a, plane_b, planes_a, planes_b, pair_eps, n_eps, extra, extra_row};
     const SandwichConv cv{conv_w, state, state_slots, state_row, state_off, taps};
     hipStream_t s = (hipStream_t)stream;
     auto ok16 = [](const void* p) { return ((uintptr_t)p % 16) == 0; };
     const bool vec = W % 4 == 0 && plane_a % 4 == 0 && plane_b % 4 == 0 && ok16(resid) && ok16(a) && ok16(b) && ok16(wa) && ok16(wb) &&
-                     ok16(bias) && ok16(nw) && ok16(nb) && ok16(scale) && ok16(w) && ok16(beta) && ok16(out) && ok16(conv_w);
+                     ok16(bias) && ok16(nw) && ok16(nb) && ok16(scale) && ok16(w) && ok16(beta) && ok16(out) && ok16(conv_w) && ok16(extra) && extra_row % 4 == 0;
     TFF_REQUIRE(vec || W <= 8192, "add_layernorm: rows of %d (more than 8192) must be a multiple of 4 wide and 16-byte aligned", W);
 #define SN_LAUNCH(TO, NT, VPT, VEC) add_layernorm_kernel<TO, NT, VPT, VEC><<<n, NT, 0, s>>>(resid, tm, w, beta, eps, (TO*)out, rows, W, cv)
 #define SN_SIZES(TO)                                                                         \

@@ -50,8 +50,9 @@ TFF_API int tff_rmsnorm(const void* x, const float* weight, float eps, void* out
 // sums [bytes / (M * N * 4), M, N] are left there for the caller to add up
 // (tff_add_rmsnorm takes them as they are) and C is not written.
 TFF_API int tff_gemm(const void* A, const void* W, void* C, int M, int N, int K, int lda,
-                     int ab_dtype, int c_dtype, int w_packed, int glu_out, const float* bias, void* workspace,
-                     size_t workspace_bytes, int keep_partials, tff_stream_t stream);
+                     int ab_dtype, int c_dtype, int w_packed, int glu_out, const float* bias, float glu_limit,
+                     float glu_alpha, float glu_up_offset, void* workspace, size_t workspace_bytes, int keep_partials,
+                     tff_stream_t stream);
 TFF_API size_t tff_gemm_workspace_bytes(int M, int N, int K, int ab_dtype, int glu, int keep_partials);
 // The bfloat16 product's plan for these sizes: rows and columns of a block tile (0: the
 // streaming kernel for up to 16 rows) and the number of parts K is split into.
@@ -75,7 +76,7 @@ TFF_API int tff_gemm_residual_prenorm(const void* A, const void* Wp, int M, int 
                                       tff_stream_t stream);
 TFF_API int tff_gemm_row_scaled(const void* A, const void* Wp, void* C, int M, int N, int K, int lda, int c_dtype,
                                 int glu_out, const float* ss, int ss_stride, int ss_count, int dim, float eps,
-                                tff_stream_t stream);
+                                float glu_limit, float glu_alpha, float glu_up_offset, tff_stream_t stream);
 
 // bfloat16 row-major [N, K] (K a multiple of 8) -> fragment order: tiles of
 // 16 rows x 32 k, each stored as the 1 KB operand of a 16x16x32 MFMA, element
@@ -296,9 +297,13 @@ TFF_API int tff_diff_combine(const void* a, size_t a_row, int P, const float* ga
 // Router: s = sigmoid(z), z = Wr h in float32 (Wr [E, width] float32), or z = logits [T, E] where given
 // (h and Wr may then be null); the `top` largest s + bias (bias may be null) are chosen; idx [T, top],
 // wts [T, top] = s / (sum of the chosen s + 1e-20).  softmax 1: s = softmax(z) over all experts, wts = the chosen s;
-// softmax 2: s = sigmoid(z) and wts = the chosen s as they are.
+// softmax 2: s = sigmoid(z) and wts = the chosen s as they are.  The E experts form `groups` groups of neighbours; only
+// experts of the `keep` groups whose two largest s + bias have the largest sum can be chosen.  The weights are times
+// `scale`.  shared > 0: z has one row more, idx and wts [T, top + shared]: the experts E .. E + shared - 1 follow the
+// chosen ones, each with the weight sigmoid(z[E]).
 TFF_API int tff_route_topk(const void* h, int h_row, const float* Wr, const float* logits, const float* bias, int T,
-                           int width, int E, int top, int softmax, int32_t* idx, float* wts, int dtype, tff_stream_t stream);
+                           int width, int E, int top, int softmax, int groups, int keep, float scale, int shared, int32_t* idx,
+                           float* wts, int dtype, tff_stream_t stream);
 // y[(t, k), :] = g * sigmoid(act_alpha * g) * (u + up_offset), g = min(Wg[e] h_t, limit), u = clamp(Wu[e] h_t, +-limit),
 // e = idx[t, k]; Wg, Wu [E, ff, width], rows ldw elements apart.  in_wts [T, top] (may be null): the pair's
 // weight multiplies the expert's input, that is both products before clamps and activation.
@@ -416,7 +421,8 @@ TFF_API int tff_mixed_attention_q16(const void* q, const void* k_cache, const vo
                                     int window, int keep_first, int sink, void* out, int T, int H, int G, int D,
                                     int page_size, int splits, int tiles_per_split, float* workspace, tff_stream_t stream);
 
-TFF_API int tff_swiglu(const void* gu, const float* bias, void* out, int T, int I, int dtype, tff_stream_t stream);
+TFF_API int tff_swiglu(const void* gu, const float* bias, void* out, int T, int I, float limit, float alpha, float up_offset, int dtype,
+                       tff_stream_t stream);
 
 // Element type conversion of n elements.
 TFF_API int tff_cast(const void* src, int src_dtype, void* dst, int dst_dtype, int64_t n,
@@ -428,7 +434,7 @@ TFF_API int tff_add_layernorm(float* resid, const float* a, int planes_a, size_t
                               const float* nw, const float* nb, float n_eps, const float* scale, const float* w,
                               const float* beta, float eps, void* out, const int32_t* rows, int n, int W, const float* conv_w,
                               int taps, float* state, size_t state_row, size_t state_off, const int32_t* state_slots,
-                              int out_dtype, tff_stream_t stream);
+                              const float* extra, size_t extra_row, int out_dtype, tff_stream_t stream);
 // items of up to `chunk` tokens (row of the step's tables, first place in its portion), chunk >= taps - 1
 TFF_API int tff_input_conv(const float* h, const float* w, int taps, float* state, size_t state_row, size_t state_off,
                            const int32_t* items, int num_items, int chunk, const int32_t* cu_tokens, const int32_t* state_slots, void* out,
@@ -449,15 +455,46 @@ TFF_API int tff_row_norm_gate(const float* o, const float* g, size_t g_row, cons
 
 // ---- around a grouped attention with a query temperature and the mean keys of blocks (grouped_attention.hip) ----
 TFF_API int tff_grouped_qkv_store(const float* proj, size_t row, const float* cos_sin, int rot_dims, int pairing, int max_pos,
-                                  float temp_coef, int temp_every, const int32_t* positions, const int32_t* slots, void* q_out,
-                                  void* k_cache, void* v_cache, int page_size, int num_pages, int T, int H, int G, int D, int E,
-                                  int P, int store, int dtype, tff_stream_t stream);
+                                  float temp_coef, int temp_every, const float* bias, const float* q_norm, const float* k_norm,
+                                  float norm_eps, const int32_t* positions, const int32_t* slots, void* q_out, void* k_cache,
+                                  void* v_cache, int page_size, int num_pages, int T, int H, int G, int D, int E, int P, int store,
+                                  int dtype, tff_stream_t stream);
 // tokens [T] (may be null: tokens 0 .. T - 1): the step's tokens to look at; those that end no block are left out.
 TFF_API int tff_pool_keys(void* k_cache, void* v_cache, const int32_t* block_tables, int bt_stride, const int32_t* pool_tables,
                           int pt_stride, const int32_t* token_req, const int32_t* positions, const int32_t* slots,
                           const int32_t* tokens, int page_size, int num_pages, int pool, int T, int G, int d, int dtype, tff_stream_t stream);
-TFF_API int tff_gate_heads(const void* o, size_t o_row, int P, const float* g, size_t g_row, void* out, int T, int H, int E,
-                           int dtype, tff_stream_t stream);
+TFF_API int tff_gate_heads(const void* o, size_t o_row, int P, const float* g, size_t g_row, float scale, void* out, size_t out_row,
+                           int T, int H, int E, int dtype, tff_stream_t stream);
+
+// ---- linear recurrences with decays or gates that depend on the token (linear_recurrence.hip) ----
+enum { TFF_LR_DECAY = 0, TFF_LR_EXP = 1 };      // a decay per key channel; exponential gates per head with a running maximum
+typedef struct TffRecurrence {
+    const float *q, *k, *v, *gate;              // columns of the joint projection: [H D], [H D], [H E], [H E]; rows ld apart
+    size_t ld;
+    const float *a1, *a2, *a_bias;              // decay: columns [rank]; [rank][H D] (transposed); [H D]
+    const float *ig, *fg, *i_bias, *f_bias;     // gates: columns [H], [H]; [H], [H]
+    const float* w;                             // the norm's weight, [E] or [H E]
+    float* state;                               // a request's row: [H][E or E + 1][D] (and [H]), rows state_row apart
+    size_t state_row;
+    const int32_t *cu_tokens, *state_slots;
+    void* out;                                  // [T][H E], rows out_row apart
+    size_t out_row;
+    int kind, R, H, D, E, rank, w_per_head, sigmoid_gate, out_dtype;
+    float inv_tau, cap, den_eps, eps, q_scale, out_scale;
+} TffRecurrence;
+// max_tokens: the most tokens a request brings (0: unknown)
+TFF_API int tff_recurrence_few(const TffRecurrence* p, int max_tokens, tff_stream_t stream);
+TFF_API int tff_recurrence_chunk(void);          // tokens an item of tff_recurrence_chunks holds at most
+TFF_API size_t tff_recurrence_workspace_bytes(int kind, int T, int items, int H, int D, int E);
+// items [num_items][2]: (row of the step's tables, first place in its portion); item_start [R + 1]: a row's items, in order
+TFF_API int tff_recurrence_chunks(const TffRecurrence* p, int T, const int32_t* items, const int32_t* item_start, int num_items,
+                                  float* workspace, size_t workspace_bytes, tff_stream_t stream);
+
+// ---- an embedding with a table for pairs of neighbouring tokens (bigram_embedding.hip) ----
+TFF_API int tff_bigram_embed(const void* table, int packed, int row_width, const void* pairs, const int32_t* ids,
+                             const int32_t* positions, const int32_t* token_req, const int32_t* cu_tokens,
+                             const int32_t* state_slots, int32_t* last, size_t last_row, int64_t mul_prev, int64_t mul_cur,
+                             int64_t buckets, float* out, float* copy, int T, int W, int V, int dtype, tff_stream_t stream);
 
 // out[r] = lowest index among the maxima of logits[r, :].
 // workspace: tff_argmax_workspace_bytes(rows, V) bytes, 16-byte aligned (0: none needed), for the

@@ -84,6 +84,8 @@ class StepBatch:
         self.cu_tokens = self.start_pos = self.context_lens = None
         self.state_slots = self.logit_rows = None
         self.groups: list[GroupTables] = []
+        #: float32 [T, hidden]: the embedding's output, where the run order adds it to the stream again
+        self.embedding_output = None
         # host copies for parts that loop over entries
         self.host_cu_tokens: list = []
         self.host_start_pos: list = []

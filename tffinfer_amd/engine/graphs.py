@@ -326,6 +326,7 @@ class DecodeGraph:
                     with torch.cuda.graph(piece.graph, stream=side):
                         piece.resid, piece.pending, piece.logits = body()
                     resid, pending = piece.resid, piece.pending
+                    piece.embedding_output = self.batch.embedding_output     # (kept for pieces that run eagerly)
         finally:
             if gc_was_on:
                 gc.enable()
@@ -377,6 +378,8 @@ class DecodeGraph:
                 continue
             if live is None:
                 live = self._context(self._live_batch(R))
+                kept = pieces[0].embedding_output
+                live.batch.embedding_output = None if kept is None else kept[:R]
             # the piece before left the residual stream and its pending term in fixed tensors;
             # this one adds to the stream's live rows in place
             before = pieces[i - 1]
@@ -391,11 +394,11 @@ class DecodeGraph:
 
 class _Piece:
     """A run of consecutive items of the step: one captured graph, or eager code."""
-    __slots__ = ("safe", "items", "graph", "resid", "pending", "logits")
+    __slots__ = ("safe", "items", "graph", "resid", "pending", "logits", "embedding_output")
 
     def __init__(self, safe: bool, items: list):
         self.safe, self.items = safe, items
-        self.graph = self.resid = self.pending = self.logits = None
+        self.graph = self.resid = self.pending = self.logits = self.embedding_output = None
 
 
 def graph_buckets(max_seqs: int) -> list[int]:

@@ -35,7 +35,8 @@ class LayerContext:
         self.kv = None
         self.state = None
         self.call_index = -1
-        self.stream_offset = None       # float32 [hidden]: a row the run order adds to the stream before this call
+        # float32 [hidden] or [tokens, hidden]: what the run order adds to the stream before this call
+        self.stream_offset = None
 
 
 class StepContext(LayerContext):

@@ -6,7 +6,7 @@ from ctypes import c_char_p, c_float, c_int, c_int64, c_size_t, c_void_p
 
 from .build import ensure_built
 
-ABI_VERSION = 35
+ABI_VERSION = 36
 
 
 class KernelLibraryError(RuntimeError):
@@ -19,16 +19,29 @@ class KernelError(RuntimeError):
 
 _P, _I, _F, _Z = c_void_p, c_int, c_float, c_size_t
 
+
+class Recurrence(ctypes.Structure):
+    """``TffRecurrence`` of csrc/tffinfer_kernels.h, field by field."""
+    _fields_ = ([(n, _P) for n in ("q", "k", "v", "gate")] + [("ld", _Z)]
+                + [(n, _P) for n in ("a1", "a2", "a_bias", "ig", "fg", "i_bias", "f_bias", "w", "state")] + [("state_row", _Z)]
+                + [(n, _P) for n in ("cu_tokens", "state_slots", "out")] + [("out_row", _Z)]
+                + [(n, _I) for n in ("kind", "R", "H", "D", "E", "rank", "w_per_head", "sigmoid_gate", "out_dtype")]
+                + [(n, _F) for n in ("inv_tau", "cap", "den_eps", "eps", "q_scale", "out_scale")])
+
+
+#: ``Recurrence.kind``: a decay per key channel; exponential gates per head with a running maximum
+LR_DECAY, LR_EXP = 0, 1
+
 _SIGNATURES = {
     "tff_embed": [_P, _P, _P, _I, _I, _I, _I, _P],
     "tff_add_rmsnorm": [_P, _P, _I, _Z, _P, _F, _P, _P, _I, _I, _I, _P],
     "tff_rmsnorm": [_P, _P, _F, _P, _I, _I, _I, _P],
-    "tff_gemm": [_P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _P, _P, _Z, _I, _P],
+    "tff_gemm": [_P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _P, _F, _F, _F, _P, _Z, _I, _P],
     "tff_gemm_workspace_bytes": [_I, _I, _I, _I, _I, _I],
     "tff_gemm_plan": [_I, _I, _I, _I, _I, _P, _P, _P],
     "tff_gemm_residual_prenorm": [_P, _P, _I, _I, _I, _I, _P, _P, _P, _P, _I, _P],
     "tff_gemm_residual_dyt": [_P, _P, _I, _I, _I, _I, _P, _F, _P, _P, _P, _P],
-    "tff_gemm_row_scaled": [_P, _P, _P, _I, _I, _I, _I, _I, _I, _P, _I, _I, _I, _F, _P],
+    "tff_gemm_row_scaled": [_P, _P, _P, _I, _I, _I, _I, _I, _I, _P, _I, _I, _I, _F, _F, _F, _F, _P],
     "tff_pack_weight": [_P, _P, _I, _I, _P],
     "tff_embed_packed": [_P, _P, _P, _I, _I, _I, _P],
     "tff_qk_norm_rope_kv": [_P, _I, _I, _I, _I, _P, _P, _F, _P, _I, _I, _I, _P, _P, _P, _P,
@@ -55,7 +68,7 @@ _SIGNATURES = {
     "tff_diff_combine": [_P, _Z, _I, _P, _Z, _F, _F, _F, _P, _Z, _I, _I, _I, _I, _P],
     "tff_scale_add_rmsnorm": [_P, _P, _I, _Z, _F, _P, _F, _P, _I, _I, _I, _P],
     "tff_gelu": [_P, _P, c_int64, _I, _I, _P],
-    "tff_route_topk": [_P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _P, _P, _I, _P],
+    "tff_route_topk": [_P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _I, _P, _P, _I, _P],
     "tff_experts_gate_up": [_P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _F, _F, _P, _P, _I, _P],
     "tff_experts_tiles_supported": [_I, _I, _I],
     "tff_experts_by_tiles": [_P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _F, _F, _P, _P, _P, _I, _P, _P, _I, _I, _P],
@@ -80,22 +93,27 @@ _SIGNATURES = {
     "tff_mixed_attention_q16_supported": [_I, _I, _I, _I],
     "tff_mixed_attention_q16": [_P, _P, _P, _P, _I, _P, _P, _P, _I, _P, _I, _P, _F, _F, _I, _I, _I, _P, _I, _I, _I, _I, _I, _I, _I, _P, _P],
     "tff_experts_down": [_P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P, _I, _I, _P, _I, _P],
-    "tff_swiglu": [_P, _P, _P, _I, _I, _I, _P],
+    "tff_swiglu": [_P, _P, _P, _I, _I, _F, _F, _F, _I, _P],
     "tff_cast": [_P, _I, _P, _I, c_int64, _P],
     "tff_argmax_workspace_bytes": [_I, _I],
     "tff_argmax": [_P, _P, _I, _I, _P, _P],
     "tff_repetition_penalty": [_P, _I, _I, _P, _P, _P, _P],
     "tff_sample": [_P, _P, _I, _I, _P, _P, _P, _P, _P, _P, _P],
     "tff_add_layernorm": [_P, _P, _I, _Z, _P, _I, _Z, _P, _P, _F, _P, _P, _P, _F, _P, _P, _P, _F, _P, _P, _I, _I, _P, _I, _P, _Z,
-                          _Z, _P, _I, _P],
+                          _Z, _P, _P, _Z, _I, _P],
     "tff_input_conv": [_P, _P, _I, _P, _Z, _Z, _P, _I, _I, _P, _P, _P, _I, _I, _P],
     "tff_lightning": [_P, _Z, _P, _P, _Z, _P, _P, _P, _I, _I, _I, _I, _P],
     "tff_lightning_chunk": [],
     "tff_lightning_chunks": [_P, _Z, _P, _P, _Z, _P, _P, _I, _P, _P, _P, _P, _I, _I, _I, _I, _P],
     "tff_row_norm_gate": [_P, _P, _Z, _P, _F, _P, _I, _I, _I, _P],
-    "tff_grouped_qkv_store": [_P, _Z, _P, _I, _I, _I, _F, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _I, _I, _P],
+    "tff_grouped_qkv_store": [_P, _Z, _P, _I, _I, _I, _F, _I, _P, _P, _P, _F, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _I, _I, _P],
     "tff_pool_keys": [_P, _P, _P, _I, _P, _I, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P],
-    "tff_gate_heads": [_P, _Z, _I, _P, _Z, _P, _I, _I, _I, _I, _P],
+    "tff_gate_heads": [_P, _Z, _I, _P, _Z, _F, _P, _Z, _I, _I, _I, _I, _P],
+    "tff_recurrence_few": [_P, _I, _P],
+    "tff_recurrence_chunk": [],
+    "tff_recurrence_workspace_bytes": [_I, _I, _I, _I, _I, _I],
+    "tff_recurrence_chunks": [_P, _I, _P, _P, _I, _P, _Z, _P],
+    "tff_bigram_embed": [_P, _I, _I, _P, _P, _P, _P, _P, _P, _P, _Z, c_int64, c_int64, c_int64, _P, _P, _I, _I, _I, _I, _P],
     "tff_probe_stream_read": [_P, _Z, _P, _I, _P],
     "tff_probe_mfma": [_P, _I, _I, _I, _P],
 }

@@ -69,11 +69,15 @@ def _ptr(t):
     return None if t is None else t.data_ptr()
 
 
+#: the constants (limit, alpha, up_offset) with which the gated activation is silu(gate) * up
+SILU = (math.inf, 1.0, 0.0)
+
+
 class PackedWeight:
     """A bfloat16 matrix [N, K] in the fragment order of the matrix-core
     products: tiles of 16 rows by 32 k stored as the 1 KB operand a wave loads,
     rows and k padded with zeros to multiples of 16 and 32."""
-    __slots__ = ("data", "N", "K", "glu_out", "k_in")
+    __slots__ = ("data", "N", "K", "glu_out", "k_in", "glu_act")
 
     def __init__(self, data: torch.Tensor, N: int, K: int, glu_out: int = 0, k_in: int | None = None):
         self.data, self.N, self.K = data, int(N), int(K)
@@ -83,6 +87,8 @@ class PackedWeight:
         #: > 0: the 16-row groups alternate between a gate and an up projection and the
         #: product yields silu(gate) * up with this many columns
         self.glu_out = int(glu_out)
+        #: (limit, alpha, up_offset) of the gated product's activation, see :func:`swiglu`
+        self.glu_act = SILU
 
     @property
     def shape(self):
@@ -125,11 +131,11 @@ def pack_weight(w: torch.Tensor) -> PackedWeight:
     return PackedWeight(out, N, K, k_in=k_in)
 
 
-def pack_gate_up(gate: torch.Tensor, up: torch.Tensor) -> PackedWeight:
+def pack_gate_up(gate: torch.Tensor, up: torch.Tensor, act: tuple = SILU) -> PackedWeight:
     """Gate and up projections [I, K] (bfloat16, on the GPU) as one weight whose
     16-row groups alternate gate, up, gate, up, ..., in fragment order.  A
     product with it yields silu(x gate^T) * (x up^T) directly: the activation
-    runs in the product's epilogue, on the float32 accumulators."""
+    runs in the product's epilogue, on the float32 accumulators.  ``act``: its constants (:func:`swiglu`)."""
     _req(gate, "gate", torch.bfloat16, 2)
     _req(up, "up", torch.bfloat16, 2)
     if gate.shape != up.shape:
@@ -142,6 +148,7 @@ def pack_gate_up(gate: torch.Tensor, up: torch.Tensor) -> PackedWeight:
     both = padded.view(2, groups, 16, K).permute(1, 0, 2, 3).reshape(groups * 32, K).contiguous()
     pw = pack_weight(both)
     pw.glu_out = I
+    pw.glu_act = tuple(float(x) for x in act)
     return pw
 
 
@@ -189,6 +196,31 @@ def embed(table, ids: torch.Tensor, out: torch.Tensor | None = None) -> torch.Te
         _lib.check(L.tff_embed(table.data_ptr(), ids.data_ptr(), out.data_ptr(), T, H, V,
                                dtype_code(table.dtype), _stream()))
     return out
+
+
+def bigram_embed(table, pairs: torch.Tensor, batch, last: torch.Tensor, mul_prev: int, mul_cur: int,
+                 copy: bool = False):
+    """Rows of ``table`` [V, H] plus rows of ``pairs`` [buckets + 1, H] (row-major, the table's type) for the step's
+    tokens: row (previous token * mul_prev + token * mul_cur) mod buckets, for a sequence's first token the last one.
+    ``last`` int32 [slots, 1]: per state slot the token before the portion, which the step's last one replaces.
+    Returns float32 [T, H], and with ``copy`` the same rows once more in a tensor of their own (else None)."""
+    packed = isinstance(table, PackedWeight)
+    width = table.k_in if packed else table.shape[1]
+    _req(pairs, "bigram table", table.dtype, 2)
+    _req(last, "bigram state", torch.int32, 2)
+    _req(batch.token_ids, "embed ids", torch.int32, 1)
+    _req(batch.positions, "positions", torch.int32, 1)
+    if pairs.shape[1] != width or pairs.shape[0] < 2:
+        raise _lib.KernelError(f"bigram_embed: a table {tuple(pairs.shape)} beside one of rows of {width}")
+    T = batch.num_tokens
+    out = torch.empty(T, width, dtype=torch.float32, device=table.device)
+    out2 = torch.empty_like(out) if copy else None
+    _lib.check(_lib.load().tff_bigram_embed(
+        table.data_ptr(), 1 if packed else 0, table.shape[1], pairs.data_ptr(), batch.token_ids.data_ptr(), batch.positions.data_ptr(),
+        batch.token_req.data_ptr(), batch.cu_tokens.data_ptr(), batch.state_slots.data_ptr(), last.data_ptr(), last.stride(0),
+        int(mul_prev), int(mul_cur), pairs.shape[0] - 1, out.data_ptr(), _ptr(out2), T, width, table.shape[0], dtype_code(table.dtype),
+        _stream()))
+    return out, out2
 
 
 class PendingProduct:
@@ -407,7 +439,7 @@ def linear(x: torch.Tensor, weight, out_dtype: torch.dtype | None = None,
             raise _lib.KernelError(f"linear out: shape {tuple(out.shape)} is not {(M, n_out)}")
     _lib.check(L.tff_gemm(x.data_ptr(), weight.data_ptr(), out.data_ptr(), M, N, K, lda,
                           dtype_code(x.dtype), dtype_code(out_dtype), 1 if packed else 0, glu_out, _ptr(bias),
-                          _ptr(ws), ws_bytes, 1 if keep else 0, _stream()))
+                          *(weight.glu_act if packed else SILU), _ptr(ws), ws_bytes, 1 if keep else 0, _stream()))
     return out
 
 
@@ -419,7 +451,7 @@ def _linear_row_scaled(x: ScaledRows, weight: "PackedWeight", out_dtype: torch.d
     L = _lib.load()
     _lib.check(L.tff_gemm_row_scaled(x.x.data_ptr(), weight.data_ptr(), out.data_ptr(), M, N, K, K,
                                      dtype_code(out_dtype), glu_out, x.ss.data_ptr(), x.ss.stride(0), x.count, K,
-                                     x.eps, _stream()))
+                                     x.eps, *weight.glu_act, _stream()))
     return out
 
 
@@ -1112,12 +1144,19 @@ def relu_squared(x: torch.Tensor) -> torch.Tensor:
 
 
 def route_topk(h: torch.Tensor | None, router: torch.Tensor | None, bias: torch.Tensor | None, top: int,
-               logits: torch.Tensor | None = None, softmax: bool = False, normalize: bool = True):
+               logits: torch.Tensor | None = None, softmax: bool = False, normalize: bool = True, groups: int = 1,
+               keep_groups: int = 1, scale: float = 1.0, shared: int = 0):
     """s = sigmoid(z) with z = h . router^T in float32 (router float32 [E, width]) or z = ``logits``
     (float32 [T, E], a product that ran before); the ``top`` experts with the largest s + bias;
     returns (int32 [T, top], float32 [T, top] = s / (sum of the chosen s + 1e-20)).  With
     ``softmax``, s = softmax(z) over all experts and the weights are the chosen s as they are; without
-    ``normalize``, s = sigmoid(z) and the weights are the chosen s as they are."""
+    ``normalize``, s = sigmoid(z) and the weights are the chosen s as they are.
+
+    ``groups``: E / groups neighbours form a group whose score is the sum of its two largest s + bias; only experts
+    of the ``keep_groups`` best groups can be chosen.  ``scale`` multiplies the weights.  ``shared`` > 0: the router has
+    one row more (z_sh), and the results [T, top + shared] end with the experts E .. E + shared - 1, each with the
+    weight sigmoid(z_sh)."""
+    extra = 1 if shared else 0
     if logits is not None:
         _req(logits, "router logits", torch.float32, 2)
         T, E = logits.shape
@@ -1130,15 +1169,18 @@ def route_topk(h: torch.Tensor | None, router: torch.Tensor | None, bias: torch.
         dev, dt = h.device, h.dtype
         if router.shape[1] != width:
             raise _lib.KernelError(f"route_topk: router {tuple(router.shape)} for rows of {width}")
+    E -= extra
     if bias is not None:
         _req(bias, "router bias", torch.float32, 1)
         if bias.numel() != E:
             raise _lib.KernelError(f"route_topk: {bias.numel()} bias terms for {E} experts")
-    idx = torch.empty(T, top, dtype=torch.int32, device=dev)
-    wts = torch.empty(T, top, dtype=torch.float32, device=dev)
+    idx = torch.empty(T, top + shared, dtype=torch.int32, device=dev)
+    wts = torch.empty(T, top + shared, dtype=torch.float32, device=dev)
     _lib.check(_lib.load().tff_route_topk(None if logits is not None else h.data_ptr(), width,
                                           None if logits is not None else router.data_ptr(), _ptr(logits), _ptr(bias),
-                                          T, width, E, int(top), 1 if softmax else (0 if normalize else 2), idx.data_ptr(), wts.data_ptr(), dtype_code(dt), _stream()))
+                                          T, width, E, int(top), 1 if softmax else (0 if normalize else 2), int(groups),
+                                          int(keep_groups), float(scale), int(shared), idx.data_ptr(), wts.data_ptr(),
+                                          dtype_code(dt), _stream()))
     return idx, wts
 
 
@@ -1581,12 +1623,14 @@ def _token_items(batch, chunk: int, device):
 
 
 def add_layernorm(resid: torch.Tensor | None, delta, weight, bias, eps: float, out_dtype: torch.dtype,
-                  rows: torch.Tensor | None = None, conv=None, batch=None) -> torch.Tensor:
+                  rows: torch.Tensor | None = None, conv=None, batch=None,
+                  extra: torch.Tensor | None = None) -> torch.Tensor:
     """``resid += delta`` (None, an :class:`OutputTerm` or anything else a sublayer may return; not added when
     ``rows`` is given) and the layer norm of the sum in ``out_dtype``; with ``rows`` (int32) of those rows only.
     ``conv`` (weights float32 [taps, W], state float32 [slots, row], offset in a state row): the normed rows leave
     with their causal convolution over time added, per request of ``batch``; the last taps - 1 normed
     rows of each request are left in its state.  A step of one token per request is one kernel.
+    ``bias`` None: the norm has none.  ``extra`` (float32, the stream's shape or one row [W]): added to the stream too.
     ``resid`` None and ``weight`` None: the term itself."""
     term = delta if isinstance(delta, OutputTerm) else OutputTerm(delta)
     if isinstance(term.term, PendingTerms):
@@ -1621,6 +1665,12 @@ def add_layernorm(resid: torch.Tensor | None, delta, weight, bias, eps: float, o
             raise _lib.KernelError(f"add_layernorm: state rows of {state.shape[1]} do not hold {taps - 1} x {W} from {off}")
         if batch.num_tokens != n or batch.cu_tokens.numel() != batch.num_reqs + 1:
             raise _lib.KernelError("add_layernorm: the step's tables do not describe the rows")
+    extra_row = 0
+    if extra is not None:
+        _req(extra, "add_layernorm extra", torch.float32)
+        if tuple(extra.shape) not in ((W,), shape):
+            raise _lib.KernelError(f"add_layernorm: rows {tuple(extra.shape)} to add to a stream {shape}")
+        extra_row = W if extra.dim() == 2 else 0
     split = conv is not None and not one
     out = torch.empty(n, W, dtype=torch.float32 if split else out_dtype, device=dev)
     L = _lib.load()
@@ -1630,7 +1680,7 @@ def add_layernorm(resid: torch.Tensor | None, delta, weight, bias, eps: float, o
     _lib.check(L.tff_add_layernorm(
         _ptr(resid), _ptr(a), pa, sa, _ptr(b), pb, sb, _ptr(wa), _ptr(wb), float(pair_eps), _ptr(tb), _ptr(nw), _ptr(nb),
         float(n_eps), _ptr(sc), _ptr(weight), _ptr(bias), float(eps), out.data_ptr(), _ptr(rows), n, W,
-        _ptr(cw) if one else None, taps, st, st_row, off, slots, dtype_code(out.dtype), _stream()))
+        _ptr(cw) if one else None, taps, st, st_row, off, slots, _ptr(extra), extra_row, dtype_code(out.dtype), _stream()))
     if not split:
         return out
     chunk = CONV_CHUNK if taps - 1 <= CONV_CHUNK else 32
@@ -1693,13 +1743,96 @@ def row_norm_gate(o: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, eps
     return out
 
 
+#: tokens of a step's longest entry from which these recurrences run in chunks on the matrix cores
+RECURRENCE_LONG_PORTION = 12
+
+
+def _recurrence(kind: int, proj, cols: dict, H: int, D: int, E: int, gate_sigmoid: bool, weight, eps: float, state, batch,
+                out: torch.Tensor, out_scale: float, chunked: bool | None, vectors: dict, numbers: dict) -> torch.Tensor:
+    """``cols``: where the projections' columns start; ``vectors``: float32 tensors; ``numbers``: constants."""
+    T = proj.shape[0]
+    last = max(c + {"q": H * D, "k": H * D, "v": H * E, "gate": H * E, "a1": numbers.get("rank", 0), "ig": H, "fg": H}[n]
+               for n, c in cols.items())
+    ld = _rows2(proj, "recurrence proj", torch.float32, last)
+    E1 = E + (1 if kind == _lib.LR_EXP else 0)
+    row = _state_rows(state, "recurrence state")
+    if row < H * E1 * D + (H if kind == _lib.LR_EXP else 0) or batch.num_tokens != T or out.shape[0] != T \
+            or batch.cu_tokens.numel() != batch.num_reqs + 1:
+        raise _lib.KernelError(f"recurrence: state rows of {row}, {T} rows for {H} heads of {D} x {E} and a step of "
+                               f"{batch.num_tokens} tokens")
+    if weight.numel() not in (E, H * E):
+        raise _lib.KernelError(f"recurrence: a norm weight of {weight.numel()} for {H} heads of {E}")
+    _req(weight, "recurrence norm weight", torch.float32, 1)
+    out_row = _rows2(out, "recurrence out", out.dtype, H * E)
+    if T == 0:
+        return out
+    base = proj.data_ptr()
+    a = _lib.Recurrence(kind=kind, ld=ld, R=batch.num_reqs, H=H, D=D, E=E, w=weight.data_ptr(),
+                        w_per_head=1 if weight.numel() == H * E and H > 1 else 0,
+                        sigmoid_gate=1 if gate_sigmoid else 0, eps=float(eps), state=state.data_ptr(), state_row=row,
+                        cu_tokens=batch.cu_tokens.data_ptr(), state_slots=batch.state_slots.data_ptr(), out=out.data_ptr(),
+                        out_row=out_row, out_dtype=dtype_code(out.dtype), out_scale=float(out_scale),
+                        **{n: base + 4 * c for n, c in cols.items()}, **{n: t.data_ptr() for n, t in vectors.items()}, **numbers)
+    L = _lib.load()
+    if chunked is None:
+        chunked = batch.max_new_tokens >= RECURRENCE_LONG_PORTION
+    if not chunked:
+        _lib.check(L.tff_recurrence_few(ctypes.byref(a), int(batch.max_new_tokens), _stream()))
+        return out
+    items, start = _token_items(batch, L.tff_recurrence_chunk(), proj.device)
+    ws_bytes = L.tff_recurrence_workspace_bytes(kind, T, items.shape[0], H, D, E)
+    ws = torch.empty(ws_bytes // 4, dtype=torch.float32, device=proj.device)
+    _lib.check(L.tff_recurrence_chunks(ctypes.byref(a), T, items.data_ptr(), start.data_ptr(), items.shape[0], ws.data_ptr(), ws_bytes,
+                                       _stream()))
+    return out
+
+
+def decay_recurrence(proj: torch.Tensor, cols: dict, a2_t: torch.Tensor, a_bias: torch.Tensor, tau: float, weight: torch.Tensor,
+                     eps: float, state: torch.Tensor, batch, H: int, D: int, E: int, out: torch.Tensor, out_scale: float = 1.0,
+                     q_scale: float = 1.0, sigmoid_gate: bool = False, chunked: bool | None = None) -> torch.Tensor:
+    """A linear recurrence with a decay per key channel, over each request's tokens of the step, per head:
+
+        z = A2 a1 + a_bias,  alpha = sigmoid(z)^(1/tau);  S <- diag(alpha) S + k v^T,  o = S^T (q_scale q)
+        out = o / sqrt(mean over the head of o^2 + eps) * weight * gate * out_scale,   gate = silu(g) or sigmoid(g)
+
+    ``proj`` float32 (rows may be strided) holds the columns q, k [H D], v, gate [H E] and a1 [rank] from ``cols[name]`` on;
+    ``a2_t`` float32 [rank, H D] (A2 transposed), ``weight`` [E] or [H E].  S lies transposed, [H][E][D], at the start of
+    the request's row of ``state`` (float32).  ``out`` [T, >= H E] in either type (rows may be strided).
+    ``chunked``: in chunks of 64 tokens on the matrix cores instead of token by token (None: by the step's longest entry)."""
+    _req(a2_t, "recurrence a2", torch.float32, 2)
+    _vec(a_bias, H * D, "recurrence decay bias")
+    if a2_t.shape[1] != H * D or tau <= 0:
+        raise _lib.KernelError(f"recurrence: a2 {tuple(a2_t.shape)} for {H} heads of {D}, tau {tau}")
+    return _recurrence(_lib.LR_DECAY, proj, cols, H, D, E, sigmoid_gate, weight, eps, state, batch, out, out_scale, chunked,
+                       {"a2": a2_t, "a_bias": a_bias}, {"rank": a2_t.shape[0], "inv_tau": 1.0 / tau, "q_scale": float(q_scale)})
+
+
+def exp_gate_recurrence(proj: torch.Tensor, cols: dict, i_bias: torch.Tensor, f_bias: torch.Tensor, cap: float, weight: torch.Tensor,
+                        eps: float, state: torch.Tensor, batch, H: int, D: int, E: int, out: torch.Tensor, out_scale: float = 1.0,
+                        q_scale: float = 1.0, den_eps: float = 1e-6, sigmoid_gate: bool = True,
+                        chunked: bool | None = None) -> torch.Tensor:
+    """A linear recurrence with exponential gates per head and a running maximum m (zero at the start):
+
+        i = cap tanh((zi + i_bias) / cap),  f = logsigmoid(cap tanh((zf + f_bias) / cap)),  m' = max(f + m, i)
+        S <- exp(f + m - m') S + exp(i - m') k v^T,  n <- the same with k alone,  o = S^T q / (max(|n . q|, exp(-m')) + den_eps)
+
+    with q times q_scale; then norm, weight and gate as in :func:`decay_recurrence`.  ``proj`` holds the columns q, k, v, gate, ig [H]
+    and fg [H]; the state row [H][E + 1][D] (the last value channel is n), then m [H]."""
+    _vec(i_bias, H, "recurrence input gate bias")
+    _vec(f_bias, H, "recurrence forget gate bias")
+    return _recurrence(_lib.LR_EXP, proj, cols, H, D, E, sigmoid_gate, weight, eps, state, batch, out, out_scale, chunked,
+                       {"i_bias": i_bias, "f_bias": f_bias}, {"cap": float(cap), "den_eps": float(den_eps), "q_scale": float(q_scale)})
+
+
 def grouped_qkv_store(proj: torch.Tensor, H: int, G: int, D: int, E: int, cos_sin: torch.Tensor | None, pairing: int,
-                      temp: tuple, positions: torch.Tensor, kv, store: bool = True) -> torch.Tensor:
+                      temp: tuple, positions: torch.Tensor, kv, store: bool = True, bias: torch.Tensor | None = None,
+                      q_norm: torch.Tensor | None = None, k_norm: torch.Tensor | None = None, eps: float = 0.0) -> torch.Tensor:
     """Queries, keys and values of a grouped attention from their projections, ``proj`` float32 [T, >= H D (+ G D + G E
     with ``store``)] (rows may be strided): the first ``2 * cos_sin.shape[1]`` elements of every head of q and k rotated,
     q times 1 + coef ln(floor((p + 1) / every) + 1) for ``temp`` = (coef, every).  Returns q [T, H P] in the cache's type,
     P the cache's head size, zeros behind a head's D elements; with ``store`` the token's key and value rows go to
-    its slot of ``kv``."""
+    its slot of ``kv``.  ``bias`` (float32, one number a column): added first; ``q_norm`` [H D], ``k_norm`` [G D] (float32): an
+    RMS norm (``eps``) over the whole of a token's q and of its k, before the rotation."""
     cols = H * D + (G * (D + E) if store else 0)
     T = proj.shape[0]
     row = _rows2(proj, "grouped_qkv_store proj", torch.float32, cols)
@@ -1718,10 +1851,13 @@ def grouped_qkv_store(proj: torch.Tensor, H: int, G: int, D: int, E: int, cos_si
     _req(kv.slot_mapping, "slot_mapping", torch.int32, 1)
     if P < D or P < E or positions.numel() < T or kv.slot_mapping.numel() < T:
         raise _lib.KernelError(f"grouped_qkv_store: a cache head of {P} for {D} and {E}, or fewer positions than tokens")
+    _vec(bias, cols, "grouped_qkv_store bias")
+    _vec(q_norm, H * D, "grouped_qkv_store q norm")
+    _vec(k_norm, G * D, "grouped_qkv_store k norm")
     q = torch.empty(T, H * P, dtype=k_cache.dtype, device=proj.device)
     _lib.check(_lib.load().tff_grouped_qkv_store(
-        proj.data_ptr(), row, _ptr(cos_sin), dims, int(pairing), max_pos, float(temp[0]), int(temp[1]), positions.data_ptr(),
-        kv.slot_mapping.data_ptr(), q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), k_cache.shape[2], k_cache.shape[0], T, H, G,
+        proj.data_ptr(), row, _ptr(cos_sin), dims, int(pairing), max_pos, float(temp[0]), int(temp[1]), _ptr(bias),
+        _ptr(q_norm), _ptr(k_norm), float(eps), positions.data_ptr(), kv.slot_mapping.data_ptr(), q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), k_cache.shape[2], k_cache.shape[0], T, H, G,
         D, E, P, 1 if store else 0, dtype_code(k_cache.dtype), _stream()))
     return q
 
@@ -1757,17 +1893,22 @@ def pool_keys(kv, batch, pool: int) -> None:
         batch.positions.data_ptr(), kv.slot_mapping.data_ptr(), _ptr(tokens), ps, pages, int(pool), T, G, d, dtype_code(k_cache.dtype), _stream()))
 
 
-def gate_heads(o: torch.Tensor, P: int, gate: torch.Tensor | None, H: int, E: int) -> torch.Tensor:
+def gate_heads(o: torch.Tensor, P: int, gate: torch.Tensor | None, H: int, E: int, out: torch.Tensor | None = None,
+               scale: float = 1.0) -> torch.Tensor:
     """The first E elements of every head of ``o`` (heads P apart) side by side, [T, H E], times sigmoid(gate[:, h])
-    (float32 [T, >= H], rows may be strided; None: as they are)."""
+    (float32 [T, >= H], rows may be strided; None: no gate) and ``scale``, into ``out`` if given (rows may be strided)."""
     T = o.shape[0]
     o_row = _rows2(o, "gate_heads o", o.dtype, H * P)
     g_row = _rows2(gate, "gate_heads gate", torch.float32, H) if gate is not None else 0
     if P < E or (gate is not None and gate.shape[0] != T):
         raise _lib.KernelError("gate_heads: o and gate must have one row per token and heads that hold E elements")
-    out = torch.empty(T, H * E, dtype=o.dtype, device=o.device)
-    _lib.check(_lib.load().tff_gate_heads(o.data_ptr(), o_row, int(P), _ptr(gate), g_row, out.data_ptr(), T, H, E,
-                                          dtype_code(o.dtype), _stream()))
+    if out is None:
+        out = torch.empty(T, H * E, dtype=o.dtype, device=o.device)
+    elif out.shape[0] != T:
+        raise _lib.KernelError("gate_heads: the result needs one row per token")
+    out_row = _rows2(out, "gate_heads out", o.dtype, H * E)
+    _lib.check(_lib.load().tff_gate_heads(o.data_ptr(), o_row, int(P), _ptr(gate), g_row, float(scale), out.data_ptr(), out_row, T, H,
+                                          E, dtype_code(o.dtype), _stream()))
     return out
 
 
@@ -1968,8 +2109,10 @@ def linear_swiglu_bias(x: torch.Tensor, weight, bias: torch.Tensor) -> torch.Ten
     return swiglu(linear(x, weight), bias=bias)
 
 
-def swiglu(gate_up: torch.Tensor, out: torch.Tensor | None = None, bias: torch.Tensor | None = None) -> torch.Tensor:
-    """``silu(gate) * up`` for gate_up [T, 2I] = [gate | up] (plus ``bias`` float32 [2I], if given)."""
+def swiglu(gate_up: torch.Tensor, out: torch.Tensor | None = None, bias: torch.Tensor | None = None,
+           act: tuple = SILU) -> torch.Tensor:
+    """``silu(gate) * up`` for gate_up [T, 2I] = [gate | up] (plus ``bias`` float32 [2I], if given).  ``act`` = (limit,
+    alpha, up_offset): g sigmoid(alpha g) (u + up_offset) with g = min(gate, limit), u = clamp(up, -limit, limit)."""
     _req(gate_up, "swiglu input", ndim=2)
     T, two_i = gate_up.shape
     if two_i % 2:
@@ -1982,7 +2125,8 @@ def swiglu(gate_up: torch.Tensor, out: torch.Tensor | None = None, bias: torch.T
     if out is None:
         out = torch.empty(T, I, dtype=gate_up.dtype, device=gate_up.device)
     L = _lib.load()
-    _lib.check(L.tff_swiglu(gate_up.data_ptr(), _ptr(bias), out.data_ptr(), T, I, dtype_code(gate_up.dtype), _stream()))
+    _lib.check(L.tff_swiglu(gate_up.data_ptr(), _ptr(bias), out.data_ptr(), T, I, *(float(x) for x in act),
+                            dtype_code(gate_up.dtype), _stream()))
     return out
 
 

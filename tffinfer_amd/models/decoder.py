@@ -14,7 +14,7 @@ import torch
 
 from ..config.base import ModelConfig
 from ..parts.base import BLOCKS, FEED_FORWARDS, MIXERS, NORMS, Part, StateSpec, WeightSpec
-from ..parts.embedding import Embedding, OutputHead
+from ..parts.embedding import BigramTable, Embedding, OutputHead
 from ..weights.loader import check_weights, normalize_stored
 from ..weights.random_init import FLOAT32_INITS, random_tensor
 
@@ -28,6 +28,8 @@ class TensorNames:
     head: str = "lm_head"
     #: the table of vectors the run order adds to the stream, for architectures that have one
     stream_offsets: str = "stream_offsets"
+    #: the embedding's table for pairs of tokens, for architectures that have one
+    bigram: str = "bigram"
     #: the block's children by the name the files use
     children: dict = field(default_factory=dict)
     #: tensors a file may hold that the model has no use for
@@ -79,8 +81,10 @@ class DecoderModel:
         self.device = None
         H, V = config.hidden_size, config.vocab_size
         emb_norm = config.embedding_norm_spec() if hasattr(config, "embedding_norm_spec") else None
+        pairs = config.bigram_spec() if hasattr(config, "bigram_spec") else None
         self.embedding = Embedding(V, H, scale=getattr(config, "embedding_scale", 1.0),
-                                   norm=NORMS.build(emb_norm) if emb_norm is not None else None)
+                                   norm=NORMS.build(emb_norm) if emb_norm is not None else None,
+                                   bigram=BigramTable(hidden_size=H, **pairs) if pairs is not None else None)
         n_off = config.stream_offset_rows() if hasattr(config, "stream_offset_rows") else 0
         self.stream_offsets = StreamOffsets(n_off, H) if n_off else None
         self.blocks = []
@@ -104,6 +108,10 @@ class DecoderModel:
             if call.offset >= (self.stream_offsets.rows if self.stream_offsets else 0):
                 raise ValueError(f"layer schedule names stream offset {call.offset}, the model has "
                                  f"{self.stream_offsets.rows if self.stream_offsets else 0}")
+            if call.add_embedding and call.offset >= 0:
+                raise ValueError("a layer call adds the embedding's output or a row of the table of offsets, not both")
+        #: some call adds the embedding's output to the stream: it is kept beside it
+        self.keeps_embedding = any(call.add_embedding for call in self.schedule)
         self.final_norm = NORMS.build(config.final_norm_spec())
         self.head = OutputHead(V, H, self.embedding if config.tie_word_embeddings else None,
                                softcap=getattr(config, "logit_softcap", None),
@@ -112,6 +120,8 @@ class DecoderModel:
     # ---- weights ---------------------------------------------------------
     def _weighted_parts(self):
         yield from _leaves(self.names.embedding, self.embedding, {})
+        if self.embedding.bigram is not None:
+            yield self.names.bigram, self.embedding.bigram
         if self.stream_offsets is not None:
             yield self.names.stream_offsets, self.stream_offsets
         for i, block in zip(self.layer_numbers, self.blocks):
@@ -199,12 +209,16 @@ class DecoderModel:
     # ---- cache needs -----------------------------------------------------
     def call_requirements(self):
         """For every entry of the run order: (cache id, writes, KVCacheSpec or
-        None, StateSpec or None), and the state's id where it is not the cache's."""
+        None, StateSpec or None), and the state's id where it is not the cache's.  Where the embedding carries state,
+        a row of its own follows those of the run order."""
         out = []
         for call in self.schedule:
             block = self.blocks[call.layer]
             row = (call.cache, call.writes_cache, block.mixer.cache_spec(), self.call_state(block))
             out.append(row if call.state < 0 or call.state == call.cache else row + (call.state,))
+        own = self.embedding.state_spec()
+        if own is not None:
+            out.append((1 + max(max(call.cache, call.state) for call in self.schedule), True, None, own))
         return out
 
     @staticmethod
@@ -238,7 +252,12 @@ class DecoderModel:
         logits = None
         for it in items:
             if it == "embed":
-                resid, pending = self.embedding.forward(ctx, b.token_ids), None
+                c = ctx.for_call(len(self.schedule)) if self.embedding.state_spec() is not None else ctx
+                pending = None
+                if self.keeps_embedding:
+                    resid, b.embedding_output = self.embedding.forward_kept(c, b.token_ids)
+                else:
+                    resid = self.embedding.forward(c, b.token_ids)
             elif it == "finish":
                 if b.num_logit_rows == 0:
                     logits = torch.empty(0, self.config.vocab_size, dtype=torch.float32, device=resid.device)
@@ -248,13 +267,14 @@ class DecoderModel:
             else:
                 call = self.schedule[it]
                 block, c = self.blocks[call.layer], ctx.for_call(it)
-                if call.offset >= 0:
+                if call.offset >= 0 or call.add_embedding:
+                    extra = b.embedding_output if call.add_embedding else self.stream_offsets.row(call.offset)
                     if getattr(block, "takes_stream_offset", False):
-                        c.stream_offset = self.stream_offsets.row(call.offset)
+                        c.stream_offset = extra
                     else:       # a block that knows nothing of offsets finds them in the stream
                         if pending is not None:
                             resid += ctx.ops.as_tensor(pending)
                             pending = None
-                        resid += self.stream_offsets.row(call.offset)
+                        resid += extra
                 pending = block.forward(c, resid, pending)
         return resid, pending, logits

@@ -333,12 +333,17 @@ class DifferentialAttention(Mixer):
 
 @register_mixer("grouped_attention")
 class GroupedAttention(Mixer):
-    """Grouped-query attention with queries, keys and values of sizes of their own, without a norm on them:
+    """Grouped-query attention with queries, keys and values of sizes of their own:
 
         q_h = temp(p) rot(Wq x)_h,  k_g = rot(Wk x)_g  (heads of ``head_dim``),  v_g = (Wv x)_g  (``value_dim``)
         temp(p) = 1 + q_temp_coef * ln(floor((p + 1) / q_temp_every) + 1)       (coef 0: 1)
         y_h(i) = sum over what i sees of softmax(scale q_h(i) . key) value,   g = h // (heads / kv_heads)
         out = Wo [y_h sigmoid(Wg x)_h]_h            (``head_gate``: one number per head; else no gate)
+
+    ``bias``: Wq, Wk and Wv have biases (``q.b``, ``k.b``, ``v.b``); ``output_bias``: Wo has one (``o.b``), left to whoever adds
+    the result to the stream.  ``qk_norm_eps``: before the rotation an RMS norm over the whole of q (all heads at once) and
+    of k, with weights as long (``q.norm``, ``k.norm``).  ``sinks``: a number per query head (``sink``) whose exponential is
+    one more term of its softmax's denominator, without a key or value, not scaled.
 
     What position i sees: every j <= i; with a ``window`` the j with i - j < window; and with a ``pool`` P
     beside them one key and one value per block of P tokens that lies wholly before the window: the means
@@ -352,16 +357,21 @@ class GroupedAttention(Mixer):
     The attention proper runs on the paged kernels with one head size for keys and values, the larger of the
     two brought up to a size they take.  The projections' results stay float32 until temperature and
     rotation are done (``ops.grouped_qkv_store``).  ``external``: the mixer is one of several that read the same
-    rows; whoever combines them forms all their projections in one product and calls ``forward_projected``.
+    rows; whoever combines them forms all their projections in one product and calls ``forward_projected``, or with
+    ``external_output`` ``inner_projected``, which stops before Wo (``w_o_host`` is the combiner's then).
     """
 
     graph_safe = True
     input_goes_to_linear = True
+    #: a combiner may form this mixer's projections and apply its output matrix
+    joint_input = True
 
     def __init__(self, hidden_size: int, num_heads: int, num_kv_heads: int, head_dim: int, value_dim: int,
                  position=None, scale: float | None = None, window: int = 0, pool: int = 0,
                  cache_window: int | None = None, cache_pools: tuple | None = None, shared_cache: bool = False,
-                 head_gate: bool = False, q_temp_coef: float = 0.0, q_temp_every: int = 1, external: bool = False):
+                 head_gate: bool = False, q_temp_coef: float = 0.0, q_temp_every: int = 1, external: bool = False,
+                 bias: bool = False, output_bias: bool = False, qk_norm_eps: float | None = None, sinks: bool = False,
+                 external_output: bool = False):
         self.hidden_size = int(hidden_size)
         self.num_heads = int(num_heads)
         self.num_kv_heads = int(num_kv_heads)
@@ -393,8 +403,15 @@ class GroupedAttention(Mixer):
             raise ConfigError(f"grouped attention: {position.rotary_dim} rotated elements of a head of {self.head_dim}")
         self.position = position
         self.external = bool(external)
+        self.external_output = bool(external_output)
+        self.has_bias, self.has_output_bias, self.has_sinks = bool(bias), bool(output_bias), bool(sinks)
+        self.qk_norm_eps = None if qk_norm_eps is None else float(qk_norm_eps)
+        if self.shared_cache and (self.has_bias or self.qk_norm_eps is not None):
+            raise ConfigError("grouped attention: a layer that reads another's cache has neither biases nor a norm on q and k")
+        if self.external_output and self.has_output_bias:
+            raise ConfigError("grouped attention: an output matrix that is left to a combiner has no bias")
         self._dtype = torch.bfloat16
-        self.w_in = self.w_o = None
+        self.w_in = self.w_o = self.w_o_host = self.in_bias = self.out_bias = self.q_norm = self.k_norm = self.sinks = None
 
     # ---- sizes -----------------------------------------------------------
     def padded_head_dim(self) -> int:
@@ -406,6 +423,11 @@ class GroupedAttention(Mixer):
         """Columns of the joint projection: q, then k and v (unless shared), then the gate."""
         n = self.num_heads * self.head_dim + (self.num_heads if self.has_gate else 0)
         return n + (0 if self.shared_cache else self.num_kv_heads * (self.head_dim + self.value_dim))
+
+    @property
+    def inner_size(self) -> int:
+        """Columns of what ``inner_projected`` leaves: the input size of Wo."""
+        return self.num_heads * self.value_dim
 
     def cache_spec(self):
         return KVCacheSpec(self.num_kv_heads, self.padded_head_dim(), self.cache_window, pools=self.cache_pools)
@@ -421,6 +443,15 @@ class GroupedAttention(Mixer):
         if self.has_gate:
             specs["g"] = WeightSpec((H, W))
         specs["o"] = WeightSpec((W, H * E))
+        if self.has_bias:
+            specs |= {"q.b": WeightSpec((H * D,), "norm_offset"), "k.b": WeightSpec((G * D,), "norm_offset"),
+                      "v.b": WeightSpec((G * E,), "norm_offset")}
+        if self.has_output_bias:
+            specs["o.b"] = WeightSpec((W,), "norm_offset")
+        if self.qk_norm_eps is not None:
+            specs |= {"q.norm": WeightSpec((H * D,), "norm"), "k.norm": WeightSpec((G * D,), "norm")}
+        if self.has_sinks:
+            specs["sink"] = WeightSpec((H,), "vector")
         return specs
 
     def stacked(self, weights) -> list:
@@ -432,27 +463,46 @@ class GroupedAttention(Mixer):
         if not self.external:
             w = self.stacked(weights)
             self.w_in = to_device(torch.cat([t.to(w[0].dtype) for t in w], 0), dtype, device)
-        self.w_o = to_device(weights["o"], dtype, device)
+        if self.external_output:
+            self.w_o_host = weights["o"]
+        else:
+            self.w_o = to_device(weights["o"], dtype, device)
+        f32 = lambda t: t.to(torch.float32).contiguous().to(device)      # noqa: E731
+        if self.has_bias:       # in the order of the joint product's columns
+            self.in_bias = f32(torch.cat([weights[n].to(torch.float32) for n in ("q.b", "k.b", "v.b")], 0))
+        if self.has_output_bias:
+            self.out_bias = f32(weights["o.b"])
+        if self.qk_norm_eps is not None:
+            self.q_norm, self.k_norm = f32(weights["q.norm"]), f32(weights["k.norm"])
+        if self.has_sinks:
+            self.sinks = f32(weights["sink"])
 
-    def forward_projected(self, ctx, proj):
-        """From the joint projection (float32 [T, >= columns], rows may be strided) to the mixer's output."""
+    def inner_projected(self, ctx, proj, out=None, out_scale: float = 1.0):
+        """From the joint projection (float32 [T, >= columns], rows may be strided) to the input of Wo, [T, heads *
+        value_dim] in the activation type, into ``out`` if given (rows may be strided), times ``out_scale``."""
         ops, kv, b = ctx.ops, ctx.kv, ctx.batch
         H, G, D, E = self.num_heads, self.num_kv_heads, self.head_dim, self.value_dim
         P = kv.k_cache.shape[3]
         table = self.position.cached_table(ctx.max_positions, proj.device) if self.position is not None else None
         pairing = 1 if (self.position is not None and self.position.pairing == "interleaved") else 0
         q = ops.grouped_qkv_store(proj, H, G, D, E, table, pairing, (self.q_temp_coef, self.q_temp_every), b.positions, kv,
-                                  store=not self.shared_cache)
+                                  store=not self.shared_cache, bias=self.in_bias, q_norm=self.q_norm, k_norm=self.k_norm,
+                                  eps=self.qk_norm_eps or 0.0)
         if not self.shared_cache:
             for p in self.cache_pools:
                 ops.pool_keys(kv, b, p)
-        o = ops.paged_attention(q, H, G, P, kv, b, self.window, self.scale, pool=self.pool)
+        o = ops.paged_attention(q, H, G, P, kv, b, self.window, self.scale, sinks=self.sinks, pool=self.pool)
         gate = proj[:, self.columns - H:self.columns] if self.has_gate else None
-        if gate is not None or P != E:
-            o = ops.gate_heads(o, P, gate, H, E)
-        return ops.linear(o, self.w_o, out_dtype=torch.float32, partials=True)
+        if gate is not None or P != E or out is not None or out_scale != 1.0:
+            o = ops.gate_heads(o, P, gate, H, E, out, out_scale)
+        return o
+
+    def forward_projected(self, ctx, proj):
+        """From the joint projection to the mixer's output."""
+        y = ctx.ops.linear(self.inner_projected(ctx, proj), self.w_o, out_dtype=torch.float32, partials=True)
+        return ctx.ops.OutputTerm(y, bias=self.out_bias) if self.has_output_bias else y
 
     def forward(self, ctx, x):
-        if self.external:
-            raise RuntimeError("grouped attention: its projections were left to a combining mixer")
+        if self.external or self.external_output:
+            raise RuntimeError("grouped attention: its projections or its output matrix were left to a combining mixer")
         return self.forward_projected(ctx, ctx.ops.linear(x, self.w_in, out_dtype=torch.float32))

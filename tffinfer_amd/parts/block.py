@@ -32,6 +32,10 @@ class PreNormBlock(Block):
         return {"norm1": self.norm1, "mixer": self.mixer, "norm2": self.norm2,
                 "feed_forward": self.feed_forward}
 
+    @property
+    def takes_stream_offset(self) -> bool:
+        return getattr(self.norm1, "adds_to_stream", False)
+
     @staticmethod
     def _norm(norm, consumer, ctx, resid, pending):
         # a norm and a consumer that both say so may pass rows that still lack the norm's factor
@@ -40,7 +44,11 @@ class PreNormBlock(Block):
         return norm.forward(ctx, resid, pending)
 
     def forward(self, ctx, resid, pending):
-        h = self._norm(self.norm1, self.mixer, ctx, resid, pending)
+        add = getattr(ctx, "stream_offset", None)
+        if add is not None:
+            h = self.norm1.forward(ctx, resid, pending, extra=add)
+        else:
+            h = self._norm(self.norm1, self.mixer, ctx, resid, pending)
         a = self.mixer.forward(ctx, h)
         if not self.has_ffn:
             return a

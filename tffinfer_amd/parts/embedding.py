@@ -3,17 +3,46 @@ from __future__ import annotations
 
 import torch
 
-from .base import Part, WeightSpec, to_device
+from ..config.base import ConfigError
+from .base import Part, StateSpec, WeightSpec, to_device
+
+
+class BigramTable(Part):
+    """A table of rows for pairs of neighbouring tokens, beside the embedding's rows for single ones: token t adds the row
+    (token_(t-1) * mul_prev + token_t * mul_cur) mod buckets, a sequence's first token the last row (number buckets).
+    The last token a request brought is its state (one int32)."""
+
+    graph_safe = True
+
+    def __init__(self, buckets: int, hidden_size: int, mul_prev: int, mul_cur: int):
+        self.buckets, self.hidden_size = int(buckets), int(hidden_size)
+        self.mul_prev, self.mul_cur = int(mul_prev), int(mul_cur)
+        if self.buckets <= 0 or max(abs(self.mul_prev), abs(self.mul_cur)) >= 1 << 31:
+            raise ConfigError(f"bigram table: {buckets} rows and factors {mul_prev}, {mul_cur}")
+        self.weight = None
+
+    def weight_specs(self):
+        return {"weight": WeightSpec((self.buckets + 1, self.hidden_size), "embedding")}
+
+    def load_weights(self, weights, dtype, device):
+        self.weight = weights["weight"].to(dtype).contiguous().to(device)     # (only looked up: row-major in both types)
+
+    def state_spec(self):
+        return StateSpec((1,), torch.int32)
 
 
 class Embedding(Part):
     """x[t, :] = scale * E[token[t], :] into the float32 residual stream (scale 1: the rows
     as they are), then through ``norm`` (an RMS norm part, named ``norm`` under the table's name)
-    if there is one.  Reference: src/kernel/cpu/embedding.cpp:34-49 (a CPU lookup there)."""
+    if there is one.  Reference: src/kernel/cpu/embedding.cpp:34-49 (a CPU lookup there).
+    ``bigram``: a table of rows for pairs of tokens whose rows are added (a part with a tensor name of its own)."""
 
     graph_safe = True
 
-    def __init__(self, vocab_size: int, hidden_size: int, scale: float = 1.0, norm=None):
+    def __init__(self, vocab_size: int, hidden_size: int, scale: float = 1.0, norm=None, bigram: BigramTable | None = None):
+        self.bigram = bigram
+        if bigram is not None and (float(scale) != 1.0 or norm is not None):
+            raise ConfigError("embedding: a table for pairs of tokens goes with neither a scale nor a norm")
         self.vocab_size = int(vocab_size)
         self.hidden_size = int(hidden_size)
         self.scale = float(scale)
@@ -29,7 +58,24 @@ class Embedding(Part):
     def load_weights(self, weights, dtype, device):
         self.weight = to_device(weights["weight"], dtype, device)
 
+    def state_spec(self) -> StateSpec | None:
+        """State per request that the embedding carries from step to step."""
+        return self.bigram.state_spec() if self.bigram is not None else None
+
+    def forward_kept(self, ctx, token_ids):
+        """(rows, the same rows once more in a tensor that the layers do not add to)."""
+        if self.bigram is not None:
+            return self._with_pairs(ctx, True)
+        x = self.forward(ctx, token_ids)
+        return x, x.clone()
+
+    def _with_pairs(self, ctx, copy: bool):
+        b = self.bigram
+        return ctx.ops.bigram_embed(self.weight, b.weight, ctx.batch, ctx.state, b.mul_prev, b.mul_cur, copy=copy)
+
     def forward(self, ctx, token_ids):
+        if self.bigram is not None:
+            return self._with_pairs(ctx, False)[0]
         x = ctx.ops.embed(self.weight, token_ids)
         if self.scale != 1.0:
             ctx.ops.scale_rows(x, self.scale)       # (in float32; the table itself also serves a tied head)

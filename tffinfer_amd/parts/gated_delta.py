@@ -113,7 +113,9 @@ class MixerPair(Mixer):
     writes its part of one matrix [T, left inner + right inner], scaled by its factor, and the two output
     matrices, put side by side, make the sum one product.  One of them may keep keys and values
     (``cache_spec``) and one a state (``state_spec``); the layer call's cache and state go to both.
-    Their tensors are named ``left.*`` and ``right.*``."""
+    Their tensors are named ``left.*`` and ``right.*``.  Where both can also start from a projection that was formed for
+    them (``joint_input``: ``external`` / ``stacked`` / ``columns`` / ``inner_projected``), the input matrices of both are one
+    product too."""
 
     graph_safe = True
 
@@ -121,21 +123,26 @@ class MixerPair(Mixer):
         self.hidden_size = int(hidden_size)
         self.left_scale = float(left_scale)
         self.right_scale = float(right_scale)
+        if not (isinstance(left, PartSpec) and isinstance(right, PartSpec)):
+            raise ConfigError("mixer pair: 'left' and 'right' are the specs of two mixers")
+        # (the two mixers' projections are one product)
+        self.joint = all(getattr(MIXERS.classes.get(s.kind), "joint_input", False) for s in (left, right))
         self.left = self._build(left)
         self.right = self._build(right)
         if sum(m.cache_spec() is not None for m in (self.left, self.right)) > 1 or \
                 sum(m.state_spec() is not None for m in (self.left, self.right)) > 1:
             raise ConfigError("mixer pair: both mixers ask for a cache, or both for a state; a layer call has one of each")
-        self.w_o = None
+        self.w_in = self.w_o = None
 
-    @staticmethod
-    def _build(spec):
-        if not isinstance(spec, PartSpec):
-            raise ConfigError("mixer pair: 'left' and 'right' are the specs of two mixers")
-        m = MIXERS.build(PartSpec(spec.kind, dict(spec.args, external_output=True)))
-        if not hasattr(m, "forward_inner"):
+    def _build(self, spec):
+        m = MIXERS.build(PartSpec(spec.kind, dict(spec.args, external_output=True, **({"external": True} if self.joint else {}))))
+        if not hasattr(m, "inner_projected" if self.joint else "forward_inner"):
             raise ConfigError(f"mixer pair: a '{spec.kind}' cannot stop before its output matrix")
         return m
+
+    @property
+    def input_goes_to_linear(self) -> bool:
+        return self.joint
 
     def cache_spec(self):
         return self.left.cache_spec() or self.right.cache_spec()
@@ -152,8 +159,19 @@ class MixerPair(Mixer):
         return specs
 
     def load_weights(self, weights, dtype, device):
+        stacked, self._right_from = [], 0
         for name, m in (("left.", self.left), ("right.", self.right)):
-            m.load_weights({k[len(name):]: v for k, v in weights.items() if k.startswith(name)}, dtype, device)
+            own = {k[len(name):]: v for k, v in weights.items() if k.startswith(name)}
+            m.load_weights(own, dtype, device)
+            if self.joint:
+                # (the right one's columns start at a multiple of 16 bytes)
+                self._right_from = sum(t.shape[0] for t in stacked)
+                if self._right_from % 4:
+                    stacked.append(torch.zeros(4 - self._right_from % 4, self.hidden_size, dtype=stacked[0].dtype))
+                    self._right_from += stacked[-1].shape[0]
+                stacked += m.stacked(own)
+        if self.joint:
+            self.w_in = to_device(torch.cat([t.to(stacked[0].dtype) for t in stacked], 0), dtype, device)
         lo, ro = self.left.w_o_host, self.right.w_o_host
         self.w_o = to_device(torch.cat([lo, ro.to(lo.dtype)], 1), dtype, device)
         self.left.w_o_host = self.right.w_o_host = None
@@ -161,6 +179,11 @@ class MixerPair(Mixer):
     def forward(self, ctx, x):
         nl, nr = self.left.inner_size, self.right.inner_size
         y = torch.empty(x.shape[0], nl + nr, dtype=ctx.act_dtype, device=x.device)
+        if self.joint:
+            proj = ctx.ops.linear(x, self.w_in, out_dtype=torch.float32)
+            self.left.inner_projected(ctx, proj, y[:, :nl], self.left_scale)
+            self.right.inner_projected(ctx, proj[:, self._right_from:], y[:, nl:], self.right_scale)
+            return ctx.ops.linear(y, self.w_o, out_dtype=torch.float32, partials=True)
         self.left.forward_inner(ctx, x, y[:, :nl], self.left_scale)
         self.right.forward_inner(ctx, x, y[:, nl:], self.right_scale)
         return ctx.ops.linear(y, self.w_o, out_dtype=torch.float32, partials=True)

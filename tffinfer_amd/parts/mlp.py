@@ -15,6 +15,8 @@ class SwiGLU(FeedForward):
     Gate and up are put into one matrix at load so that one product streams both.
     ``bias``: all three projections have one (``<name>.b``, float32 where it is added), f =
     Wdown (silu(Wgate z + bg) * (Wup z + bu)) + bd; the last one is left to whoever adds f to the stream.
+    ``limit``, ``act_alpha``, ``up_offset``: the activation with constants instead, g = min(Wgate z, limit), u = clamp(Wup z,
+    -limit, limit), f = Wdown (g sigmoid(act_alpha g) (u + up_offset)).
     """
 
     graph_safe = True
@@ -22,7 +24,8 @@ class SwiGLU(FeedForward):
     input_goes_to_linear = True
 
     def __init__(self, hidden_size: int, intermediate_size: int,
-                 names=("gate_proj.weight", "up_proj.weight", "down_proj.weight"), bias: bool = False):
+                 names=("gate_proj.weight", "up_proj.weight", "down_proj.weight"), bias: bool = False,
+                 limit: float | None = None, act_alpha: float = 1.0, up_offset: float = 0.0):
         self.hidden_size = int(hidden_size)
         self.intermediate_size = int(intermediate_size)
         self.names = tuple(names)       # how the files call gate, up and down
@@ -30,6 +33,10 @@ class SwiGLU(FeedForward):
             from ..config.base import ConfigError
             raise ConfigError("swiglu: 'names' are the names of gate, up and down")
         self.has_bias = bool(bias)
+        self.act = (float("inf") if limit is None else float(limit), float(act_alpha), float(up_offset))
+        if self.has_bias and self.act != (float("inf"), 1.0, 0.0):
+            from ..config.base import ConfigError
+            raise ConfigError("swiglu: biases go with silu(gate) * up")
         self.w_gate_up = None
         self.w_down = None
         self.gate_up_bias = self.down_bias = None
@@ -62,7 +69,7 @@ class SwiGLU(FeedForward):
             # product streams both and applies silu(gate) * up to its float32 accumulators
             from ..kernels import ops
             self.w_gate_up = ops.pack_gate_up(gate.to(dtype).contiguous().to(device),
-                                              up.to(dtype).contiguous().to(device))
+                                              up.to(dtype).contiguous().to(device), self.act)
         else:
             # float32: gate and up stacked to [2I, H]; the activation is a kernel of its own
             self.w_gate_up = to_device(torch.cat([gate, up], 0), dtype, device)
@@ -74,7 +81,7 @@ class SwiGLU(FeedForward):
             return ctx.ops.OutputTerm(ctx.ops.linear(m, self.w_down, out_dtype=torch.float32, partials=True),
                                       bias=self.down_bias)
         gu = ctx.ops.linear(x, self.w_gate_up)
-        m = gu if getattr(self.w_gate_up, "glu_out", 0) else ctx.ops.swiglu(gu)
+        m = gu if getattr(self.w_gate_up, "glu_out", 0) else ctx.ops.swiglu(gu, act=self.act)
         return ctx.ops.linear(m, self.w_down, out_dtype=torch.float32, partials=True)
 
 
@@ -143,6 +150,11 @@ class RoutedExperts(FeedForward):
     instead of what comes out.
     ``identity``: that many experts more, behind the others in the router's outputs, have no matrices and hand
     their input on, f_e = z.
+    ``groups``, ``keep_groups``: neighbouring experts form ``groups`` equal groups, a group's score is the sum of its two
+    largest s + b, and only experts of the ``keep_groups`` best groups can be chosen.  ``weight_scale``: w_e is multiplied by it.
+    ``shared``: the inner size of one more expert (``shared.gate``, ``shared.up``, ``shared.down``) that every token uses, with the
+    weight sigmoid(Wsg z) (``shared.sg``, one row).  Its hidden units lie behind the others' in the stacked matrices, cut into
+    experts of ``intermediate_size`` (the last one filled up with zeros), and run in the same launches.
 
     The experts' matrices lie stacked, [experts, out, in], so that a kernel finds an expert's
     rows by its number."""
@@ -152,8 +164,12 @@ class RoutedExperts(FeedForward):
     def __init__(self, hidden_size: int, intermediate_size: int, num_experts: int, top: int,
                  limit: float | None, act_alpha: float = 1.702, correction: bool = True,
                  router_softmax: bool = False, up_offset: float = 1.0, normalize: bool = True,
-                 weight_input: bool = False, identity: int = 0):
+                 weight_input: bool = False, identity: int = 0, groups: int = 1, keep_groups: int = 1,
+                 weight_scale: float = 1.0, shared: int = 0):
         self.identity = int(identity)
+        self.groups, self.keep_groups = int(groups), int(keep_groups)
+        self.weight_scale = float(weight_scale)
+        self.shared = int(shared)
         self.router_softmax = bool(router_softmax)
         self.normalize = bool(normalize)
         self.weight_input = bool(weight_input)
@@ -172,6 +188,20 @@ class RoutedExperts(FeedForward):
         if self.identity and self.weight_input:
             from ..config.base import ConfigError
             raise ConfigError("routed experts: experts that hand their input on take the weight on their output")
+        if self.groups < 1 or (self.num_experts + self.identity) % self.groups or not 1 <= self.keep_groups <= self.groups \
+                or self.top > self.keep_groups * ((self.num_experts + self.identity) // self.groups):
+            from ..config.base import ConfigError
+            raise ConfigError(f"routed experts: top={self.top} from {self.keep_groups} of {self.groups} groups of "
+                              f"{self.num_experts + self.identity} experts")
+        if self.shared < 0 or (self.shared and (self.identity or self.weight_input)):
+            from ..config.base import ConfigError
+            raise ConfigError("routed experts: a shared expert goes neither with experts that hand their input on nor with "
+                              "weights on the input")
+        #: experts of ``intermediate_size`` that the shared one is cut into
+        self.shared_parts = -(-self.shared // self.intermediate_size)
+        if self.top + self.shared_parts > 64:
+            from ..config.base import ConfigError
+            raise ConfigError(f"routed experts: {self.top} chosen experts and {self.shared_parts} parts of a shared one (up to 64)")
         self.w_gate = self.w_up = self.w_down = self.router = self.router_w = self.correction = None
 
     def weight_specs(self):
@@ -184,14 +214,17 @@ class RoutedExperts(FeedForward):
             specs[f"e{e}.gate"] = WeightSpec((I, H))
             specs[f"e{e}.up"] = WeightSpec((I, H))
             specs[f"e{e}.down"] = WeightSpec((H, I))
+        if self.shared:
+            specs |= {"shared.gate": WeightSpec((self.shared, H)), "shared.up": WeightSpec((self.shared, H)),
+                      "shared.down": WeightSpec((H, self.shared)), "shared.sg": WeightSpec((1, H))}
         return specs
 
     def active_matrix_elements(self) -> int:
-        """Matrix elements a token multiplies with: the router and its ``top`` experts."""
+        """Matrix elements a token multiplies with: the router and its ``top`` experts (and the shared one)."""
         H, I = self.hidden_size, self.intermediate_size
         # (on average over the experts, where some have no matrices)
         share = self.num_experts / (self.num_experts + self.identity)
-        return (self.num_experts + self.identity) * H + round(self.top * share * 3 * H * I)
+        return (self.num_experts + self.identity) * H + round(self.top * share * 3 * H * I) + 3 * H * self.shared
 
     def streamed_matrix_elements(self, rows: int) -> int:
         """Matrix elements a step of ``rows`` tokens reads at least: the router and as many
@@ -199,37 +232,51 @@ class RoutedExperts(FeedForward):
         H, I = self.hidden_size, self.intermediate_size
         share = self.num_experts / (self.num_experts + self.identity)
         return ((self.num_experts + self.identity) * H
-                + round(min(self.num_experts, rows * self.top * share) * 3 * H * I))
+                + round(min(self.num_experts, rows * self.top * share) * 3 * H * I) + 3 * H * self.shared)
 
     def load_weights(self, weights, dtype, device):
-        E = self.num_experts
+        E, I = self.num_experts, self.intermediate_size
 
         def stack(which):
             from ..kernels.ops import pad_expert_rows
-            return pad_expert_rows(torch.stack([weights[f"e{e}.{which}"].to(dtype) for e in range(E)], 0)).to(device)
+            mats = [weights[f"e{e}.{which}"].to(dtype) for e in range(E)]
+            if self.shared:
+                w = weights[f"shared.{which}"].to(dtype)
+                fill = self.shared_parts * I - self.shared
+                if which == "down":
+                    mats += torch.nn.functional.pad(w, (0, fill)).split(I, 1)
+                else:
+                    mats += torch.nn.functional.pad(w, (0, 0, 0, fill)).split(I, 0)
+            return pad_expert_rows(torch.stack(mats, 0)).to(device)
 
         self.w_gate, self.w_up, self.w_down = stack("gate"), stack("up"), stack("down")
+        router = weights["router"]
+        if self.shared:         # (the shared expert's gate is one more row of the router)
+            sg = weights["shared.sg"]
+            kind = router.dtype if router.dtype == sg.dtype else torch.float32
+            router = torch.cat([router.to(kind), sg.to(kind)], 0)
         # The router's logits are float32 sums.  A router stored in bfloat16 multiplies exactly with
         # bfloat16 rows on the matrix cores (the products of two bfloat16 numbers are float32 numbers,
         # the sums are float32): the engine's own product serves.  One stored in more bits keeps them,
         # and the routing kernel forms the logits itself.
         self.router_w = None
-        if dtype == torch.float32 or weights["router"].dtype == torch.bfloat16:
-            self.router_w = to_device(weights["router"], dtype, device)
-        self.router = weights["router"].to(torch.float32).contiguous().to(device) if self.router_w is None else None
+        if dtype == torch.float32 or router.dtype == torch.bfloat16:
+            self.router_w = to_device(router, dtype, device)
+        self.router = router.to(torch.float32).contiguous().to(device) if self.router_w is None else None
         self.correction = (weights["correction"].to(torch.float32).contiguous().to(device)
                            if self.has_correction else None)
 
     def forward(self, ctx, x):
         ops = ctx.ops
         x = ops.as_tensor(x)
+        how = {"softmax": self.router_softmax, "normalize": self.normalize}
+        if self.groups > 1 or self.weight_scale != 1.0 or self.shared:
+            how |= {"groups": self.groups, "keep_groups": self.keep_groups, "scale": self.weight_scale, "shared": self.shared_parts}
         if self.router_w is not None:
             idx, wts = ops.route_topk(None, None, self.correction, self.top,
-                                      logits=ops.linear(x, self.router_w, out_dtype=torch.float32),
-                                      softmax=self.router_softmax, normalize=self.normalize)
+                                      logits=ops.linear(x, self.router_w, out_dtype=torch.float32), **how)
         else:
-            idx, wts = ops.route_topk(x, self.router, self.correction, self.top, softmax=self.router_softmax,
-                                      normalize=self.normalize)
+            idx, wts = ops.route_topk(x, self.router, self.correction, self.top, **how)
         return ops.routed_experts(x, self.w_gate, self.w_up, self.w_down, idx, wts, self.limit, self.act_alpha,
                                   up_offset=self.up_offset, weight_input=self.weight_input,
                                   **({"identity": self.identity} if self.identity else {}))

@@ -134,35 +134,40 @@ class DynamicTanh(Norm):
 class LayerNorm(Norm):
     """y = (v - mean(v)) / sqrt(variance + eps) * w + b over rows of ``size`` elements, the variance being the mean
     of the squared deviations; v is the residual stream plus the term still pending.  float32 throughout.  The
-    tensors are called ``weight`` and ``b``.  ``optional``: a file may leave them out (the norm of a sublayer that
-    a layer does not have)."""
+    tensors are called ``weight`` and ``b`` (``has_bias`` False: there is no b).  ``optional``: a file may leave them out
+    (the norm of a sublayer that a layer does not have)."""
 
     graph_safe = True
+    #: ``forward`` takes ``extra``: rows (or one row for all) that are added to the stream beside ``delta``
+    adds_to_stream = True
 
-    def __init__(self, size: int, eps: float, optional: bool = False):
+    def __init__(self, size: int, eps: float, optional: bool = False, has_bias: bool = True):
         self.size = int(size)
         self.eps = float(eps)
         self.optional = bool(optional)
+        self.has_bias = bool(has_bias)
         self.weight = self.bias = None
 
     def weight_specs(self):
-        return {"weight": WeightSpec((self.size,), "norm", optional=self.optional),
-                "b": WeightSpec((self.size,), "norm_offset", optional=self.optional)}
+        specs = {"weight": WeightSpec((self.size,), "norm", optional=self.optional)}
+        if self.has_bias:
+            specs["b"] = WeightSpec((self.size,), "norm_offset", optional=self.optional)
+        return specs
 
     def load_weights(self, weights, dtype, device):
-        if not all(k in weights for k in ("weight", "b")):
+        if not all(k in weights for k in self.weight_specs()):
             self.weight = self.bias = None
             return
         self.weight = weights["weight"].to(torch.float32).contiguous().to(device)
-        self.bias = weights["b"].to(torch.float32).contiguous().to(device)
+        self.bias = weights["b"].to(torch.float32).contiguous().to(device) if self.has_bias else None
 
     def output_term(self, ctx, delta, scale=None):
         """A sublayer's result on its way into the stream through this norm (then times ``scale`` [size], if
         given), for the norm that adds it there (``ops.OutputTerm``)."""
         return ctx.ops.output_term(delta, norm=(self.weight, self.bias, self.eps), scale=scale)
 
-    def forward(self, ctx, resid, delta, rows=None, for_linear=False, conv=None):
+    def forward(self, ctx, resid, delta, rows=None, for_linear=False, conv=None, extra=None):
         """``conv`` (weights [taps, size], the layer call's state, where in a state row the convolution's inputs
         lie): the rows leave with their causal convolution over time added."""
         return ctx.ops.add_layernorm(resid, delta, self.weight, self.bias, self.eps, ctx.act_dtype, rows=rows,
-                                     conv=conv, batch=ctx.batch)
+                                     conv=conv, batch=ctx.batch, extra=extra)

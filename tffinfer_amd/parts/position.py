@@ -100,3 +100,17 @@ class ScaledRotaryEmbedding(RotaryEmbedding):
         mid = (1.0 - s) * f / self.factor + s * f
         f = torch.where(wave < self.original / self.high, f, torch.where(wave > self.original / self.low, f / self.factor, mid))
         return torch.arange(max_positions, dtype=torch.float64)[:, None] * f[None, :]
+
+
+@register_position_encoding("rope_linear")
+class LinearRotaryEmbedding(RotaryEmbedding):
+    """The rotation with every angle divided by ``factor``, as if positions lay that much closer together."""
+
+    def __init__(self, head_dim: int, theta: float, factor: float, pairing: str = "half", rotary_dim: int | None = None):
+        super().__init__(head_dim, theta, pairing, rotary_dim)
+        self.factor = float(factor)
+        if not self.factor > 0:
+            raise ConfigError(f"linear rope: factor {factor} must be positive")
+
+    def angles(self, max_positions: int) -> torch.Tensor:
+        return super().angles(max_positions) / self.factor
