@@ -177,9 +177,43 @@ GOPUZEN_SHAPES = {
                       expert_ff=1536)),
 }
 
+def pupinex_shape(width, heads, kv_heads, dim, window, gla_heads, gla_dim, gla_vdim, left_heads, left_kv_heads, left_dim, right_heads,
+                  right_dim, right_vdim, dense_ff, experts, top, groups, keep, expert_ff, layers, vocab=151936):
+    """A Pupinex configuration of ``layers`` layers: a windowed attention with a sink, a linear recurrence with a decay per
+    key channel, a windowed attention beside a matrix memory, and so on; dense feed-forwards and mixtures of
+    experts with a shared one in turn."""
+    def att(h, g, d, base):
+        return {"heads": h, "kv_heads": g, "dim": d, "vdim": d, "scale": d ** -0.5, "mask": {"size": window},
+                "rot": {"base": base, "dims": d}}
+    left = att(left_heads, left_kv_heads, left_dim, 50000.0)
+    left["rot"]["scaling"] = {"factor": 8.0}
+    kinds = [{"type": "attention", "mixer": att(heads, kv_heads, dim, 10000.0)},
+             {"type": "gla", "mixer": {"heads": gla_heads, "dim": gla_dim, "vdim": gla_vdim, "tau": 16.0, "decay_rank": 16}},
+             {"type": "parallel", "mixer": {"left": left, "left_scale": 0.5, "right_scale": 0.5,
+                                            "right": {"heads": right_heads, "dim": right_dim, "vdim": right_vdim, "gate_cap": 15.0}}}]
+    mlps = [{"kind": "dense", "ff": dense_ff, "limit": 7.0},
+            {"kind": "moe", "expert": {"ff": expert_ff}, "shared": {"ff": expert_ff},
+             "router": {"experts": experts, "top": top, "groups": {"count": groups, "keep": keep}, "scale": 2.5}}]
+    return {"architecture": "Pupinex", "width": width, "vocab": vocab, "norm": {"eps": 1e-5},
+            "embedding": {"bigram": {"buckets": 65521, "mul_prev": 1009, "mul_cur": 31}},
+            "layers": [dict(kinds[i % 3], mlp=mlps[i % 2]) for i in range(layers)]}
+
+
+# Pupinex at sizes that resemble a real model's layers, beside the Qwen3 shape of the same width (the same dense
+# feed-forward) and, with --design-beside gopuzen, beside the design whose layers are closest: a windowed attention, an
+# attention beside a recurrence of as many heads and channels, routed experts of the same sizes
+PUPINEX_SHAPES = {
+    "2k": ("1.7b", dict(width=2048, heads=16, kv_heads=4, dim=128, window=1024, gla_heads=8, gla_dim=128, gla_vdim=256, left_heads=16,
+                        left_kv_heads=4, left_dim=128, right_heads=8, right_dim=128, right_vdim=128, dense_ff=6144, experts=16, top=2,
+                        groups=4, keep=2, expert_ff=1536)),
+    "4k": ("8b", dict(width=4096, heads=32, kv_heads=8, dim=128, window=1024, gla_heads=16, gla_dim=128, gla_vdim=256, left_heads=32,
+                      left_kv_heads=8, left_dim=128, right_heads=16, right_dim=128, right_vdim=128, dense_ff=12288, experts=32, top=4,
+                      groups=8, keep=4, expert_ff=1536)),
+}
+
 DESIGNS = {"disunex": ("Disunex", DISUNEX_SHAPES, disunex_shape), "netovik": ("Netovik", NETOVIK_SHAPES, netovik_shape),
            "sipilorn": ("Sipilorn", SIPILORN_SHAPES, sipilorn_shape), "rutevik": ("Rutevik", RUTEVIK_SHAPES, rutevik_shape),
-           "gopuzen": ("Gopuzen", GOPUZEN_SHAPES, gopuzen_shape)}
+           "gopuzen": ("Gopuzen", GOPUZEN_SHAPES, gopuzen_shape), "pupinex": ("Pupinex", PUPINEX_SHAPES, pupinex_shape)}
 
 
 def design_points(args):

@@ -61,6 +61,14 @@ def gopuzen_dirs(tmp_path_factory):
     return {name: make_gopuzen_dir(str(base / name), cfg, seed) for name, (cfg, seed) in GOPUZEN_CONFIGS.items()}
 
 
+@pytest.fixture(scope="session")
+def pupinex_dirs(tmp_path_factory):
+    """Model folders of the tiny Pupinex configurations (sharpened weights), once per session."""
+    from pupinex_models import PUPINEX_CONFIGS, make_pupinex_dir
+    base = tmp_path_factory.mktemp("pupinex")
+    return {name: make_pupinex_dir(str(base / name), cfg, seed) for name, (cfg, seed) in PUPINEX_CONFIGS.items()}
+
+
 @pytest.fixture(autouse=True)
 def _seeded():
     """Every test draws the same random inputs in every run."""

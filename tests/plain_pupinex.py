@@ -126,13 +126,13 @@ def gla(m: dict, P: dict, h: torch.Tensor, eps: float) -> torch.Tensor:
     return (o.reshape(T, -1) * silu(h @ P["g"].T)) @ P["o"].T
 
 
-def mlstm_states(q, k, v, i, f, max_start: float = 0.0) -> torch.Tensor:
+def mlstm_states(q, k, v, i, f, floor: bool = True) -> torch.Tensor:
     """q, k [T, H, D], v [T, H, E], log gates i, f [T, H]: the matrix S and the vector n kept relative to exp(m),
-    m the running maximum; o [T, H, E]."""
+    m the running maximum (zero at the start); ``floor`` False: the denominator without its floor; o [T, H, E]."""
     T, H, D = q.shape
     S = torch.zeros(H, D, v.shape[2], dtype=q.dtype)
     n = torch.zeros(H, D, dtype=q.dtype)
-    m = torch.full((H,), max_start, dtype=q.dtype)
+    m = torch.zeros(H, dtype=q.dtype)
     out = torch.zeros(T, H, v.shape[2], dtype=q.dtype)
     for t in range(T):
         new = torch.maximum(f[t] + m, i[t])
@@ -140,7 +140,8 @@ def mlstm_states(q, k, v, i, f, max_start: float = 0.0) -> torch.Tensor:
         m = new
         S = keep[:, None, None] * S + put[:, None, None] * k[t][:, :, None] * v[t][:, None, :]
         n = keep[:, None] * n + put[:, None] * k[t]
-        den = torch.maximum((n * q[t]).sum(-1).abs(), torch.exp(-m)) + 1e-6
+        den = (n * q[t]).sum(-1).abs()
+        den = (torch.maximum(den, torch.exp(-m)) if floor else den) + 1e-6
         out[t] = torch.einsum("hde,hd->he", S, q[t]) / den[:, None]
     return out
 

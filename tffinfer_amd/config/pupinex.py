@@ -84,7 +84,9 @@ def _mixer_spec(i: int, width: int, eps: float, kind: str, m) -> PartSpec:
     if kind == "attention":
         return _attention(width, m, "interleaved", where, output_bias=True, sinks=True)
     if kind == "gla":
-        return PartSpec("gated_linear_attention", dict(_recurrence_sizes(width, eps, m, where), tau=require(m, "tau", float, where)))
+        # (the decay's inner size comes from its tensors; a caller that draws random weights names it)
+        return PartSpec("gated_linear_attention", dict(_recurrence_sizes(width, eps, m, where), tau=require(m, "tau", float, where),
+                                                       decay_rank=optional(m, "decay_rank", int, None, where)))
     if kind == "parallel":
         left, right = _obj(m, "left", where), _obj(m, "right", where)
         rw = where + ".right"

@@ -16,26 +16,22 @@ struct GroupedRot {
     int pairing;         // 0: (i, i + dims/2), 1: (2i, 2i+1)
 };
 
-// Element e of a head whose elements are value(0), value(1), ...
-template <typename F>
-__device__ __forceinline__ float grouped_rotated(F value, int e, const GroupedRot r) {
-    const float v = value(e);
-    if (!r.cs || e >= r.dims) return v;
-    int i, other;
-    bool first;
-    if (r.pairing == 0) {
-        const int half = r.dims >> 1;
-        first = e < half;
-        i = first ? e : e - half;
-        other = first ? e + half : e - half;
+// Elements of a head come two by two: place p < dims / 2 is the p-th pair that turns, the others two neighbours behind
+// the turned part.  f(element, its value): elements from D to P - 1 are zeros.
+template <typename V, typename F>
+__device__ __forceinline__ void grouped_pair(int p, int D, const GroupedRot r, V value, F f) {
+    const int half = r.cs ? r.dims >> 1 : 0;
+    if (p < half) {
+        const int i = r.pairing == 0 ? p : 2 * p, j = r.pairing == 0 ? p + half : 2 * p + 1;
+        const float u = value(i), w = value(j), c = r.cs[2 * p], s = r.cs[2 * p + 1];
+        // the pair (u, w) becomes (u c - w s, w c + u s)
+        f(i, fmaf(u, c, -(w * s)));
+        f(j, fmaf(w, c, u * s));
     } else {
-        first = !(e & 1);
-        i = e >> 1;
-        other = e ^ 1;
+        const int i = 2 * p;
+        f(i, i < D ? value(i) : 0.f);
+        f(i + 1, i + 1 < D ? value(i + 1) : 0.f);
     }
-    const float o = value(other), c = r.cs[2 * i], s = r.cs[2 * i + 1];
-    // the pair (u, w) becomes (u c - w s, w c + u s)
-    return first ? fmaf(v, c, -(o * s)) : fmaf(v, c, o * s);
 }
 
 // What happens to the projections before rotation.
@@ -45,18 +41,31 @@ struct GroupedPre {
     float eps;
 };
 
-// Blocks (token, y): y < q_blocks works through GQ_HEADS query heads; the others are one kv head each: its key row and
-// its value row into the token's slot.  Elements past a head's own size are zeros.  With a norm every block forms the
+// Blocks (token, y): y < q_blocks works through `per_q` query heads; the others through `per_kv` kv heads each: their key
+// and value rows into the token's slot.  Elements past a head's own size are zeros.  With a norm every block forms the
 // sum of squares it needs by itself, always in the same order.
 #define GQ_THREADS 128
 #define GQ_HEADS 8
 
 // 1 / sqrt(mean over x[0 .. n) of (x + bias)^2 + eps), the result in every thread of the block
-__device__ __forceinline__ float grouped_rms(const float* __restrict__ x, const float* __restrict__ bias, int n, float eps, float* red) {
+__device__ __forceinline__ float grouped_rms(const float* __restrict__ x, const float* __restrict__ bias, int n, float eps, bool vec,
+                                             float* red) {
     float ss = 0.f;
-    for (int c = threadIdx.x; c < n; c += GQ_THREADS) {
-        const float v = x[c] + (bias ? bias[c] : 0.f);
-        ss = fmaf(v, v, ss);
+    if (vec) {
+#pragma unroll 8
+        for (int c = threadIdx.x * 4; c < n; c += GQ_THREADS * 4) {
+            float4 v = *reinterpret_cast<const float4*>(x + c);
+            if (bias) {
+                const float4 b = *reinterpret_cast<const float4*>(bias + c);
+                v.x += b.x; v.y += b.y; v.z += b.z; v.w += b.w;
+            }
+            ss = fmaf(v.x, v.x, fmaf(v.y, v.y, fmaf(v.z, v.z, fmaf(v.w, v.w, ss))));
+        }
+    } else {
+        for (int c = threadIdx.x; c < n; c += GQ_THREADS) {
+            const float v = x[c] + (bias ? bias[c] : 0.f);
+            ss = fmaf(v, v, ss);
+        }
     }
     ss = rows_sum(row16_sum(ss));
     if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = ss;
@@ -72,48 +81,55 @@ __global__ __launch_bounds__(GQ_THREADS) void grouped_qkv_store_kernel(
     const float* __restrict__ proj, size_t row, const float* __restrict__ cos_sin, int rot_dims, int pairing, int max_pos,
     float temp_coef, int temp_every, const GroupedPre pre, const int32_t* __restrict__ positions, const int32_t* __restrict__ slots,
     TC* __restrict__ q_out, TC* __restrict__ k_cache, TC* __restrict__ v_cache, int page_size, int H, int G, int D, int E, int P,
-    int q_blocks) {
+    int q_blocks, int per_q, int per_kv, int vec) {
     __shared__ float red[GQ_THREADS / 64];
     const int t = blockIdx.x, y = blockIdx.y, tid = threadIdx.x;
     const float* x = proj + (size_t)t * row;
     const int pos = max(positions[t], 0), tpos = min(pos, max(max_pos - 1, 0));
     const GroupedRot rot{(cos_sin && rot_dims) ? cos_sin + (size_t)tpos * rot_dims : nullptr, rot_dims, pairing};
+    const int half = P >> 1;                 // places of a head
     if (y < q_blocks) {
         const float temp = temp_coef != 0.f ? 1.0f + temp_coef * logf((float)((pos + 1) / temp_every + 1)) : 1.0f;
-        const float rr = pre.q_norm ? grouped_rms(x, pre.bias, H * D, pre.eps, red) : 1.0f;
+        const float rr = pre.q_norm ? grouped_rms(x, pre.bias, H * D, pre.eps, vec, red) : 1.0f;
         TC* qo = q_out + (size_t)t * H * P;
-        const int h0 = y * GQ_HEADS, h1 = min(H, h0 + GQ_HEADS);
-        for (int h = h0; h < h1; ++h) {
-            const int c0 = h * D;
-            auto value = [&](int e) {
-                float v = x[c0 + e];
-                if (pre.bias) v += pre.bias[c0 + e];
-                return pre.q_norm ? v * rr * pre.q_norm[c0 + e] : v;
-            };
-            for (int e = tid; e < P; e += GQ_THREADS)
-                qo[(size_t)h * P + e] = from_f32<TC>(e < D ? grouped_rotated(value, e, rot) * temp : 0.f);
+        const int h0 = y * per_q, count = (min(H, h0 + per_q) - h0) * half;
+        for (int idx = tid; idx < count; idx += GQ_THREADS) {
+            const int h = h0 + idx / half, p = idx % half, c0 = h * D;
+            TC* const qh = qo + (size_t)h * P;
+            grouped_pair(p, D, rot,
+                [&](int e) {
+                    float v = x[c0 + e];
+                    if (pre.bias) v += pre.bias[c0 + e];
+                    return pre.q_norm ? v * rr * pre.q_norm[c0 + e] : v;
+                },
+                [&](int e, float v) { qh[e] = from_f32<TC>(v * temp); });
         }
         return;
     }
     const int slot = slots[t];
     if (slot < 0) return;      // (the whole block: a token that writes no key)
-    const int g = y - q_blocks;
     const int page = slot / page_size, off = slot - page * page_size;
-    const size_t ck = (size_t)H * D, cv = ck + (size_t)G * D + (size_t)g * E;
+    const size_t ck = (size_t)H * D;
     const float* xk = x + ck;
     const float* bk = pre.bias ? pre.bias + ck : nullptr;
-    const float rr = pre.k_norm ? grouped_rms(xk, bk, G * D, pre.eps, red) : 1.0f;
-    const int c0 = g * D;
-    auto value = [&](int e) {
-        float v = xk[c0 + e];
-        if (bk) v += bk[c0 + e];
-        return pre.k_norm ? v * rr * pre.k_norm[c0 + e] : v;
-    };
-    TC* kd = k_cache + (((size_t)page * G + g) * page_size + off) * P;
-    TC* vd = v_cache + ((size_t)page * G + g) * P * page_size + off;
-    for (int e = tid; e < P; e += GQ_THREADS) {
-        kd[e] = from_f32<TC>(e < D ? grouped_rotated(value, e, rot) : 0.f);
-        vd[(size_t)e * page_size] = from_f32<TC>(e < E ? x[cv + e] + (pre.bias ? pre.bias[cv + e] : 0.f) : 0.f);
+    const float rr = pre.k_norm ? grouped_rms(xk, bk, G * D, pre.eps, vec, red) : 1.0f;
+    const int g0 = (y - q_blocks) * per_kv, groups = min(G, g0 + per_kv) - g0;
+    for (int idx = tid; idx < groups * half; idx += GQ_THREADS) {
+        const int g = g0 + idx / half, p = idx % half, c0 = g * D;
+        TC* const kd = k_cache + (((size_t)page * G + g) * page_size + off) * P;
+        grouped_pair(p, D, rot,
+            [&](int e) {
+                float v = xk[c0 + e];
+                if (bk) v += bk[c0 + e];
+                return pre.k_norm ? v * rr * pre.k_norm[c0 + e] : v;
+            },
+            [&](int e, float v) { kd[e] = from_f32<TC>(v); });
+    }
+    for (int idx = tid; idx < groups * P; idx += GQ_THREADS) {
+        const int g = g0 + idx / P, e = idx % P;
+        const size_t cv = ck + (size_t)G * D + (size_t)g * E + e;
+        TC* const vd = v_cache + ((size_t)page * G + g) * P * page_size + off;
+        vd[(size_t)e * page_size] = from_f32<TC>(e < E ? x[cv] + (pre.bias ? pre.bias[cv] : 0.f) : 0.f);
     }
 }
 
@@ -125,19 +141,24 @@ TFF_API int tff_grouped_qkv_store(const float* proj, size_t row, const float* co
     TFF_REQUIRE(proj && positions && q_out && (!store || (slots && k_cache && v_cache)), "grouped_qkv_store: null pointer");
     TFF_REQUIRE(T >= 0 && H > 0 && G > 0 && H % G == 0 && D > 0 && E > 0 && P >= D && P >= E && temp_every > 0,
                 "grouped_qkv_store: bad sizes H=%d G=%d D=%d E=%d P=%d", H, G, D, E, P);
+    TFF_REQUIRE(P % 2 == 0, "grouped_qkv_store: a cache head of %d elements must be even", P);
     TFF_REQUIRE(row >= (size_t)H * D + (store ? (size_t)G * (D + E) : 0), "grouped_qkv_store: rows of %zu are too short", row);
     TFF_REQUIRE(rot_dims >= 0 && rot_dims <= D && rot_dims % 2 == 0 && (rot_dims == 0 || (cos_sin && max_pos > 0)) &&
                 (pairing == 0 || pairing == 1), "grouped_qkv_store: %d rotated elements of a head of %d need an even count and a table", rot_dims, D);
     TFF_REQUIRE(page_size > 0 && num_pages > 0, "grouped_qkv_store: bad cache geometry");
     if (T == 0) return 0;
     hipStream_t s = (hipStream_t)stream;
-    const int q_blocks = (H + GQ_HEADS - 1) / GQ_HEADS, kv_blocks = store ? G : 0;
+    // (with a norm over all heads, many tokens fill the GPU with a block each for q and for k: nothing is summed twice)
+    const bool whole = (q_norm || k_norm) && T >= 128;
+    const int per_q = whole ? H : GQ_HEADS, per_kv = whole ? G : 1;
+    const int q_blocks = (H + per_q - 1) / per_q, kv_blocks = store ? (G + per_kv - 1) / per_kv : 0;
+    const int vec = D % 4 == 0 && row % 4 == 0 && ((uintptr_t)proj % 16) == 0 && ((uintptr_t)bias % 16) == 0;
     TFF_REQUIRE(q_blocks + kv_blocks <= 65535, "grouped_qkv_store: too many heads");
     const dim3 grid(T, q_blocks + kv_blocks);
 #define GQ_LAUNCH(TC)                                                                                                          \
     grouped_qkv_store_kernel<TC><<<grid, GQ_THREADS, 0, s>>>(proj, row, cos_sin, rot_dims, pairing, max_pos, temp_coef, temp_every, \
                                                              GroupedPre{bias, q_norm, k_norm, norm_eps}, positions, slots, (TC*)q_out, (TC*)k_cache, (TC*)v_cache, page_size, H, \
-                                                             G, D, E, P, q_blocks)
+                                                             G, D, E, P, q_blocks, per_q, per_kv, vec)
     if (dtype == TFF_F32) GQ_LAUNCH(float);
     else if (dtype == TFF_BF16) GQ_LAUNCH(bf16_t);
     else return tff_fail("grouped_qkv_store: unknown dtype %d", dtype);

@@ -41,17 +41,17 @@ __device__ __forceinline__ float lr_gate(float z, int sigmoid) {
 // Block: one head of one request, its threads in rows of sixteen lanes; a row shares a value channel, lane s holding
 // the key channels 64 m + 4 s .. + 3.  Up to `tm` tokens pass at a time: their q, k, v, gates and decays go to LDS,
 // every row takes its value channels through all of them with S in registers, then a wave per token norms and gates.
-template <int KIND, int M, bool VEC, typename TO>
+template <int KIND, int M, int IT, bool VEC, typename TO>
 __global__ __launch_bounds__(1024) void lr_few_kernel(const TffRecurrence a, int tm) {
     extern __shared__ __attribute__((aligned(16))) float lr_lds[];
     constexpr bool EXPG = KIND == TFF_LR_EXP;
-    constexpr int DP = 64 * M, KPL = 4 * M, IT = M >= 4 ? 1 : 2;
+    constexpr int DP = 64 * M, KPL = 4 * M, NS = EXPG ? IT + 1 : IT;      // (the last place of the first row is for n)
     const int D = a.D, E = a.E, E1 = EXPG ? E + 1 : E;
     float* const lq = lr_lds;
     float* const lk = lq + tm * DP;
     float* const la = lk + tm * DP;                        // decays (channel-wise), or nothing
     float* const lv = la + (EXPG ? 0 : tm * DP);
-    float* const lg = lv + tm * E;
+    float* const lg = lv + tm * E;                         // the norm's weight times the gate
     float* const lo = lg + tm * E;
     float* const lc = lo + tm * E1;                        // exponential gates: keep, put, exp(-m) of a token
     const int h = blockIdx.x, r = blockIdx.y, tid = threadIdx.x, nt = blockDim.x;
@@ -62,11 +62,17 @@ __global__ __launch_bounds__(1024) void lr_few_kernel(const TffRecurrence a, int
     float* const S0 = srow + (size_t)h * E1 * D;
     float* const mp = srow + (size_t)a.H * E1 * D + h;     // (exponential gates)
     float m_run = (EXPG && wave == 0) ? *mp : 0.f;
-    float S[IT][KPL];
+    float S[NS][KPL];
+    // the value channel of place u of a row; E1: none
+    auto channel = [&](int e0, int u) {
+        if (u == IT) return e0 == 0 ? E : E1;
+        const int e = e0 + u * rows;
+        return e < E ? e : E1;
+    };
     auto load = [&](int e0) {
 #pragma unroll
-        for (int u = 0; u < IT; ++u) {
-            const int e = e0 + u * rows;
+        for (int u = 0; u < NS; ++u) {
+            const int e = channel(e0, u);
             const float* p = S0 + (size_t)e * D;
 #pragma unroll
             for (int m = 0; m < M; ++m) {
@@ -84,8 +90,8 @@ __global__ __launch_bounds__(1024) void lr_few_kernel(const TffRecurrence a, int
     };
     auto store = [&](int e0) {
 #pragma unroll
-        for (int u = 0; u < IT; ++u) {
-            const int e = e0 + u * rows;
+        for (int u = 0; u < NS; ++u) {
+            const int e = channel(e0, u);
             float* p = S0 + (size_t)e * D;
 #pragma unroll
             for (int m = 0; m < M; ++m) {
@@ -125,8 +131,15 @@ __global__ __launch_bounds__(1024) void lr_few_kernel(const TffRecurrence a, int
                     const float* a1 = a.a1 + (tp + tk) * a.ld;
                     const float* a2 = a.a2 + c;
                     const size_t step = (size_t)a.H * D;
-#pragma unroll 8
-                    for (int i = 0; i < a.rank; ++i) z = fmaf(a2[i * step], a1[i], z);
+                    int i = 0;
+                    for (; i + 16 <= a.rank; i += 16) {      // (sixteen loads in flight)
+                        float x[16], y[16];
+#pragma unroll
+                        for (int j = 0; j < 16; ++j) { x[j] = a2[(i + j) * step]; y[j] = a1[i + j]; }
+#pragma unroll
+                        for (int j = 0; j < 16; ++j) z = fmaf(x[j], y[j], z);
+                    }
+                    for (; i < a.rank; ++i) z = fmaf(a2[i * step], a1[i], z);
                     al = expf(lr_logsigmoid(z) * a.inv_tau);
                 }
                 la[x] = al;
@@ -136,7 +149,7 @@ __global__ __launch_bounds__(1024) void lr_few_kernel(const TffRecurrence a, int
             const int tk = x / E, e = x - tk * E;
             const size_t at = (tp + tk) * a.ld + (size_t)h * E + e;
             lv[x] = a.v[at];
-            lg[x] = a.gate[at];
+            lg[x] = lr_gate(a.gate[at], a.sigmoid_gate) * a.w[(a.w_per_head ? (size_t)h * E : 0) + e];
         }
         if constexpr (EXPG) {
             if (wave == 0) {
@@ -156,7 +169,7 @@ __global__ __launch_bounds__(1024) void lr_few_kernel(const TffRecurrence a, int
             }
         }
         __syncthreads();
-        for (int e0 = row, base = 0; base < E1; base += rows * IT, e0 += rows * IT) {
+        for (int e0 = row, base = 0; base < E; base += rows * IT, e0 += rows * IT) {
             if (base) load(e0);
             for (int tk = 0; tk < cnt; ++tk) {
                 float kk[KPL], qq[KPL], al[EXPG ? 1 : KPL];
@@ -165,8 +178,9 @@ __global__ __launch_bounds__(1024) void lr_few_kernel(const TffRecurrence a, int
                 if constexpr (!EXPG) take(al, la + tk * DP);
                 const float keep = EXPG ? lc[3 * tk] : 0.f, put = EXPG ? lc[3 * tk + 1] : 1.f;
 #pragma unroll
-                for (int u = 0; u < IT; ++u) {
-                    const int e = e0 + u * rows;
+                for (int u = 0; u < NS; ++u) {
+                    if (u == IT && e0 != 0) break;
+                    const int e = channel(e0, u);
                     const float v = e < E ? lv[tk * E + e] * put : put;
                     float acc = 0.f;
 #pragma unroll
@@ -192,10 +206,9 @@ __global__ __launch_bounds__(1024) void lr_few_kernel(const TffRecurrence a, int
             ss = rows_sum(row16_sum(ss));
             const float rr = a.out_scale / sqrtf(ss / (float)E + a.eps);
             TO* out = reinterpret_cast<TO*>(a.out) + (tp + tk) * a.out_row + (size_t)h * E;
-            const float* w = a.w + (a.w_per_head ? (size_t)h * E : 0);
             for (int e = lane; e < E; e += 64) {
                 const float o = EXPG ? x[e] / den : x[e];
-                out[e] = from_f32<TO>(o * rr * w[e] * lr_gate(lg[tk * E + e], a.sigmoid_gate));
+                out[e] = from_f32<TO>(o * rr * lg[tk * E + e]);
             }
         }
     }
@@ -236,7 +249,7 @@ TFF_API int tff_recurrence_few(const TffRecurrence* p, int max_tokens, tff_strea
     const int nt = a.E <= 16 ? 256 : a.E <= 32 ? 512 : 1024;
     const bool vec = a.D % 4 == 0 && a.state_row % 4 == 0 && ((uintptr_t)a.state % 16) == 0;
     const dim3 grid(a.H, a.R);
-#define LR_GO(K, MM, V, TO) lr_few_kernel<K, MM, V, TO><<<grid, nt, lds, s>>>(a, tm)
+#define LR_GO(K, MM, V, TO) lr_few_kernel<K, MM, 2, V, TO><<<grid, nt, lds, s>>>(a, tm)
 #define LR_M(K, V, TO) do { if (M == 1) LR_GO(K, 1, V, TO); else if (M == 2) LR_GO(K, 2, V, TO); else LR_GO(K, 4, V, TO); } while (0)
 #define LR_V(K, TO) do { if (vec) LR_M(K, true, TO); else LR_M(K, false, TO); } while (0)
     if (ex && a.out_dtype == TFF_BF16) LR_V(TFF_LR_EXP, bf16_t);
@@ -256,17 +269,29 @@ TFF_API int tff_recurrence_few(const TffRecurrence* p, int max_tokens, tff_strea
 #define LRC 64
 #define LRS 68       // floats between rows whose lanes read four neighbours (the inner index runs along the row)
 #define LRV 80       // floats between rows whose lanes read one column each (the inner index runs down the rows)
+#define LR_FUSED_E 256   // value channels up to which the outputs' kernel also norms and gates
 #define LRR 32       // inner size of the decay's second product that is worked through at a time
 
-// (0a) channel-wise decay: cum[t][h D + d] = the sum of log2 alpha from the chunk's first token to t.
+// -log1p(e^(-|z|)) + min(z, 0) with the hardware's exponential and logarithm: log u for u = 1 + e is off by the rounding of
+// the sum, which the factor e / (u - 1) takes out again.
+__device__ __forceinline__ float lr_logsigmoid_fast(float z) {
+    const float e = __expf(-fabsf(z)), u = 1.0f + e, d = u - 1.0f;
+    return fminf(z, 0.f) - (d == 0.f ? e : __logf(u) * (e * __builtin_amdgcn_rcpf(d)));
+}
+
+// (0a) channel-wise decay: cum[t][h D + d] = the sum of log2 alpha from the chunk's first token to t.  A wave takes sixteen
+// of the chunk's tokens, its lanes 64 channels; the waves' sums meet in LDS.
 __global__ __launch_bounds__(256) void lr_decay_kernel(const TffRecurrence a, const int32_t* __restrict__ items, float* __restrict__ cum) {
     __shared__ __attribute__((aligned(16))) float a1s[LRR * LRS];
+    __shared__ float tot[4][64];
     const int r = items[2 * blockIdx.x], i0 = items[2 * blockIdx.x + 1];
     const int t0 = a.cu_tokens[r] + i0, n = min(LRC, a.cu_tokens[r + 1] - t0);
-    const int HD = a.H * a.D, c = blockIdx.y * 256 + threadIdx.x, cc = min(c, HD - 1);
-    float z[LRC];
+    const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
+    const int HD = a.H * a.D, c = blockIdx.y * 64 + lane, cc = min(c, HD - 1);
+    float z[16];
+    const float b = a.a_bias[cc];
 #pragma unroll
-    for (int t = 0; t < LRC; ++t) z[t] = 0.f;
+    for (int t = 0; t < 16; ++t) z[t] = b;
     for (int r0 = 0; r0 < a.rank; r0 += LRR) {
         if (r0) __syncthreads();
         const int nr = min(LRR, a.rank - r0);
@@ -275,26 +300,34 @@ __global__ __launch_bounds__(256) void lr_decay_kernel(const TffRecurrence a, co
             a1s[i * LRS + t] = (t < n && i < nr) ? a.a1[(size_t)(t0 + t) * a.ld + r0 + i] : 0.f;
         }
         __syncthreads();
+#pragma unroll 4
         for (int i = 0; i < nr; ++i) {
-            const float w = a.a2[(size_t)(r0 + i) * HD + cc];
+            const float q = a.a2[(size_t)(r0 + i) * HD + cc];
 #pragma unroll
-            for (int t = 0; t < LRC; t += 4) {
-                const float4 x = *reinterpret_cast<const float4*>(a1s + i * LRS + t);
-                z[t] = fmaf(w, x.x, z[t]);
-                z[t + 1] = fmaf(w, x.y, z[t + 1]);
-                z[t + 2] = fmaf(w, x.z, z[t + 2]);
-                z[t + 3] = fmaf(w, x.w, z[t + 3]);
+            for (int t = 0; t < 16; t += 4) {
+                const float4 x = *reinterpret_cast<const float4*>(a1s + i * LRS + w * 16 + t);
+                z[t] = fmaf(q, x.x, z[t]);
+                z[t + 1] = fmaf(q, x.y, z[t + 1]);
+                z[t + 2] = fmaf(q, x.z, z[t + 2]);
+                z[t + 3] = fmaf(q, x.w, z[t + 3]);
             }
         }
     }
-    const float b = a.a_bias[cc], f = a.inv_tau * LR_LOG2E;
+    const float f = a.inv_tau * LR_LOG2E;
     float sum = 0.f;
-    float* out = cum + (size_t)t0 * HD + c;
 #pragma unroll
-    for (int t = 0; t < LRC; ++t) {
-        sum = fmaf(lr_logsigmoid(z[t] + b), f, sum);
-        if (t < n && c < HD) out[(size_t)t * HD] = sum;
+    for (int t = 0; t < 16; ++t) {
+        sum = fmaf(lr_logsigmoid_fast(z[t]), f, sum);
+        z[t] = sum;
     }
+    tot[w][lane] = sum;
+    __syncthreads();
+    sum = 0.f;
+    for (int j = 0; j < w; ++j) sum += tot[j][lane];
+    float* out = cum + (size_t)(t0 + w * 16) * HD + c;
+#pragma unroll
+    for (int t = 0; t < 16; ++t)
+        if (w * 16 + t < n && c < HD) out[(size_t)t * HD] = sum + z[t];
 }
 
 // (0b) exponential gates, per request and head, sixteen chunks at a time (a wave each).  With b the sums of f within a
@@ -779,7 +812,7 @@ TFF_API size_t tff_recurrence_workspace_bytes(int kind, int T, int items, int H,
     n = (n + 3) & ~(size_t)3;
     n += ex ? 3 * (size_t)T * H + 2 * (size_t)items * H : (size_t)T * H * D;
     n = (n + 3) & ~(size_t)3;
-    if (E > 128) n += (size_t)T * H * E;
+    if (E > LR_FUSED_E) n += (size_t)T * H * E;
     return n * sizeof(float);
 }
 
@@ -792,7 +825,7 @@ TFF_API int tff_recurrence_chunks(const TffRecurrence* p, int T, const int32_t* 
     TFF_REQUIRE(workspace_bytes >= tff_recurrence_workspace_bytes(a.kind, T, num_items, a.H, a.D, a.E), "recurrence_chunks: a workspace of %zu bytes is too small", workspace_bytes);
     const bool ex = a.kind == TFF_LR_EXP;
     const int E1 = a.E + (ex ? 1 : 0), d_blocks = (a.D + 63) / 64, e_blocks = (a.E + 63) / 64;
-    TFF_REQUIRE((long)d_blocks * e_blocks <= 65535, "recurrence_chunks: too many channels");
+    TFF_REQUIRE((long)d_blocks * e_blocks <= 65535 && ((long)a.H * a.D + 63) / 64 <= 65535, "recurrence_chunks: too many channels");
     hipStream_t s = (hipStream_t)stream;
     LrWork k{items, item_start, nullptr, nullptr, nullptr, nullptr, nullptr, nullptr, workspace, nullptr};
     float* q = workspace + ((((size_t)num_items * a.H * E1 * a.D) + 3) & ~(size_t)3);
@@ -804,7 +837,7 @@ TFF_API int tff_recurrence_chunks(const TffRecurrence* p, int T, const int32_t* 
         if (int rc = tff_check_launch("recurrence_gates")) return rc;
     } else {
         k.cum = q;
-        lr_decay_kernel<<<dim3(num_items, (a.H * a.D + 255) / 256), 256, 0, s>>>(a, items, q);
+        lr_decay_kernel<<<dim3(num_items, (a.H * a.D + 63) / 64), 256, 0, s>>>(a, items, q);
         q += (size_t)T * a.H * a.D;
         if (int rc = tff_check_launch("recurrence_decay")) return rc;
     }
@@ -820,24 +853,26 @@ TFF_API int tff_recurrence_chunks(const TffRecurrence* p, int T, const int32_t* 
     else lr_scan_kernel<TFF_LR_DECAY><<<g2, 256, 0, s>>>(a, k);
     if (int rc = tff_check_launch("recurrence_scan")) return rc;
     const bool bf = a.out_dtype == TFF_BF16;
-    const int eb = a.E <= 64 ? 1 : 2;
+    const int eb = a.E <= 64 ? 1 : a.E <= 128 ? 2 : 4;
     const dim3 g3(num_items, a.H, (e_blocks + eb - 1) / eb);
 #define LR_OUT(K, EB, V, TO, FU) lr_outputs_kernel<K, EB, V, TO, FU><<<g3, 256, 0, s>>>(a, k)
 #define LR_OUT_V(K, EB, TO, FU) do { if (vec) LR_OUT(K, EB, true, TO, FU); else LR_OUT(K, EB, false, TO, FU); } while (0)
 #define LR_OUT_K(K)                                          \
     do {                                                     \
-        if (a.E > 128) LR_OUT_V(K, 2, float, false);         \
+        if (a.E > LR_FUSED_E) LR_OUT_V(K, 4, float, false);  \
         else if (eb == 1 && bf) LR_OUT_V(K, 1, bf16_t, true); \
         else if (eb == 1) LR_OUT_V(K, 1, float, true);       \
-        else if (bf) LR_OUT_V(K, 2, bf16_t, true);           \
-        else LR_OUT_V(K, 2, float, true);                    \
+        else if (eb == 2 && bf) LR_OUT_V(K, 2, bf16_t, true); \
+        else if (eb == 2) LR_OUT_V(K, 2, float, true);       \
+        else if (bf) LR_OUT_V(K, 4, bf16_t, true);           \
+        else LR_OUT_V(K, 4, float, true);                    \
     } while (0)
     if (ex) LR_OUT_K(TFF_LR_EXP); else LR_OUT_K(TFF_LR_DECAY);
 #undef LR_OUT_K
 #undef LR_OUT_V
 #undef LR_OUT
     if (int rc = tff_check_launch("recurrence_outputs")) return rc;
-    if (a.E > 128) {
+    if (a.E > LR_FUSED_E) {
         const int pairs = T * a.H;
         if (bf) lr_norm_gate_kernel<bf16_t><<<(pairs + 3) / 4, 256, 0, s>>>(a, k.o, pairs);
         else lr_norm_gate_kernel<float><<<(pairs + 3) / 4, 256, 0, s>>>(a, k.o, pairs);
