@@ -46,8 +46,8 @@ def test_every_size_and_constant_comes_from_the_file():
     assert isinstance(p.right, MatrixMemory) and (p.right.num_heads, p.right.head_dim, p.right.value_dim, p.right.gate_cap) == (3, 8, 12, 10.0)
     assert p.state_spec().shape[0] >= 3 * 8 * 13 + 3 and p.state_spec().shape[0] % 4 == 0
     e = model.blocks[2].feed_forward
-    assert (e.num_experts, e.top, e.groups, e.keep_groups, e.intermediate_size, e.shared, e.shared_parts, e.weight_scale) == \
-        (6, 2, 3, 2, 16, 40, 3, 1.0)
+    assert (e.num_experts, e.top, e.groups, e.keep_groups, e.intermediate_size, e.shared, e.shared_expert.intermediate_size,
+            e.weight_scale) == (6, 2, 3, 2, 16, 40, 40, 1.0)
     assert not e.has_correction and not e.router_softmax and e.normalize and (e.limit, e.act_alpha, e.up_offset) == (math.inf, 1.0, 0.0)
     assert model.blocks[0].feed_forward.act == (1.5, 1.702, 1.0)
     assert isinstance(model.final_norm, LayerNorm) and not model.final_norm.has_bias and model.final_norm.eps == 1e-2

@@ -155,16 +155,18 @@ def _spans(plan, i):
 
 @pytest.mark.parametrize("W", [48, 321, 1030, 2052, 4100, 4099, 12288])
 def test_layer_norm_without_bias_and_rows_added_beside_the_term(W):
-    """resid += term + extra (a row each, or one for all) and the layer norm of the sum without a bias."""
+    """resid += term + extra (a row each, or one for all) and the layer norm of the sum without a bias; the term may be a
+    second result with a factor per row."""
     ops = _ops()
     n, eps = 5, 1e-3
     x, one, rows = (_rand(n, W, seed=i, scale=s) for i, s in ((1, 3.0), (2, 0.7), (3, 2.0)))
     one = one + 2.0                 # (a mean far from zero)
-    planes, w, vec, bias = _rand(3, n, W, seed=4), _rand(W, seed=5), _rand(W, seed=6), _rand(W, seed=7)
+    planes, w, vec, bias, fac = _rand(3, n, W, seed=4), _rand(W, seed=5), _rand(W, seed=6), _rand(W, seed=7), _rand(n, seed=8)
     d = lambda t: t.to(DEV)                  # noqa: E731
     dd = lambda t: t.double()                # noqa: E731
     for term, want in ((None, 0 * dd(x)), (d(one), dd(one)), (d(planes), dd(planes).sum(0)),
-                       (ops.OutputTerm(d(planes), bias=d(bias)), dd(planes).sum(0) + dd(bias))):
+                       (ops.OutputTerm(d(planes), bias=d(bias)), dd(planes).sum(0) + dd(bias)),
+                       (ops.OutputTerm(d(one), beside=(d(planes), d(fac))), dd(one) + dd(fac)[:, None] * dd(planes).sum(0))):
         for extra, add in ((None, 0 * dd(x)), (d(rows), dd(rows)), (d(vec), dd(vec))):
             total = dd(x) + want + add
             ref = plain.layer_norm(total, dd(w), eps)
@@ -209,15 +211,15 @@ def test_clamps_in_the_gated_product(M, I, K, limit):
     (256, 8, 8, 4, 8, 16, 2.5), (3, 3, 1, 1, 16, 130, 1.0), (90, 1, 30, 1, 8, 8, 1.0)])
 def test_experts_from_the_best_groups_beside_a_shared_one(E, top, groups, keep, ff, shared, scale):
     """The choice and its weights against the plain router (groups of one expert to many), the shared expert narrower,
-    as wide and wider than the others, by pairs and by tiles; a token's result does not depend on its batch."""
+    as wide and wider than the others, experts by pairs and by tiles; a token's result does not depend on its batch."""
     from tffinfer_amd.parts import RoutedExperts
     ops = _ops()
     T, W = 40, 48
     part = RoutedExperts(W, ff, E, top, None, act_alpha=1.0, up_offset=0.0, correction=False, groups=groups, keep_groups=keep,
                          weight_scale=scale, shared=shared)
-    w = _draw(part, E + top)
+    w, ws = _draw(part, E + top), _draw(part.shared_expert, E + top + 1)
     w["router"] = (w["router"].float() * 0.8).to(BF)
-    P = {k: v.double() for k, v in w.items()}
+    P = {k: v.double() for k, v in w.items()} | {"shared." + k: v.double() for k, v in ws.items()}
     m = {"router": {"top": top, "experts": E, "groups": {"count": groups, "keep": keep}, "scale": scale}}
     x = _rand(400, W, seed=E).to(BF).float()
     # rows whose choice rests on no close call
@@ -227,18 +229,18 @@ def test_experts_from_the_best_groups_beside_a_shared_one(E, top, groups, keep, 
     s = plain.sigmoid(x.double() @ P["router"].T)
     want = [plain.router_choice(m["router"], s[t])[0] for t in range(T)]
     ref = plain.routed_experts(m, P, x.double())
-    S = part.shared_parts
-    idx, wts = ops.route_topk(x.to(DEV), torch.cat([w["router"], w["shared.sg"]]).float().to(DEV), None, top, groups=groups,
-                              keep_groups=keep, scale=scale, shared=S)
-    assert idx.shape == (T, top + S) and torch.equal(idx.cpu().long(), torch.tensor([c + list(range(E, E + S)) for c in want]))
+    idx, wts, gate = ops.route_topk(x.to(DEV), torch.cat([w["router"], w["shared.sg"]]).float().to(DEV), None, top, groups=groups,
+                              keep_groups=keep, scale=scale, shared=True)
+    assert torch.equal(idx.cpu().long(), torch.tensor(want))
     chosen = torch.gather(s, 1, torch.tensor(want))
-    assert _err(wts[:, :top], chosen / chosen.sum(1, keepdim=True) * scale) < 2e-6
-    assert _err(wts[:, top:], plain.sigmoid(x.double() @ P["shared.sg"].T).expand(T, S)) < 2e-6
+    assert _err(wts, chosen / chosen.sum(1, keepdim=True) * scale) < 2e-6
+    assert _err(gate, plain.sigmoid(x.double() @ P["shared.sg"].T)[:, 0]) < 2e-6
     if keep < groups < E:       # the groups matter
         free = dict(m["router"], groups={"count": groups, "keep": groups})
         assert any(set(plain.router_choice(free, s[t])[0]) != set(want[t]) for t in range(T))
     for dtype, limit in ((F32, 2e-5), (BF, 3e-2)):
         part.load_weights(w, dtype, DEV)
+        part.shared_expert.load_weights(ws, dtype, DEV)
         ctx = _ctx(None, dtype)
         full = ops.as_tensor(part.forward(ctx, x.to(dtype).to(DEV)))
         assert _err(full, ref) < limit

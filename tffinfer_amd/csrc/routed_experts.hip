@@ -6,8 +6,8 @@
 //                   s = softmax(z) over all experts and the weights are the chosen s as they are.
 //                   With `groups`, E / groups neighbours form a group whose score is the sum of its two
 //                   largest s + bias, and only experts of the best `keep` groups can be chosen.  The weights
-//                   are multiplied by `scale`.  With `shared`, every token also gets the experts E .. E + shared - 1,
-//                   each with the weight sigmoid(row E of z).
+//                   are multiplied by `scale`.  With `shared`, z has one row more, whose sigmoid goes there (the
+//                   weight of an expert that every token uses).
 // tff_experts_gate_up: for every (token, chosen expert): g = min(Wg h, limit),
 //                   u = clamp(Wu h, -limit, limit), y = g * sigmoid(act_alpha * g) * (u + up_offset)
 //                   (limit = infinity, act_alpha = 1, up_offset = 0: silu(g) * u).
@@ -65,14 +65,14 @@ __global__ __launch_bounds__(64 * RT_WAVES) void route_topk_kernel(const T* __re
                                                                    const float* __restrict__ logits,
                                                                    const float* __restrict__ bias, int width, int E,
                                                                    int top, int softmax, int groups, int keep, float scale,
-                                                                   int shared, int32_t* __restrict__ idx,
+                                                                   float* __restrict__ shared, int32_t* __restrict__ idx,
                                                                    float* __restrict__ wts) {
     __shared__ float s_all[RT_MAX_E + 1];
     __shared__ float c_all[RT_MAX_E];
     __shared__ float g_all[RT_MAX_E];       // a group's score; of the chosen groups -infinity
     __shared__ int chosen[64];
     const int t = blockIdx.x, lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
-    const int rows = E + (shared > 0 ? 1 : 0), out_cols = top + shared;
+    const int rows = E + (shared ? 1 : 0);
     if (logits) {
         for (int e = threadIdx.x; e < rows; e += blockDim.x) s_all[e] = logits[(size_t)t * rows + e];
     } else {
@@ -156,7 +156,7 @@ __global__ __launch_bounds__(64 * RT_WAVES) void route_topk_kernel(const T* __re
         const int bi = largest(c_all, E);
         // (one wave from here on: LDS works through its accesses in order)
         if (lane == 0) {
-            idx[(size_t)t * out_cols + k] = bi;
+            idx[(size_t)t * top + k] = bi;
             chosen[k] = bi;
             c_all[bi] = -INFINITY;
         }
@@ -165,21 +165,17 @@ __global__ __launch_bounds__(64 * RT_WAVES) void route_topk_kernel(const T* __re
         __builtin_amdgcn_wave_barrier();
     }
     const float inv = softmax ? 1.0f : 1.0f / (sum + 1e-20f);      // (mode 2: sigmoid scores as they are)
-    if (lane < top) {
-        wts[(size_t)t * out_cols + lane] = s_all[chosen[lane]] * inv * scale;
-    } else if (lane < out_cols) {
-        idx[(size_t)t * out_cols + lane] = E + lane - top;
-        wts[(size_t)t * out_cols + lane] = 1.0f / (1.0f + expf(-s_all[E]));
-    }
+    if (lane < top) wts[(size_t)t * top + lane] = s_all[chosen[lane]] * inv * scale;
+    if (shared && lane == 0) shared[t] = 1.0f / (1.0f + expf(-s_all[E]));
 }
 
 TFF_API int tff_route_topk(const void* h, int h_row, const float* Wr, const float* logits, const float* bias, int T,
-                           int width, int E, int top, int softmax, int groups, int keep, float scale, int shared, int32_t* idx,
+                           int width, int E, int top, int softmax, int groups, int keep, float scale, float* shared, int32_t* idx,
                            float* wts, int dtype, tff_stream_t stream) {
     TFF_REQUIRE(idx && wts && (logits || (h && Wr)), "route_topk: null pointer");
     TFF_REQUIRE(T >= 0 && (logits || (width > 0 && h_row >= width)), "route_topk: bad sizes T=%d width=%d row=%d", T, width, h_row);
-    TFF_REQUIRE(E > 0 && E <= RT_MAX_E && top > 0 && top <= E && shared >= 0 && top + shared <= 64,
-                "route_topk: %d of %d experts and %d for every token (up to 64 of up to %d)", top, E, shared, RT_MAX_E);
+    TFF_REQUIRE(E > 0 && E <= RT_MAX_E && top > 0 && top <= E && top <= 64,
+                "route_topk: %d of %d experts (up to 64 of up to %d)", top, E, RT_MAX_E);
     TFF_REQUIRE(groups >= 1 && E % groups == 0 && keep >= 1 && keep <= groups && top <= keep * (E / groups),
                 "route_topk: %d of %d experts from %d of %d groups", top, E, keep, groups);
     if (T == 0) return 0;

@@ -3,6 +3,7 @@
 //
 // tff_add_layernorm, per row:
 //   d = (planes of a, in order) + bias                                       one sublayer's result, or
+//   d = (planes of a) + bias + b_scale[row] * (planes of b)                  two results, one with a factor per row, or
 //   d = (rms(a) * wa + rms(b) * wb) / 2                                      two normed results side by side
 //   y = layernorm(d; nw, nb) * scale                                         (nw null: y = d; scale null: 1)
 //   resid <- resid + y + extra;   h = layernorm(resid; w, b)                 -> out
@@ -25,8 +26,9 @@
 
 struct SandwichTerm {
     const float* a;            // null: no term
-    const float* b;            // the second of two normed results, or null
-    const float *wa, *wb;      // their RMS norms' weights
+    const float* b;            // the second of two results, or null
+    const float* b_scale;      // a factor per row on b (null: 1), where the two are not normed
+    const float *wa, *wb;      // their RMS norms' weights, or null
     const float* bias;         // added to a
     const float *nw, *nb;      // the layer norm of the term, or null
     const float* scale;
@@ -131,6 +133,7 @@ __global__ __launch_bounds__(NT) void add_layernorm_kernel(float* __restrict__ r
     float* const xr = resid ? resid + at : nullptr;
     const float* const ar = tm.a ? tm.a + at : nullptr;
     const float* const br = tm.b ? tm.b + at : nullptr;
+    const float bs = br && tm.b_scale ? tm.b_scale[row] : 1.0f;
     const int slot = cv.w ? cv.slots[i] : 0;
     float x[IT][VEC], d[IT][VEC], p2[IT][VEC];
 #pragma unroll
@@ -196,6 +199,10 @@ __global__ __launch_bounds__(NT) void add_layernorm_kernel(float* __restrict__ r
 #pragma unroll
                 for (int u = 0; u < VEC; ++u) p2[it][u] += t[u];
             }
+            if (br && !tm.wa) {
+#pragma unroll
+                for (int u = 0; u < VEC; ++u) d[it][u] = fmaf(p2[it][u], bs, d[it][u]);
+            }
             if (tm.bias) {
                 vbias.take(t, it, e);
 #pragma unroll
@@ -233,7 +240,7 @@ __global__ __launch_bounds__(NT) void add_layernorm_kernel(float* __restrict__ r
             }
         }
     };
-    if (br) {
+    if (br && tm.wa) {
         float s0 = 0.f, s1 = 0.f;
 #pragma unroll
         for (int it = 0; it < IT; ++it)
@@ -339,7 +346,7 @@ __global__ __launch_bounds__(NT) void add_layernorm_kernel(float* __restrict__ r
 }
 
 TFF_API int tff_add_layernorm(float* resid, const float* a, int planes_a, size_t plane_a, const float* b, int planes_b,
-                              size_t plane_b, const float* wa, const float* wb, float pair_eps, const float* bias,
+                              size_t plane_b, const float* b_scale, const float* wa, const float* wb, float pair_eps, const float* bias,
                               const float* nw, const float* nb, float n_eps, const float* scale, const float* w,
                               const float* beta, float eps, void* out, const int32_t* rows, int n, int W, const float* conv_w,
                               int taps, float* state, size_t state_row, size_t state_off, const int32_t* state_slots,
@@ -347,14 +354,14 @@ TFF_API int tff_add_layernorm(float* resid, const float* a, int planes_a, size_t
     TFF_REQUIRE((resid || a) && out, "add_layernorm: null pointer");
     TFF_REQUIRE(n >= 0 && W > 0 && W <= SN_MAX_W, "add_layernorm: rows of %d (up to %d)", W, SN_MAX_W);
     TFF_REQUIRE(!a || planes_a >= 1, "add_layernorm: a term without planes");
-    TFF_REQUIRE(!b || (a && wa && wb && planes_b >= 1), "add_layernorm: the second of two results needs the first and both weights");
+    TFF_REQUIRE(!b || (a && (!wa) == (!wb) && planes_b >= 1), "add_layernorm: the second of two results needs the first, and both weights or none");
     TFF_REQUIRE((nw || !nb) && (w || !beta) && (!nw || a), "add_layernorm: a norm takes a weight, and a bias or none");
     TFF_REQUIRE(!extra || (resid && (extra_row == 0 || extra_row >= (size_t)W)), "add_layernorm: rows of %zu to add to a stream of %d", extra_row, W);
     TFF_REQUIRE(!rows || resid, "add_layernorm: chosen rows of no stream");
     TFF_REQUIRE(!conv_w || (taps >= 1 && taps <= SN_MAX_TAPS && !rows && (taps == 1 || (state && state_slots &&
                 state_off + (size_t)(taps - 1) * W <= state_row))), "add_layernorm: a convolution of %d taps (up to %d) needs its state", taps, SN_MAX_TAPS);
     if (n == 0) return 0;
-    const SandwichTerm tm{a, b, wa, wb, bias, nw, nb, scale, plane_a, plane_b, planes_a, planes_b, pair_eps, n_eps, extra, extra_row};
+    const SandwichTerm tm{a, b, b_scale, wa, wb, bias, nw, nb, scale, plane_a, plane_b, planes_a, planes_b, pair_eps, n_eps, extra, extra_row};
     const SandwichConv cv{conv_w, state, state_slots, state_row, state_off, taps};
     hipStream_t s = (hipStream_t)stream;
     auto ok16 = [](const void* p) { return ((uintptr_t)p % 16) == 0; };

@@ -299,10 +299,9 @@ TFF_API int tff_diff_combine(const void* a, size_t a_row, int P, const float* ga
 // wts [T, top] = s / (sum of the chosen s + 1e-20).  softmax 1: s = softmax(z) over all experts, wts = the chosen s;
 // softmax 2: s = sigmoid(z) and wts = the chosen s as they are.  The E experts form `groups` groups of neighbours; only
 // experts of the `keep` groups whose two largest s + bias have the largest sum can be chosen.  The weights are times
-// `scale`.  shared > 0: z has one row more, idx and wts [T, top + shared]: the experts E .. E + shared - 1 follow the
-// chosen ones, each with the weight sigmoid(z[E]).
+// `scale`.  shared [T] (may be null): z has one row more, shared = sigmoid(z[E]).
 TFF_API int tff_route_topk(const void* h, int h_row, const float* Wr, const float* logits, const float* bias, int T,
-                           int width, int E, int top, int softmax, int groups, int keep, float scale, int shared, int32_t* idx,
+                           int width, int E, int top, int softmax, int groups, int keep, float scale, float* shared, int32_t* idx,
                            float* wts, int dtype, tff_stream_t stream);
 // y[(t, k), :] = g * sigmoid(act_alpha * g) * (u + up_offset), g = min(Wg[e] h_t, limit), u = clamp(Wu[e] h_t, +-limit),
 // e = idx[t, k]; Wg, Wu [E, ff, width], rows ldw elements apart.  in_wts [T, top] (may be null): the pair's
@@ -430,7 +429,7 @@ TFF_API int tff_cast(const void* src, int src_dtype, void* dst, int dst_dtype, i
 
 // ---- norms before and after a sublayer, and the convolution of its input (sandwich_norm.hip) ----
 TFF_API int tff_add_layernorm(float* resid, const float* a, int planes_a, size_t plane_a, const float* b, int planes_b,
-                              size_t plane_b, const float* wa, const float* wb, float pair_eps, const float* bias,
+                              size_t plane_b, const float* b_scale, const float* wa, const float* wb, float pair_eps, const float* bias,
                               const float* nw, const float* nb, float n_eps, const float* scale, const float* w,
                               const float* beta, float eps, void* out, const int32_t* rows, int n, int W, const float* conv_w,
                               int taps, float* state, size_t state_row, size_t state_off, const int32_t* state_slots,

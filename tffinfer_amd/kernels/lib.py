@@ -6,7 +6,7 @@ from ctypes import c_char_p, c_float, c_int, c_int64, c_size_t, c_void_p
 
 from .build import ensure_built
 
-ABI_VERSION = 36
+ABI_VERSION = 37
 
 
 class KernelLibraryError(RuntimeError):
@@ -68,7 +68,7 @@ _SIGNATURES = {
     "tff_diff_combine": [_P, _Z, _I, _P, _Z, _F, _F, _F, _P, _Z, _I, _I, _I, _I, _P],
     "tff_scale_add_rmsnorm": [_P, _P, _I, _Z, _F, _P, _F, _P, _I, _I, _I, _P],
     "tff_gelu": [_P, _P, c_int64, _I, _I, _P],
-    "tff_route_topk": [_P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _I, _P, _P, _I, _P],
+    "tff_route_topk": [_P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _P, _P, _P, _I, _P],
     "tff_experts_gate_up": [_P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _F, _F, _P, _P, _I, _P],
     "tff_experts_tiles_supported": [_I, _I, _I],
     "tff_experts_by_tiles": [_P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _F, _F, _P, _P, _P, _I, _P, _P, _I, _I, _P],
@@ -99,7 +99,7 @@ _SIGNATURES = {
     "tff_argmax": [_P, _P, _I, _I, _P, _P],
     "tff_repetition_penalty": [_P, _I, _I, _P, _P, _P, _P],
     "tff_sample": [_P, _P, _I, _I, _P, _P, _P, _P, _P, _P, _P],
-    "tff_add_layernorm": [_P, _P, _I, _Z, _P, _I, _Z, _P, _P, _F, _P, _P, _P, _F, _P, _P, _P, _F, _P, _P, _I, _I, _P, _I, _P, _Z,
+    "tff_add_layernorm": [_P, _P, _I, _Z, _P, _I, _Z, _P, _P, _P, _F, _P, _P, _P, _F, _P, _P, _P, _F, _P, _P, _I, _I, _P, _I, _P, _Z,
                           _Z, _P, _P, _Z, _I, _P],
     "tff_input_conv": [_P, _P, _I, _P, _Z, _Z, _P, _I, _I, _P, _P, _P, _I, _I, _P],
     "tff_lightning": [_P, _Z, _P, _P, _Z, _P, _P, _P, _I, _I, _I, _I, _P],

@@ -1145,7 +1145,7 @@ def relu_squared(x: torch.Tensor) -> torch.Tensor:
 
 def route_topk(h: torch.Tensor | None, router: torch.Tensor | None, bias: torch.Tensor | None, top: int,
                logits: torch.Tensor | None = None, softmax: bool = False, normalize: bool = True, groups: int = 1,
-               keep_groups: int = 1, scale: float = 1.0, shared: int = 0):
+               keep_groups: int = 1, scale: float = 1.0, shared: bool = False):
     """s = sigmoid(z) with z = h . router^T in float32 (router float32 [E, width]) or z = ``logits``
     (float32 [T, E], a product that ran before); the ``top`` experts with the largest s + bias;
     returns (int32 [T, top], float32 [T, top] = s / (sum of the chosen s + 1e-20)).  With
@@ -1153,9 +1153,8 @@ def route_topk(h: torch.Tensor | None, router: torch.Tensor | None, bias: torch.
     ``normalize``, s = sigmoid(z) and the weights are the chosen s as they are.
 
     ``groups``: E / groups neighbours form a group whose score is the sum of its two largest s + bias; only experts
-    of the ``keep_groups`` best groups can be chosen.  ``scale`` multiplies the weights.  ``shared`` > 0: the router has
-    one row more (z_sh), and the results [T, top + shared] end with the experts E .. E + shared - 1, each with the
-    weight sigmoid(z_sh)."""
+    of the ``keep_groups`` best groups can be chosen.  ``scale`` multiplies the weights.  ``shared``: the router has
+    one row more, and its sigmoid (float32 [T]) is returned as a third tensor."""
     extra = 1 if shared else 0
     if logits is not None:
         _req(logits, "router logits", torch.float32, 2)
@@ -1174,14 +1173,15 @@ def route_topk(h: torch.Tensor | None, router: torch.Tensor | None, bias: torch.
         _req(bias, "router bias", torch.float32, 1)
         if bias.numel() != E:
             raise _lib.KernelError(f"route_topk: {bias.numel()} bias terms for {E} experts")
-    idx = torch.empty(T, top + shared, dtype=torch.int32, device=dev)
-    wts = torch.empty(T, top + shared, dtype=torch.float32, device=dev)
+    idx = torch.empty(T, top, dtype=torch.int32, device=dev)
+    wts = torch.empty(T, top, dtype=torch.float32, device=dev)
+    gate = torch.empty(T, dtype=torch.float32, device=dev) if shared else None
     _lib.check(_lib.load().tff_route_topk(None if logits is not None else h.data_ptr(), width,
                                           None if logits is not None else router.data_ptr(), _ptr(logits), _ptr(bias),
                                           T, width, E, int(top), 1 if softmax else (0 if normalize else 2), int(groups),
-                                          int(keep_groups), float(scale), int(shared), idx.data_ptr(), wts.data_ptr(),
+                                          int(keep_groups), float(scale), _ptr(gate), idx.data_ptr(), wts.data_ptr(),
                                           dtype_code(dt), _stream()))
-    return idx, wts
+    return (idx, wts, gate) if shared else (idx, wts)
 
 
 def pad_expert_rows(w: torch.Tensor) -> torch.Tensor:
@@ -1576,14 +1576,17 @@ def add_rmsnorm_pair(resid: torch.Tensor, delta, bias: torch.Tensor | None, w1: 
 class OutputTerm:
     """A sublayer's result on its way into the residual stream, with everything that happens to it there:
 
-        d = term + bias,   or with ``pair`` (b, wa, wb, eps)   d = (rms(term) * wa + rms(b) * wb) / 2
+        d = term + bias,   with ``beside`` (b, f)   d = term + bias + f b, f a factor per row (float32 [T]),
+        or with ``pair`` (b, wa, wb, eps)   d = (rms(term) * wa + rms(b) * wb) / 2
         d <- layernorm(d) with ``norm`` (weight, bias, eps);   d <- d * scale
 
     ``term`` and ``b`` are what ``linear`` may return with ``partials=True``.  ``add_layernorm`` adds it to the
     stream in the kernel that norms the sum; ``as_tensor`` makes a tensor of it."""
 
-    def __init__(self, term, bias=None, pair=None, norm=None, scale=None):
-        self.term, self.bias, self.pair, self.norm, self.scale = term, bias, pair, norm, scale
+    def __init__(self, term, bias=None, pair=None, norm=None, scale=None, beside=None):
+        self.term, self.bias, self.pair, self.norm, self.scale, self.beside = term, bias, pair, norm, scale, beside
+        if pair is not None and beside is not None:
+            raise _lib.KernelError("output term: two results are either normed or weighed")
 
 
 def output_term(delta, norm=None, scale=None) -> OutputTerm:
@@ -1591,7 +1594,7 @@ def output_term(delta, norm=None, scale=None) -> OutputTerm:
     t = delta if isinstance(delta, OutputTerm) else OutputTerm(delta)
     if t.norm is not None or t.scale is not None:
         raise _lib.KernelError("output term: it has a norm already")
-    return OutputTerm(t.term, t.bias, t.pair, norm, scale)
+    return OutputTerm(t.term, t.bias, t.pair, norm, scale, t.beside)
 
 
 def _vec(t, n: int, what: str):
@@ -1634,14 +1637,18 @@ def add_layernorm(resid: torch.Tensor | None, delta, weight, bias, eps: float, o
     ``resid`` None and ``weight`` None: the term itself."""
     term = delta if isinstance(delta, OutputTerm) else OutputTerm(delta)
     if isinstance(term.term, PendingTerms):
-        term = OutputTerm(as_tensor(term.term), term.bias, term.pair, term.norm, term.scale)
+        term = OutputTerm(as_tensor(term.term), term.bias, term.pair, term.norm, term.scale, term.beside)
     shape = tuple(resid.shape) if resid is not None else tuple(term.term.shape[-2:])
     W = shape[1]
     if resid is not None:
         _req(resid, "add_layernorm resid", torch.float32, 2)
     dev = resid.device if resid is not None else term.term.device
     a, pa, sa = _planes_of(term.term, shape, "add_layernorm term")
-    b, pb, sb, wa, wb, pair_eps = None, 0, 0, None, None, 0.0
+    b, pb, sb, wa, wb, pair_eps, b_scale = None, 0, 0, None, None, 0.0, None
+    if term.beside is not None:
+        b, b_scale = term.beside
+        b, pb, sb = _planes_of(b, shape, "add_layernorm second term")
+        b_scale = _vec(b_scale, shape[0], "add_layernorm factors")
     if term.pair is not None:
         b, wa, wb, pair_eps = term.pair
         b, pb, sb = _planes_of(b, shape, "add_layernorm second term")
@@ -1678,7 +1685,7 @@ def add_layernorm(resid: torch.Tensor | None, delta, weight, bias, eps: float, o
     st_row = state.stride(0) if taps > 1 else 0
     slots = batch.state_slots.data_ptr() if conv is not None else None
     _lib.check(L.tff_add_layernorm(
-        _ptr(resid), _ptr(a), pa, sa, _ptr(b), pb, sb, _ptr(wa), _ptr(wb), float(pair_eps), _ptr(tb), _ptr(nw), _ptr(nb),
+        _ptr(resid), _ptr(a), pa, sa, _ptr(b), pb, sb, _ptr(b_scale), _ptr(wa), _ptr(wb), float(pair_eps), _ptr(tb), _ptr(nw), _ptr(nb),
         float(n_eps), _ptr(sc), _ptr(weight), _ptr(bias), float(eps), out.data_ptr(), _ptr(rows), n, W,
         _ptr(cw) if one else None, taps, st, st_row, off, slots, _ptr(extra), extra_row, dtype_code(out.dtype), _stream()))
     if not split:

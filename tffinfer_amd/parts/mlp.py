@@ -152,9 +152,9 @@ class RoutedExperts(FeedForward):
     their input on, f_e = z.
     ``groups``, ``keep_groups``: neighbouring experts form ``groups`` equal groups, a group's score is the sum of its two
     largest s + b, and only experts of the ``keep_groups`` best groups can be chosen.  ``weight_scale``: w_e is multiplied by it.
-    ``shared``: the inner size of one more expert (``shared.gate``, ``shared.up``, ``shared.down``) that every token uses, with the
-    weight sigmoid(Wsg z) (``shared.sg``, one row).  Its hidden units lie behind the others' in the stacked matrices, cut into
-    experts of ``intermediate_size`` (the last one filled up with zeros), and run in the same launches.
+    ``shared``: the inner size of one more expert (a gated feed-forward with silu, ``shared.gate``, ``shared.up``, ``shared.down``)
+    that every token uses, with the weight sigmoid(Wsg z) (``shared.sg``, one row, which rides in the router's product).  It
+    runs on the dense products; its weight meets its output where the sum goes into the stream (``ops.OutputTerm``).
 
     The experts' matrices lie stacked, [experts, out, in], so that a kernel finds an expert's
     rows by its number."""
@@ -197,11 +197,7 @@ class RoutedExperts(FeedForward):
             from ..config.base import ConfigError
             raise ConfigError("routed experts: a shared expert goes neither with experts that hand their input on nor with "
                               "weights on the input")
-        #: experts of ``intermediate_size`` that the shared one is cut into
-        self.shared_parts = -(-self.shared // self.intermediate_size)
-        if self.top + self.shared_parts > 64:
-            from ..config.base import ConfigError
-            raise ConfigError(f"routed experts: {self.top} chosen experts and {self.shared_parts} parts of a shared one (up to 64)")
+        self.shared_expert = SwiGLU(hidden_size, self.shared, names=("gate", "up", "down")) if self.shared else None
         self.w_gate = self.w_up = self.w_down = self.router = self.router_w = self.correction = None
 
     def weight_specs(self):
@@ -215,9 +211,11 @@ class RoutedExperts(FeedForward):
             specs[f"e{e}.up"] = WeightSpec((I, H))
             specs[f"e{e}.down"] = WeightSpec((H, I))
         if self.shared:
-            specs |= {"shared.gate": WeightSpec((self.shared, H)), "shared.up": WeightSpec((self.shared, H)),
-                      "shared.down": WeightSpec((H, self.shared)), "shared.sg": WeightSpec((1, H))}
+            specs["shared.sg"] = WeightSpec((1, H))
         return specs
+
+    def children(self):
+        return {"shared": self.shared_expert} if self.shared else {}
 
     def active_matrix_elements(self) -> int:
         """Matrix elements a token multiplies with: the router and its ``top`` experts (and the shared one)."""
@@ -235,19 +233,11 @@ class RoutedExperts(FeedForward):
                 + round(min(self.num_experts, rows * self.top * share) * 3 * H * I) + 3 * H * self.shared)
 
     def load_weights(self, weights, dtype, device):
-        E, I = self.num_experts, self.intermediate_size
+        E = self.num_experts
 
         def stack(which):
             from ..kernels.ops import pad_expert_rows
-            mats = [weights[f"e{e}.{which}"].to(dtype) for e in range(E)]
-            if self.shared:
-                w = weights[f"shared.{which}"].to(dtype)
-                fill = self.shared_parts * I - self.shared
-                if which == "down":
-                    mats += torch.nn.functional.pad(w, (0, fill)).split(I, 1)
-                else:
-                    mats += torch.nn.functional.pad(w, (0, 0, 0, fill)).split(I, 0)
-            return pad_expert_rows(torch.stack(mats, 0)).to(device)
+            return pad_expert_rows(torch.stack([weights[f"e{e}.{which}"].to(dtype) for e in range(E)], 0)).to(device)
 
         self.w_gate, self.w_up, self.w_down = stack("gate"), stack("up"), stack("down")
         router = weights["router"]
@@ -271,15 +261,16 @@ class RoutedExperts(FeedForward):
         x = ops.as_tensor(x)
         how = {"softmax": self.router_softmax, "normalize": self.normalize}
         if self.groups > 1 or self.weight_scale != 1.0 or self.shared:
-            how |= {"groups": self.groups, "keep_groups": self.keep_groups, "scale": self.weight_scale, "shared": self.shared_parts}
+            how |= {"groups": self.groups, "keep_groups": self.keep_groups, "scale": self.weight_scale, "shared": self.shared > 0}
         if self.router_w is not None:
-            idx, wts = ops.route_topk(None, None, self.correction, self.top,
-                                      logits=ops.linear(x, self.router_w, out_dtype=torch.float32), **how)
+            idx, wts, *gate = ops.route_topk(None, None, self.correction, self.top,
+                                             logits=ops.linear(x, self.router_w, out_dtype=torch.float32), **how)
         else:
-            idx, wts = ops.route_topk(x, self.router, self.correction, self.top, **how)
-        return ops.routed_experts(x, self.w_gate, self.w_up, self.w_down, idx, wts, self.limit, self.act_alpha,
-                                  up_offset=self.up_offset, weight_input=self.weight_input,
-                                  **({"identity": self.identity} if self.identity else {}))
+            idx, wts, *gate = ops.route_topk(x, self.router, self.correction, self.top, **how)
+        y = ops.routed_experts(x, self.w_gate, self.w_up, self.w_down, idx, wts, self.limit, self.act_alpha,
+                               up_offset=self.up_offset, weight_input=self.weight_input,
+                               **({"identity": self.identity} if self.identity else {}))
+        return ops.OutputTerm(y, beside=(self.shared_expert.forward(ctx, x), gate[0])) if self.shared else y
 
 
 @register_feed_forward("table_experts")
