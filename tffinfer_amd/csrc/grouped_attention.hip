@@ -43,17 +43,19 @@ struct GroupedPre {
 
 // Blocks (token, y): y < q_blocks works through `per_q` query heads; the others through `per_kv` kv heads each: their key
 // and value rows into the token's slot.  Elements past a head's own size are zeros.  With a norm every block forms the
-// sum of squares it needs by itself, always in the same order.
+// sum of squares it needs by itself, always in the same order (its threads are as many whatever the step).
 #define GQ_THREADS 128
+#define GQ_WIDE 512      // threads with a norm, and where few tokens wait for one another's loads
 #define GQ_HEADS 8
 
 // 1 / sqrt(mean over x[0 .. n) of (x + bias)^2 + eps), the result in every thread of the block
+template <int NT>
 __device__ __forceinline__ float grouped_rms(const float* __restrict__ x, const float* __restrict__ bias, int n, float eps, bool vec,
                                              float* red) {
     float ss = 0.f;
     if (vec) {
 #pragma unroll 8
-        for (int c = threadIdx.x * 4; c < n; c += GQ_THREADS * 4) {
+        for (int c = threadIdx.x * 4; c < n; c += NT * 4) {
             float4 v = *reinterpret_cast<const float4*>(x + c);
             if (bias) {
                 const float4 b = *reinterpret_cast<const float4*>(bias + c);
@@ -62,7 +64,7 @@ __device__ __forceinline__ float grouped_rms(const float* __restrict__ x, const 
             ss = fmaf(v.x, v.x, fmaf(v.y, v.y, fmaf(v.z, v.z, fmaf(v.w, v.w, ss))));
         }
     } else {
-        for (int c = threadIdx.x; c < n; c += GQ_THREADS) {
+        for (int c = threadIdx.x; c < n; c += NT) {
             const float v = x[c] + (bias ? bias[c] : 0.f);
             ss = fmaf(v, v, ss);
         }
@@ -72,17 +74,17 @@ __device__ __forceinline__ float grouped_rms(const float* __restrict__ x, const 
     __syncthreads();
     ss = 0.f;
 #pragma unroll
-    for (int i = 0; i < GQ_THREADS / 64; ++i) ss += red[i];
+    for (int i = 0; i < NT / 64; ++i) ss += red[i];
     return 1.0f / sqrtf(ss / (float)n + eps);
 }
 
-template <typename TC>
-__global__ __launch_bounds__(GQ_THREADS) void grouped_qkv_store_kernel(
+template <typename TC, int NT>
+__global__ __launch_bounds__(NT) void grouped_qkv_store_kernel(
     const float* __restrict__ proj, size_t row, const float* __restrict__ cos_sin, int rot_dims, int pairing, int max_pos,
     float temp_coef, int temp_every, const GroupedPre pre, const int32_t* __restrict__ positions, const int32_t* __restrict__ slots,
     TC* __restrict__ q_out, TC* __restrict__ k_cache, TC* __restrict__ v_cache, int page_size, int H, int G, int D, int E, int P,
     int q_blocks, int per_q, int per_kv, int vec) {
-    __shared__ float red[GQ_THREADS / 64];
+    __shared__ float red[NT / 64];
     const int t = blockIdx.x, y = blockIdx.y, tid = threadIdx.x;
     const float* x = proj + (size_t)t * row;
     const int pos = max(positions[t], 0), tpos = min(pos, max(max_pos - 1, 0));
@@ -90,10 +92,10 @@ __global__ __launch_bounds__(GQ_THREADS) void grouped_qkv_store_kernel(
     const int half = P >> 1;                 // places of a head
     if (y < q_blocks) {
         const float temp = temp_coef != 0.f ? 1.0f + temp_coef * logf((float)((pos + 1) / temp_every + 1)) : 1.0f;
-        const float rr = pre.q_norm ? grouped_rms(x, pre.bias, H * D, pre.eps, vec, red) : 1.0f;
+        const float rr = pre.q_norm ? grouped_rms<NT>(x, pre.bias, H * D, pre.eps, vec, red) : 1.0f;
         TC* qo = q_out + (size_t)t * H * P;
         const int h0 = y * per_q, count = (min(H, h0 + per_q) - h0) * half;
-        for (int idx = tid; idx < count; idx += GQ_THREADS) {
+        for (int idx = tid; idx < count; idx += NT) {
             const int h = h0 + idx / half, p = idx % half, c0 = h * D;
             TC* const qh = qo + (size_t)h * P;
             grouped_pair(p, D, rot,
@@ -112,9 +114,9 @@ __global__ __launch_bounds__(GQ_THREADS) void grouped_qkv_store_kernel(
     const size_t ck = (size_t)H * D;
     const float* xk = x + ck;
     const float* bk = pre.bias ? pre.bias + ck : nullptr;
-    const float rr = pre.k_norm ? grouped_rms(xk, bk, G * D, pre.eps, vec, red) : 1.0f;
+    const float rr = pre.k_norm ? grouped_rms<NT>(xk, bk, G * D, pre.eps, vec, red) : 1.0f;
     const int g0 = (y - q_blocks) * per_kv, groups = min(G, g0 + per_kv) - g0;
-    for (int idx = tid; idx < groups * half; idx += GQ_THREADS) {
+    for (int idx = tid; idx < groups * half; idx += NT) {
         const int g = g0 + idx / half, p = idx % half, c0 = g * D;
         TC* const kd = k_cache + (((size_t)page * G + g) * page_size + off) * P;
         grouped_pair(p, D, rot,
@@ -125,7 +127,7 @@ __global__ __launch_bounds__(GQ_THREADS) void grouped_qkv_store_kernel(
             },
             [&](int e, float v) { kd[e] = from_f32<TC>(v); });
     }
-    for (int idx = tid; idx < groups * P; idx += GQ_THREADS) {
+    for (int idx = tid; idx < groups * P; idx += NT) {
         const int g = g0 + idx / P, e = idx % P;
         const size_t cv = ck + (size_t)G * D + (size_t)g * E + e;
         TC* const vd = v_cache + ((size_t)page * G + g) * P * page_size + off;
@@ -155,12 +157,15 @@ TFF_API int tff_grouped_qkv_store(const float* proj, size_t row, const float* co
     const int vec = D % 4 == 0 && row % 4 == 0 && ((uintptr_t)proj % 16) == 0 && ((uintptr_t)bias % 16) == 0;
     TFF_REQUIRE(q_blocks + kv_blocks <= 65535, "grouped_qkv_store: too many heads");
     const dim3 grid(T, q_blocks + kv_blocks);
-#define GQ_LAUNCH(TC)                                                                                                          \
-    grouped_qkv_store_kernel<TC><<<grid, GQ_THREADS, 0, s>>>(proj, row, cos_sin, rot_dims, pairing, max_pos, temp_coef, temp_every, \
-                                                             GroupedPre{bias, q_norm, k_norm, norm_eps}, positions, slots, (TC*)q_out, (TC*)k_cache, (TC*)v_cache, page_size, H, \
-                                                             G, D, E, P, q_blocks, per_q, per_kv, vec)
-    if (dtype == TFF_F32) GQ_LAUNCH(float);
-    else if (dtype == TFF_BF16) GQ_LAUNCH(bf16_t);
+    const bool wide = q_norm || k_norm || T < 128;
+#define GQ_LAUNCH(TC, NT)                                                                                                      \
+    grouped_qkv_store_kernel<TC, NT><<<grid, NT, 0, s>>>(proj, row, cos_sin, rot_dims, pairing, max_pos, temp_coef, temp_every, \
+                                                         GroupedPre{bias, q_norm, k_norm, norm_eps}, positions, slots, (TC*)q_out, \
+                                                         (TC*)k_cache, (TC*)v_cache, page_size, H, G, D, E, P, q_blocks, per_q, per_kv, vec)
+    if (dtype == TFF_F32 && wide) GQ_LAUNCH(float, GQ_WIDE);
+    else if (dtype == TFF_F32) GQ_LAUNCH(float, GQ_THREADS);
+    else if (dtype == TFF_BF16 && wide) GQ_LAUNCH(bf16_t, GQ_WIDE);
+    else if (dtype == TFF_BF16) GQ_LAUNCH(bf16_t, GQ_THREADS);
     else return tff_fail("grouped_qkv_store: unknown dtype %d", dtype);
 #undef GQ_LAUNCH
     return tff_check_launch("grouped_qkv_store");

@@ -273,7 +273,8 @@ TFF_API int tff_recurrence_few(const TffRecurrence* p, int max_tokens, tff_strea
 #define LRR 32       // inner size of the decay's second product that is worked through at a time
 
 // -log1p(e^(-|z|)) + min(z, 0) with the hardware's exponential and logarithm: log u for u = 1 + e is off by the rounding of
-// the sum, which the factor e / (u - 1) takes out again.
+// the sum, which the factor e / (u - 1) takes out again (D. Goldberg, "What Every Computer Scientist Should Know About
+// Floating-Point Arithmetic", theorem 4).
 __device__ __forceinline__ float lr_logsigmoid_fast(float z) {
     const float e = __expf(-fabsf(z)), u = 1.0f + e, d = u - 1.0f;
     return fminf(z, 0.f) - (d == 0.f ? e : __logf(u) * (e * __builtin_amdgcn_rcpf(d)));
